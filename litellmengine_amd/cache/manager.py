@@ -11,8 +11,8 @@ no zero-filling of reused pages (lengths say what is valid).  Different:
    slot; only new entries travel (the reference packs and uploads the whole
    table per layer per step, src/ops/attention.cu:959-1020);
  * cache layers with the same needs form a group with pages and tables of its
-   own; a group with a window gives pages back as soon as the window has
-   passed them;
+   own; a group with a window (or chunks) gives pages back as soon as the window
+   has passed them (the chunk is over), but for those of first tokens that are kept;
  * mixers may ask for fixed-size state rows, zeroed at admission.
 
 Pool layout of a group: [layer, page, elements of a page]; a page holds the fields of
@@ -68,7 +68,9 @@ class CacheGroup:
         self.window = spec.window
         self.max_requests = max_requests
         self.max_pages_per_request = max_pages_per_request
-        self.native = PageTables(num_pages, page_size, max_requests, max_pages_per_request, spec.window)
+        self.forgets = spec.span is not None  # pages are given back while their request lives
+        self.native = PageTables(num_pages, page_size, max_requests, max_pages_per_request, spec.window, spec.chunk,
+                                 spec.keep_first)
         self._lib, self._h = self.native.lib, self.native.handle
         self.pool = PagePool(num_pages, self.native)
         # One page more than the pool hands out: page `num_pages` is never written (it stays zero)
@@ -109,7 +111,8 @@ class CacheGroup:
 
     def trim(self, slot: int, length: int) -> None:
         """Give back the pages that no later query can see: with a window w the
-        next query (position `length`) sees keys >= length - w + 1."""
+        next query (position `length`) sees keys >= length - w + 1, with chunks of c
+        positions keys >= length // c * c; pages of kept first positions stay."""
         self._lib.lle_pt_trim(self._h, slot, length)
 
     def release(self, slot: int) -> None:
@@ -188,8 +191,8 @@ class CacheManager:
         of its own:
           * page size: `group_sizes[spec].page_size`, else the spec's own, else `page_size`;
           * pool: `group_sizes[spec].num_pages`, else pages for the same number of tokens; a
-            group with a window needs no more than the window and one step's tokens per
-            request, and is sized so when `max_tokens_per_step` says how long a step may be
+            group with a window (or chunks) needs no more than the window and one step's tokens per
+            request (and the kept first tokens), and is sized so when `max_tokens_per_step` says how long a step may be
             (the reference has one geometry and one pool for all layers,
             src/engine/paged_kv_cache.cpp:26-52).
         `max_pages_per_request` counts pages of `page_size` tokens: the longest request."""
@@ -218,9 +221,9 @@ class CacheManager:
             pages = asked.num_pages
             if pages is None:
                 pages = -(-capacity // P)
-                if spec.window is not None and max_tokens_per_step is not None:
-                    # positions past - window + 1 .. past + step - 1 of a request, wherever they start in a page
-                    each = -(-(spec.window - 1 + max_tokens_per_step) // P) + 1
+                if spec.span is not None and max_tokens_per_step is not None:
+                    # positions past - span + 1 .. past + step - 1 of a request, wherever they start in a page, and the kept first ones
+                    each = -(-(spec.span - 1 + max_tokens_per_step) // P) + 1 + -(-spec.keep_first // P)
                     pages = min(pages, max_requests * each)
             self.groups.append(CacheGroup(g, spec, ids, P, pages, max_requests, -(-longest // P), dtype, device))
         where: Dict[int, Tuple[CacheGroup, int]] = {}
@@ -342,7 +345,7 @@ class CacheManager:
         self._check_live(slot)
         self._length[slot] = new_len
         for group in self.groups:
-            if group.window is not None:
+            if group.forgets:
                 group.trim(slot, new_len)
 
     def commit_many(self, wants: Sequence[Tuple[int, int]]) -> None:
@@ -350,7 +353,7 @@ class CacheManager:
         for slot, new_len in wants:
             self._check_live(slot)
             self._length[slot] = new_len
-        if any(group.window is not None for group in self.groups):
+        if any(group.forgets for group in self.groups):
             n, slots, lens, keep = self._arrays(wants)
             for group in self.groups:
                 group._lib.lle_pt_trim_many(group._h, n, slots, lens)

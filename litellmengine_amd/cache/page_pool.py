@@ -18,7 +18,7 @@ OK, OUT_OF_PAGES, NO_SUCH_PAGE, FREED_TWICE, TOO_MANY_PAGES, BAD_TOKEN, NO_PAGE_
 
 _I, _P, _L = ctypes.c_int, ctypes.c_void_p, ctypes.c_int64
 _SIGNATURES = {
-    "lle_pt_create": ([_I, _I, _I, _I, _I], _P),
+    "lle_pt_create": ([_I, _I, _I, _I, _I, _I, _I], _P),
     "lle_pt_destroy": ([_P], None),
     "lle_pt_num_pages": ([_P], _I),
     "lle_pt_num_free": ([_P], _I),
@@ -66,12 +66,13 @@ class PageTables:
     tables of `max_requests` request slots."""
 
     def __init__(self, num_pages: int, page_size: int = 1, max_requests: int = 0, max_pages_per_request: int = 0,
-                 window: Optional[int] = None):
+                 window: Optional[int] = None, chunk: Optional[int] = None, keep_first: int = 0):
         if num_pages <= 0:
             raise ValueError("a page pool needs at least one page")
         self.lib = host_library()
         self.handle = self.lib.lle_pt_create(num_pages, page_size, max_requests, max_pages_per_request,
-                                             -1 if window is None else int(window))
+                                             -1 if window is None else int(window), int(chunk or 0),
+                                             int(keep_first))
         if not self.handle:
             raise ValueError("page tables need positive sizes")
 

@@ -3,6 +3,7 @@ from .visadra_config import VisadraConfig
 from .kezasun_config import KezasunConfig
 from .malilorn_config import MalilornConfig
 from .birelix_config import BirelixConfig
+from .telulorn_config import TelulornConfig
 from .registry import (
     Architecture,
     architecture_of,
@@ -20,6 +21,7 @@ __all__ = [
     "KezasunConfig",
     "MalilornConfig",
     "BirelixConfig",
+    "TelulornConfig",
     "FULL_ATTENTION",
     "SLIDING_ATTENTION",
     "architecture_of",

@@ -9,7 +9,9 @@
 // of the step's tokens are already in their pages, the block tables live on the
 // device, and every query token attends through them:
 //   query at cache position p (= kv_len - q_len + its index in the portion)
-//   sees keys lo..p,  lo = max(0, p - window + 1) with a window, else 0
+//   sees keys lo..p,  lo = max(0, p - window + 1) with a window, else 0, and with `keep_first`
+//   also the first keys, 0 .. min(keep_first, lo) - 1: every kernel walks that range first, with
+//   the same running maximum and sums, then lo..p
 //   score_j = (q . k_j) * scale;  softmax over j streamed in 32-bit (m, l, acc)
 //   kv head of q head h = h / (nq / nkv)                  (:577-668 for the maths)
 // A cache page holds K as [nkv][page_size][d], then V as [nkv][d][page_size].
@@ -43,7 +45,7 @@ __global__ __launch_bounds__(ATT_WAVES* LLE_WAVE) void paged_attention_generic_k
     const T* __restrict__ q, const T* __restrict__ kv_layer, const int32_t* __restrict__ block_tables,
     const int32_t* __restrict__ seq_slots, const int32_t* __restrict__ cu_tokens,
     const int32_t* __restrict__ kv_lens, const int32_t* __restrict__ token_seq, T* __restrict__ out, int nq,
-    int nkv, int d, int page_size, int64_t page_stride, int max_pages, int window, float scale,
+    int nkv, int d, int page_size, int64_t page_stride, int max_pages, int window, int keep_first, float scale,
     const float* __restrict__ sinks) {
     __shared__ float s_m[ATT_WAVES], s_l[ATT_WAVES];
     __shared__ float s_acc[ATT_WAVES][ATT_MAX_R * LLE_WAVE];
@@ -55,8 +57,9 @@ __global__ __launch_bounds__(ATT_WAVES* LLE_WAVE) void paged_attention_generic_k
     const int kv_len = kv_lens[s];
     const int q_start = cu_tokens[s];
     const int q_len = cu_tokens[s + 1] - q_start;
-    const int pos = kv_len - q_len + (int)(tok - q_start);
-    const int lo = window > 0 ? max(0, pos - window + 1) : 0;
+    const int query_pos = kv_len - q_len + (int)(tok - q_start);
+    const int query_lo = window > 0 ? max(0, query_pos - window + 1) : 0;
+    const int kept = min(keep_first, query_lo);
     const int kvh = h / (nq / nkv);
     const int32_t* table = block_tables + (int64_t)seq_slots[s] * max_pages;
 
@@ -75,6 +78,8 @@ __global__ __launch_bounds__(ATT_WAVES* LLE_WAVE) void paged_attention_generic_k
     // (keys j0 .. j0 + ATT_KEYS - 1 lie in one page, side by side, when the steps start at a
     // multiple of ATT_KEYS and pages hold a multiple of it; the last step of a row may reach
     // past `pos`, but not past its page)
+    for (int range = kept > 0 ? 0 : 1; range < 2; ++range) {
+    const int lo = range == 0 ? 0 : query_lo, pos = range == 0 ? kept - 1 : query_pos;
     const bool keys_in_one_piece = lo % ATT_KEYS == 0 && page_size % ATT_KEYS == 0;
     for (int j0 = lo + wave * ATT_KEYS; j0 <= pos; j0 += ATT_WAVES * ATT_KEYS) {
         const T* vp[ATT_KEYS];
@@ -145,6 +150,7 @@ __global__ __launch_bounds__(ATT_WAVES* LLE_WAVE) void paged_attention_generic_k
         }
         m = new_m;
     }
+    }
     if (lane == 0) {
         s_m[wave] = m;
         s_l[wave] = l;
@@ -171,20 +177,21 @@ extern "C" int lle_paged_attention_generic(const void* q, const void* kv_layer, 
                                            const void* seq_slots, const void* cu_tokens, const void* kv_lens,
                                            const void* token_seq, void* out, int N, int nq, int nkv, int d,
                                            int page_size, int64_t page_stride, int max_pages, int window,
-                                           float scale, int dtype, const void* sinks, hipStream_t stream) {
+                                           int keep_first, float scale, int dtype, const void* sinks,
+                                           hipStream_t stream) {
     if (N <= 0) return 0;
-    if (d > ATT_MAX_R * LLE_WAVE) return (int)hipErrorInvalidValue;
+    if (keep_first < 0 || d > ATT_MAX_R * LLE_WAVE) return (int)hipErrorInvalidValue;
     dim3 grid(N, nq);
     if (dtype == LLE_F32)
         paged_attention_generic_kernel<float><<<grid, ATT_WAVES * LLE_WAVE, 0, stream>>>(
             (const float*)q, (const float*)kv_layer, (const int32_t*)block_tables, (const int32_t*)seq_slots,
             (const int32_t*)cu_tokens, (const int32_t*)kv_lens, (const int32_t*)token_seq, (float*)out, nq, nkv, d,
-            page_size, page_stride, max_pages, window, scale, (const float*)sinks);
+            page_size, page_stride, max_pages, window, keep_first, scale, (const float*)sinks);
     else
         paged_attention_generic_kernel<bf16_t><<<grid, ATT_WAVES * LLE_WAVE, 0, stream>>>(
             (const bf16_t*)q, (const bf16_t*)kv_layer, (const int32_t*)block_tables, (const int32_t*)seq_slots,
             (const int32_t*)cu_tokens, (const int32_t*)kv_lens, (const int32_t*)token_seq, (bf16_t*)out, nq, nkv,
-            d, page_size, page_stride, max_pages, window, scale, (const float*)sinks);
+            d, page_size, page_stride, max_pages, window, keep_first, scale, (const float*)sinks);
     LLE_RETURN_LAUNCH_STATUS();
 }
 
@@ -243,6 +250,23 @@ struct RowState {
     float m[RT], l[RT];            // running maximum (base 2) and this lane's share of the sum
 };
 
+// the steps that every row of a tile sees whole (the rows' lo and pos are what they see of the range walked now)
+template <int DK, int RT>
+__device__ __forceinline__ void set_open_range(RowState<DK, RT>& st, const RowInfo (&row)[RT]) {
+#pragma unroll
+    for (int t = 0; t < RT; ++t) {
+        int lo_max = row[t].q ? row[t].lo : 0, pos_min = row[t].q ? row[t].pos : 0x7fffffff;
+#pragma unroll
+        for (int off = 1; off < LLE_WAVE; off <<= 1) {
+            lo_max = max(lo_max, __shfl_xor(lo_max, off, LLE_WAVE));
+            pos_min = min(pos_min, __shfl_xor(pos_min, off, LLE_WAVE));
+        }
+        // (the same in every lane: kept in scalar registers, so that the test is a scalar branch)
+        st.open_lo[t] = __builtin_amdgcn_readfirstlane(lo_max);
+        st.open_hi[t] = __builtin_amdgcn_readfirstlane(pos_min == 0x7fffffff ? -1 : pos_min);
+    }
+}
+
 // LOAD_Q = false: the caller has filled st.qv itself
 template <int DK, int RT, bool LOAD_Q = true>
 __device__ __forceinline__ void init_rows(RowState<DK, RT>& st, const RowInfo (&row)[RT]) {
@@ -264,16 +288,8 @@ __device__ __forceinline__ void init_rows(RowState<DK, RT>& st, const RowInfo (&
         for (int n = 0; n < 2 * DK; ++n) st.o[t][n] = f32x4{0.f, 0.f, 0.f, 0.f};
         st.m[t] = NEG_BIG;
         st.l[t] = 0.f;
-        int lo_max = row[t].q ? row[t].lo : 0, pos_min = row[t].q ? row[t].pos : 0x7fffffff;
-#pragma unroll
-        for (int off = 1; off < LLE_WAVE; off <<= 1) {
-            lo_max = max(lo_max, __shfl_xor(lo_max, off, LLE_WAVE));
-            pos_min = min(pos_min, __shfl_xor(pos_min, off, LLE_WAVE));
-        }
-        // (the same in every lane: kept in scalar registers, so that the test is a scalar branch)
-        st.open_lo[t] = __builtin_amdgcn_readfirstlane(lo_max);
-        st.open_hi[t] = __builtin_amdgcn_readfirstlane(pos_min == 0x7fffffff ? -1 : pos_min);
     }
+    set_open_range<DK, RT>(st, row);
     // The rows of Q are waited for here, once.  Left pending, their first use lies inside the
     // key loop, where the wait for them also waits for the K/V loads just issued for a later
     // step: the loop would run at the latency of memory.
@@ -416,7 +432,9 @@ struct StepOperands {
 // `before_keys()` runs when the first table lookup is on its way and no operand is asked for yet:
 // what the caller loads there travels beside the lookup, what it stores there is stored before
 // this wavefront reads any key.  `after_first_loads()` runs once the first two steps are asked for.
-template <int DK, int RT, bool LOAD_Q = true, typename BeforeKeys, typename AfterFirstLoads>
+// A second range of keys is walked by a call with FIRST = false (the rows' lo and pos are the range's
+// then, what the first call has summed up stays); all calls but the last have LAST = false.
+template <int DK, int RT, bool LOAD_Q = true, bool FIRST = true, bool LAST = true, typename BeforeKeys, typename AfterFirstLoads>
 __device__ __forceinline__ void attend_rows(RowState<DK, RT>& st, const RowInfo (&row)[RT],
                                             const bf16_t* kv_layer, const int32_t* __restrict__ table,
                                             int kvh, int nkv, int P, int64_t page_stride, int step_begin,
@@ -425,7 +443,8 @@ __device__ __forceinline__ void attend_rows(RowState<DK, RT>& st, const RowInfo 
     constexpr int D = DK * 32;
     const int lane = threadIdx.x % LLE_WAVE;
     const int c = lane / 16, r16 = lane % 16;
-    init_rows<DK, RT, LOAD_Q>(st, row);
+    if constexpr (FIRST) init_rows<DK, RT, LOAD_Q>(st, row);
+    else set_open_range<DK, RT>(st, row);
     // the lane's keys of tile x lie in the 16-key half r16 / 8 of the step, its eight V keys in half c / 2
     const int k_half = r16 / 8, v_half = c / 2;
     const int64_t k_lane[2] = {(int64_t)kvh * P * D + (int64_t)(KEY_OF_ROW(r16, 0) % 16) * D + 8 * c,
@@ -484,7 +503,7 @@ __device__ __forceinline__ void attend_rows(RowState<DK, RT>& st, const RowInfo 
         multiply(odd, step + step_stride);
         load(odd);
     }
-    finish_rows<DK, RT>(st);
+    if constexpr (LAST) finish_rows<DK, RT>(st);
 }
 
 // row `r` of the (token, head-in-group) rows of one request and kv head
@@ -687,13 +706,14 @@ __device__ __forceinline__ void fused_kv_write(const FusedQKV& f, int64_t tok, i
 #ifndef DEC_WAVES
 #define DEC_WAVES 4
 #endif
-template <int DK, bool FUSED>
+template <int DK, bool FUSED, bool KEEP>
 __global__ __launch_bounds__(DEC_WAVES* LLE_WAVE) void mfma_decode_kernel(
     const bf16_t* __restrict__ q, bf16_t* kv_layer, const int32_t* __restrict__ block_tables,
     const int32_t* __restrict__ seq_slots, const int32_t* __restrict__ cu_tokens,
     const int32_t* __restrict__ kv_lens, bf16_t* __restrict__ out, float* __restrict__ ws_o,
     float* __restrict__ ws_ml, int ws_stride, int nq, int nkv, int P, int64_t page_stride, int max_pages,
-    int window, float scale_log2, FusedQKV fused, const float* __restrict__ sinks) {
+    int window, float scale_log2, FusedQKV fused, const float* __restrict__ sinks, int keep_first) {
+    static_assert(!(FUSED && KEEP), "kept first keys: the launch that reads ready-made queries");
     constexpr int D = DK * 32;
     extern __shared__ float smem[];  // [waves][16][D] acc, then [waves][16] m, [waves][16] l
     float* s_o = smem;
@@ -765,6 +785,22 @@ __global__ __launch_bounds__(DEC_WAVES* LLE_WAVE) void mfma_decode_kernel(
                 }
             },
             [&]() { qrow.finish(st.qv[0], r16 < nrows, fused); });
+    } else if constexpr (KEEP) {
+        // the kept first keys are the first split's work (few steps)
+        init_rows<DK, 1, true>(st, row);
+        const int kept = min(keep_first, max(0, hi - window + 1));  // of the row that sees the most of them
+        if (split == 0 && kept > 0) {
+            const RowInfo main_row = row[0];
+            if (row[0].q) row[0].pos = min(keep_first, row[0].lo) - 1;
+            row[0].lo = 0;
+            attend_rows<DK, 1, true, false, false>(
+                st, row, kv_layer, table, kvh, nkv, P, page_stride, wave, (kept + KSTEP - 1) / KSTEP, DEC_WAVES, 0, kept - 1,
+                scale_log2, []() {}, []() {});
+            row[0] = main_row;
+        }
+        attend_rows<DK, 1, true, false, true>(
+            st, row, kv_layer, table, kvh, nkv, P, page_stride, sb + wave, se, DEC_WAVES, lo_min, hi_loads, scale_log2,
+            []() {}, []() {});
     } else {
         attend_rows<DK, 1, true>(
             st, row, kv_layer, table, kvh, nkv, P, page_stride, sb + wave, se, DEC_WAVES, lo_min, hi_loads, scale_log2,
@@ -897,14 +933,14 @@ __global__ __launch_bounds__(LLE_WAVE) void mfma_combine_kernel(const float* __r
 #define PRE_RT_MAX 2
 #endif
 #define PRE_RT_OF(DK) ((DK) <= 4 ? PRE_RT_MAX : 1)
-template <int DK, int PRE_RT, int PRE_WAVES = 4>
+template <int DK, int PRE_RT, int PRE_WAVES, bool KEEP>
 // (heads over 192 elements need more than the 256 registers a lane that two workgroups a CU leave)
 __global__ __launch_bounds__(PRE_WAVES* LLE_WAVE, DK <= 6 ? 2 : 1) void mfma_prefill_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ kv_layer, const int32_t* __restrict__ block_tables,
     const int32_t* __restrict__ seq_slots, const int32_t* __restrict__ cu_tokens,
     const int32_t* __restrict__ kv_lens, bf16_t* __restrict__ out, float* __restrict__ ws_o,
     float* __restrict__ ws_ml, int ws_stride, int nsplit, int nq, int nkv, int P, int64_t page_stride, int max_pages,
-    int window, float scale_log2, int complement_order, const float* __restrict__ sinks) {
+    int window, float scale_log2, int complement_order, const float* __restrict__ sinks, int keep_first) {
     constexpr int D = DK * 32;
     static_assert(PRE_RT <= PRE_RT_OF(DK), "the accumulators of two row tiles fit the registers up to heads of 128");
     constexpr int PRE_ROWS = PRE_WAVES * 16 * PRE_RT;
@@ -939,9 +975,9 @@ __global__ __launch_bounds__(PRE_WAVES* LLE_WAVE, DK <= 6 ? 2 : 1) void mfma_pre
 
     // the workgroup's key range, and this wavefront's own
     const int block_last_row = min(nrows, block_row0 + PRE_ROWS) - 1;
-    const int hi = past + block_last_row / G;
+    int hi = past + block_last_row / G;
     const int block_first_pos = past + block_row0 / G;
-    const int lo_min = window > 0 ? max(0, block_first_pos - window + 1) : 0;
+    int lo_min = window > 0 ? max(0, block_first_pos - window + 1) : 0;
     int first_step = lo_min / KSTEP, end_step = hi / KSTEP + 1;
     if (nsplit > 1) {  // this workgroup's share of the steps (it may be empty)
         const int per_split = (end_step - first_step + nsplit - 1) / nsplit;
@@ -985,7 +1021,7 @@ __global__ __launch_bounds__(PRE_WAVES* LLE_WAVE, DK <= 6 ? 2 : 1) void mfma_pre
     // page and offset of the next half are carried along instead of divided out (the page size
     // is no constant).  A half wholly outside [lo_min, hi] may lie in a page that is not there:
     // the page index is clamped to those of keys that are.
-    const int page_lo = lo_min / P, page_hi = hi / P;
+    int page_lo = lo_min / P, page_hi = hi / P;
     int look_page = __builtin_amdgcn_readfirstlane((first_step * KSTEP) / P);
     int look_off = __builtin_amdgcn_readfirstlane((first_step * KSTEP) % P);
     int page_id[2], page_off[2];
@@ -1001,7 +1037,7 @@ __global__ __launch_bounds__(PRE_WAVES* LLE_WAVE, DK <= 6 ? 2 : 1) void mfma_pre
             }
         }
     };
-    lookup();
+    if constexpr (!KEEP) lookup();
     // Piece `piece` of a tile: the wavefront-sized run it lies in belongs to ONE 16-key half
     // (half = run / DK), so the half's page is the same for the whole wavefront and its address
     // stays in scalar registers; what differs between the threads is fixed for the kernel.
@@ -1068,6 +1104,39 @@ __global__ __launch_bounds__(PRE_WAVES* LLE_WAVE, DK <= 6 ? 2 : 1) void mfma_pre
         __syncthreads();
     };
 
+    // With kept first keys the walk has two ranges: those keys (the first split's work), then the window's.
+    // What the loops above and below know of a range is set anew for each; the rows' sums run on.
+    [[maybe_unused]] const int w_hi = hi, w_lo_min = lo_min, w_first = first_step, w_end = end_step, w_my_first = my_first,
+                               w_my_end = my_end;
+    auto set_range = [&](int range) {
+        const int kept = min(keep_first, max(0, w_hi - window + 1));  // of the row that sees the most of them
+#pragma unroll
+        for (int t = 0; t < PRE_RT; ++t) {
+            row[t] = make_row(q, row0 + 16 * t + r16, nrows, G, q_start, past, nq, kvh, D, window);
+            if (range == 0) {
+                if (row[t].q) row[t].pos = min(keep_first, row[t].lo) - 1;
+                row[t].lo = 0;
+            }
+        }
+        hi = range == 0 ? max(0, kept - 1) : w_hi;
+        lo_min = range == 0 ? 0 : w_lo_min;
+        first_step = range == 0 ? 0 : w_first;
+        end_step = range == 0 ? (split == 0 ? (kept + KSTEP - 1) / KSTEP : 0) : w_end;
+        my_first = __builtin_amdgcn_readfirstlane(range == 0 ? 0 : w_my_first);
+        my_end = __builtin_amdgcn_readfirstlane(range == 0 ? (row0 < nrows ? end_step : 0) : w_my_end);
+        page_lo = lo_min / P;
+        page_hi = hi / P;
+        look_page = __builtin_amdgcn_readfirstlane((first_step * KSTEP) / P);
+        look_off = __builtin_amdgcn_readfirstlane((first_step * KSTEP) % P);
+        set_open_range<DK, PRE_RT>(st, row);
+        lookup();
+    };
+
+    for (int range = KEEP ? 0 : 1; range < 2; ++range) {
+    if constexpr (KEEP) {
+        set_range(range);
+        if (first_step >= end_step) continue;  // (the same for the whole workgroup: nothing of this range is its work)
+    }
     if constexpr (DMA) {
         // Tiles go from the pages straight into LDS (no registers, no stores by the wavefronts):
         // a wavefront's load writes 1 KB of LDS in lane order (M0 holds where), so the swizzle is
@@ -1182,6 +1251,7 @@ __global__ __launch_bounds__(PRE_WAVES* LLE_WAVE, DK <= 6 ? 2 : 1) void mfma_pre
             one_step(step + 1, 1, std::integral_constant<int, 0>{});  // multiplies nothing past my_end
         }
     }
+    }
     finish_rows<DK, PRE_RT>(st);
 #pragma unroll
     for (int t = 0; t < PRE_RT; ++t) {
@@ -1237,7 +1307,7 @@ __global__ __launch_bounds__(F32_WAVES* LLE_WAVE) void mfma_f32_attention_kernel
     const int32_t* __restrict__ seq_slots, const int32_t* __restrict__ cu_tokens,
     const int32_t* __restrict__ kv_lens, float* __restrict__ out, float* __restrict__ ws_o,
     float* __restrict__ ws_ml, int nsplit, int nq, int nkv, int P, int64_t page_stride, int max_pages, int window,
-    float scale_log2, const float* __restrict__ sinks) {
+    int keep_first, float scale_log2, const float* __restrict__ sinks) {
     constexpr int D = 16 * DQ;
     extern __shared__ float smem[];  // [waves][16][D] acc, then [waves][16] m, [waves][16] l
     float* s_o = smem;
@@ -1266,8 +1336,8 @@ __global__ __launch_bounds__(F32_WAVES* LLE_WAVE) void mfma_f32_attention_kernel
     const bool exists = row < nrows;
     const int tok = exists ? row / G : 0, g = exists ? row - tok * G : 0;
     const int64_t head_row = (int64_t)(q_start + tok) * nq + kvh * G + g;
-    const int pos = exists ? past + tok : -1;
-    const int lo = (exists && window > 0) ? max(0, pos - window + 1) : 0;
+    int pos = exists ? past + tok : -1;
+    int lo = (exists && window > 0) ? max(0, pos - window + 1) : 0;
     f32x4 qf[DQ];
 #pragma unroll
     for (int i = 0; i < DQ; ++i)
@@ -1275,10 +1345,12 @@ __global__ __launch_bounds__(F32_WAVES* LLE_WAVE) void mfma_f32_attention_kernel
 
     // the keys of this wavefront's tile, in steps of 16, and its share of them
     int step_begin = 0, step_end = 0, step_stride = 1;
+    int kept_end = 0;  // steps of the kept first keys, which are the first split's work
     if (wave_has_rows) {
         const int last_row = min(nrows, row0 + 16) - 1;
         const int hi = past + last_row / G;
         const int lo_tile = window > 0 ? max(0, past + row0 / G - window + 1) : 0;
+        if (keep_first > 0 && split == 0) kept_end = (min(keep_first, max(0, hi - window + 1)) + F32_KEYS - 1) / F32_KEYS;
         const int first = lo_tile / F32_KEYS, end = hi / F32_KEYS + 1;
         const int per_split = (end - first + nsplit - 1) / nsplit;
         step_begin = first + split * per_split;
@@ -1342,6 +1414,12 @@ __global__ __launch_bounds__(F32_WAVES* LLE_WAVE) void mfma_f32_attention_kernel
             for (int e = 0; e < 4; ++e) o[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(vf[buf][n][e], p[e], o[n], 0, 0, 0);
         }
     };
+    const int w_pos = pos, w_lo = lo, w_begin = step_begin, w_end = step_end;
+    for (int range = kept_end > 0 ? 0 : 1; range < 2; ++range) {
+    pos = range == 0 ? (exists ? min(keep_first, w_lo) - 1 : -1) : w_pos;
+    lo = range == 0 ? 0 : w_lo;
+    step_begin = range == 0 ? (few ? wave : 0) : w_begin;
+    step_end = range == 0 ? kept_end : w_end;
     if constexpr (NBUF == 2) {
         // the operands of the next step are asked for before this one is multiplied
         if (step_begin < step_end) load(0, step_begin);
@@ -1358,6 +1436,7 @@ __global__ __launch_bounds__(F32_WAVES* LLE_WAVE) void mfma_f32_attention_kernel
             load(0, step);
             multiply(0, step);
         }
+    }
     }
     l += __shfl_xor(l, 16, LLE_WAVE);
     l += __shfl_xor(l, 32, LLE_WAVE);
@@ -1449,13 +1528,14 @@ extern "C" int lle_paged_attention_mfma_f32(const void* q, const void* kv_layer,
                                             const void* seq_slots, const void* cu_tokens, const void* kv_lens,
                                             void* out, void* ws_o, void* ws_ml, int N, int S, int nq, int nkv, int d,
                                             int page_size, int64_t page_stride, int max_pages, int window,
-                                            float scale, int row_blocks, int nsplit, const void* sinks,
+                                            int keep_first, float scale, int row_blocks, int nsplit, const void* sinks,
                                             hipStream_t stream) {
     if (N <= 0) return 0;
     if (d % 16 != 0 || d > 256 || d <= 0 || page_size % 16 != 0 || nq % nkv != 0) return (int)hipErrorInvalidValue;
     if (S > 65535 || nkv <= 0 || row_blocks < 1 || nsplit < 1 || nsplit > 64 || (int64_t)row_blocks * nsplit > 65535)
         return (int)hipErrorInvalidValue;
     if (nsplit > 1 && (!ws_o || !ws_ml)) return (int)hipErrorInvalidValue;
+    if (keep_first < 0 || (keep_first > 0 && window <= 0)) return (int)hipErrorInvalidValue;
     const float scale_log2 = scale * 1.44269504088896340736f;
     const dim3 grid(nkv, row_blocks * nsplit, S);
     const size_t smem = (size_t)(F32_WAVES * 16 * d + 2 * F32_WAVES * 16) * sizeof(float);
@@ -1469,7 +1549,7 @@ extern "C" int lle_paged_attention_mfma_f32(const void* q, const void* kv_layer,
         mfma_f32_attention_kernel<DQV><<<grid, F32_WAVES * LLE_WAVE, smem, stream>>>(                             \
             (const float*)q, (const float*)kv_layer, (const int32_t*)block_tables, (const int32_t*)seq_slots,     \
             (const int32_t*)cu_tokens, (const int32_t*)kv_lens, (float*)out, (float*)ws_o, (float*)ws_ml, nsplit, \
-            nq, nkv, page_size, page_stride, max_pages, window, scale_log2, (const float*)sinks);                \
+            nq, nkv, page_size, page_stride, max_pages, window, keep_first, scale_log2, (const float*)sinks);    \
         break;
     switch (d / 16) {
         LLE_F32_CASE(1) LLE_F32_CASE(2) LLE_F32_CASE(3) LLE_F32_CASE(4) LLE_F32_CASE(5) LLE_F32_CASE(6)
@@ -1496,21 +1576,22 @@ static int compute_units() {
     return cached[dev];
 }
 
-template <int DK, bool FUSED>
+template <int DK, bool FUSED, bool KEEP>
 static int launch_decode(const bf16_t* q, bf16_t* kv_layer, const int32_t* block_tables, const int32_t* seq_slots,
                          const int32_t* cu_tokens, const int32_t* kv_lens, bf16_t* out, float* ws_o, float* ws_ml,
                          int ws_stride, int S, int nq, int nkv, int P, int64_t page_stride, int max_pages, int window,
-                         float scale_log2, int nsplit, const FusedQKV& fused, const float* sinks, hipStream_t stream) {
+                         float scale_log2, int nsplit, const FusedQKV& fused, const float* sinks, int keep_first,
+                         hipStream_t stream) {
     constexpr int D = DK * 32;
     const size_t smem = (size_t)(DEC_WAVES * 16 * D + 2 * DEC_WAVES * 16) * sizeof(float);
     if (smem > 64 * 1024) {
-        hipError_t e = hipFuncSetAttribute((const void*)mfma_decode_kernel<DK, FUSED>,
+        hipError_t e = hipFuncSetAttribute((const void*)mfma_decode_kernel<DK, FUSED, KEEP>,
                                            hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
         if (e != hipSuccess) return (int)e;
     }
-    mfma_decode_kernel<DK, FUSED><<<dim3(S, nkv, nsplit), DEC_WAVES * LLE_WAVE, smem, stream>>>(
+    mfma_decode_kernel<DK, FUSED, KEEP><<<dim3(S, nkv, nsplit), DEC_WAVES * LLE_WAVE, smem, stream>>>(
         q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out, ws_o, ws_ml, ws_stride, nq, nkv, P,
-        page_stride, max_pages, window, scale_log2, fused, sinks);
+        page_stride, max_pages, window, scale_log2, fused, sinks, keep_first);
     return 0;
 }
 
@@ -1545,13 +1626,13 @@ static int launch_mfma(const bf16_t* q, bf16_t* kv_layer, const int32_t* block_t
                        const int32_t* token_seq, bf16_t* out, float* ws_o, float* ws_ml, int N, int S, int nq,
                        int nkv, int P, int64_t page_stride, int max_pages, int window, float scale_log2,
                        int run_decode, int nsplit_decode, int run_prefill, int nsplit_prefill, int max_q_len,
-                       int prefill_form, const FusedQKV& fused, const float* sinks, hipStream_t stream) {
+                       int prefill_form, const FusedQKV& fused, const float* sinks, int keep_first, hipStream_t stream) {
     constexpr int D = DK * 32;
     const int G = nq / nkv;
     if (!run_decode) nsplit_decode = 1;
     if (!run_prefill) nsplit_prefill = 1;
     const int ws_stride = nsplit_decode > nsplit_prefill ? nsplit_decode : nsplit_prefill;
-    if (fused.qkv && (run_prefill || !run_decode || DK % 2 != 0)) return (int)hipErrorInvalidValue;
+    if (fused.qkv && (run_prefill || !run_decode || DK % 2 != 0 || keep_first)) return (int)hipErrorInvalidValue;
     // both kinds in one batch: the decode kernel goes to the side stream, forked from and joined to `stream`
     SideLane* lane = (run_decode && run_prefill) ? side_lane() : nullptr;
     hipStream_t prefill_stream = stream;
@@ -1562,17 +1643,21 @@ static int launch_mfma(const bf16_t* q, bf16_t* kv_layer, const int32_t* block_t
     if (lane) stream = lane->stream;  // for the decode kernel below
     if (run_decode) {
         int e;
-        if constexpr (DK % 2 == 0) {
-            e = fused.qkv ? launch_decode<DK, true>(q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out, ws_o,
+        if (keep_first > 0) {
+            e = launch_decode<DK, false, true>(q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out, ws_o, ws_ml,
+                                               ws_stride, S, nq, nkv, P, page_stride, max_pages, window, scale_log2,
+                                               nsplit_decode, fused, sinks, keep_first, stream);
+        } else if constexpr (DK % 2 == 0) {
+            e = fused.qkv ? launch_decode<DK, true, false>(q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out, ws_o,
                                                     ws_ml, ws_stride, S, nq, nkv, P, page_stride, max_pages, window,
-                                                    scale_log2, nsplit_decode, fused, sinks, stream)
-                          : launch_decode<DK, false>(q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out,
+                                                    scale_log2, nsplit_decode, fused, sinks, 0, stream)
+                          : launch_decode<DK, false, false>(q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out,
                                                      ws_o, ws_ml, ws_stride, S, nq, nkv, P, page_stride, max_pages,
-                                                     window, scale_log2, nsplit_decode, fused, sinks, stream);
+                                                     window, scale_log2, nsplit_decode, fused, sinks, 0, stream);
         } else {
-            e = launch_decode<DK, false>(q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out, ws_o, ws_ml,
+            e = launch_decode<DK, false, false>(q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out, ws_o, ws_ml,
                                          ws_stride, S, nq, nkv, P, page_stride, max_pages, window, scale_log2,
-                                         nsplit_decode, fused, sinks, stream);
+                                         nsplit_decode, fused, sinks, 0, stream);
         }
         if (e != 0) {
             if (lane) (void)hipStreamSynchronize(lane->stream);
@@ -1596,9 +1681,14 @@ static int launch_mfma(const bf16_t* q, bf16_t* kv_layer, const int32_t* block_t
             constexpr int PRE_ROWS = WAVES * 16 * RT;
             const int blocks = (rows + PRE_ROWS - 1) / PRE_ROWS;
             const int64_t workgroups = (int64_t)nkv * blocks * nsplit_prefill * S;
-            mfma_prefill_kernel<DK, RT, WAVES><<<dim3(nkv, blocks * nsplit_prefill, S), WAVES * LLE_WAVE, 0, stream>>>(
-                q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out, ws_o, ws_ml, ws_stride, nsplit_prefill,
-                nq, nkv, P, page_stride, max_pages, window, scale_log2, workgroups <= 2 * compute_units() ? 1 : 0, sinks);
+            auto go = [&](auto kernel) {
+                kernel<<<dim3(nkv, blocks * nsplit_prefill, S), WAVES * LLE_WAVE, 0, stream>>>(
+                    q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out, ws_o, ws_ml, ws_stride, nsplit_prefill,
+                    nq, nkv, P, page_stride, max_pages, window, scale_log2, workgroups <= 2 * compute_units() ? 1 : 0, sinks,
+                    keep_first);
+            };
+            if (keep_first > 0) go(mfma_prefill_kernel<DK, RT, WAVES, true>);
+            else go(mfma_prefill_kernel<DK, RT, WAVES, false>);
         };
         using Four = std::integral_constant<int, 4>;
         if (DK == 4 && prefill_form == 3) {
@@ -1631,8 +1721,10 @@ static int paged_attention_mfma(const void* q, void* kv_layer, const void* block
                                 void* ws_o, void* ws_ml, int N, int S, int nq, int nkv, int d, int page_size,
                                 int64_t page_stride, int max_pages, int window, float scale, int run_decode,
                                 int nsplit_decode, int run_prefill, int nsplit_prefill, int max_q_len,
-                                int prefill_form, const FusedQKV& fused, const float* sinks, hipStream_t stream) {
+                                int prefill_form, const FusedQKV& fused, const float* sinks, int keep_first,
+                                hipStream_t stream) {
     if (N <= 0) return 0;
+    if (keep_first < 0 || (keep_first > 0 && window <= 0)) return (int)hipErrorInvalidValue;
     if (d % 32 != 0 || d > 256 || page_size % 16 != 0 || nq % nkv != 0) return (int)hipErrorInvalidValue;
     if (S > 65535 || nkv > 65535 || page_stride < 0 || page_stride >= ((int64_t)1 << 32)) return (int)hipErrorInvalidValue;
     if (nsplit_decode < 1 || nsplit_decode > 64 || nsplit_prefill < 1 || nsplit_prefill > 64)
@@ -1644,7 +1736,7 @@ static int paged_attention_mfma(const void* q, void* kv_layer, const void* block
                                 (const int32_t*)seq_slots, (const int32_t*)cu_tokens, (const int32_t*)kv_lens,      \
                                 (const int32_t*)token_seq, (bf16_t*)out, (float*)ws_o, (float*)ws_ml, N, S, nq, nkv, \
                                 page_size, page_stride, max_pages, window, scale_log2, run_decode, nsplit_decode,   \
-                                run_prefill, nsplit_prefill, max_q_len, prefill_form, fused, sinks, stream);
+                                run_prefill, nsplit_prefill, max_q_len, prefill_form, fused, sinks, keep_first, stream);
     switch (d / 32) {
         LLE_ATT_CASE(1)
         LLE_ATT_CASE(2)
@@ -1665,12 +1757,12 @@ extern "C" int lle_paged_attention_mfma(const void* q, const void* kv_layer, con
                                         int nq, int nkv, int d, int page_size, int64_t page_stride, int max_pages,
                                         int window, float scale, int run_decode, int nsplit_decode, int run_prefill,
                                         int nsplit_prefill, int max_q_len, int prefill_form, const void* sinks,
-                                        hipStream_t stream) {
+                                        int keep_first, hipStream_t stream) {
     const FusedQKV none = {};
     return paged_attention_mfma(q, (void*)kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, token_seq, out, ws_o,
                                 ws_ml, N, S, nq, nkv, d, page_size, page_stride, max_pages, window, scale, run_decode,
                                 nsplit_decode, run_prefill, nsplit_prefill, max_q_len, prefill_form, none,
-                                (const float*)sinks, stream);
+                                (const float*)sinks, keep_first, stream);
 }
 
 // Decode steps only (every request has at most 16 / group tokens), head_dim a multiple of 64, a
@@ -1699,5 +1791,5 @@ extern "C" int lle_qk_norm_rope_attention_decode(const void* qkv, const void* sl
     fused.write_kv = write_kv;
     return paged_attention_mfma(nullptr, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, token_seq, out, ws_o,
                                 ws_ml, N, S, nq, nkv, d, page_size, page_stride, max_pages, window, scale, 1,
-                                nsplit_decode, 0, 1, 1, 0, fused, nullptr, stream);
+                                nsplit_decode, 0, 1, 1, 0, fused, nullptr, 0, stream);
 }

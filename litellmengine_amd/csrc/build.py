@@ -37,6 +37,8 @@ LIBRARIES: Dict[str, List[str]] = {
     "moe": ["moe.hip"],
     "wkv": ["wkv.hip"],
     "delta": ["delta.hip"],
+    "gla": ["gla.hip"],
+    "talking": ["talking.hip"],
     "probe": ["probe.hip"],
 }
 # libraries without GPU code: compiled with the host's C++ compiler

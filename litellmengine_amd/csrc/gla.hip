@@ -1,0 +1,283 @@
+// Gated linear attention: a recurrence with a matrix state per head whose rows decay each at a rate of its own,
+// made from the data.
+//
+//   decay_t = sigmoid(z_t)^(1 / tau),  z_t = a2 low_t + b       per head and key channel, 32-bit        gla_decay
+//   S[i][j] <- decay_t[i] S[i][j] + k_t[i] v_t[j]                                                       gla_scan
+//   o_t[j]   = sum_i q_scale q_t[i] S[i][j]                     (the read-out sees the token's own write)
+//   y_t      = o_t / rms(o_t) * norm_w * silu(g_t)              per head, eps inside the root, norm_w [vdim] for all heads
+//
+// The state is float32 [head][key i][value j] per request slot.  A row of `u` holds q [H dim], k [H dim], v [H vdim]
+// and g [H vdim] of a token as the projection left them.  A thread owns one value channel j of one head and a
+// quarter of the key channels of S[:, j] in registers; q, k and the decays of a few tokens are staged in LDS,
+// where every thread reads the same word at a time (a broadcast).
+//
+// The state is linear in what came before: S_out = diag(A) S_in + B, A the product of a stretch's decays.  A long
+// portion is therefore cut into pieces that are walked side by side:
+//   pass 1  every piece but a request's last, from a zero state: A and B                (no outputs)
+//   carry   a short walk over the pieces leaves every piece's entry state
+//   pass 2  every piece again from its entry state, with outputs; the last writes the state back
+// A step of single tokens, or of short portions, is one launch from the state itself.
+#include "common.h"
+
+LLE_DEFINE_ERROR_STRING()
+
+// decay[n][c] = exp(log(sigmoid(z)) / tau), z = sum_r low[n][r] a2[r][c] + b[c]; low float32 [N, R], a2 float32 [R, C].
+// grid = (blocks of 256 channels, runs of GD_TOKENS tokens): a thread reads its column of a2 once for the run.
+#define GD_TOKENS 8
+__device__ __forceinline__ float gla_decay_of(float z, float inv_tau) {
+    return expf((fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau);  // log(sigmoid(z)), both ends without overflow
+}
+
+__global__ __launch_bounds__(256) void gla_decay_kernel(const float* __restrict__ low, const float* __restrict__ a2,
+                                                         const float* __restrict__ b, float* __restrict__ decay, int N,
+                                                         int R, int C, float inv_tau) {
+    const int c = blockIdx.x * blockDim.x + threadIdx.x;
+    const int n0 = blockIdx.y * GD_TOKENS;
+    if (c >= C) return;
+    float z[GD_TOKENS];
+#pragma unroll
+    for (int t = 0; t < GD_TOKENS; ++t) z[t] = b[c];
+    for (int r = 0; r < R; ++r) {
+        const float w = a2[(int64_t)r * C + c];
+#pragma unroll
+        for (int t = 0; t < GD_TOKENS; ++t) z[t] = fmaf(low[(int64_t)min(n0 + t, N - 1) * R + r], w, z[t]);  // (the same for all lanes)
+    }
+#pragma unroll
+    for (int t = 0; t < GD_TOKENS; ++t)
+        if (n0 + t < N) decay[(int64_t)(n0 + t) * C + c] = gla_decay_of(z[t], inv_tau);
+}
+
+extern "C" int lle_gla_decay(const void* low, const void* a2, const void* b, void* decay, int N, int R, int C, float tau,
+                             hipStream_t stream) {
+    if (N <= 0 || C <= 0) return 0;
+    if (R <= 0 || !(tau > 0.f)) return (int)hipErrorInvalidValue;
+    const int64_t runs = ((int64_t)N + GD_TOKENS - 1) / GD_TOKENS;
+    if (runs > 65535) return (int)hipErrorInvalidValue;
+    gla_decay_kernel<<<dim3((C + 255) / 256, (int)runs), 256, 0, stream>>>((const float*)low, (const float*)a2, (const float*)b,
+                                                                           (float*)decay, N, R, C, 1.0f / tau);
+    LLE_RETURN_LAUNCH_STATUS();
+}
+
+struct GlaArgs {
+    const void* u;  // [N, cols], activation type
+    int cols;
+    const float* decay;  // [N, H dim]
+    float q_scale;
+    const float* norm_w;  // [vdim]
+    float eps;
+    float* state;  // [slots, state_stride]
+    int64_t state_stride;
+    const int32_t* seq_slots;
+    const int32_t* cu_tokens;
+    void* out;  // [N, H vdim], activation type
+    int H, dim, vdim;
+    int jt;  // threads of a group: 64, 128 or 256, at least vdim
+    int pieces, piece_len;
+    float* part;  // [S, pieces, H, dim * vdim + dim]: B (then the entry state) and A of every piece
+};
+
+#define GLA_FROM_STATE 0  // one walk over a request's tokens
+#define GLA_SUMMARY 1     // pass 1
+#define GLA_FROM_ENTRY 2  // pass 2
+#define GLA_TC 8          // tokens staged at a time
+#define GLA_IG 4          // groups of threads that share a value channel's key channels
+
+// grid = (requests x pieces, heads).  KD >= dim (a multiple of 16) key channels are kept; a workgroup is GLA_IG groups
+// of `jt` threads: thread (ig, j) owns value channel j and the key channels [ig KD / GLA_IG, (ig + 1) KD / GLA_IG).
+// The groups' shares of o_t meet in LDS (dynamic: [GLA_IG][GLA_TC][jt]).
+template <int KD, typename T, int MODE>
+__global__ __launch_bounds__(1024) void gla_scan_kernel(GlaArgs a) {
+    constexpr bool OUT = MODE != GLA_SUMMARY;
+    constexpr int KI = KD / GLA_IG;
+    static_assert(KD % GLA_IG == 0, "the key channels are dealt to the groups in equal shares");
+    __shared__ float s_q[GLA_TC][KD], s_k[GLA_TC][KD], s_w[GLA_TC][KD];
+    __shared__ float s_inv[GLA_TC];
+    extern __shared__ float s_o[];
+    const int dim = a.dim, vdim = a.vdim, HK = a.H * dim, HV = a.H * vdim, jt = a.jt;
+    const int s = blockIdx.x / a.pieces, piece = blockIdx.x % a.pieces;
+    const int h = blockIdx.y;
+    const int tid = threadIdx.x;
+    const int j = tid & (jt - 1), ig = tid / jt, i0 = ig * KI;
+    const int q0 = a.cu_tokens[s], q1 = a.cu_tokens[s + 1];
+    const int live = (q1 - q0 + a.piece_len - 1) / a.piece_len;  // pieces of this request that hold tokens
+    if (piece >= live) return;
+    if (MODE == GLA_SUMMARY && piece == live - 1) return;  // nobody comes after the last piece
+    const int t0 = q0 + piece * a.piece_len, t1 = min(q1, t0 + a.piece_len);
+    float* srow = a.state + (int64_t)a.seq_slots[s] * a.state_stride + (int64_t)h * dim * vdim;
+    float* prow = a.part ? a.part + ((int64_t)(s * a.pieces + piece) * a.H + h) * (dim * vdim + dim) : nullptr;
+    const T* u = (const T*)a.u;
+
+    float S[KI];
+#pragma unroll
+    for (int ii = 0; ii < KI; ++ii) {
+        const int i = i0 + ii;
+        float x = 0.f;
+        if (MODE == GLA_FROM_STATE && i < dim && j < vdim) x = srow[i * vdim + j];
+        if (MODE == GLA_FROM_ENTRY && i < dim && j < vdim) x = prow[i * vdim + j];
+        S[ii] = x;
+    }
+    float A = 1.0f;  // (threads tid < KD: the product of the piece's decays of key channel tid)
+
+    for (int c0 = t0; c0 < t1; c0 += GLA_TC) {
+        const int nt = min(GLA_TC, t1 - c0);
+        __syncthreads();  // (the chunk before has been read)
+        for (int idx = tid; idx < GLA_TC * KD; idx += blockDim.x) {
+            const int t = idx / KD, i = idx - t * KD;
+            // past the chunk's last token: nothing is written and nothing decays
+            float qq = 0.f, kk = 0.f, ww = 1.0f;
+            if (t < nt && i < dim) {
+                const T* row = u + (int64_t)(c0 + t) * a.cols + h * dim + i;
+                if (OUT) qq = to_f32<T>(row[0]) * a.q_scale;
+                kk = to_f32<T>(row[HK]);
+                ww = a.decay[(int64_t)(c0 + t) * HK + h * dim + i];
+            }
+            if (OUT) s_q[t][i] = qq;
+            s_k[t][i] = kk;
+            s_w[t][i] = ww;
+        }
+        float vv[GLA_TC];
+#pragma unroll
+        for (int t = 0; t < GLA_TC; ++t)
+            vv[t] = (t < nt && j < vdim) ? to_f32<T>(u[(int64_t)(c0 + t) * a.cols + 2 * HK + h * vdim + j]) : 0.f;
+        __syncthreads();
+#pragma unroll
+        for (int t = 0; t < GLA_TC; ++t) {
+            float o = 0.f;
+#pragma unroll
+            for (int ii = 0; ii < KI; ++ii) {
+                const int i = i0 + ii;
+                S[ii] = fmaf(s_w[t][i], S[ii], s_k[t][i] * vv[t]);
+                if (OUT) o = fmaf(s_q[t][i], S[ii], o);
+            }
+            if (OUT) s_o[(ig * GLA_TC + t) * jt + j] = o;
+        }
+        if (!OUT && tid < KD) {
+#pragma unroll
+            for (int t = 0; t < GLA_TC; ++t) A *= s_w[t][tid];
+        }
+        if (OUT) {
+            __syncthreads();
+            // the groups' shares are added up, and every token's head is divided by its own root mean square:
+            // a wavefront per token
+            const int wave = tid / LLE_WAVE, lane = tid % LLE_WAVE, waves = blockDim.x / LLE_WAVE;
+            for (int t = wave; t < nt; t += waves) {
+                float ss = 0.f;
+                for (int e = lane; e < vdim; e += LLE_WAVE) {
+                    float o = s_o[t * jt + e];
+#pragma unroll
+                    for (int g2 = 1; g2 < GLA_IG; ++g2) o += s_o[(g2 * GLA_TC + t) * jt + e];
+                    s_o[t * jt + e] = o;
+                    ss += o * o;
+                }
+                ss = wave_sum(ss);
+                if (lane == 0) s_inv[t] = 1.0f / sqrtf(ss / (float)vdim + a.eps);
+            }
+            __syncthreads();
+            for (int idx = tid; idx < nt * vdim; idx += blockDim.x) {
+                const int t = idx / vdim, e = idx - t * vdim;
+                const float gate = to_f32<T>(u[(int64_t)(c0 + t) * a.cols + 2 * HK + HV + h * vdim + e]);
+                const float y = s_o[t * jt + e] * s_inv[t] * a.norm_w[e] * (gate / (1.0f + expf(-gate)));
+                ((T*)a.out)[(int64_t)(c0 + t) * HV + h * vdim + e] = from_f32<T>(y);
+            }
+        }
+    }
+    if (MODE == GLA_SUMMARY) {
+        if (j < vdim) {
+#pragma unroll
+            for (int ii = 0; ii < KI; ++ii)
+                if (i0 + ii < dim) prow[(i0 + ii) * vdim + j] = S[ii];
+        }
+        if (tid < dim) prow[dim * vdim + tid] = A;
+        return;
+    }
+    if (piece != live - 1) return;
+    if (j < vdim) {
+#pragma unroll
+        for (int ii = 0; ii < KI; ++ii)
+            if (i0 + ii < dim) srow[(i0 + ii) * vdim + j] = S[ii];
+    }
+}
+
+// grid = (requests, heads, blocks of 256 state elements): a thread walks one element S[i][j] through the
+// pieces and leaves every piece's entry state in the place of its B (eight pieces' A and B are asked
+// for together: one after the other, each would wait for the memory on its own)
+__global__ __launch_bounds__(256) void gla_carry_kernel(GlaArgs a) {
+    const int s = blockIdx.x, h = blockIdx.y;
+    const int elems = a.dim * a.vdim;
+    const int e = blockIdx.z * blockDim.x + threadIdx.x;
+    if (e >= elems) return;
+    const int i = e / a.vdim;
+    const int q0 = a.cu_tokens[s], q1 = a.cu_tokens[s + 1];
+    const int live = (q1 - q0 + a.piece_len - 1) / a.piece_len;
+    const int64_t stride = (int64_t)a.H * (elems + a.dim);
+    float* base = a.part + ((int64_t)s * a.pieces * a.H + h) * (elems + a.dim);
+    float S = a.state[(int64_t)a.seq_slots[s] * a.state_stride + (int64_t)h * elems + e];
+    for (int p0 = 0; p0 < live; p0 += 8) {
+        float A[8], B[8];
+#pragma unroll
+        for (int n = 0; n < 8; ++n) {
+            const int p = min(p0 + n, live - 1);
+            B[n] = base[p * stride + e];
+            A[n] = base[p * stride + elems + i];
+        }
+#pragma unroll
+        for (int n = 0; n < 8; ++n) {
+            if (p0 + n < live) {
+                base[(p0 + n) * stride + e] = S;
+                S = A[n] * S + B[n];  // (the last piece has left no A and B; what S becomes there is not used)
+            }
+        }
+    }
+}
+
+template <int KD, typename T>
+static int gla_launch(const GlaArgs& a, int S, hipStream_t stream) {
+    const int threads = a.jt * GLA_IG;
+    const size_t smem = (size_t)GLA_IG * GLA_TC * a.jt * sizeof(float);
+    const dim3 grid(S * a.pieces, a.H);
+    if (a.pieces == 1) {
+        gla_scan_kernel<KD, T, GLA_FROM_STATE><<<grid, threads, smem, stream>>>(a);
+        return (int)hipGetLastError();
+    }
+    gla_scan_kernel<KD, T, GLA_SUMMARY><<<grid, threads, 0, stream>>>(a);
+    hipError_t e = hipGetLastError();
+    if (e != hipSuccess) return (int)e;
+    gla_carry_kernel<<<dim3(S, a.H, (a.dim * a.vdim + 255) / 256), 256, 0, stream>>>(a);
+    e = hipGetLastError();
+    if (e != hipSuccess) return (int)e;
+    gla_scan_kernel<KD, T, GLA_FROM_ENTRY><<<grid, threads, smem, stream>>>(a);
+    return (int)hipGetLastError();
+}
+
+extern "C" int lle_gla_max_dim(void) { return 256; }
+
+// u [N, cols] in `dtype`: q, k, v, g in this order; decay float32 [N, H dim]; state float32 rows of `state_stride` floats
+// that begin with H dim vdim of the matrix state.  `pieces` > 1 needs `part`, float32 [S pieces H (dim vdim + dim)]; every
+// request has at most pieces * piece_len tokens.
+extern "C" int lle_gla_scan(const void* u, int cols, const void* decay, float q_scale, const void* norm_w, float eps, void* state,
+                            int64_t state_stride, const void* seq_slots, const void* cu_tokens, void* out, int S, int H, int dim,
+                            int vdim, int pieces, int piece_len, void* part, int dtype, hipStream_t stream) {
+    if (S <= 0 || H <= 0) return 0;
+    if (dim <= 0 || dim > 256 || vdim <= 0 || vdim > 256 || pieces < 1 || piece_len < 1 || (pieces > 1 && part == nullptr) ||
+        H > 65535 || (int64_t)S * pieces > 0x7fffffff || cols < 2 * H * (dim + vdim))
+        return (int)hipErrorInvalidValue;
+    // a group has as many threads as there are value channels, and the groups together as many as key channels
+    // (so that pass 1 finds a thread for every channel's product of decays)
+    const int jt = vdim <= 64 ? 64 : vdim <= 128 ? 128 : 256;
+    const GlaArgs a{u, cols, (const float*)decay, q_scale, (const float*)norm_w, eps, (float*)state, state_stride,
+                    (const int32_t*)seq_slots, (const int32_t*)cu_tokens, out, H, dim, vdim, jt, pieces, piece_len,
+                    (float*)part};
+#define GLA_CASE(KD)                                                                    \
+    if (dim <= KD)                                                                      \
+        return dtype == LLE_F32 ? gla_launch<KD, float>(a, S, stream) : gla_launch<KD, bf16_t>(a, S, stream);
+    GLA_CASE(16)
+    GLA_CASE(32)
+    GLA_CASE(48)
+    GLA_CASE(64)
+    GLA_CASE(96)
+    GLA_CASE(128)
+    GLA_CASE(192)
+    GLA_CASE(256)
+#undef GLA_CASE
+    return (int)hipErrorInvalidValue;
+}

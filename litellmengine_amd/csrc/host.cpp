@@ -30,7 +30,9 @@ namespace {
 
 struct PageTables {
     int num_pages = 0, page_size = 1, max_requests = 0, max_pages_per_request = 0;
-    int window = -1;                    // < 0: every key stays needed
+    int window = -1;                    // < 0: no window
+    int chunk = 0;                      // > 0: a position sees keys of its own chunk of so many positions only
+    int keep_first = 0;                 // positions below stay needed whatever the window says
     std::vector<int32_t> free_list;     // a stack: back() is handed out next
     std::vector<uint8_t> held;
     std::vector<std::vector<int32_t>> tables;  // per request slot: logical page -> physical page, -1 once given back
@@ -38,6 +40,12 @@ struct PageTables {
     std::vector<int32_t> pending_index, pending_page;  // entries of the device table not yet sent
 
     int pages_for(int length) const { return (length + page_size - 1) / page_size; }
+    bool forgets() const { return window >= 0 || chunk > 0; }
+    // the first position past the kept ones that the next query (position `length`) may still see
+    int first_needed(int length) const {
+        if (chunk > 0) return length / chunk * chunk;
+        return window >= 0 ? std::max(0, length - window + 1) : 0;
+    }
     int new_pages_needed(int slot, int new_len) const {
         return std::max(0, pages_for(new_len) - (int)tables[slot].size());
     }
@@ -67,14 +75,18 @@ const char* lle_error_string(int code) {
     return "unknown";
 }
 
-void* lle_pt_create(int num_pages, int page_size, int max_requests, int max_pages_per_request, int window) {
+void* lle_pt_create(int num_pages, int page_size, int max_requests, int max_pages_per_request, int window, int chunk,
+                    int keep_first) {
     if (num_pages <= 0 || page_size <= 0 || max_requests < 0 || max_pages_per_request < 0) return nullptr;
+    if (chunk < 0 || keep_first < 0 || (chunk > 0 && window >= 0)) return nullptr;
     PageTables* t = new PageTables;
     t->num_pages = num_pages;
     t->page_size = page_size;
     t->max_requests = max_requests;
     t->max_pages_per_request = max_pages_per_request;
     t->window = window;
+    t->chunk = chunk;
+    t->keep_first = keep_first;
     t->free_list.resize(num_pages);
     for (int i = 0; i < num_pages; ++i) t->free_list[i] = num_pages - 1 - i;  // page 0 on top
     t->held.assign(num_pages, 0);
@@ -205,17 +217,19 @@ void lle_pt_shrink_many(void* h, int n, const int32_t* slots, const int32_t* len
     for (int i = n - 1; i >= 0; --i) lle_pt_shrink(h, slots[i], lengths[i]);
 }
 
-// With a window w the next query (position `length`) sees keys >= length - w + 1: the pages
-// before that one's are given back.
+// With a window w the next query (position `length`) sees keys >= length - w + 1, with chunks of c
+// positions keys >= length / c * c: the pages before that one's are given back, except those that
+// hold the first positions where these are kept.
 void lle_pt_trim(void* h, int slot, int length) {
     PageTables* t = pt(h);
-    if (t->window < 0) return;
-    const int first_needed = std::max(0, length - t->window + 1) / t->page_size;
+    if (!t->forgets()) return;
+    const int first_needed = t->first_needed(length) / t->page_size;
+    const int kept = t->pages_for(t->keep_first);
     std::vector<int32_t>& table = t->tables[slot];
     const int first = t->first_live[slot];
     if (first_needed > first) {
         const int last = std::min(first_needed, (int)table.size());
-        for (int i = first; i < last; ++i) {
+        for (int i = std::max(first, kept); i < last; ++i) {
             t->give_back(table[i]);
             table[i] = -1;
         }
@@ -224,7 +238,7 @@ void lle_pt_trim(void* h, int slot, int length) {
 }
 
 void lle_pt_trim_many(void* h, int n, const int32_t* slots, const int32_t* lengths) {
-    if (pt(h)->window < 0) return;
+    if (!pt(h)->forgets()) return;
     for (int i = 0; i < n; ++i) lle_pt_trim(h, slots[i], lengths[i]);
 }
 
@@ -232,7 +246,8 @@ void lle_pt_trim_many(void* h, int n, const int32_t* slots, const int32_t* lengt
 void lle_pt_release_slot(void* h, int slot) {
     PageTables* t = pt(h);
     std::vector<int32_t>& table = t->tables[slot];
-    for (size_t i = (size_t)t->first_live[slot]; i < table.size(); ++i) t->give_back(table[i]);
+    for (size_t i = 0; i < table.size(); ++i)
+        if (table[i] >= 0) t->give_back(table[i]);
     table.clear();
     t->first_live[slot] = 0;
 }

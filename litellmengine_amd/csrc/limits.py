@@ -11,6 +11,19 @@ MAX_WKV_HEAD_DIM = 256
 # the delta rule's walk keeps a column of a head's state in the registers of sixteen lanes, up to sixteen each;
 # its convolution keeps a head in a wavefront, four elements a lane
 MAX_DELTA_HEAD_DIM = 256
+# gated linear attention: as the recurrence with a matrix state, key and value channels each
+MAX_GLA_HEAD_DIM = 256
+# heads whose weights are mixed keep a tile of scores, one of weights and their sums in LDS
+MAX_TALKING_LDS = 160 * 1024
+TALKING_KEYS = 64
+
+
+def check_talking_sizes(heads: int, head_dim: int) -> None:
+    """Raises ValueError for sizes whose heads' weights no kernel mixes."""
+    need = 4 * (2 * heads * TALKING_KEYS + heads * head_dim + 2 * heads)
+    if need > MAX_TALKING_LDS:
+        raise ValueError(f"{heads} heads of {head_dim} elements whose weights are mixed need {need} bytes of LDS, "
+                         f"there are {MAX_TALKING_LDS}")
 
 
 def check_head_dim(head_dim: int, rotary_dim: int = 0) -> None:

@@ -543,3 +543,123 @@ extern "C" int lle_rmsnorm_add_rmsnorm(void* hidden, const void* y, int y_dtype,
                                                                        w_next, weight_dtype, (bf16_t*)out, H, eps_out, eps_next);
     LLE_RETURN_LAUNCH_STATUS();
 }
+
+// Between two blocks something enters the stream: hidden[n] += a[n] (+ b[n]) (+ vec) (+ table[id(n)] * scale), all in
+// 32-bit and in place, then out[n] = norm(hidden[n]) * w, one launch.  `a` (float32 or bfloat16, null: nothing is left
+// to be added) may come as `slices` partial sums, `slice_stride` elements apart, added in slice order; `b` (or null)
+// is another summand of a's kind with a type of its own; `vec` float32 [H] or null; `table` [V, H] or null: the
+// embedding's rows once more, ids as in the embedding kernel.  The new row waits in registers where rows are no wider
+// than 256 x 4 x NORM_CHUNKS and a multiple of 4 (a plain loop otherwise).
+struct InjectArgs {
+    float* hidden;
+    const void* a;
+    int a_dtype, slices;
+    int64_t slice_stride;
+    const void* b;
+    int b_dtype;
+    const float* vec;
+    const int32_t* ids;
+    const void* table;
+    int table_dtype;
+    float scale;
+    const int32_t *feedback, *token_seq, *seq_slots;
+    const void* weight;
+    int weight_dtype;
+    void* out;
+    int H;
+    float eps;
+};
+
+__device__ __forceinline__ float4 load_quad(const void* p, int64_t i, int dtype) {
+    return dtype == LLE_F32 ? Quad<float>::load((const float*)p + i) : Quad<bf16_t>::load((const bf16_t*)p + i);
+}
+__device__ __forceinline__ void add_quad(float4& v, float4 d) {
+    v.x += d.x;
+    v.y += d.y;
+    v.z += d.z;
+    v.w += d.w;
+}
+
+template <typename TO>
+__global__ __launch_bounds__(256) void inject_rmsnorm_kernel(InjectArgs x) {
+    __shared__ float red[16];
+    const int64_t n = blockIdx.x, at = n * x.H;
+    const int H = x.H;
+    int64_t row = 0;
+    if (x.table) {
+        int id = x.ids[n];
+        if (id < 0) id = x.feedback ? x.feedback[x.seq_slots[x.token_seq[n]]] : 0;
+        row = (int64_t)id * H;
+    }
+    TO* out = (TO*)x.out;
+    float ss = 0.f;
+    if (H % 4 == 0 && H <= 256 * 4 * NORM_CHUNKS) {
+        float4 keep[NORM_CHUNKS], wv[NORM_CHUNKS];
+#pragma unroll
+        for (int k = 0; k < NORM_CHUNKS; ++k) {
+            const int i = (k * 256 + threadIdx.x) * 4;
+            if (i < H) {
+                wv[k] = load_weight4(x.weight, i, x.weight_dtype);
+                float4 v = *(const float4*)(x.hidden + at + i);
+                if (x.a) {
+                    float4 d = load_quad(x.a, at + i, x.a_dtype);
+                    for (int s = 1; s < x.slices; ++s) add_quad(d, load_quad(x.a, s * x.slice_stride + at + i, x.a_dtype));
+                    if (x.b) add_quad(d, load_quad(x.b, at + i, x.b_dtype));
+                    add_quad(v, d);
+                }
+                if (x.table) {
+                    const float4 e = load_quad(x.table, row + i, x.table_dtype);
+                    add_quad(v, make_float4(e.x * x.scale, e.y * x.scale, e.z * x.scale, e.w * x.scale));
+                }
+                if (x.vec) add_quad(v, Quad<float>::load(x.vec + i));
+                *(float4*)(x.hidden + at + i) = v;
+                keep[k] = v;
+                ss += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
+            }
+        }
+        ss = block_sum(ss, red);
+        const float inv = 1.0f / sqrtf(ss / (float)H + x.eps);
+#pragma unroll
+        for (int k = 0; k < NORM_CHUNKS; ++k) {
+            const int i = (k * 256 + threadIdx.x) * 4;
+            if (i < H)
+                Quad<TO>::store(out + at + i, make_float4(keep[k].x * inv * wv[k].x, keep[k].y * inv * wv[k].y,
+                                                          keep[k].z * inv * wv[k].z, keep[k].w * inv * wv[k].w));
+        }
+        return;
+    }
+    for (int i = threadIdx.x; i < H; i += blockDim.x) {
+        float v = x.hidden[at + i];
+        if (x.a) {
+            float d = load_as_f32(x.a, at + i, x.a_dtype);
+            for (int s = 1; s < x.slices; ++s) d += load_as_f32(x.a, s * x.slice_stride + at + i, x.a_dtype);
+            if (x.b) d += load_as_f32(x.b, at + i, x.b_dtype);
+            v += d;
+        }
+        if (x.table) v += load_as_f32(x.table, row + i, x.table_dtype) * x.scale;
+        if (x.vec) v += x.vec[i];
+        x.hidden[at + i] = v;
+        ss += v * v;
+    }
+    ss = block_sum(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)H + x.eps);
+    for (int i = threadIdx.x; i < H; i += blockDim.x)  // (each thread reads back the elements that it wrote itself)
+        out[at + i] = from_f32<TO>(x.hidden[at + i] * inv * load_as_f32(x.weight, i, x.weight_dtype));
+}
+
+extern "C" int lle_inject_rmsnorm(void* hidden, const void* a, int a_dtype, int slices, int64_t slice_stride, const void* b,
+                                  int b_dtype, const void* vec, const void* ids, const void* table, int table_dtype,
+                                  float scale, const void* feedback, const void* token_seq, const void* seq_slots,
+                                  const void* weight, int weight_dtype, void* out, int N, int H, float eps, int out_dtype,
+                                  hipStream_t stream) {
+    if (N <= 0 || H <= 0) return 0;
+    if (slices < 1 || (b && !a) || (table && !ids) || (feedback != nullptr) != (token_seq != nullptr) ||
+        (feedback != nullptr) != (seq_slots != nullptr))
+        return (int)hipErrorInvalidValue;
+    const InjectArgs x{(float*)hidden, a, a_dtype, slices, slice_stride, b, b_dtype, (const float*)vec, (const int32_t*)ids,
+                       table, table_dtype, scale, (const int32_t*)feedback, (const int32_t*)token_seq,
+                       (const int32_t*)seq_slots, weight, weight_dtype, out, H, eps};
+    if (out_dtype == LLE_F32) inject_rmsnorm_kernel<float><<<N, 256, 0, stream>>>(x);
+    else inject_rmsnorm_kernel<bf16_t><<<N, 256, 0, stream>>>(x);
+    LLE_RETURN_LAUNCH_STATUS();
+}

@@ -10,10 +10,10 @@ from typing import Optional
 
 import torch
 
-from ..parts.base import PartialSums, Prenormed
+from ..parts.base import PartialSums, Prenormed, ScaledSum
 from . import build
 from .tuning import ProductTuning
-from .limits import MAX_DELTA_HEAD_DIM, MAX_HEAD_DIM, MAX_SUMMED_NORM_WIDTH, MAX_WKV_HEAD_DIM
+from .limits import MAX_DELTA_HEAD_DIM, MAX_GLA_HEAD_DIM, MAX_HEAD_DIM, MAX_SUMMED_NORM_WIDTH, MAX_WKV_HEAD_DIM
 
 F32, BF16 = 0, 1
 _P = ctypes.c_void_p
@@ -441,8 +441,9 @@ class HipOps:
 
     def paged_attention(self, q, kv_layer, block_table, seq_slots, cu_tokens, kv_lens, token_seq,
                         window: Optional[int], scale: float, min_q_len: int = 0, max_q_len: int = 0,
-                        max_kv_len: int = 0, sinks=None) -> torch.Tensor:
-        """q [N, nq, d] against the pages -> [N, nq * d].  `sinks` (float32 [nq], or None): every head's
+                        max_kv_len: int = 0, sinks=None, keep_first: int = 0) -> torch.Tensor:
+        """q [N, nq, d] against the pages -> [N, nq * d].  `keep_first`: beside a window the first so many keys stay
+        in sight too.  `sinks` (float32 [nq], or None): every head's
         softmax has one more place, with that score and no value: p_j = exp(s_j) / (exp(sink) + sum exp(s_j)).
         `min_q_len`, `max_q_len`
         and `max_kv_len` are host-side bounds of this batch; they choose the kernels
@@ -468,6 +469,8 @@ class HipOps:
             _need(sinks.shape == (nq,), "sinks must be [nq]")
         out = torch.empty((N, nq * d), dtype=q.dtype, device=q.device)
         win = int(window) if window else 0
+        keep = int(keep_first) if win else 0
+        _need(keep >= 0, "keep_first must not be negative")
         mfma = (q.dtype == torch.bfloat16 and d % 32 == 0 and page_size % 16 == 0 and max_q_len > 0
                 and max_kv_len > 0 and S <= 65535 and not self.force_generic_attention)
         group = nq // nkv
@@ -482,17 +485,17 @@ class HipOps:
                 ws_o = torch.empty((N * nq * ns * d,), dtype=torch.float32, device=q.device)
                 ws_ml = torch.empty((N * nq * ns * 2,), dtype=torch.float32, device=q.device)
             self._run("attention", "lle_paged_attention_mfma_f32",
-                      [_P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _L, _I, _I, _F, _I, _I, _P, _P],
+                      [_P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _L, _I, _I, _I, _F, _I, _I, _P, _P],
                       _ptr(q), _ptr(kv_layer), _ptr(block_table), _ptr(seq_slots), _ptr(cu_tokens), _ptr(kv_lens),
                       _ptr(out), _ptr(ws_o), _ptr(ws_ml), N, S, nq, nkv, d, page_size, kv_layer.stride(0),
-                      block_table.shape[1], win, float(scale), row_blocks, ns, _ptr(sinks))
+                      block_table.shape[1], win, keep, float(scale), row_blocks, ns, _ptr(sinks))
             return out
         if not mfma:
             self._run("attention", "lle_paged_attention_generic",
-                      [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _L, _I, _I, _F, _I, _P, _P],
+                      [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _L, _I, _I, _I, _F, _I, _P, _P],
                       _ptr(q), _ptr(kv_layer), _ptr(block_table), _ptr(seq_slots), _ptr(cu_tokens), _ptr(kv_lens),
                       _ptr(token_seq), _ptr(out), N, nq, nkv, d, page_size, kv_layer.stride(0), block_table.shape[1],
-                      win, float(scale), dtype_code(q.dtype), _ptr(sinks))
+                      win, keep, float(scale), dtype_code(q.dtype), _ptr(sinks))
             return out
         min_q_len = min_q_len or 1
         run_decode = min_q_len * group <= 16
@@ -508,11 +511,11 @@ class HipOps:
             ws_ml = torch.empty((N * nq * ns * 2,), dtype=torch.float32, device=q.device)
         self._run("attention", "lle_paged_attention_mfma",
                   [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _L, _I, _I, _F, _I, _I, _I, _I, _I, _I,
-                   _P, _P],
+                   _P, _I, _P],
                   _ptr(q), _ptr(kv_layer), _ptr(block_table), _ptr(seq_slots), _ptr(cu_tokens), _ptr(kv_lens),
                   _ptr(token_seq), _ptr(out), _ptr(ws_o), _ptr(ws_ml), N, S, nq, nkv, d, page_size,
                   kv_layer.stride(0), block_table.shape[1], win, float(scale), int(run_decode), ns_decode,
-                  int(run_prefill), ns_prefill, max_q_len, row_tiles, _ptr(sinks))
+                  int(run_prefill), ns_prefill, max_q_len, row_tiles, _ptr(sinks), keep)
         return out
 
     def can_fuse_rope_attention(self, dtype, head_dim: int, rotary_dim: int, page_size: int, group: int,
@@ -1152,6 +1155,197 @@ class HipOps:
                   _ptr(r), _ptr(k), _ptr(v), _ptr(wraw), _ptr(w0), _ptr(u), _ptr(g), _ptr(norm_w),
                   dtype_code(norm_w.dtype), float(eps), _ptr(x), _ptr(state), state.stride(0), HD * dim, _ptr(seq_slots),
                   _ptr(cu_tokens), _ptr(out), S, heads, dim, W, pieces, piece, _ptr(part), dtype_code(out_dtype))
+        return out
+
+    # -- what enters the stream between two blocks ------------------------------------------------
+    def inject_rmsnorm(self, hidden, delta, vector, again, weight, eps: float, out_dtype) -> torch.Tensor:
+        """hidden float32 [N, H] += delta + vector + the embedding's rows, in 32-bit and in place, then
+        RMSNorm(hidden) * weight in `out_dtype`.  `delta`: [N, H] in either type, PartialSums, a ScaledSum with a
+        factor of one, or None; `vector` float32 [H] or None; `again` a parts.base.EmbeddedRows or None."""
+        _dev(hidden, "hidden", torch.float32)
+        _dev(weight, "norm weight")
+        N, H = hidden.shape
+        _need(weight.shape == (H,), f"norm weight must be [{H}]")
+        a, b, slices, stride = delta, None, 1, 0
+        if isinstance(delta, PartialSums):
+            a = delta.sums
+            slices, stride = a.shape[0], a.stride(0)
+            _dev(a, "partial sums", torch.float32)
+            _need(a.dim() == 3 and a.shape[1:] == hidden.shape, "partial sums must be [slices, N, H]")
+        elif isinstance(delta, ScaledSum):
+            a, b = delta.a, delta.b
+            if delta.mult != 1.0:
+                a, b = delta.total(), None
+        if a is not None and not isinstance(delta, PartialSums):
+            for t, name in ((a, "delta"), (b, "delta's second summand")):
+                if t is not None:
+                    _dev(t, name)
+                    _need(t.shape == hidden.shape, f"{name} must have the shape of hidden")
+        if vector is not None:
+            _dev(vector, "vector", torch.float32)
+            _need(vector.shape == (H,), f"vector must be [{H}]")
+        ids = table = feedback = token_seq = seq_slots = None
+        scale = 1.0
+        if again is not None:
+            ids, table, scale = again.ids, again.table, float(again.scale)
+            feedback, token_seq, seq_slots = again.feedback, again.token_seq, again.seq_slots
+            _dev(ids, "ids", torch.int32)
+            _dev(table, "embedding table")
+            _need(ids.shape == (N,) and table.dim() == 2 and table.shape[1] == H, "the embedding's rows must fit hidden")
+            if feedback is not None:
+                for t, name in ((feedback, "feedback"), (token_seq, "token_seq"), (seq_slots, "seq_slots")):
+                    _need(t is not None, "feedback, token_seq and seq_slots come together")
+                    _dev(t, name, torch.int32)
+                _need(token_seq.shape == (N,), "token_seq must be [N]")
+        out = torch.empty((N, H), dtype=out_dtype, device=hidden.device)
+        code = lambda t: 0 if t is None else dtype_code(t.dtype)
+        self._run("norm", "lle_inject_rmsnorm",
+                  [_P, _P, _I, _I, _L, _P, _I, _P, _P, _P, _I, _F, _P, _P, _P, _P, _I, _P, _I, _I, _F, _I, _P],
+                  _ptr(hidden), _ptr(a), code(a), slices, stride, _ptr(b), code(b), _ptr(vector), _ptr(ids), _ptr(table),
+                  code(table), scale, _ptr(feedback), _ptr(token_seq) if feedback is not None else None,
+                  _ptr(seq_slots) if feedback is not None else None, _ptr(weight), dtype_code(weight.dtype), _ptr(out), N, H,
+                  float(eps), dtype_code(out_dtype))
+        return out
+
+    # -- attention gated element by element, heads' weights mixed ----------------------------------
+    def pair_rope_write(self, u, bias, slots, cos_sin, v_cos_sin, kv_layer, num_q_heads: int, num_kv_heads: int, dim: int,
+                        vdim: int, write_kv: bool = True) -> torch.Tensor:
+        """A row of u holds q [nq dim], k [nkv dim], v [nkv vdim], then columns that are left alone; `bias` (or None)
+        covers those three.  The first elements of every q and k head turn in neighbouring pairs by cos_sin
+        [N, rot / 2, 2] (None: not), whole values by v_cos_sin [N, vdim / 2, 2] (None: not).  Returns q [N, nq, D] with
+        D = kv_layer.shape[4] >= max(dim, vdim), zeros past dim; K and V^T go to the pages `kv_layer`
+        [pages, 2, nkv, page_size, D] at `slots` [N] with zeros past dim and vdim."""
+        _dev(u, "u")
+        _dev(slots, "slots", torch.int32)
+        _dev(kv_layer, "kv_layer", u.dtype)
+        nq, nkv = num_q_heads, num_kv_heads
+        N, cols = u.shape
+        used = nq * dim + nkv * (dim + vdim)
+        _need(cols >= used, "u has too few columns")
+        _need(slots.shape == (N,), "slots must be [N]")
+        _need(kv_layer.dim() == 5 and kv_layer.shape[1] == 2 and kv_layer.shape[2] == nkv, "kv_layer must be [pages, 2, nkv, page_size, D]")
+        D, page_size = kv_layer.shape[4], kv_layer.shape[3]
+        _need(D >= max(dim, vdim) and D % 2 == 0, "the cache's heads are smaller than the model's, or odd")
+        if bias is not None:
+            _dev(bias, "bias", u.dtype)
+            _need(bias.shape == (used,), "bias must cover q, k and v")
+        rot = 0
+        for t, name, most in ((cos_sin, "cos_sin", dim), (v_cos_sin, "v_cos_sin", vdim)):
+            if t is not None:
+                _dev(t, name, torch.float32)
+                _need(t.dim() == 3 and t.shape[0] == N and t.shape[2] == 2 and 2 * t.shape[1] <= most, f"{name} must be [N, pairs, 2]")
+        if cos_sin is not None:
+            rot = 2 * cos_sin.shape[1]
+        _need(v_cos_sin is None or 2 * v_cos_sin.shape[1] == vdim, "v_cos_sin must cover the whole value")
+        q_out = torch.empty((N, nq, D), dtype=u.dtype, device=u.device)
+        self._run("rope_kv", "lle_pair_rope_write",
+                  [_P, _I, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _L, _I, _I, _P],
+                  _ptr(u), cols, _ptr(bias), _ptr(slots), _ptr(cos_sin), rot, _ptr(v_cos_sin), _ptr(q_out), _ptr(kv_layer), N,
+                  nq, nkv, dim, vdim, D, page_size, kv_layer.stride(0), 1 if write_kv else 0, dtype_code(u.dtype))
+        return q_out
+
+    def turn_back_gate(self, a, u, gate_col: int, heads: int, vdim: int, v_cos_sin, out_scale: float = 1.0) -> torch.Tensor:
+        """a [N, heads * D], D >= vdim -> [N, heads * vdim]: every head's first vdim elements, turned back in
+        neighbouring pairs by v_cos_sin [N, vdim / 2, 2] (None: not), times sigmoid(u[n, gate_col + ...]) element by
+        element, times out_scale."""
+        _dev(a, "a")
+        _dev(u, "u", a.dtype)
+        N = a.shape[0]
+        _need(a.dim() == 2 and a.shape[1] % heads == 0 and a.shape[1] // heads >= vdim, "a must be [N, heads * D], D >= vdim")
+        _need(u.dim() == 2 and u.shape[0] == N and 0 <= gate_col and gate_col + heads * vdim <= u.shape[1], "u [N, >= gate_col + heads * vdim]")
+        if v_cos_sin is not None:
+            _dev(v_cos_sin, "v_cos_sin", torch.float32)
+            _need(v_cos_sin.shape == (N, vdim // 2, 2) and vdim % 2 == 0, "v_cos_sin must cover the whole value")
+        out = torch.empty((N, heads * vdim), dtype=a.dtype, device=a.device)
+        self._run("rope_kv", "lle_turn_back_gate", [_P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _F, _I, _P], _ptr(a), _ptr(u),
+                  u.shape[1], int(gate_col), _ptr(v_cos_sin), _ptr(out), N, heads, a.shape[1] // heads, vdim, float(out_scale),
+                  dtype_code(a.dtype))
+        return out
+
+    def talking_attention(self, q, kv_layer, block_table, seq_slots, cu_tokens, kv_lens, token_seq, chunk: Optional[int],
+                          scale: float, slopes, talk, min_q_len: int = 0, max_q_len: int = 0,
+                          max_kv_len: int = 0) -> torch.Tensor:
+        """q [N, H, D] against the pages -> [N, H * D].  Position p sees the keys p // chunk * chunk .. p (chunk None:
+        all from 0 on); scores (q . k) * scale - slopes[h] * (p - j) (slopes float32 [H] or None), softmax, then the
+        heads' weights mixed, w_h <- sum_g talk[h, g] w_g (talk float32 [H, H]), head h on its own key/value head's
+        values.  `min_q_len`, `max_q_len` and `max_kv_len` are host-side bounds of this batch; they choose the
+        kernels, never the result."""
+        _dev(q, "q")
+        _dev(kv_layer, "kv_layer", q.dtype)
+        for t, name in ((block_table, "block_table"), (seq_slots, "seq_slots"), (cu_tokens, "cu_tokens"),
+                        (kv_lens, "kv_lens"), (token_seq, "token_seq")):
+            _dev(t, name, torch.int32)
+        N, H, D = q.shape
+        G, P = kv_layer.shape[2], kv_layer.shape[3]
+        _need(kv_layer.dim() == 5 and kv_layer.shape[4] == D and kv_layer.shape[1] == 2, "kv_layer must be [pages, 2, G, page_size, D]")
+        _need(H % G == 0, "query heads must be a multiple of key/value heads")
+        _need(token_seq.shape == (N,), "token_seq must be [N]")
+        S = seq_slots.shape[0]
+        _need(cu_tokens.shape == (S + 1,) and kv_lens.shape == (S,), "cu_tokens [S + 1], kv_lens [S]")
+        _need(block_table.dim() == 2, "block_table must be [slots, pages]")
+        _need(chunk is None or chunk > 0, "a chunk must be positive")
+        _dev(talk, "talk", torch.float32)
+        _need(talk.shape == (H, H), "talk must be [H, H]")
+        if slopes is not None:
+            _dev(slopes, "slopes", torch.float32)
+            _need(slopes.shape == (H,), "slopes must be [H]")
+        out = torch.empty((N, H * D), dtype=q.dtype, device=q.device)
+        self._run("talking", "lle_talking_generic",
+                  [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _L, _I, _I, _F, _P, _P, _I, _P],
+                  _ptr(q), _ptr(kv_layer), _ptr(block_table), _ptr(seq_slots), _ptr(cu_tokens), _ptr(kv_lens), _ptr(token_seq),
+                  _ptr(out), N, H, G, D, P, kv_layer.stride(0), block_table.shape[1], int(chunk or 0), float(scale),
+                  _ptr(slopes), _ptr(talk), dtype_code(q.dtype))
+        return out
+
+    # -- gated linear attention -----------------------------------------------------------------------
+    GLA_PIECE = 64  # tokens of one request that are walked in a row before the walk is cut into pieces
+
+    def gla_decay(self, low, a2, bias, tau: float) -> torch.Tensor:
+        """sigmoid(low @ a2 + bias)^(1 / tau), all float32: low [N, R], a2 [R, C], bias [C] -> [N, C]."""
+        for t, name in ((low, "low"), (a2, "a2"), (bias, "bias")):
+            _dev(t, name, torch.float32)
+        N, R = low.shape
+        C = bias.shape[0]
+        _need(a2.shape == (R, C), "a2 must be [R, C]")
+        out = torch.empty((N, C), dtype=torch.float32, device=low.device)
+        self._run("gla", "lle_gla_decay", [_P, _P, _P, _P, _I, _I, _I, _F, _P], _ptr(low), _ptr(a2), _ptr(bias), _ptr(out), N, R,
+                  C, float(tau))
+        return out
+
+    def gla_scan(self, u, decay, q_scale: float, norm_w, eps: float, state, heads: int, dim: int, vdim: int, seq_slots,
+                 cu_tokens, max_q_len: int = 0) -> torch.Tensor:
+        """Per head, with the matrix state S [dim, vdim] of the request (float32, `state[slot, : heads dim vdim]`):
+            S <- diag(decay_t) S + k_t v_t^T;   o_t = S^T (q_scale q_t)
+        and the result [N, heads * vdim] is o_t / rms(o_t) (per head, eps inside the root) * norm_w [vdim] * silu(g_t).
+        A row of u holds q [heads dim], k [heads dim], v [heads vdim], g [heads vdim]; decay float32 [N, heads * dim].
+        `max_q_len` (a host-side bound) only decides into how many pieces a walk is cut."""
+        _dev(u, "u")
+        _dev(decay, "decay", torch.float32)
+        _dev(norm_w, "norm weight", torch.float32)
+        _rows(state, "state", torch.float32)
+        _dev(seq_slots, "seq_slots", torch.int32)
+        _dev(cu_tokens, "cu_tokens", torch.int32)
+        N, cols = u.shape
+        S = seq_slots.shape[0]
+        _need(0 < dim <= MAX_GLA_HEAD_DIM and 0 < vdim <= MAX_GLA_HEAD_DIM, f"a head of the recurrence holds at most {MAX_GLA_HEAD_DIM} channels")
+        _need(cols >= 2 * heads * (dim + vdim), "u has too few columns")
+        _need(decay.shape == (N, heads * dim), "decay must be [N, heads * dim]")
+        _need(norm_w.shape == (vdim,), "the norm weight must be [vdim]")
+        _need(state.dim() == 2 and state.shape[1] >= heads * dim * vdim, "a state row holds heads * dim * vdim floats")
+        _need(cu_tokens.shape == (S + 1,), "cu_tokens must be [S + 1]")
+        out = torch.empty((N, heads * vdim), dtype=u.dtype, device=u.device)
+        piece = self.GLA_PIECE
+        pieces = -(-max_q_len // piece) if max_q_len > 2 * piece else 1
+        part = None
+        if pieces > 1:
+            part = torch.empty((S * pieces * heads * (dim * vdim + dim),), dtype=torch.float32, device=u.device)
+        else:
+            piece = 1 << 30
+        self._run("gla", "lle_gla_scan",
+                  [_P, _I, _P, _F, _P, _F, _P, _L, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _I, _P],
+                  _ptr(u), cols, _ptr(decay), float(q_scale), _ptr(norm_w), float(eps), _ptr(state), state.stride(0),
+                  _ptr(seq_slots), _ptr(cu_tokens), _ptr(out), S, heads, dim, vdim, pieces, piece, _ptr(part),
+                  dtype_code(u.dtype))
         return out
 
     # -- activations, caps, chained norms ---------------------------------------------------------

@@ -880,3 +880,183 @@ extern "C" int lle_conv_state_update(const void* u, int cols, void* state, int64
                                                              (const int32_t*)cu_tokens, (const int32_t*)seq_slots);
     LLE_RETURN_LAUNCH_STATUS();
 }
+
+// ---------------------------------------------------------------------------------
+// Projections whose heads are rotated in neighbouring pairs.  A row of `u` holds q [nq dim], k [nkv dim] and
+// v [nkv vdim], then columns that are left alone; `bias` (or null) covers the first three.  Elements 2i and 2i + 1
+// of the first `rot` elements of every q and k head turn by cos_sin [N, rot / 2, 2] (null: no rotation), those of
+// a whole value by v_cos_sin [N, vdim / 2, 2] (null: not).  q leaves as [N, nq, D] (zeros past dim), K and V^T go
+// to the pages with zeros past dim and vdim.  All in 32-bit.  A workgroup takes PR_TOKENS consecutive tokens:
+// a thread of the value part holds one element pair of one head for a run of tokens, so that tokens that lie side
+// by side in a page are stored in one piece (V^T holds an element's tokens side by side).
+// ---------------------------------------------------------------------------------
+#define PR_TOKENS 8
+
+template <typename T>
+__device__ __forceinline__ float2 pr_pair(const T* __restrict__ row, const T* __restrict__ bias, int col0, int e, int n,
+                                          const float* __restrict__ cs, int rot) {
+    // elements e and e + 1 (e even) of a head of n elements that starts at column col0
+    float2 x = {0.f, 0.f};
+    if (e < n) x.x = to_f32<T>(row[col0 + e]) + (bias ? to_f32<T>(bias[col0 + e]) : 0.f);
+    if (e + 1 < n) x.y = to_f32<T>(row[col0 + e + 1]) + (bias ? to_f32<T>(bias[col0 + e + 1]) : 0.f);
+    if (e < rot) {
+        const float c = cs[e], s = cs[e + 1];
+        x = make_float2(x.x * c - x.y * s, x.y * c + x.x * s);
+    }
+    return x;
+}
+
+template <typename T> struct PrPair;
+template <> struct PrPair<float> { typedef float2 vec; };
+template <> struct PrPair<bf16_t> { typedef bf16_t vec __attribute__((ext_vector_type(2))); };
+template <typename T>
+__device__ __forceinline__ void pr_store(T* p, float2 x) {  // p on a multiple of two elements (D is even)
+    typename PrPair<T>::vec v;
+    v.x = from_f32<T>(x.x);
+    v.y = from_f32<T>(x.y);
+    *(typename PrPair<T>::vec*)p = v;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void pair_rope_write_kernel(
+    const T* __restrict__ u, int cols, const T* __restrict__ bias, const int32_t* __restrict__ slots,
+    const float* __restrict__ cos_sin, int rot, const float* __restrict__ v_cos_sin, T* __restrict__ q_out,
+    T* __restrict__ kv_layer, int N, int nq, int nkv, int dim, int vdim, int D, int page_size, int64_t page_stride,
+    int write_kv) {
+    const int64_t n0 = (int64_t)blockIdx.x * PR_TOKENS;
+    const int count = (int)min((int64_t)PR_TOKENS, N - n0);
+    const int half = D / 2, q_pairs = nq * half, k_pairs = nkv * half;
+    const int per_token = q_pairs + (write_kv ? k_pairs : 0);
+    for (int idx = threadIdx.x; idx < count * per_token; idx += blockDim.x) {
+        const int t = idx / per_token, p = idx - t * per_token;
+        const int64_t n = n0 + t;
+        const T* row = u + n * cols;
+        const float* cs = cos_sin + n * rot;
+        const bool is_q = p < q_pairs;
+        const int pp = is_q ? p : p - q_pairs;
+        const int h = pp / half, e = 2 * (pp - h * half);
+        const float2 x = pr_pair<T>(row, bias, (is_q ? 0 : nq * dim) + h * dim, e, dim, cs, rot);
+        if (is_q) {
+            pr_store<T>(q_out + (n * nq + h) * D + e, x);
+        } else {
+            const int slot = slots[n];
+            if (slot >= 0) {
+                const int page = slot / page_size, off = slot - page * page_size;
+                pr_store<T>(kv_layer + (int64_t)page * page_stride + ((int64_t)h * page_size + off) * D + e, x);
+            }
+        }
+    }
+    if (!write_kv) return;
+    const int v_col = (nq + nkv) * dim;
+    int my_slots[PR_TOKENS];
+    bool run = count == PR_TOKENS && PR_TOKENS % 8 == 0;  // the tokens lie side by side in one page, from a multiple of 8 on
+#pragma unroll
+    for (int t = 0; t < PR_TOKENS; ++t) {
+        my_slots[t] = t < count ? slots[n0 + t] : -1;
+        run = run && my_slots[t] == my_slots[0] + t;
+    }
+    const int first_off = my_slots[0] >= 0 ? my_slots[0] % page_size : 0;
+    run = run && my_slots[0] >= 0 && first_off % PR_TOKENS == 0 && page_size % PR_TOKENS == 0;
+    for (int p = threadIdx.x; p < k_pairs; p += blockDim.x) {
+        const int h = p / half, e = 2 * (p - h * half);
+        float2 x[PR_TOKENS];
+#pragma unroll
+        for (int t = 0; t < PR_TOKENS; ++t)
+            x[t] = t < count ? pr_pair<T>(u + (n0 + t) * cols, bias, v_col + h * vdim, e, vdim,
+                                          v_cos_sin + (n0 + t) * vdim, v_cos_sin ? vdim : 0)
+                             : make_float2(0.f, 0.f);
+        const int64_t at = (int64_t)nkv * page_size * D + ((int64_t)h * D + e) * page_size;
+        if (run) {
+            typedef T piece_t __attribute__((ext_vector_type(PR_TOKENS)));
+            T* dst = kv_layer + (int64_t)(my_slots[0] / page_size) * page_stride + at + first_off;
+            piece_t a, b;
+#pragma unroll
+            for (int t = 0; t < PR_TOKENS; ++t) {
+                a[t] = from_f32<T>(x[t].x);
+                b[t] = from_f32<T>(x[t].y);
+            }
+            *(piece_t*)dst = a;
+            *(piece_t*)(dst + page_size) = b;
+        } else {
+#pragma unroll
+            for (int t = 0; t < PR_TOKENS; ++t) {
+                if (my_slots[t] >= 0) {
+                    const int page = my_slots[t] / page_size, off = my_slots[t] - page * page_size;
+                    T* dst = kv_layer + (int64_t)page * page_stride + at + off;
+                    dst[0] = from_f32<T>(x[t].x);
+                    dst[page_size] = from_f32<T>(x[t].y);
+                }
+            }
+        }
+    }
+}
+
+extern "C" int lle_pair_rope_write(const void* u, int cols, const void* bias, const void* slots, const void* cos_sin, int rot,
+                                   const void* v_cos_sin, void* q_out, void* kv_layer, int N, int nq, int nkv, int dim,
+                                   int vdim, int D, int page_size, int64_t page_stride, int write_kv, int dtype,
+                                   hipStream_t stream) {
+    if (N <= 0) return 0;
+    if (rot % 2 || rot > dim || dim > D || vdim > D || D % 2 || (rot > 0 && !cos_sin) || (v_cos_sin && vdim % 2) ||
+        cols < nq * dim + nkv * (dim + vdim))
+        return (int)hipErrorInvalidValue;
+    const int grid = (N + PR_TOKENS - 1) / PR_TOKENS;
+    if (dtype == LLE_F32)
+        pair_rope_write_kernel<float><<<grid, 256, 0, stream>>>(
+            (const float*)u, cols, (const float*)bias, (const int32_t*)slots, (const float*)cos_sin, rot,
+            (const float*)v_cos_sin, (float*)q_out, (float*)kv_layer, N, nq, nkv, dim, vdim, D, page_size, page_stride, write_kv);
+    else
+        pair_rope_write_kernel<bf16_t><<<grid, 256, 0, stream>>>(
+            (const bf16_t*)u, cols, (const bf16_t*)bias, (const int32_t*)slots, (const float*)cos_sin, rot,
+            (const float*)v_cos_sin, (bf16_t*)q_out, (bf16_t*)kv_layer, N, nq, nkv, dim, vdim, D, page_size, page_stride,
+            write_kv);
+    LLE_RETURN_LAUNCH_STATUS();
+}
+
+// out[n, h, e] = out_scale * a'[n, h, e] * sigmoid(u[n, gate_col + h vdim + e]) with a' the first vdim elements of the
+// heads of D that an attention left, turned back by the token's own rotation over all of them (v_cos_sin [N, vdim / 2, 2];
+// null: as they are).  A thread takes a neighbouring pair.
+template <typename T>
+__global__ __launch_bounds__(256) void turn_back_gate_kernel(const T* __restrict__ a, const T* __restrict__ u, int cols,
+                                                              int gate_col, const float* __restrict__ v_cos_sin,
+                                                              T* __restrict__ out, int64_t total, int heads, int D, int vdim,
+                                                              float out_scale) {
+    const int half = (vdim + 1) / 2;
+    for (int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total;
+         idx += (int64_t)gridDim.x * blockDim.x) {
+        const int64_t nh = idx / half;
+        const int e = 2 * (int)(idx - nh * half);
+        const int64_t n = nh / heads;
+        const int h = (int)(nh - n * heads);
+        const bool two = e + 1 < vdim;
+        const T* src = a + nh * D + e;
+        float x = to_f32<T>(src[0]), y = two ? to_f32<T>(src[1]) : 0.f;
+        if (v_cos_sin) {
+            const float c = v_cos_sin[n * vdim + e], s = v_cos_sin[n * vdim + e + 1];
+            const float t = x * c + y * s;
+            y = y * c - x * s;
+            x = t;
+        }
+        const T* g = u + n * cols + gate_col + h * vdim + e;
+        T* o = out + nh * vdim + e;
+        o[0] = from_f32<T>(x * out_scale / (1.0f + expf(-to_f32<T>(g[0]))));
+        if (two) o[1] = from_f32<T>(y * out_scale / (1.0f + expf(-to_f32<T>(g[1]))));
+    }
+}
+
+extern "C" int lle_turn_back_gate(const void* a, const void* u, int cols, int gate_col, const void* v_cos_sin, void* out, int N,
+                                  int heads, int D, int vdim, float out_scale, int dtype, hipStream_t stream) {
+    const int64_t total = (int64_t)N * heads * ((vdim + 1) / 2);
+    if (total <= 0) return 0;
+    if (vdim > D || (v_cos_sin && vdim % 2) || gate_col < 0 || cols < gate_col + heads * vdim) return (int)hipErrorInvalidValue;
+    int64_t blocks = (total + 255) / 256;
+    if (blocks > 65536) blocks = 65536;
+    if (dtype == LLE_F32)
+        turn_back_gate_kernel<float><<<(int)blocks, 256, 0, stream>>>((const float*)a, (const float*)u, cols, gate_col,
+                                                                       (const float*)v_cos_sin, (float*)out, total, heads, D,
+                                                                       vdim, out_scale);
+    else
+        turn_back_gate_kernel<bf16_t><<<(int)blocks, 256, 0, stream>>>((const bf16_t*)a, (const bf16_t*)u, cols, gate_col,
+                                                                        (const float*)v_cos_sin, (bf16_t*)out, total, heads, D,
+                                                                        vdim, out_scale);
+    LLE_RETURN_LAUNCH_STATUS();
+}

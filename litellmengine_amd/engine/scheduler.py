@@ -96,7 +96,7 @@ class Scheduler:
         longest = prompt_len + max_new_tokens - 1  # the last token drawn is never cached
         for group in self.cache.groups:
             pages = group.pages_for(longest)
-            if group.window is None and pages > group.pool.num_pages:
+            if not group.forgets and pages > group.pool.num_pages:
                 raise ValueError(
                     f"request of {prompt_len} prompt + {max_new_tokens} new tokens needs {pages} pages, "
                     f"the cache has {group.pool.num_pages}"

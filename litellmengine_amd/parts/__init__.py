@@ -1,10 +1,13 @@
 from .attention import ConvAttention, PagedAttention, SinkAttention
-from .base import (Block, BuildContext, CacheField, Carried, CacheSpec, FeedForward, KVCacheSpec, Mixer, Norm, NormFold, Part,
-                   Normed, PartialSums, PositionEncoding, Prenormed, ScaledSum, StateSpec)
+from .base import (Block, BuildContext, CacheField, Carried, CacheSpec, EmbeddedRows, FeedForward, Injected, KVCacheSpec, Mixer,
+                   Norm, NormFold, Part, Normed, PartialSums, PositionEncoding, Prenormed, ScaledSum, StateSpec)
 from .block import ParallelBlock, PostNormBlock, PreNormBlock, SandwichBlock
 from .delta import GatedDeltaMixer
 from .embedding import Embedding
 from .feed_forward import GatedMLP, PlainMLP
+from .gated_attention import GatedAttention, geometric_slopes
+from .gla import GatedLinearAttention
+from .injection import PassVectors
 from .latent_attention import LatentAttention
 from .linear import Linear
 from .moe import GroupLimitedMLP, RoutedMLP, ScoreRoutedMLP
@@ -20,4 +23,5 @@ __all__ = [
     "NoPositionEncoding", "Norm", "NormFold", "Normed", "PagedAttention", "Part", "PartialSums", "PositionEncoding", "PreNormBlock", "Prenormed", "RMSNorm",
     "RotaryHalfSplit", "StateSpec", "GroupLimitedMLP", "ParallelBlock", "ScaledSum", "SinkAttention", "WKVMixer",
     "ConvAttention", "SandwichBlock", "PlainMLP", "ScoreRoutedMLP", "SideBySideMixer", "GatedDeltaMixer",
+    "EmbeddedRows", "GatedAttention", "GatedLinearAttention", "Injected", "PassVectors", "geometric_slopes",
 ]

@@ -48,7 +48,10 @@ class CacheField:
 class CacheSpec:
     """Per-token cache need of a mixer: a record of named fields for every token.  A page
     holds the fields one after the other, each for all of the page's tokens.  With a
-    `window` only the last `window` positions stay needed and pages behind it are given back.
+    `window` only the last `window` positions stay needed and pages behind it are given back,
+    but for the first `keep_first` positions, which are kept.  With a `chunk` a position needs the
+    earlier ones of its own chunk of so many positions (counted from a request's first token), and the
+    pages of chunks that are over are given back.
     `page_size`: tokens per page, if the mixer's kernels want a size of their own (None: the
     engine's).  Mixers with equal specs share a group of pages and block tables; every group
     has a page size and a pool of its own."""
@@ -56,8 +59,16 @@ class CacheSpec:
     fields: Tuple[CacheField, ...]
     window: Optional[int] = None
     page_size: Optional[int] = None
+    chunk: Optional[int] = None
+    keep_first: int = 0
 
     def __post_init__(self):
+        if self.window is not None and self.chunk is not None:
+            raise ValueError("a cache record has a window or chunks, not both")
+        if (self.chunk is not None and self.chunk <= 0) or self.keep_first < 0:
+            raise ValueError("a cache record's chunk must be positive and its kept positions not negative")
+        if self.keep_first and self.window is None:
+            raise ValueError("first positions are kept beside a window only")
         names = [f.name for f in self.fields]
         if not names or len(set(names)) != len(names):
             raise ValueError("a cache record needs at least one field, and every field a name of its own")
@@ -66,6 +77,12 @@ class CacheSpec:
                 raise ValueError(f"cache field {f.name!r} needs positive sizes")
         if self.page_size is not None and self.page_size <= 0:
             raise ValueError("a cache record's page size must be positive")
+
+    @property
+    def span(self) -> Optional[int]:
+        """The most positions behind a query, itself counted, that stay needed (None: all of them);
+        kept first positions come on top."""
+        return self.window if self.window is not None else self.chunk
 
     @property
     def elems_per_token(self) -> int:
@@ -82,12 +99,12 @@ class CacheSpec:
         return k.num_heads, k.width
 
 
-def KVCacheSpec(num_kv_heads: int, head_dim: int, window: Optional[int] = None,
-                page_size: Optional[int] = None) -> CacheSpec:
+def KVCacheSpec(num_kv_heads: int, head_dim: int, window: Optional[int] = None, page_size: Optional[int] = None,
+                chunk: Optional[int] = None, keep_first: int = 0) -> CacheSpec:
     """Keys and values of `num_kv_heads` heads of `head_dim`, in the layout the attention
     kernels read: K as [head][token][d], V transposed as [head][d][token]."""
     return CacheSpec((CacheField("k", num_kv_heads, head_dim), CacheField("v", num_kv_heads, head_dim, True)), window,
-                     page_size)
+                     page_size, chunk, keep_first)
 
 
 @dataclasses.dataclass(frozen=True)
@@ -180,13 +197,55 @@ class ScaledSum:
         return t * self.mult
 
 
+@dataclasses.dataclass
+class EmbeddedRows:
+    """The embedding's rows of a step's tokens once more, named and not made: table[id(n)] * scale, where an
+    id below zero stands for the token that the step before left on the device (feedback, token_seq and
+    seq_slots; None where every id is given).  A kernel that adds them reads the table itself."""
+
+    ids: torch.Tensor
+    table: torch.Tensor
+    scale: float = 1.0
+    feedback: Optional[torch.Tensor] = None
+    token_seq: Optional[torch.Tensor] = None
+    seq_slots: Optional[torch.Tensor] = None
+
+    def rows(self, ops) -> torch.Tensor:
+        """float32 [N, width] (the plain way to take them)."""
+        return ops.embedding(self.ids, self.table, self.feedback, self.token_seq, self.seq_slots, scale=self.scale)
+
+
+@dataclasses.dataclass
+class Injected:
+    """What is left to be added to the residual stream where something enters it between two blocks:
+    `delta` (what the block before has left: a tensor, PartialSums, a ScaledSum or nothing), a `vector`
+    [width] in 32-bit that every row gets (or None), and the embedding's rows once more (`again`, or None).
+    Norm.forward takes it where it takes a delta; `total()` is the plain way to take it."""
+
+    delta: Any
+    vector: Optional[torch.Tensor]
+    again: Optional[EmbeddedRows]
+    ops: Any
+
+    def total(self) -> torch.Tensor:
+        parts = []
+        if self.delta is not None:
+            parts.append((self.delta.total() if hasattr(self.delta, "total") else self.delta).float())
+        if self.again is not None:
+            parts.append(self.again.rows(self.ops))
+        t = parts[0] if parts else 0.0
+        for p in parts[1:]:
+            t = t + p
+        return t if self.vector is None else t + self.vector
+
+
 class Norm(Part):
     """forward(hidden, delta) adds `delta` (or nothing) into the 32-bit residual
     stream `hidden` in place and returns the normed rows in the activation type;
     with `rows` only those rows are read and `hidden` is left alone.  `delta` is
     [N, hidden] in the activation type, or the PartialSums that a Linear made with
     `to_residual` may leave, or the ScaledSum of a block whose sublayers run side by
-    side (`delta.total()` is the plain way to take either).
+    side, or an Injected (`delta.total()` is the plain way to take any of them).
 
     fold(hidden) may return a NormFold when the step is small enough that the
     products on both sides of the norm can do its work (None: call forward).

@@ -37,6 +37,12 @@ class PreNormBlock(Block):
         for p in self._parts():
             p.bind(weights, ctx)
 
+    @staticmethod
+    def _sum(y):
+        """A mixer may hand its result on as a pair whose sum is meant (two mixers side by side): the norm's
+        kernel that takes it adds the two."""
+        return ScaledSum(y[0], y[1], 1.0) if isinstance(y, tuple) else y
+
     def entry_norm(self):
         return self.norm_in if self.mixer.folds_norm else None
 
@@ -53,12 +59,12 @@ class PreNormBlock(Block):
         else:
             x = self.norm_in.forward(hidden, delta)
         if self.feed_forward is None:
-            return self.mixer.forward(x, step, cache)
+            return self._sum(self.mixer.forward(x, step, cache))
         fold = self.norm_post.fold(hidden) if self.mixer.folds_norm and self.feed_forward.folds_norm else None
         if fold is not None:
             x = self.mixer.forward(x, step, cache, fold=fold)
         else:
-            x = self.norm_post.forward(hidden, self.mixer.forward(x, step, cache))
+            x = self.norm_post.forward(hidden, self._sum(self.mixer.forward(x, step, cache)))
         fold = next_norm.fold(hidden) if next_norm is not None and self.feed_forward.folds_norm else None
         if fold is not None:
             return self.feed_forward.forward(x, fold=fold)

@@ -7,7 +7,7 @@ from typing import Dict, Optional
 import torch
 
 from ..weights.spec import INIT_NORMAL, TensorSpec
-from .base import BuildContext, Normed, Part
+from .base import BuildContext, EmbeddedRows, Normed, Part
 
 
 class Embedding(Part):
@@ -25,6 +25,12 @@ class Embedding(Part):
     def bind(self, weights, ctx: BuildContext) -> None:
         self.ctx = ctx
         self.weight = weights[self.name].to(ctx.dtype).contiguous()
+
+    def again(self, step) -> EmbeddedRows:
+        """The rows that forward(step.token_ids, step) gives, for whoever adds them once more later in the step."""
+        deferred = step.token_feedback is not None
+        return EmbeddedRows(step.token_ids, self.weight, self.scale, step.token_feedback,
+                            step.token_seq if deferred else None, step.seq_slots if deferred else None)
 
     def forward(self, ids: torch.Tensor, step=None, norm=None):
         """`step` (engine.batch.StepState): where it carries `token_feedback`, ids below zero are

@@ -59,13 +59,14 @@ class PlainMLP(FeedForward):
     the factor enters with the activation, in 32-bit, since the last product is linear in it."""
 
     def __init__(self, prefix: str, hidden_size: int, intermediate_size: int, names=("up", "down"),
-                 activation: str = "relu2"):
+                 activation: str = "relu2", to_residual: bool = False):
+        """`to_residual`: the result goes nowhere but into Norm.forward(hidden, delta) (it may then come as PartialSums)."""
         if activation not in ("relu2", "relu", "silu"):
             raise ValueError(f"a plain feed-forward's activation is relu2, relu or silu, not {activation!r}")
         self.activation = activation
         up, down = names
         self.up = Linear([prefix + up], hidden_size, [intermediate_size])
-        self.down = Linear([prefix + down], intermediate_size, [hidden_size])
+        self.down = Linear([prefix + down], intermediate_size, [hidden_size], to_residual=to_residual)
 
     def tensor_specs(self) -> Dict[str, TensorSpec]:
         return {**self.up.tensor_specs(), **self.down.tensor_specs()}

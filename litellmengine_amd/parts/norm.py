@@ -8,7 +8,7 @@ from typing import Dict, Optional
 import torch
 
 from ..weights.spec import INIT_NORM, INIT_NORMAL, TensorSpec
-from .base import BuildContext, Norm, NormFold, ScaledSum
+from .base import BuildContext, Injected, Norm, NormFold, ScaledSum
 
 
 class RMSNorm(Norm):
@@ -43,6 +43,9 @@ class RMSNorm(Norm):
         return then.forward(hidden, None)
 
     def forward(self, hidden, delta, rows=None) -> torch.Tensor:
+        if isinstance(delta, Injected) and rows is None:  # everything that enters the stream, and the norm, in one launch
+            return self.ctx.ops.inject_rmsnorm(hidden, delta.delta, delta.vector, delta.again, self.weight, self.eps,
+                                               self.ctx.dtype)
         if isinstance(delta, ScaledSum):  # the add, times its constant, and the norm in one launch
             return self.ctx.ops.scaled_add_rmsnorm(hidden, delta.a, delta.b, delta.mult, self.weight, self.eps,
                                                    self.ctx.dtype, rows)

@@ -115,7 +115,7 @@ class TorchOps:
         return q.to(qkv.dtype).contiguous()
 
     def paged_attention(self, q, kv_layer, block_table, seq_slots, cu_tokens, kv_lens, token_seq, window, scale,
-                        min_q_len=0, max_q_len=0, max_kv_len=0, sinks=None):
+                        min_q_len=0, max_q_len=0, max_kv_len=0, sinks=None, keep_first=0):
         N, nq, d = q.shape
         nkv, P = kv_layer.shape[2], kv_layer.shape[3]
         group = nq // nkv
@@ -127,7 +127,8 @@ class TorchOps:
             for t in range(q0, q1):
                 pos = kv_len - (q1 - q0) + (t - q0)
                 lo = max(0, pos - window + 1) if window else 0
-                idx = torch.arange(lo, pos + 1, device=q.device)
+                idx = torch.cat([torch.arange(0, min(lo, keep_first), device=q.device),
+                                 torch.arange(lo, pos + 1, device=q.device)])
                 pages = block_table[slot, (idx // P).long()].long()
                 assert int(pages.min()) >= 0, "attention reads a page that was given back"
                 offs = (idx % P).long()
@@ -531,6 +532,99 @@ class TorchOps:
             h = hidden[rows.long()] + mult * d[rows.long()]
         x = h.to(self.cd)
         return (x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * weight.to(self.cd)).to(out_dtype)
+
+    # -- what enters the stream between two blocks -----------------------------------------------
+    def inject_rmsnorm(self, hidden, delta, vector, again, weight, eps, out_dtype):
+        if delta is not None:
+            hidden += (delta.total() if hasattr(delta, "total") else delta).to(torch.float32)
+        if vector is not None:
+            hidden += vector
+        if again is not None:
+            hidden += again.rows(self)
+        return self.add_rmsnorm(hidden, None, weight, eps, out_dtype)
+
+    # -- attention gated element by element, heads' weights mixed ---------------------------------
+    def _turned(self, t, cos_sin, sign):
+        """t [N, heads, n]: neighbouring pairs of the first 2 cos_sin.shape[1] elements turned."""
+        if cos_sin is None:
+            return t
+        rot = 2 * cos_sin.shape[1]
+        c, s = cos_sin[:, None, :, 0].to(self.cd), sign * cos_sin[:, None, :, 1].to(self.cd)
+        u, v = t[..., 0:rot:2], t[..., 1:rot:2]
+        pairs = torch.stack([u * c - v * s, v * c + u * s], dim=-1).flatten(-2)
+        return torch.cat([pairs, t[..., rot:]], dim=-1)
+
+    def pair_rope_write(self, u, bias, slots, cos_sin, v_cos_sin, kv_layer, num_q_heads, num_kv_heads, dim, vdim,
+                        write_kv=True):
+        nq, nkv, N = num_q_heads, num_kv_heads, u.shape[0]
+        D, P = kv_layer.shape[4], kv_layer.shape[3]
+        widths = [nq * dim, nkv * dim, nkv * vdim]
+        x = u[:, : sum(widths)].to(self.cd)
+        if bias is not None:
+            x = x + bias.to(self.cd)
+        q, k, v = (t.reshape(N, -1, n) for t, n in zip(x.split(widths, dim=1), (dim, dim, vdim)))
+        padded = lambda t: torch.nn.functional.pad(t, (0, D - t.shape[-1]))
+        q, k, v = padded(self._turned(q, cos_sin, 1)), padded(self._turned(k, cos_sin, 1)), padded(self._turned(v, v_cos_sin, 1))
+        if write_kv:
+            for n in range(N):
+                slot = int(slots[n])
+                if slot >= 0:
+                    kv_layer[slot // P, 0, :, slot % P, :] = k[n].to(kv_layer.dtype)
+                    v_pages(kv_layer)[slot // P, :, :, slot % P] = v[n].to(kv_layer.dtype)
+        return q.to(u.dtype).contiguous()
+
+    def turn_back_gate(self, a, u, gate_col, heads, vdim, v_cos_sin, out_scale):
+        N = a.shape[0]
+        o = self._turned(a.to(self.cd).view(N, heads, -1)[..., :vdim], v_cos_sin, -1).reshape(N, heads * vdim)
+        g = u[:, gate_col : gate_col + heads * vdim].to(self.cd)
+        return (o * torch.sigmoid(g) * out_scale).to(a.dtype).contiguous()
+
+    def talking_attention(self, q, kv_layer, block_table, seq_slots, cu_tokens, kv_lens, token_seq, chunk, scale, slopes,
+                          talk, min_q_len=0, max_q_len=0, max_kv_len=0):
+        N, nq, d = q.shape
+        nkv, P = kv_layer.shape[2], kv_layer.shape[3]
+        group = nq // nkv
+        out = torch.zeros((N, nq, d), dtype=self.cd, device=q.device)
+        for s in range(seq_slots.shape[0]):
+            slot = int(seq_slots[s])
+            q0, q1 = int(cu_tokens[s]), int(cu_tokens[s + 1])
+            for t in range(q0, q1):
+                pos = int(kv_lens[s]) - (q1 - q0) + (t - q0)
+                idx = torch.arange(pos // chunk * chunk if chunk else 0, pos + 1, device=q.device)
+                pages = block_table[slot, (idx // P).long()].long()
+                assert int(pages.min()) >= 0, "attention reads a page that was given back"
+                offs = (idx % P).long()
+                keys = kv_layer[pages, 0, :, offs, :].to(self.cd).repeat_interleave(group, dim=1)  # [n, nq, d]
+                vals = v_pages(kv_layer)[pages, :, :, offs].to(self.cd).repeat_interleave(group, dim=1)
+                sc = (q[t].to(self.cd)[None] * keys).sum(-1).t() * scale  # [nq, n]
+                if slopes is not None:
+                    sc = sc - slopes.to(self.cd)[:, None] * (pos - idx).to(self.cd)[None]
+                p = talk.to(self.cd) @ torch.softmax(sc, dim=-1)
+                out[t] = (p.t()[:, :, None] * vals).sum(0)
+        return out.reshape(N, nq * d).to(q.dtype)
+
+    # -- gated linear attention --------------------------------------------------------------------
+    def gla_decay(self, low, a2, bias, tau):
+        z = low.to(self.cd) @ a2.to(self.cd) + bias.to(self.cd)
+        return torch.exp(torch.nn.functional.logsigmoid(z) / tau).to(torch.float32)
+
+    def gla_scan(self, u, decay, q_scale, norm_w, eps, state, heads, dim, vdim, seq_slots, cu_tokens, max_q_len=0):
+        N = u.shape[0]
+        q, k, v, g = (t.to(self.cd) for t in u.split([heads * dim, heads * dim, heads * vdim, heads * vdim], dim=1))
+        q, k, w = (t.reshape(N, heads, dim) for t in (q * q_scale, k, decay.to(self.cd)))
+        v = v.reshape(N, heads, vdim)
+        out = torch.zeros((N, heads, vdim), dtype=self.cd, device=u.device)
+        for s in range(seq_slots.shape[0]):
+            slot, q0, q1 = int(seq_slots[s]), int(cu_tokens[s]), int(cu_tokens[s + 1])
+            if q1 <= q0:
+                continue
+            S = state[slot].to(self.cd).view(heads, dim, vdim).clone()
+            for t in range(q0, q1):
+                S = w[t][:, :, None] * S + k[t][:, :, None] * v[t][:, None, :]
+                out[t] = (q[t][:, :, None] * S).sum(1)
+            state[slot] = S.reshape(-1).to(state.dtype)
+        out = out / torch.sqrt((out * out).mean(-1, keepdim=True) + eps) * norm_w.to(self.cd)
+        return (out.reshape(N, heads * vdim) * g * torch.sigmoid(g)).to(u.dtype)
 
     # -- recurrence with a matrix state ----------------------------------------------------------
     def shift_mix(self, x, state, prev_offset, mu, token_seq, cu_tokens, seq_slots):
