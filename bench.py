@@ -12,6 +12,7 @@
     python bench.py --workload kezasun [--sizes small|mid|wide]   # Kezasun beside Visadra, kernel by kernel
     python bench.py --workload malilorn [--sizes small|mid|wide]  # Malilorn beside Kezasun, kernel by kernel
     python bench.py --workload birelix [--sizes small|mid|wide]   # Birelix beside Kezasun, kernel by kernel
+    python bench.py --workload telulorn [--sizes small|mid|wide]  # Telulorn beside Malilorn, kernel by kernel
 
 A "step" is one decode step of the whole engine (scheduler, model step over the
 paged cache, sampling) with `batch` live requests whose context ends at
@@ -1139,6 +1140,197 @@ def birelix_workload(args):
     return 0
 
 
+TELULORN_SIZES = {
+    # width; both attentions: q heads, kv heads, dim, vdim; chunk; window, kept first tokens, rotated; linear attention: heads,
+    # dim, vdim, decay rank; dense ff
+    "small": (1024, 8, 2, 128, 128, 512, 1024, 64, 64, 16, 64, 64, 16, 4096),
+    "mid": (2048, 16, 4, 128, 128, 1024, 2048, 64, 64, 32, 64, 64, 16, 8192),
+    "wide": (4096, 32, 8, 128, 128, 1024, 4096, 64, 64, 64, 64, 64, 16, 12288),
+}
+
+
+def telulorn_config(which, groups):
+    from litellmengine_amd.config import TelulornConfig
+
+    W, H, G, dim, vdim, chunk, window, keep, rot, LH, ldim, lvdim, rank, ff = TELULORN_SIZES[which]
+    mlp = {"kind": "dense", "ff": ff}
+    parallel = {"type": "parallel", "mlp": mlp, "mixer": {
+        "left": {"heads": H, "kv_heads": G, "dim": dim, "vdim": vdim, "scale": dim ** -0.5, "mask": {"size": chunk}},
+        "right": {"heads": LH, "dim": ldim, "vdim": lvdim, "tau": 16.0, "decay_rank": rank}, "left_scale": 0.7, "right_scale": 0.8}}
+    attention = {"type": "attention", "mlp": mlp, "mixer": {
+        "heads": H, "kv_heads": G, "dim": dim, "vdim": vdim, "scale": dim ** -0.5, "rot": {"base": 250000.0, "dims": rot},
+        "mask": {"size": window, "keep_first": keep}}}
+    layers = [parallel, attention, parallel, parallel] * groups
+    return TelulornConfig.from_dict({"architecture": "Telulorn", "vocab": 32768, "width": W, "norm": {"eps": 1e-6},
+                                     "layers": layers, "loop": {"start": 1, "stop": 3, "times": 2}})
+
+
+def malilorn_dense_config(which, layers):
+    """Malilorn at its sizes of that name with `layers` layers, all of them with its dense feed-forward."""
+    from litellmengine_amd.config import MalilornConfig
+
+    d = malilorn_config(which, 1).to_dict()
+    d["layers"] = [d["layers"][0]] * layers
+    return MalilornConfig.from_dict(d)
+
+
+def telulorn_kernels(which):
+    """Each kernel of Telulorn's own at two shapes (a 2048-token prompt; 8 decoded tokens after 4096) beside the like
+    kernel of Kezasun and Malilorn (attention over a window with a sink, the recurrence with a matrix state, the
+    projections' way into the cache, the add with its norm) at their sizes of the same name: microseconds and the
+    share of its roofline."""
+    import torch
+
+    from litellmengine_amd.csrc.ops import default_ops
+    from litellmengine_amd.parts.base import EmbeddedRows
+
+    ops = default_ops()
+    W, H, G, dim, vdim, chunk, window, keep, rot, LH, ldim, lvdim, rank, ff = TELULORN_SIZES[which]
+    KW, kwh, kwd, krank, KH, KG, kdim, kvdim, krot, kwindow, *_ = KEZASUN_SIZES[which]
+    dev, bf = "cuda", torch.bfloat16
+    P = PAGE_SIZE
+    rnd = lambda *shape, dtype=bf, scale=1.0: (torch.randn(shape, device=dev) * scale).to(dtype)
+    ints = lambda values: torch.tensor(values, dtype=torch.int32, device=dev)
+    out = {}
+
+    def entry(name, seconds, flops, nbytes, like=None):
+        floor = max(flops / MFMA_PEAK["bf16"], nbytes / HBM_PEAK)
+        e = {"us": round(seconds * 1e6, 1), "roofline_us": round(floor * 1e6, 2), "frac": round(floor / seconds, 4),
+             "bound": "mfma" if flops / MFMA_PEAK["bf16"] > nbytes / HBM_PEAK else "hbm"}
+        if like is not None:
+            e["like"] = like
+            e["times_farther_from_roofline"] = round(like["frac"] / e["frac"], 2) if e["frac"] > 0 else None
+        out[name] = e
+        return e
+
+    for shape, S, q_len, past in (("prefill_2048", 1, 2048, 0), ("decode_b8_ctx4096", 8, 1, 4095)):
+        N, kv = S * q_len, past + q_len
+        pages_each = -(-kv // P)
+        table = torch.arange(S * pages_each, dtype=torch.int32, device=dev).view(S, pages_each).contiguous()
+        seq_slots, cu = ints(list(range(S))), ints([i * q_len for i in range(S + 1)])
+        kv_lens = ints([kv] * S)
+        token_seq = ints([i // q_len for i in range(N)])
+        positions = ints([past + i % q_len for i in range(N)])
+        slots = (table.long().repeat_interleave(P, 1)[:, past:kv] * P + torch.arange(past, kv, device=dev) % P).reshape(-1).int()
+        where = (table, seq_slots, cu, kv_lens, token_seq)
+        # attention over a window that keeps the first tokens, and chunked attention whose heads' weights are mixed,
+        # beside attention over a window with a sink
+        D = -(-max(dim, vdim) // 32) * 32
+        kv_layer = rnd(S * pages_each + 1, 2, G, P, D)
+        q, sinks = rnd(N, H, D, scale=0.1), torch.zeros(H, device=dev)
+        KD = -(-max(kdim, kvdim) // 32) * 32
+        kq, ksinks = rnd(N, KH, KD, scale=0.1), torch.zeros(KH, device=dev)
+        kkv = rnd(S * pages_each + 1, 2, KG, P, KD)
+        tk = timed_launches(lambda: ops.paged_attention(kq, kkv, *where, kwindow, 0.1, q_len, q_len, kv, sinks=ksinks))
+        seen = sum(min(kwindow, past + i + 1) for i in range(q_len)) * S
+        like = entry(f"{shape}/paged_attention, window and sink (Kezasun)", tk, 4.0 * KH * KD * seen,
+                     2.0 * (S * min(kv, kwindow + q_len - 1) * 2 * KG * KD + 2 * N * KH * KD))
+        like = dict(like, name="paged_attention")
+        t = timed_launches(lambda: ops.paged_attention(q, kv_layer, *where, window, 0.1, q_len, q_len, kv, sinks=sinks, keep_first=keep))
+        seen = sum(min(past + i + 1, window + min(keep, max(0, past + i + 1 - window))) for i in range(q_len)) * S
+        entry(f"{shape}/paged_attention, window, kept first tokens and sink", t, 4.0 * H * D * seen,
+              2.0 * (S * min(kv, keep + window + q_len - 1) * 2 * G * D + 2 * N * H * D), like)
+        slopes, talk = torch.rand(H, device=dev), torch.randn(H, H, device=dev)
+        t = timed_launches(lambda: ops.talking_attention(q, kv_layer, *where, chunk, 0.1, slopes, talk, q_len, q_len, kv))
+        seen = sum((past + i) % chunk + 1 for i in range(q_len)) * S
+        first = past // chunk * chunk
+        entry(f"{shape}/talking_attention, chunks", t, (4.0 * H * D + 2.0 * H * H) * seen,
+              2.0 * (S * (kv - first) * 2 * G * D + 2 * N * H * D), like)
+        # rotations and the cache write beside the projection norm's kernel; the turn back under the gate beside the head gates
+        used = H * dim + G * (dim + vdim)
+        u, bias = rnd(N, used + H * vdim), rnd(used)
+        cos_sin = ops.rope_table(positions, torch.ones(rot // 2, device=dev))
+        v_cos_sin = ops.rope_table(positions, torch.ones(vdim // 2, device=dev))
+        kcols = KH * kdim + KG * (kdim + kvdim) + KH
+        kqkv, kbias = rnd(N, kcols), rnd(kcols)
+        kqw, kkw = torch.ones(KH * kdim, device=dev), torch.ones(KG * kdim, device=dev)
+        kcs = ops.rope_table(positions, torch.ones(krot // 2, device=dev))
+        tk = timed_launches(lambda: ops.proj_norm_rope_write(kqkv, kbias, slots, kqw, kkw, kcs, krot, 1e-6, kkv, KH, KG, kdim, kvdim))
+        like = dict(entry(f"{shape}/proj_norm_rope_write (Kezasun)", tk, 0, 2.0 * N * (kcols + KH * KD + 2 * KG * KD)), name="proj_norm_rope_write")
+        nbytes = 2.0 * N * (used + H * D + 2 * G * D)
+        t = timed_launches(lambda: ops.pair_rope_write(u, bias, slots, cos_sin, v_cos_sin, kv_layer, H, G, dim, vdim))
+        entry(f"{shape}/pair_rope_write, rotated values", t, 0, nbytes + 4.0 * N * (rot + vdim), like)
+        t = timed_launches(lambda: ops.pair_rope_write(u, None, slots, None, None, kv_layer, H, G, dim, vdim))
+        entry(f"{shape}/pair_rope_write, no rotation", t, 0, nbytes, like)
+        a, ka = rnd(N, H * D), rnd(N, KH * KD)
+        tk = timed_launches(lambda: ops.head_gate(ka, kqkv, kcols - KH, KH, kvdim))
+        like = dict(entry(f"{shape}/head_gate (Kezasun)", tk, 0, 2.0 * N * (KH * KD + KH * kvdim)), name="head_gate")
+        t = timed_launches(lambda: ops.turn_back_gate(a, u, used, H, vdim, v_cos_sin, 1.0))
+        entry(f"{shape}/turn_back_gate", t, 0, 2.0 * N * (H * D + 2 * H * vdim) + 4.0 * N * vdim, like)
+        # gated linear attention (decays and walk) beside the recurrence with a matrix state
+        KHD = kwh * kwd
+        r, k, v, wraw = (rnd(N, KHD, dtype=torch.float32, scale=0.5) for _ in range(4))
+        w0 = bonus = torch.zeros(KHD, device=dev)
+        g, x = rnd(N, KHD), rnd(N, KW)
+        kstate = torch.zeros(S + 1, KHD * kwd + KW, device=dev)
+        tk = timed_launches(lambda: ops.wkv_scan(r, k, v, wraw, w0, bonus, g, torch.ones(KHD, device=dev), 1e-6, x, kstate, kwh, kwd,
+                                                 seq_slots, cu, bf, q_len))
+        like = dict(entry(f"{shape}/wkv_scan (Kezasun)", tk, 0, N * KHD * (16 + 2 + 2.0) + 2.0 * S * KHD * kwd * 4), name="wkv_scan")
+        gu, low = rnd(N, 2 * LH * (ldim + lvdim), scale=0.5), rnd(N, rank, dtype=torch.float32)
+        a2, ab = rnd(rank, LH * ldim, dtype=torch.float32), torch.zeros(LH * ldim, device=dev)
+        state = torch.zeros(S + 1, LH * ldim * lvdim, device=dev)
+        nw = torch.ones(lvdim, device=dev)
+
+        def walk():
+            ops.gla_scan(gu, ops.gla_decay(low, a2, ab, 16.0), 0.125, nw, 1e-6, state, LH, ldim, lvdim, seq_slots, cu, q_len)
+
+        t = timed_launches(walk)
+        entry(f"{shape}/gla_decay + gla_scan", t, 0, N * (4.0 * LH * (ldim + lvdim) + 4.0 * rank + 2.0 * LH * lvdim) + 8.0 * S * LH * ldim * lvdim, like)
+        out[f"{shape}/gla_decay + gla_scan"]["fp32_flops_T"] = round(6.0 * N * LH * ldim * lvdim / t / 1e12, 2)
+        # what enters the stream between two blocks, with its norm, beside the scaled add with its norm
+        hidden, da = rnd(N, W, dtype=torch.float32), rnd(N, W)
+        w = torch.ones(W, device=dev, dtype=bf)
+        tablew, vec = rnd(32768, W), torch.zeros(W, device=dev)
+        ids = torch.randint(0, 32768, (N,), device=dev, dtype=torch.int32)
+        kh, kda, kdb, kw2 = rnd(N, KW, dtype=torch.float32), rnd(N, KW), rnd(N, KW, dtype=torch.float32), torch.ones(KW, device=dev)
+        tk = timed_launches(lambda: ops.scaled_add_rmsnorm(kh, kda, kdb, 0.3, kw2, 1e-6, bf))
+        like = dict(entry(f"{shape}/scaled_add_rmsnorm (Kezasun)", tk, 0, N * KW * (4 + 4 + 2 + 4 + 2.0)), name="scaled_add_rmsnorm")
+        again = EmbeddedRows(ids, tablew)
+        t = timed_launches(lambda: ops.inject_rmsnorm(hidden, da, vec, again, w, 1e-6, bf))
+        entry(f"{shape}/inject_rmsnorm", t, 0, N * W * (4 + 4 + 2 + 2 + 2.0), like)
+        # the square of relu beside silu_mul
+        z, z2 = rnd(N, ff), rnd(N, 2 * ff)
+        tk = timed_launches(lambda: ops.silu_mul(z2))
+        like = dict(entry(f"{shape}/silu_mul (Qwen3)", tk, 0, 2.0 * N * 3 * ff), name="silu_mul")
+        t = timed_launches(lambda: ops.bias_act(z, "relu2", False))
+        entry(f"{shape}/bias_act, square of relu", t, 0, 2.0 * N * 2 * ff, like)
+        del kv_layer, kkv, tablew
+    return out
+
+
+def telulorn_workload(args):
+    import torch
+
+    from litellmengine_amd.models import random_model
+
+    which = args.sizes if args.sizes in TELULORN_SIZES else "mid"
+    groups = max(1, args.layers // 4) if args.layers != SIZES["num_hidden_layers"] else 1
+    tcfg = telulorn_config(which, groups)
+    runs = len(tcfg.layers) + 2
+    mcfg = malilorn_dense_config(which, runs)
+    line = {"metric": f"Telulorn beside Malilorn at layer sizes of the same name ({which}): prefill tok/s @ 2048 and decode tok/s "
+                      f"@ batch {args.batch}, context {args.context}", "unit": "tok/s", "n_gpus": 1, "dtype": "bf16",
+            "data": "synthetic: seeded random weights, uniform random token ids", "higher_is_better": True,
+            "config": {"sizes": dict(zip(("width", "heads", "kv_heads", "dim", "vdim", "chunk", "window", "keep_first", "rotated",
+                                          "linear_heads", "linear_dim", "linear_vdim", "decay_rank", "dense_ff"), TELULORN_SIZES[which])),
+                       "layers": len(tcfg.layers), "layer_runs": runs, "pattern": "parallel, attention, parallel, parallel; the second and "
+                       "third layer run twice", "beside": f"Malilorn with {runs} layers, every one with its dense (gated) feed-forward"}}
+    steps, warmup = min(args.steps, 16), min(args.warmup, 4)
+    for name, cfg in (("telulorn", tcfg), ("malilorn", mcfg)):
+        model = random_model(cfg, seed=0, dtype="bfloat16")
+        dt = time_decode(model, cfg, args.batch, args.context, steps, warmup)
+        pt = time_prefill(model, cfg, PREFILL_TOKENS)
+        line[name] = {"decode_tok_s": round(args.batch / dt, 1), "decode_ms_per_step": round(dt * 1e3, 3),
+                      "prefill_tok_s": round(PREFILL_TOKENS / pt, 1), "prefill_ms": round(pt * 1e3, 3)}
+        del model
+        torch.cuda.empty_cache()
+    line["value"] = line["telulorn"]["decode_tok_s"]
+    line["steps"], line["warmup"] = steps, warmup
+    line["kernels"] = telulorn_kernels(which)
+    print(json.dumps(line))
+    return 0
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -1152,8 +1344,8 @@ def main():
     ap.add_argument("--no-more", action="store_true", help="skip the other workloads that the default line carries")
     ap.add_argument("--sizes", default="8b", choices=["8b", "0p6b", "32b", "small", "mid", "wide"],
                     help="layer sizes of the decode workload: Qwen3-8B (default, the headline), Qwen3-0.6B or Qwen3-32B; "
-                         "small, mid or wide: the layer sizes of --workload visadra, kezasun, malilorn and birelix")
-    ap.add_argument("--workload", default="decode", choices=["decode", "reference-0p6b", "mixed-32b", "serving", "visadra", "kezasun", "malilorn", "birelix"],
+                         "small, mid or wide: the layer sizes of --workload visadra, kezasun, malilorn, birelix and telulorn")
+    ap.add_argument("--workload", default="decode", choices=["decode", "reference-0p6b", "mixed-32b", "serving", "visadra", "kezasun", "malilorn", "birelix", "telulorn"],
                     help="decode (default: the headline line), the reference's own benchmark shape at Qwen3-0.6B "
                          "sizes, a mixed prompt-portion + decode step at Qwen3-32B sizes, requests arriving over time, "
                          "Visadra beside Qwen3 at equal layer sizes with every kernel against its roofline, Kezasun "
@@ -1179,6 +1371,8 @@ def main():
             return malilorn_workload(args)
         if args.workload == "birelix":
             return birelix_workload(args)
+        if args.workload == "telulorn":
+            return telulorn_workload(args)
         args.steps, args.warmup = min(args.steps, 3), min(args.warmup, 1)
         return mixed_workload(args)
 

@@ -1290,6 +1290,28 @@ class HipOps:
             _dev(slopes, "slopes", torch.float32)
             _need(slopes.shape == (H,), "slopes must be [H]")
         out = torch.empty((N, H * D), dtype=q.dtype, device=q.device)
+        run_decode, run_prefill = min_q_len <= 1, max_q_len > 1
+        if (q.dtype == torch.bfloat16 and D % 32 == 0 and D <= 128 and P % 16 == 0 and max_q_len > 0 and max_kv_len > 0
+                and S <= 65535 and (H <= 32 if run_prefill else H <= 512) and not self.force_generic_attention):
+            K = splits = 0
+            ws_s = ws_ml = None
+            if run_decode:
+                seen = min(chunk, max_kv_len) if chunk else max_kv_len  # keys that a query sees at most
+                K = -(-(seen + 15) // 16) * 16
+                # a wavefront should have a tile of 16 keys or two, and the workgroups fill the CUs once or twice
+                splits = int(max(1, min(-(-K // 64), 2 * self.compute_units() // max(1, S * G))))
+                ws_s = torch.empty((S * H * K,), dtype=torch.float32, device=q.device)
+                ws_ml = torch.empty((S * H * (K // 16) * 2,), dtype=torch.float32, device=q.device)
+            # one output head a wavefront twice the workgroups, which make all scores again: where the tiles leave CUs idle
+            out_heads = 1 if -(-max_q_len // 16) * S * 4 <= self.compute_units() else 2
+            self._run("talking", "lle_talking_mfma",
+                      [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _L, _I, _I, _F, _P, _P, _I, _I, _I, _P, _P, _I, _I, _I,
+                       _P],
+                      _ptr(q), _ptr(kv_layer), _ptr(block_table), _ptr(seq_slots), _ptr(cu_tokens), _ptr(kv_lens),
+                      _ptr(token_seq), _ptr(out), S, H, G, D, P, kv_layer.stride(0), block_table.shape[1], int(chunk or 0),
+                      float(scale), _ptr(slopes), _ptr(talk), int(run_decode), splits, K, _ptr(ws_s), _ptr(ws_ml),
+                      int(run_prefill), max_q_len, out_heads)
+            return out
         self._run("talking", "lle_talking_generic",
                   [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _L, _I, _I, _F, _P, _P, _I, _P],
                   _ptr(q), _ptr(kv_layer), _ptr(block_table), _ptr(seq_slots), _ptr(cu_tokens), _ptr(kv_lens), _ptr(token_seq),

@@ -7,8 +7,14 @@
 //
 // Position p sees the keys floor(p / chunk) * chunk .. p (chunk 0: all from 0 on), chunks counted from the
 // request's first token; slopes may be null (no distance bias).  The mix needs every head's weight of a key,
-// already divided by its sum, so scores are made twice: once for the rows' maxima and sums, once for the weights.
+// already divided by its sum, so maxima and sums come first and the weights after them.
 // A cache page holds K as [G][page_size][D], then V as [G][D][page_size].
+//
+// Kernels:
+//  * talking_prefill_kernel: bfloat16 on the matrix cores, heads of a multiple of 32 up to 128, up to 32 heads, pages of
+//    a multiple of 16: requests of more than one token.  A workgroup takes 16 tokens of a request and ALL heads.
+//  * talking_scores_kernel + talking_values_kernel: the same sizes, decoded tokens (any number of heads).
+//  * talking_generic_kernel: any type and size.
 #include "common.h"
 
 LLE_DEFINE_ERROR_STRING()
@@ -150,4 +156,462 @@ extern "C" int lle_talking_generic(const void* q, const void* kv, const void* bl
     if (dtype == LLE_F32) talking_generic_kernel<float><<<N, 256, smem, stream>>>(a);
     else talking_generic_kernel<bf16_t><<<N, 256, smem, stream>>>(a);
     LLE_RETURN_LAUNCH_STATUS();
+}
+
+// ---------------------------------------------------------------------------------
+// matrix-core kernels (bfloat16)
+// ---------------------------------------------------------------------------------
+typedef bf16_t bf16x8 __attribute__((ext_vector_type(8)));
+typedef bf16_t bf16x4 __attribute__((ext_vector_type(4)));
+typedef bf16_t bf16x2 __attribute__((ext_vector_type(2)));
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+
+#define NEG_BIG (-1.0e30f)
+#define LOG2E 1.44269504088896340736f
+// row r of tile x of a 32-key step stands for this key of the step: a lane's eight scores are consecutive keys then
+#define KEY_OF_ROW(r, x) (8 * ((r) / 4) + 4 * (x) + (r) % 4)
+
+// Decoded tokens, first launch: scores.  grid = (requests, G, key splits), four wavefronts; a wavefront takes every
+// (4 x splits)-th tile of 16 keys.  ws_s [S][H][K] holds the base-2 scores from the 16-key tile on in which the chunk
+// begins (NEG_BIG where the query does not see the key), ws_ml [S][H][K / 16] every tile's maximum and sum.
+template <int DK>
+__global__ __launch_bounds__(256) void talking_scores_kernel(TalkArgs a, float* __restrict__ ws_s, float2* __restrict__ ws_ml, int K) {
+    constexpr int D = DK * 32;
+    const int s = blockIdx.x, kvh = blockIdx.y;
+    const int q_start = a.cu_tokens[s];
+    if (a.cu_tokens[s + 1] - q_start != 1) return;
+    const int pos = a.kv_lens[s] - 1;
+    const int lo = a.chunk > 0 ? pos / a.chunk * a.chunk : 0, lo16 = lo & ~15;
+    const int tiles = (pos - lo16) / 16 + 1;
+    const int wave = threadIdx.x / LLE_WAVE, lane = threadIdx.x % LLE_WAVE, c = lane / 16, r16 = lane % 16;
+    const int32_t* table = a.block_tables + (int64_t)a.seq_slots[s] * a.max_pages;
+    const int group = a.H / a.G;
+    const bf16_t* kv = (const bf16_t*)a.kv;
+    for (int g0 = 0; g0 < group; g0 += 16) {  // 16 heads of the group at a time
+        const int g = g0 + r16, h = kvh * group + g;
+        const bool exists = g < group;
+        bf16x8 qv[DK];
+        const bf16_t* q = (const bf16_t*)a.q + ((int64_t)q_start * a.H + kvh * group + (exists ? g : g0)) * D;
+#pragma unroll
+        for (int ks = 0; ks < DK; ++ks) qv[ks] = *(const bf16x8*)(q + 32 * ks + 8 * c);
+        const float slope = a.slopes && exists ? a.slopes[h] * LOG2E : 0.f;
+        for (int tile = blockIdx.z * 4 + wave; tile < tiles; tile += 4 * gridDim.z) {
+            const int j0 = lo16 + 16 * tile;
+            const int lp = j0 / a.P, off = j0 - lp * a.P;
+            const bf16_t* k = kv + (int64_t)table[__builtin_amdgcn_readfirstlane(lp)] * a.page_stride +
+                              ((int64_t)kvh * a.P + off + r16) * D + 8 * c;
+            f32x4 sc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int ks = 0; ks < DK; ++ks) sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8*)(k + 32 * ks), qv[ks], sc, 0, 0, 0);
+            float top = NEG_BIG;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int j = j0 + 4 * c + i;
+                sc[i] = j < lo || j > pos ? NEG_BIG : fmaf(sc[i], a.scale * LOG2E, slope * (float)(j - pos));
+                top = fmaxf(top, sc[i]);
+            }
+            top = fmaxf(top, __shfl_xor(top, 16, LLE_WAVE));
+            top = fmaxf(top, __shfl_xor(top, 32, LLE_WAVE));
+            float sum = 0.f;  // (every tile holds a key that the query sees: its maximum is a score)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) sum += __builtin_amdgcn_exp2f(sc[i] - top);
+            sum += __shfl_xor(sum, 16, LLE_WAVE);
+            sum += __shfl_xor(sum, 32, LLE_WAVE);
+            if (exists) {
+                const int64_t row = (int64_t)s * a.H + h;
+                *(f32x4*)(ws_s + row * K + 16 * tile + 4 * c) = sc;
+                if (c == 0) ws_ml[row * (K / 16) + tile] = make_float2(top, sum);
+            }
+        }
+    }
+}
+
+// Decoded tokens, second launch: weights, mix, values.  grid = (requests, G, blocks of 64 value elements), four
+// wavefronts of 16 elements each.  256 keys at a time: a thread makes one key's weights of all heads and mixes them
+// for the key/value head's own query heads (16 at a time), the weights cross through LDS, and the values, asked for
+// before that, are multiplied on the matrix cores.  LDS: maxima [H], talk / sum [16][H], weights [16][256 + 8].
+#define TV_KEYS 256
+__global__ __launch_bounds__(256) void talking_values_kernel(TalkArgs a, const float* __restrict__ ws_s,
+                                                             const float2* __restrict__ ws_ml, int K) {
+    extern __shared__ float lds[];
+    float* s_m = lds;
+    float* s_t = s_m + a.H;  // [16][H]
+    bf16_t* s_w = (bf16_t*)(s_t + 16 * a.H + (a.H % 4 ? 4 - a.H % 4 : 0));  // [16][TV_KEYS + 8], 16-byte aligned
+    const int s = blockIdx.x, kvh = blockIdx.y;
+    const int q_start = a.cu_tokens[s];
+    if (a.cu_tokens[s + 1] - q_start != 1) return;
+    const int pos = a.kv_lens[s] - 1;
+    const int lo = a.chunk > 0 ? pos / a.chunk * a.chunk : 0, lo16 = lo & ~15;
+    const int tiles = (pos - lo16) / 16 + 1;
+    const int wave = threadIdx.x / LLE_WAVE, lane = threadIdx.x % LLE_WAVE, c = lane / 16, r16 = lane % 16;
+    const int32_t* table = a.block_tables + (int64_t)a.seq_slots[s] * a.max_pages;
+    const int group = a.H / a.G;
+    const int e0 = blockIdx.z * 64 + wave * 16;  // this wavefront's value elements
+    const bool has_values = e0 < a.D;            // (the same for the whole wavefront)
+    const bf16_t* v_base = (const bf16_t*)a.kv + ((int64_t)a.G + kvh) * a.P * a.D + (int64_t)(has_values ? e0 + r16 : 0) * a.P;
+    const float* s_row = ws_s + (int64_t)s * a.H * K;
+    for (int g0 = 0; g0 < group; g0 += 16) {
+        const int count = min(16, group - g0);
+        __syncthreads();
+        for (int h = wave; h < a.H; h += 4) {
+            const float2* ml = ws_ml + ((int64_t)s * a.H + h) * (K / 16);
+            float top = NEG_BIG;
+            for (int t = lane; t < tiles; t += LLE_WAVE) top = fmaxf(top, ml[t].x);
+            top = wave_max(top);
+            float sum = 0.f;
+            for (int t = lane; t < tiles; t += LLE_WAVE) sum += ml[t].y * __builtin_amdgcn_exp2f(ml[t].x - top);
+            sum = wave_sum(sum);
+            if (lane == 0) s_m[h] = top;
+            if (lane < count) s_t[lane * a.H + h] = a.talk[(kvh * group + g0 + lane) * a.H + h] / sum;
+        }
+        __syncthreads();
+        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+        for (int b0 = 0; b0 < 16 * tiles; b0 += TV_KEYS) {
+            bf16x8 vv[TV_KEYS / 32];
+#pragma unroll
+            for (int st = 0; st < TV_KEYS / 32; ++st) {  // keys past the last one read again: their weights are 0
+                const int j = min(lo16 + b0 + 32 * st + 16 * (c / 2), lo16 + 16 * (tiles - 1));
+                const int lp = j / a.P, off = j - lp * a.P;
+                vv[st] = *(const bf16x8*)(v_base + (int64_t)table[lp] * a.page_stride + off + 8 * (c % 2));
+            }
+            const int key = b0 + threadIdx.x;
+            float w[16];
+#pragma unroll
+            for (int i = 0; i < 16; ++i) w[i] = 0.f;
+            if (key < 16 * tiles) {
+#pragma unroll 8
+                for (int g = 0; g < a.H; ++g) {
+                    const float p = __builtin_amdgcn_exp2f(s_row[(int64_t)g * K + key] - s_m[g]);
+#pragma unroll
+                    for (int i = 0; i < 16; ++i)
+                        if (i < count) w[i] = fmaf(s_t[i * a.H + g], p, w[i]);  // (the same for all threads)
+                }
+            }
+            __syncthreads();  // (the keys before have been multiplied)
+#pragma unroll
+            for (int i = 0; i < 16; ++i) s_w[i * (TV_KEYS + 8) + threadIdx.x] = (bf16_t)w[i];
+            __syncthreads();
+#pragma unroll
+            for (int st = 0; st < TV_KEYS / 32; ++st)
+                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                    vv[st], *(const bf16x8*)(s_w + r16 * (TV_KEYS + 8) + 32 * st + 8 * c), acc, 0, 0, 0);
+        }
+        if (has_values && r16 < count) {
+            bf16x4 o;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) o[i] = (bf16_t)acc[i];
+            *(bf16x4*)((bf16_t*)a.out + ((int64_t)q_start * a.H + kvh * group + g0 + r16) * a.D + e0 + 4 * c) = o;
+        }
+    }
+}
+
+// Requests of more than one token.  grid = (blocks of 16 tokens, output splits, requests), eight wavefronts.  A wavefront
+// makes the scores of HW heads (all of the model's heads over the eight), one query token a lane column:
+//   pass 1  every row's maximum and sum over its chunk;
+//   pass 2  32 keys at a time: scores again, weights into LDS as bfloat16 pairs (high and low part: 16 bits of
+//           mantissa), [key][token][head], barrier; mixed on the matrix cores ([4 tokens x 4 keys] x heads times
+//           heads x 16 heads of this workgroup's split), [token][head][key] in LDS as bfloat16, barrier; O^T += V^T W^T for
+//           the OW heads of the wavefront.
+// A split computes all scores and the sums of 8 OW output heads: OW bounds the accumulators.
+// LDS rows of 64 bytes are cut into four 16-byte pieces whose order is swizzled so that neither the writes nor the
+// reads of the two exchanges meet in a bank.
+template <int HW>
+struct TalkTile {
+    static constexpr int KT = HW == 4 ? 2 : 1;  // up to 16 heads: high and low parts share a row; up to 32: a row each
+    static constexpr int P_BYTES = KT * 512 * 64, W_BYTES = 16 * 17 * 64;
+};
+__device__ __forceinline__ int talk_p_at(int key, int q, int piece) {  // byte offset of a 16-byte piece of a weight row
+    return (key * 16 + q) * 64 + ((piece ^ (q >> 2) ^ key) & 3) * 16;
+}
+__device__ __forceinline__ int talk_w_at(int q, int h, int piece) {  // of a mixed-weight row (32 keys)
+    return (q * 17 + h) * 64 + ((piece ^ (q >> 2) ^ (h >> 2)) & 3) * 16;
+}
+
+template <int DK, int HW, int OW>
+__global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a) {
+    constexpr int D = DK * 32;
+    constexpr int KT = TalkTile<HW>::KT;
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    char* s_p = smem;
+    char* s_w = smem + TalkTile<HW>::P_BYTES;
+    const int s = blockIdx.z, out0 = blockIdx.y * 8 * OW;
+    const int q_start = a.cu_tokens[s], q_len = a.cu_tokens[s + 1] - q_start;
+    const int t0 = blockIdx.x * 16;
+    if (q_len <= 1 || t0 >= q_len) return;
+    const int past = a.kv_lens[s] - q_len;
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / LLE_WAVE), lane = threadIdx.x % LLE_WAVE;
+    const int c = lane / 16, r16 = lane % 16;
+    const int32_t* table = a.block_tables + (int64_t)a.seq_slots[s] * a.max_pages;
+    const int group = a.H / a.G, P = a.P;
+    const bf16_t* kv = (const bf16_t*)a.kv;
+    const int last = min(q_len, t0 + 16) - 1;
+    const bool exists = t0 + r16 <= last;
+    const int pos = exists ? past + t0 + r16 : -1;
+    const int lo = exists && a.chunk > 0 ? pos / a.chunk * a.chunk : 0;
+    const int key_lo = a.chunk > 0 ? (past + t0) / a.chunk * a.chunk : 0, key_hi = past + last;  // of all rows
+    const int first_step = key_lo / 32, end_step = key_hi / 32 + 1;
+    const int half_lo = key_lo / 16, half_hi = key_hi / 16;  // 16-key halves that hold keys: others may have no page
+    const int h0 = wave * HW;
+    const int heads_here = max(0, min(HW, a.H - h0));  // (the same for the whole wavefront)
+
+    // weights of heads that do not exist stay zero
+    for (int i = threadIdx.x; i < TalkTile<HW>::P_BYTES / 16; i += 512) ((uint4*)s_p)[i] = make_uint4(0, 0, 0, 0);
+
+    bf16x8 qv[HW][DK];
+    float slope[HW];
+#pragma unroll
+    for (int i = 0; i < HW; ++i) {
+        const int h = min(h0 + i, a.H - 1);
+        const bf16_t* q = (const bf16_t*)a.q + ((int64_t)(q_start + min(t0 + r16, last)) * a.H + h) * D + 8 * c;
+#pragma unroll
+        for (int ks = 0; ks < DK; ++ks) qv[i][ks] = *(const bf16x8*)(q + 32 * ks);
+        slope[i] = a.slopes ? a.slopes[h] * LOG2E : 0.f;
+    }
+    const float scale = a.scale * LOG2E;
+
+    // a step's two 16-key halves lie in one page each
+    auto half_page = [&](int half) {
+        const int j = min(max(half, half_lo), half_hi) * 16;
+        const int lp = j / P;
+        return kv + (int64_t)table[lp] * a.page_stride;
+    };
+    auto half_off = [&](int half) {
+        const int j = min(max(half, half_lo), half_hi) * 16;
+        return j - j / P * P;
+    };
+    bf16x8 kreg[2][DK], vreg[2 * DK];
+    auto load_k = [&](int step, int kvh) {
+        const int half = 2 * step + r16 / 8;
+        const bf16_t* k = half_page(half) + ((int64_t)kvh * P + half_off(half)) * D + 8 * c;
+#pragma unroll
+        for (int x = 0; x < 2; ++x)
+#pragma unroll
+            for (int ks = 0; ks < DK; ++ks) kreg[x][ks] = *(const bf16x8*)(k + (int64_t)(KEY_OF_ROW(r16, x) % 16) * D + 32 * ks);
+    };
+    auto load_v = [&](int step, int kvh) {
+        const int half = 2 * step + c / 2;
+        const bf16_t* v = half_page(half) + ((int64_t)a.G + kvh) * P * D + (int64_t)r16 * P + half_off(half) + 8 * (c % 2);
+#pragma unroll
+        for (int n = 0; n < 2 * DK; ++n) vreg[n] = *(const bf16x8*)(v + (int64_t)16 * n * P);
+    };
+    // the lane's eight base-2 scores of head h0 + i: keys 32 step + 8 c .. + 7 of the row's token
+    auto scores = [&](int step, int i, float (&x)[8]) {
+        f32x4 sc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+            for (int ks = 0; ks < DK; ++ks) sc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kreg[t][ks], qv[i][ks], sc[t], 0, 0, 0);
+        const int j0 = 32 * step + 8 * c;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            const int j = j0 + e;
+            x[e] = j < lo || j > pos ? NEG_BIG : fmaf(sc[e / 4][e % 4], scale, slope[i] * (float)(j - pos));
+        }
+    };
+    const int first_kvh = min(h0, a.H - 1) / group;
+
+    // pass 1: every lane keeps the maximum and the sum of its own keys; the four lanes of a row meet at the end
+    float m[HW], l[HW];
+#pragma unroll
+    for (int i = 0; i < HW; ++i) {
+        m[i] = NEG_BIG;
+        l[i] = 0.f;
+    }
+    if (heads_here > 0) {
+        int kvh = first_kvh;
+        load_k(first_step, kvh);
+        for (int step = first_step; step < end_step; ++step) {
+#pragma unroll
+            for (int i = 0; i < HW; ++i) {
+                if (i < heads_here) {
+                    const int own = (h0 + i) / group;
+                    if (own != kvh) load_k(step, kvh = own);
+                    float x[8];
+                    scores(step, i, x);
+                    float top = m[i];
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) top = fmaxf(top, x[e]);
+                    const float base = top <= NEG_BIG ? 0.f : top;
+                    float sum = 0.f;
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) sum += __builtin_amdgcn_exp2f(x[e] - base);
+                    l[i] = l[i] * __builtin_amdgcn_exp2f(m[i] - base) + sum;
+                    m[i] = top;
+                }
+            }
+            load_k(min(step + 1, end_step - 1), kvh = first_kvh);
+        }
+#pragma unroll
+        for (int i = 0; i < HW; ++i) {
+            float top = fmaxf(m[i], __shfl_xor(m[i], 16, LLE_WAVE));
+            top = fmaxf(top, __shfl_xor(top, 32, LLE_WAVE));
+            const float base = top <= NEG_BIG ? 0.f : top;
+            float sum = l[i] * __builtin_amdgcn_exp2f(m[i] - base);
+            sum += __shfl_xor(sum, 16, LLE_WAVE);
+            sum += __shfl_xor(sum, 32, LLE_WAVE);
+            m[i] = base;
+            l[i] = sum > 0.f ? 1.0f / sum : 0.f;  // (a row that does not exist has seen no key)
+        }
+    }
+
+    // talk's rows of this split's heads: element e of lane (c, r16) is talk[out0 + r16][8 c + e] (KT = 1: both halves of
+    // the contraction are the heads 0 .. 15)
+    bf16x8 talk;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+        const int g = KT == 1 ? (8 * c + e) % 16 : 8 * c + e, h = out0 + r16;
+        talk[e] = (bf16_t)(r16 < 8 * OW && h < a.H && g < a.H ? a.talk[h * a.H + g] : 0.f);
+    }
+    const int oh0 = out0 + wave * OW;
+    const int outs_here = max(0, min(OW, a.H - oh0));
+    const int first_vkv = min(oh0, a.H - 1) / group;
+    f32x4 o[OW][2 * DK];
+#pragma unroll
+    for (int i = 0; i < OW; ++i)
+#pragma unroll
+        for (int n = 0; n < 2 * DK; ++n) o[i][n] = f32x4{0.f, 0.f, 0.f, 0.f};
+
+    load_k(first_step, first_kvh);
+    __syncthreads();  // (the zeros are there)
+    for (int step = first_step; step < end_step; ++step) {
+        load_v(step, first_vkv);  // used behind the second barrier
+        int kvh = first_kvh;
+        if (heads_here > 0) {
+            bf16_t hi[8][HW], low[8][HW];
+#pragma unroll
+            for (int i = 0; i < HW; ++i) {
+                if (i < heads_here) {
+                    const int own = (h0 + i) / group;
+                    if (own != kvh) load_k(step, kvh = own);
+                    float x[8];
+                    scores(step, i, x);
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) {
+                        const float p = __builtin_amdgcn_exp2f(x[e] - m[i]) * l[i];
+                        hi[e][i] = (bf16_t)p;
+                        low[e][i] = (bf16_t)(p - (float)hi[e][i]);
+                    }
+                } else {
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) hi[e][i] = low[e][i] = (bf16_t)0.f;
+                }
+            }
+            load_k(min(step + 1, end_step - 1), first_kvh);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                const int key = 8 * c + e;
+                char* at_hi = s_p + talk_p_at(key, r16, h0 / 8) + (h0 % 8) * 2;
+                char* at_lo = KT == 1 ? s_p + talk_p_at(key, r16, 2 + h0 / 8) + (h0 % 8) * 2 : at_hi + 512 * 64;
+                if constexpr (HW == 1) {
+                    *(bf16_t*)at_hi = hi[e][0];
+                    *(bf16_t*)at_lo = low[e][0];
+                } else if constexpr (HW == 2) {
+                    *(bf16x2*)at_hi = bf16x2{hi[e][0], hi[e][1]};
+                    *(bf16x2*)at_lo = bf16x2{low[e][0], low[e][1]};
+                } else {
+                    *(bf16x4*)at_hi = bf16x4{hi[e][0], hi[e][1], hi[e][2], hi[e][3]};
+                    *(bf16x4*)at_lo = bf16x4{low[e][0], low[e][1], low[e][2], low[e][3]};
+                }
+            }
+        }
+        __syncthreads();
+        // 32 tiles of (4 tokens x 4 keys), four a wavefront: row r of a tile is token 4 qa + r / 4, key 4 kq + r % 4
+#pragma unroll
+        for (int t = 0; t < 4; ++t) {
+            const int tile = wave * 4 + t, qa = tile % 4, kq = tile / 4;
+            f32x4 w = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int kt = 0; kt < KT; ++kt) {
+                const bf16x8 p = *(const bf16x8*)(s_p + kt * 512 * 64 + talk_p_at(4 * kq + r16 % 4, 4 * qa + r16 / 4, c));
+                w = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p, talk, w, 0, 0, 0);
+            }
+            // lane (c, r16): head r16 of the split, token 4 qa + c, keys 4 kq .. + 3
+            *(bf16x4*)(s_w + talk_w_at(4 * qa + c, r16, kq / 2) + (kq % 2) * 8) = bf16x4{(bf16_t)w[0], (bf16_t)w[1], (bf16_t)w[2], (bf16_t)w[3]};
+        }
+        __syncthreads();
+        int vkv = first_vkv;
+#pragma unroll
+        for (int i = 0; i < OW; ++i) {
+            if (i < outs_here) {
+                const int own = (oh0 + i) / group;
+                if (own != vkv) load_v(step, vkv = own);
+                const bf16x8 w = *(const bf16x8*)(s_w + talk_w_at(r16, wave * OW + i, c));
+#pragma unroll
+                for (int n = 0; n < 2 * DK; ++n) o[i][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vreg[n], w, o[i][n], 0, 0, 0);
+            }
+        }
+    }
+    if (!exists) return;
+#pragma unroll
+    for (int i = 0; i < OW; ++i) {
+        if (i < outs_here) {
+            bf16_t* dst = (bf16_t*)a.out + ((int64_t)(q_start + t0 + r16) * a.H + oh0 + i) * D + 4 * c;
+#pragma unroll
+            for (int n = 0; n < 2 * DK; ++n)
+                *(bf16x4*)(dst + 16 * n) = bf16x4{(bf16_t)o[i][n][0], (bf16_t)o[i][n][1], (bf16_t)o[i][n][2], (bf16_t)o[i][n][3]};
+        }
+    }
+}
+
+template <int DK, int HW, int OW>
+static int talk_prefill_launch(const TalkArgs& a, int S, int max_q_len, hipStream_t stream) {
+    const size_t smem = TalkTile<HW>::P_BYTES + TalkTile<HW>::W_BYTES;
+    if (smem > 64 * 1024) {
+        hipError_t e = hipFuncSetAttribute((const void*)talking_prefill_kernel<DK, HW, OW>,
+                                           hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+        if (e != hipSuccess) return (int)e;
+    }
+    const int splits = (a.H + 8 * OW - 1) / (8 * OW);
+    talking_prefill_kernel<DK, HW, OW><<<dim3((max_q_len + 15) / 16, splits, S), 512, smem, stream>>>(a);
+    return (int)hipGetLastError();
+}
+
+template <int DK>
+static int talk_launch(const TalkArgs& a, int S, int run_decode, int splits, int K, float* ws_s, float2* ws_ml, int run_prefill,
+                       int max_q_len, int out_heads, hipStream_t stream) {
+    if (run_decode) {
+        const size_t smem = (size_t)(a.H + 16 * a.H + 4) * sizeof(float) + 16 * (TV_KEYS + 8) * sizeof(bf16_t);
+        if (smem > 64 * 1024) return (int)hipErrorInvalidValue;
+        talking_scores_kernel<DK><<<dim3(S, a.G, splits), 256, 0, stream>>>(a, ws_s, ws_ml, K);
+        hipError_t e = hipGetLastError();
+        if (e != hipSuccess) return (int)e;
+        talking_values_kernel<<<dim3(S, a.G, (a.D + 63) / 64), 256, smem, stream>>>(a, ws_s, ws_ml, K);
+        e = hipGetLastError();
+        if (e != hipSuccess) return (int)e;
+    }
+    if (run_prefill) {
+        if (a.H <= 8) return talk_prefill_launch<DK, 1, 1>(a, S, max_q_len, stream);
+        if (a.H <= 16)
+            return out_heads == 1 ? talk_prefill_launch<DK, 2, 1>(a, S, max_q_len, stream)
+                                  : talk_prefill_launch<DK, 2, 2>(a, S, max_q_len, stream);
+        return out_heads == 1 ? talk_prefill_launch<DK, 4, 1>(a, S, max_q_len, stream)
+                              : talk_prefill_launch<DK, 4, 2>(a, S, max_q_len, stream);
+    }
+    return 0;
+}
+
+// bfloat16, D 32, 64, 96 or 128, pages of a multiple of 16 keys; with run_prefill up to 32 heads.  run_decode: the batch
+// holds requests of one token (ws_s float32 [S H K], ws_ml float32 [S H K / 8]; K a multiple of 16, at least 15 more than
+// the keys that a query sees); run_prefill: it holds longer ones.  out_heads: output heads a wavefront sums up, 1 or 2.
+extern "C" int lle_talking_mfma(const void* q, const void* kv, const void* block_tables, const void* seq_slots,
+                                const void* cu_tokens, const void* kv_lens, const void* token_seq, void* out, int S, int H, int G,
+                                int D, int P, int64_t page_stride, int max_pages, int chunk, float scale, const void* slopes,
+                                const void* talk, int run_decode, int splits, int K, void* ws_s, void* ws_ml, int run_prefill,
+                                int max_q_len, int out_heads, hipStream_t stream) {
+    if (S <= 0) return 0;
+    if (H <= 0 || G <= 0 || H % G != 0 || D % 32 != 0 || D <= 0 || D > 128 || P % 16 != 0 || P <= 0 || chunk < 0 || !talk ||
+        S > 65535 || G > 65535)
+        return (int)hipErrorInvalidValue;
+    if (run_decode && (!ws_s || !ws_ml || K % 16 != 0 || K < 16 || splits < 1 || splits > 65535)) return (int)hipErrorInvalidValue;
+    if (run_prefill && (H > 32 || max_q_len < 2)) return (int)hipErrorInvalidValue;
+    const TalkArgs a{q, kv, (const int32_t*)block_tables, (const int32_t*)seq_slots, (const int32_t*)cu_tokens,
+                     (const int32_t*)kv_lens, (const int32_t*)token_seq, out, H, G, D, P, max_pages, chunk, page_stride, scale,
+                     (const float*)slopes, (const float*)talk};
+    switch (D / 32) {
+        case 1: return talk_launch<1>(a, S, run_decode, splits, K, (float*)ws_s, (float2*)ws_ml, run_prefill, max_q_len, out_heads, stream);
+        case 2: return talk_launch<2>(a, S, run_decode, splits, K, (float*)ws_s, (float2*)ws_ml, run_prefill, max_q_len, out_heads, stream);
+        case 3: return talk_launch<3>(a, S, run_decode, splits, K, (float*)ws_s, (float2*)ws_ml, run_prefill, max_q_len, out_heads, stream);
+        case 4: return talk_launch<4>(a, S, run_decode, splits, K, (float*)ws_s, (float2*)ws_ml, run_prefill, max_q_len, out_heads, stream);
+    }
+    return (int)hipErrorInvalidValue;
 }
