@@ -85,8 +85,9 @@ struct GlaArgs {
 // grid = (requests x pieces, heads).  KD >= dim (a multiple of 16) key channels are kept; a workgroup is GLA_IG groups
 // of `jt` threads: thread (ig, j) owns value channel j and the key channels [ig KD / GLA_IG, (ig + 1) KD / GLA_IG).
 // The groups' shares of o_t meet in LDS (dynamic: [GLA_IG][GLA_TC][jt]).
-template <int KD, typename T, int MODE>
-__global__ __launch_bounds__(1024) void gla_scan_kernel(GlaArgs a) {
+// MAXT: the most threads of a workgroup (wide heads take 512 where these are enough: twice the registers a thread).
+template <int KD, typename T, int MODE, int MAXT>
+__global__ __launch_bounds__(MAXT) void gla_scan_kernel(GlaArgs a) {
     constexpr bool OUT = MODE != GLA_SUMMARY;
     constexpr int KI = KD / GLA_IG;
     static_assert(KD % GLA_IG == 0, "the key channels are dealt to the groups in equal shares");
@@ -142,14 +143,18 @@ __global__ __launch_bounds__(1024) void gla_scan_kernel(GlaArgs a) {
         __syncthreads();
 #pragma unroll
         for (int t = 0; t < GLA_TC; ++t) {
-            float o = 0.f;
+            // (the branch also keeps a token's operands from being read long before its turn: all of a chunk's at
+            // once do not fit the registers)
+            if (t < nt) {
+                float o = 0.f;
 #pragma unroll
-            for (int ii = 0; ii < KI; ++ii) {
-                const int i = i0 + ii;
-                S[ii] = fmaf(s_w[t][i], S[ii], s_k[t][i] * vv[t]);
-                if (OUT) o = fmaf(s_q[t][i], S[ii], o);
+                for (int ii = 0; ii < KI; ++ii) {
+                    const int i = i0 + ii;
+                    S[ii] = fmaf(s_w[t][i], S[ii], s_k[t][i] * vv[t]);
+                    if (OUT) o = fmaf(s_q[t][i], S[ii], o);
+                }
+                if (OUT) s_o[(ig * GLA_TC + t) * jt + j] = o;
             }
-            if (OUT) s_o[(ig * GLA_TC + t) * jt + j] = o;
         }
         if (!OUT && tid < KD) {
 #pragma unroll
@@ -230,23 +235,31 @@ __global__ __launch_bounds__(256) void gla_carry_kernel(GlaArgs a) {
     }
 }
 
-template <int KD, typename T>
-static int gla_launch(const GlaArgs& a, int S, hipStream_t stream) {
+template <int KD, typename T, int MAXT>
+static int gla_launch_of(const GlaArgs& a, int S, hipStream_t stream) {
     const int threads = a.jt * GLA_IG;
     const size_t smem = (size_t)GLA_IG * GLA_TC * a.jt * sizeof(float);
     const dim3 grid(S * a.pieces, a.H);
     if (a.pieces == 1) {
-        gla_scan_kernel<KD, T, GLA_FROM_STATE><<<grid, threads, smem, stream>>>(a);
+        gla_scan_kernel<KD, T, GLA_FROM_STATE, MAXT><<<grid, threads, smem, stream>>>(a);
         return (int)hipGetLastError();
     }
-    gla_scan_kernel<KD, T, GLA_SUMMARY><<<grid, threads, 0, stream>>>(a);
+    gla_scan_kernel<KD, T, GLA_SUMMARY, MAXT><<<grid, threads, 0, stream>>>(a);
     hipError_t e = hipGetLastError();
     if (e != hipSuccess) return (int)e;
     gla_carry_kernel<<<dim3(S, a.H, (a.dim * a.vdim + 255) / 256), 256, 0, stream>>>(a);
     e = hipGetLastError();
     if (e != hipSuccess) return (int)e;
-    gla_scan_kernel<KD, T, GLA_FROM_ENTRY><<<grid, threads, smem, stream>>>(a);
+    gla_scan_kernel<KD, T, GLA_FROM_ENTRY, MAXT><<<grid, threads, smem, stream>>>(a);
     return (int)hipGetLastError();
+}
+
+template <int KD, typename T>
+static int gla_launch(const GlaArgs& a, int S, hipStream_t stream) {
+    if constexpr (KD >= 96) {
+        if (a.jt * GLA_IG <= 512) return gla_launch_of<KD, T, 512>(a, S, stream);
+    }
+    return gla_launch_of<KD, T, 1024>(a, S, stream);
 }
 
 extern "C" int lle_gla_max_dim(void) { return 256; }

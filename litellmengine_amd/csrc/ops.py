@@ -1292,7 +1292,7 @@ class HipOps:
         out = torch.empty((N, H * D), dtype=q.dtype, device=q.device)
         run_decode, run_prefill = min_q_len <= 1, max_q_len > 1
         if (q.dtype == torch.bfloat16 and D % 32 == 0 and D <= 128 and P % 16 == 0 and max_q_len > 0 and max_kv_len > 0
-                and S <= 65535 and (H <= 32 if run_prefill else H <= 512) and not self.force_generic_attention):
+                and S <= 65535 and (H <= 32 if run_prefill else H <= 128) and not self.force_generic_attention):
             K = splits = 0
             ws_s = ws_ml = None
             if run_decode:
@@ -1302,15 +1302,16 @@ class HipOps:
                 splits = int(max(1, min(-(-K // 64), 2 * self.compute_units() // max(1, S * G))))
                 ws_s = torch.empty((S * H * K,), dtype=torch.float32, device=q.device)
                 ws_ml = torch.empty((S * H * (K // 16) * 2,), dtype=torch.float32, device=q.device)
-            # one output head a wavefront twice the workgroups, which make all scores again: where the tiles leave CUs idle
-            out_heads = 1 if -(-max_q_len // 16) * S * 4 <= self.compute_units() else 2
+            ws_sums = torch.empty((N * H,), dtype=torch.float32, device=q.device) if run_prefill else None
+            # one output head a wavefront: twice the workgroups, which make all scores again; where the tiles leave CUs idle
+            out_heads = 1 if -(-max_q_len // 16) * S * (2 if H > 16 else 1) * 2 <= self.compute_units() else 2
             self._run("talking", "lle_talking_mfma",
                       [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _L, _I, _I, _F, _P, _P, _I, _I, _I, _P, _P, _I, _I, _I,
-                       _P],
+                       _P, _P],
                       _ptr(q), _ptr(kv_layer), _ptr(block_table), _ptr(seq_slots), _ptr(cu_tokens), _ptr(kv_lens),
                       _ptr(token_seq), _ptr(out), S, H, G, D, P, kv_layer.stride(0), block_table.shape[1], int(chunk or 0),
                       float(scale), _ptr(slopes), _ptr(talk), int(run_decode), splits, K, _ptr(ws_s), _ptr(ws_ml),
-                      int(run_prefill), max_q_len, out_heads)
+                      int(run_prefill), max_q_len, out_heads, _ptr(ws_sums))
             return out
         self._run("talking", "lle_talking_generic",
                   [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _L, _I, _I, _F, _P, _P, _I, _P],

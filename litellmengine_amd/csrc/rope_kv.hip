@@ -906,50 +906,68 @@ __device__ __forceinline__ float2 pr_pair(const T* __restrict__ row, const T* __
     return x;
 }
 
-template <typename T> struct PrPair;
-template <> struct PrPair<float> { typedef float2 vec; };
-template <> struct PrPair<bf16_t> { typedef bf16_t vec __attribute__((ext_vector_type(2))); };
-template <typename T>
-__device__ __forceinline__ void pr_store(T* p, float2 x) {  // p on a multiple of two elements (D is even)
-    typename PrPair<T>::vec v;
-    v.x = from_f32<T>(x.x);
-    v.y = from_f32<T>(x.y);
-    *(typename PrPair<T>::vec*)p = v;
-}
-
-template <typename T>
+// grid = (runs of PR_TOKENS tokens, shares of a run's heads)
+template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void pair_rope_write_kernel(
     const T* __restrict__ u, int cols, const T* __restrict__ bias, const int32_t* __restrict__ slots,
     const float* __restrict__ cos_sin, int rot, const float* __restrict__ v_cos_sin, T* __restrict__ q_out,
     T* __restrict__ kv_layer, int N, int nq, int nkv, int dim, int vdim, int D, int page_size, int64_t page_stride,
     int write_kv) {
+    // q and k: a thread takes EPT elements of a head; VEC (rows, heads and the cache's heads of a multiple of eight
+    // elements): eight, in one load and one store
+    constexpr int EPT = VEC ? 8 : 2;
+    typedef T vec_t __attribute__((ext_vector_type(EPT)));
     const int64_t n0 = (int64_t)blockIdx.x * PR_TOKENS;
     const int count = (int)min((int64_t)PR_TOKENS, N - n0);
-    const int half = D / 2, q_pairs = nq * half, k_pairs = nkv * half;
-    const int per_token = q_pairs + (write_kv ? k_pairs : 0);
-    for (int idx = threadIdx.x; idx < count * per_token; idx += blockDim.x) {
+    const int first = blockIdx.y * blockDim.x + threadIdx.x, stride = gridDim.y * blockDim.x;
+    const int per_head = D / EPT, q_items = nq * per_head;
+    const int per_token = q_items + (write_kv ? nkv * per_head : 0);
+    for (int idx = first; idx < count * per_token; idx += stride) {
         const int t = idx / per_token, p = idx - t * per_token;
         const int64_t n = n0 + t;
+        const bool is_q = p < q_items;
+        const int pp = is_q ? p : p - q_items;
+        const int h = pp / per_head, e = EPT * (pp - h * per_head);
         const T* row = u + n * cols;
-        const float* cs = cos_sin + n * rot;
-        const bool is_q = p < q_pairs;
-        const int pp = is_q ? p : p - q_pairs;
-        const int h = pp / half, e = 2 * (pp - h * half);
-        const float2 x = pr_pair<T>(row, bias, (is_q ? 0 : nq * dim) + h * dim, e, dim, cs, rot);
-        if (is_q) {
-            pr_store<T>(q_out + (n * nq + h) * D + e, x);
-        } else {
-            const int slot = slots[n];
-            if (slot >= 0) {
-                const int page = slot / page_size, off = slot - page * page_size;
-                pr_store<T>(kv_layer + (int64_t)page * page_stride + ((int64_t)h * page_size + off) * D + e, x);
+        const int col0 = (is_q ? 0 : nq * dim) + h * dim;
+        const int slot = is_q ? 0 : slots[n];
+        vec_t out;
+        if constexpr (VEC) {
+            if (e < dim) {
+                const vec_t x = *(const vec_t*)(row + col0 + e);
+                vec_t b;
+                if (bias) b = *(const vec_t*)(bias + col0 + e);
+#pragma unroll
+                for (int i = 0; i < EPT; i += 2) {
+                    float2 y = make_float2(to_f32<T>(x[i]), to_f32<T>(x[i + 1]));
+                    if (bias) y = make_float2(y.x + to_f32<T>(b[i]), y.y + to_f32<T>(b[i + 1]));
+                    if (e + i < rot) {
+                        const float2 cs = *(const float2*)(cos_sin + n * rot + e + i);
+                        y = make_float2(y.x * cs.x - y.y * cs.y, y.y * cs.x + y.x * cs.y);
+                    }
+                    out[i] = from_f32<T>(y.x);
+                    out[i + 1] = from_f32<T>(y.y);
+                }
+            } else {
+#pragma unroll
+                for (int i = 0; i < EPT; ++i) out[i] = from_f32<T>(0.f);
             }
+        } else {
+            const float2 y = pr_pair<T>(row, bias, col0, e, dim, cos_sin + n * rot, rot);
+            out[0] = from_f32<T>(y.x);
+            out[1] = from_f32<T>(y.y);
+        }
+        if (is_q) {
+            *(vec_t*)(q_out + (n * nq + h) * D + e) = out;
+        } else if (slot >= 0) {
+            const int page = slot / page_size, off = slot - page * page_size;
+            *(vec_t*)(kv_layer + (int64_t)page * page_stride + ((int64_t)h * page_size + off) * D + e) = out;
         }
     }
     if (!write_kv) return;
-    const int v_col = (nq + nkv) * dim;
+    const int half = D / 2, v_col = (nq + nkv) * dim;
     int my_slots[PR_TOKENS];
-    bool run = count == PR_TOKENS && PR_TOKENS % 8 == 0;  // the tokens lie side by side in one page, from a multiple of 8 on
+    bool run = count == PR_TOKENS;  // the tokens lie side by side in one page, from a multiple of PR_TOKENS on
 #pragma unroll
     for (int t = 0; t < PR_TOKENS; ++t) {
         my_slots[t] = t < count ? slots[n0 + t] : -1;
@@ -957,7 +975,7 @@ __global__ __launch_bounds__(256) void pair_rope_write_kernel(
     }
     const int first_off = my_slots[0] >= 0 ? my_slots[0] % page_size : 0;
     run = run && my_slots[0] >= 0 && first_off % PR_TOKENS == 0 && page_size % PR_TOKENS == 0;
-    for (int p = threadIdx.x; p < k_pairs; p += blockDim.x) {
+    for (int p = first; p < nkv * half; p += stride) {
         const int h = p / half, e = 2 * (p - h * half);
         float2 x[PR_TOKENS];
 #pragma unroll
@@ -999,16 +1017,22 @@ extern "C" int lle_pair_rope_write(const void* u, int cols, const void* bias, co
     if (rot % 2 || rot > dim || dim > D || vdim > D || D % 2 || (rot > 0 && !cos_sin) || (v_cos_sin && vdim % 2) ||
         cols < nq * dim + nkv * (dim + vdim))
         return (int)hipErrorInvalidValue;
-    const int grid = (N + PR_TOKENS - 1) / PR_TOKENS;
-    if (dtype == LLE_F32)
-        pair_rope_write_kernel<float><<<grid, 256, 0, stream>>>(
-            (const float*)u, cols, (const float*)bias, (const int32_t*)slots, (const float*)cos_sin, rot,
-            (const float*)v_cos_sin, (float*)q_out, (float*)kv_layer, N, nq, nkv, dim, vdim, D, page_size, page_stride, write_kv);
-    else
-        pair_rope_write_kernel<bf16_t><<<grid, 256, 0, stream>>>(
-            (const bf16_t*)u, cols, (const bf16_t*)bias, (const int32_t*)slots, (const float*)cos_sin, rot,
-            (const float*)v_cos_sin, (bf16_t*)q_out, (bf16_t*)kv_layer, N, nq, nkv, dim, vdim, D, page_size, page_stride,
-            write_kv);
+    const bool vec = dtype == LLE_BF16 && cols % 8 == 0 && dim % 8 == 0 && D % 8 == 0 && page_stride % 8 == 0;
+    // a thread should have a few items, and a step of few tokens as many workgroups as it has work for
+    const int runs = (N + PR_TOKENS - 1) / PR_TOKENS;
+    const int64_t items = (int64_t)(N < PR_TOKENS ? N : PR_TOKENS) * (nq + nkv) * (D / (vec ? 8 : 2));
+    int shares = (int)((items + 255) / 256);
+    const int most = runs >= 256 ? 4 : 1024 / runs;
+    if (shares > most) shares = most;
+    const dim3 grid(runs, shares < 1 ? 1 : shares);
+#define LLE_PR_LAUNCH(T, VEC)                                                                                            \
+    pair_rope_write_kernel<T, VEC><<<grid, 256, 0, stream>>>(                                                            \
+        (const T*)u, cols, (const T*)bias, (const int32_t*)slots, (const float*)cos_sin, rot, (const float*)v_cos_sin,   \
+        (T*)q_out, (T*)kv_layer, N, nq, nkv, dim, vdim, D, page_size, page_stride, write_kv)
+    if (dtype == LLE_F32) LLE_PR_LAUNCH(float, false);
+    else if (vec) LLE_PR_LAUNCH(bf16_t, true);
+    else LLE_PR_LAUNCH(bf16_t, false);
+#undef LLE_PR_LAUNCH
     LLE_RETURN_LAUNCH_STATUS();
 }
 

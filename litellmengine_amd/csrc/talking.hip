@@ -11,8 +11,9 @@
 // A cache page holds K as [G][page_size][D], then V as [G][D][page_size].
 //
 // Kernels:
-//  * talking_prefill_kernel: bfloat16 on the matrix cores, heads of a multiple of 32 up to 128, up to 32 heads, pages of
-//    a multiple of 16: requests of more than one token.  A workgroup takes 16 tokens of a request and ALL heads.
+//  * talking_sums_kernel + talking_prefill_kernel: bfloat16 on the matrix cores, heads of a multiple of 32 up to 128, up
+//    to 32 heads, pages of a multiple of 16: requests of more than one token.  The first leaves every row's log of the
+//    softmax's sum; in the second a workgroup takes 16 tokens of a request and ALL heads.
 //  * talking_scores_kernel + talking_values_kernel: the same sizes, decoded tokens (any number of heads).
 //  * talking_generic_kernel: any type and size.
 #include "common.h"
@@ -226,17 +227,19 @@ __global__ __launch_bounds__(256) void talking_scores_kernel(TalkArgs a, float* 
     }
 }
 
-// Decoded tokens, second launch: weights, mix, values.  grid = (requests, G, blocks of 64 value elements), four
-// wavefronts of 16 elements each.  256 keys at a time: a thread makes one key's weights of all heads and mixes them
-// for the key/value head's own query heads (16 at a time), the weights cross through LDS, and the values, asked for
-// before that, are multiplied on the matrix cores.  LDS: maxima [H], talk / sum [16][H], weights [16][256 + 8].
-#define TV_KEYS 256
-__global__ __launch_bounds__(256) void talking_values_kernel(TalkArgs a, const float* __restrict__ ws_s,
-                                                             const float2* __restrict__ ws_ml, int K) {
-    extern __shared__ float lds[];
-    float* s_m = lds;
-    float* s_t = s_m + a.H;  // [16][H]
-    bf16_t* s_w = (bf16_t*)(s_t + 16 * a.H + (a.H % 4 ? 4 - a.H % 4 : 0));  // [16][TV_KEYS + 8], 16-byte aligned
+// Decoded tokens, second launch: weights, mix, values.  grid = (requests, G, blocks of 64 value elements), sixteen
+// wavefronts.  1024 keys at a time: a thread makes one key's weights of all heads and mixes them for CNT query heads of
+// the key/value head, the weights cross through LDS, and the values, asked for before that, are multiplied on the matrix
+// cores: wavefront w takes elements 16 (w % 4) .. and keys 256 (w / 4) .. of them; the four shares meet in LDS.
+#define TV_KEYS 1024
+#define TV_ROW (TV_KEYS + 8)  // (rows of the weights in LDS: 16 bytes more, so that rows start in different banks)
+template <int CNT>
+__global__ __launch_bounds__(1024) void talking_values_kernel(TalkArgs a, const float* __restrict__ ws_s,
+                                                              const float2* __restrict__ ws_ml, int K) {
+    extern __shared__ __attribute__((aligned(16))) float lds[];
+    bf16_t* s_w = (bf16_t*)lds;          // [CNT][TV_ROW], then the shares [4][CNT][64] in the same place
+    float* s_m = lds + CNT * TV_ROW / 2;  // [H]
+    float* s_t = s_m + a.H;               // [H][CNT]: talk / sum
     const int s = blockIdx.x, kvh = blockIdx.y;
     const int q_start = a.cu_tokens[s];
     if (a.cu_tokens[s + 1] - q_start != 1) return;
@@ -246,14 +249,14 @@ __global__ __launch_bounds__(256) void talking_values_kernel(TalkArgs a, const f
     const int wave = threadIdx.x / LLE_WAVE, lane = threadIdx.x % LLE_WAVE, c = lane / 16, r16 = lane % 16;
     const int32_t* table = a.block_tables + (int64_t)a.seq_slots[s] * a.max_pages;
     const int group = a.H / a.G;
-    const int e0 = blockIdx.z * 64 + wave * 16;  // this wavefront's value elements
-    const bool has_values = e0 < a.D;            // (the same for the whole wavefront)
+    const int e0 = blockIdx.z * 64 + (wave % 4) * 16, part = wave / 4;
+    const bool has_values = e0 < a.D;  // (the same for the whole wavefront)
     const bf16_t* v_base = (const bf16_t*)a.kv + ((int64_t)a.G + kvh) * a.P * a.D + (int64_t)(has_values ? e0 + r16 : 0) * a.P;
     const float* s_row = ws_s + (int64_t)s * a.H * K;
-    for (int g0 = 0; g0 < group; g0 += 16) {
-        const int count = min(16, group - g0);
+    for (int g0 = 0; g0 < group; g0 += CNT) {
+        const int count = min(CNT, group - g0);
         __syncthreads();
-        for (int h = wave; h < a.H; h += 4) {
+        for (int h = wave; h < a.H; h += 16) {
             const float2* ml = ws_ml + ((int64_t)s * a.H + h) * (K / 16);
             float top = NEG_BIG;
             for (int t = lane; t < tiles; t += LLE_WAVE) top = fmaxf(top, ml[t].x);
@@ -262,82 +265,221 @@ __global__ __launch_bounds__(256) void talking_values_kernel(TalkArgs a, const f
             for (int t = lane; t < tiles; t += LLE_WAVE) sum += ml[t].y * __builtin_amdgcn_exp2f(ml[t].x - top);
             sum = wave_sum(sum);
             if (lane == 0) s_m[h] = top;
-            if (lane < count) s_t[lane * a.H + h] = a.talk[(kvh * group + g0 + lane) * a.H + h] / sum;
+            if (lane < CNT) s_t[h * CNT + lane] = lane < count ? a.talk[(kvh * group + g0 + lane) * a.H + h] / sum : 0.f;
         }
         __syncthreads();
         f32x4 acc = {0.f, 0.f, 0.f, 0.f};
         for (int b0 = 0; b0 < 16 * tiles; b0 += TV_KEYS) {
-            bf16x8 vv[TV_KEYS / 32];
+            bf16x8 vv[8];
 #pragma unroll
-            for (int st = 0; st < TV_KEYS / 32; ++st) {  // keys past the last one read again: their weights are 0
-                const int j = min(lo16 + b0 + 32 * st + 16 * (c / 2), lo16 + 16 * (tiles - 1));
+            for (int st = 0; st < 8; ++st) {  // keys past the last one read again: their weights are 0
+                const int j = min(lo16 + b0 + 256 * part + 32 * st + 16 * (c / 2), lo16 + 16 * (tiles - 1));
                 const int lp = j / a.P, off = j - lp * a.P;
                 vv[st] = *(const bf16x8*)(v_base + (int64_t)table[lp] * a.page_stride + off + 8 * (c % 2));
             }
             const int key = b0 + threadIdx.x;
-            float w[16];
+            float w[CNT];
 #pragma unroll
-            for (int i = 0; i < 16; ++i) w[i] = 0.f;
+            for (int i = 0; i < CNT; ++i) w[i] = 0.f;
             if (key < 16 * tiles) {
 #pragma unroll 8
                 for (int g = 0; g < a.H; ++g) {
                     const float p = __builtin_amdgcn_exp2f(s_row[(int64_t)g * K + key] - s_m[g]);
 #pragma unroll
-                    for (int i = 0; i < 16; ++i)
-                        if (i < count) w[i] = fmaf(s_t[i * a.H + g], p, w[i]);  // (the same for all threads)
+                    for (int i = 0; i < CNT; ++i) w[i] = fmaf(s_t[g * CNT + i], p, w[i]);  // (the same for all threads)
                 }
             }
             __syncthreads();  // (the keys before have been multiplied)
 #pragma unroll
-            for (int i = 0; i < 16; ++i) s_w[i * (TV_KEYS + 8) + threadIdx.x] = (bf16_t)w[i];
+            for (int i = 0; i < CNT; ++i) s_w[i * TV_ROW + threadIdx.x] = (bf16_t)w[i];
             __syncthreads();
 #pragma unroll
-            for (int st = 0; st < TV_KEYS / 32; ++st)
-                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                    vv[st], *(const bf16x8*)(s_w + r16 * (TV_KEYS + 8) + 32 * st + 8 * c), acc, 0, 0, 0);
+            for (int st = 0; st < 8; ++st) {
+                const bf16x8 p = *(const bf16x8*)(s_w + (r16 % CNT) * TV_ROW + 256 * part + 32 * st + 8 * c);
+                acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv[st], p, acc, 0, 0, 0);
+            }
         }
-        if (has_values && r16 < count) {
-            bf16x4 o;
+        __syncthreads();
+        float* s_o = lds;  // [4][CNT][64]
+        if (r16 < CNT) *(f32x4*)(s_o + (part * CNT + r16) * 64 + (wave % 4) * 16 + 4 * c) = acc;
+        __syncthreads();
+        for (int i = threadIdx.x; i < count * 64; i += blockDim.x) {
+            const int e = blockIdx.z * 64 + i % 64;
+            if (e < a.D) {
+                float o = 0.f;
 #pragma unroll
-            for (int i = 0; i < 4; ++i) o[i] = (bf16_t)acc[i];
-            *(bf16x4*)((bf16_t*)a.out + ((int64_t)q_start * a.H + kvh * group + g0 + r16) * a.D + e0 + 4 * c) = o;
+                for (int p = 0; p < 4; ++p) o += s_o[p * CNT * 64 + i];
+                ((bf16_t*)a.out)[((int64_t)q_start * a.H + kvh * group + g0 + i / 64) * a.D + e] = (bf16_t)o;
+            }
         }
     }
 }
 
-// Requests of more than one token.  grid = (blocks of 16 tokens, output splits, requests), eight wavefronts.  A wavefront
-// makes the scores of HW heads (all of the model's heads over the eight), one query token a lane column:
-//   pass 1  every row's maximum and sum over its chunk;
-//   pass 2  32 keys at a time: scores again, weights into LDS as bfloat16 pairs (high and low part: 16 bits of
-//           mantissa), [key][token][head], barrier; mixed on the matrix cores ([4 tokens x 4 keys] x heads times
-//           heads x 16 heads of this workgroup's split), [token][head][key] in LDS as bfloat16, barrier; O^T += V^T W^T for
-//           the OW heads of the wavefront.
-// A split computes all scores and the sums of 8 OW output heads: OW bounds the accumulators.
-// LDS rows of 64 bytes are cut into four 16-byte pieces whose order is swizzled so that neither the writes nor the
-// reads of the two exchanges meet in a bank.
+// Portions, first launch: the base-2 log of every row's sum, ws [N][H].  grid = (blocks of 16 tokens, G, requests), four
+// wavefronts that take every fourth 32-key step; a wavefront makes the scores of four of the key/value head's query heads
+// with the keys in its registers (the other four and so on in further rounds).
+#define TS_HEADS 4
+template <int DK>
+__global__ __launch_bounds__(256) void talking_sums_kernel(TalkArgs a, float* __restrict__ ws) {
+    constexpr int D = DK * 32;
+    __shared__ float s_m[4][TS_HEADS][16], s_l[4][TS_HEADS][16];
+    const int s = blockIdx.z, kvh = blockIdx.y;
+    const int q_start = a.cu_tokens[s], q_len = a.cu_tokens[s + 1] - q_start;
+    const int blocks = (q_len + 15) / 16;
+    if (q_len <= 1 || (int)blockIdx.x >= blocks) return;
+    const int t0 = (blocks - 1 - (int)blockIdx.x) * 16;
+    const int past = a.kv_lens[s] - q_len;
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / LLE_WAVE), lane = threadIdx.x % LLE_WAVE;
+    const int c = lane / 16, r16 = lane % 16;
+    const int32_t* table = a.block_tables + (int64_t)a.seq_slots[s] * a.max_pages;
+    const int group = a.H / a.G, P = a.P;
+    const bf16_t* kv = (const bf16_t*)a.kv;
+    const int last = min(q_len, t0 + 16) - 1;
+    const bool exists = t0 + r16 <= last;
+    const int pos = exists ? past + t0 + r16 : -1;
+    const int lo = exists && a.chunk > 0 ? pos / a.chunk * a.chunk : 0;
+    const int key_lo = a.chunk > 0 ? (past + t0) / a.chunk * a.chunk : 0, key_hi = past + last;
+    const int open_lo = a.chunk > 0 ? key_hi / a.chunk * a.chunk : 0, open_hi = past + t0;  // keys that every row sees
+    const int first_step = key_lo / 32, end_step = key_hi / 32 + 1;
+    const int half_lo = key_lo / 16, half_hi = key_hi / 16;
+    const float scale = a.scale * LOG2E;
+    bf16x8 kreg[2][DK];
+    auto page_of = [&](int step) {
+        const int j = min(max(2 * step + r16 / 8, half_lo), half_hi) * 16;
+        return table[j / P];
+    };
+    auto load_k = [&](int step, int page) {
+        const int j = min(max(2 * step + r16 / 8, half_lo), half_hi) * 16;
+        const bf16_t* k = kv + (int64_t)page * a.page_stride + ((int64_t)kvh * P + (j - j / P * P)) * D + 8 * c;
+#pragma unroll
+        for (int x = 0; x < 2; ++x)
+#pragma unroll
+            for (int ks = 0; ks < DK; ++ks) kreg[x][ks] = *(const bf16x8*)(k + (int64_t)(KEY_OF_ROW(r16, x) % 16) * D + 32 * ks);
+    };
+    for (int g0 = 0; g0 < group; g0 += TS_HEADS) {
+        bf16x8 qv[TS_HEADS][DK];
+        float slope[TS_HEADS], m[TS_HEADS], l[TS_HEADS];
+#pragma unroll
+        for (int i = 0; i < TS_HEADS; ++i) {
+            const int h = kvh * group + min(g0 + i, group - 1);
+            const bf16_t* q = (const bf16_t*)a.q + ((int64_t)(q_start + min(t0 + r16, last)) * a.H + h) * D + 8 * c;
+#pragma unroll
+            for (int ks = 0; ks < DK; ++ks) qv[i][ks] = *(const bf16x8*)(q + 32 * ks);
+            slope[i] = a.slopes ? a.slopes[h] * LOG2E : 0.f;
+            m[i] = NEG_BIG;
+            l[i] = 0.f;
+        }
+        const int heads = min(TS_HEADS, group - g0);
+        int page = page_of(first_step + wave);
+        load_k(first_step + wave, page);
+        page = page_of(first_step + wave + 4);
+        for (int step = first_step + wave; step < end_step; step += 4) {
+            f32x4 sc[TS_HEADS][2];
+#pragma unroll
+            for (int i = 0; i < TS_HEADS; ++i) {
+                sc[i][0] = sc[i][1] = f32x4{0.f, 0.f, 0.f, 0.f};
+                if (i < heads) {
+#pragma unroll
+                    for (int t = 0; t < 2; ++t)
+#pragma unroll
+                        for (int ks = 0; ks < DK; ++ks)
+                            sc[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kreg[t][ks], qv[i][ks], sc[i][t], 0, 0, 0);
+                }
+            }
+            load_k(step + 4, page);  // (past the last step: keys that are there)
+            page = page_of(step + 8);
+            const bool open = 32 * step >= open_lo && 32 * step + 31 <= open_hi;  // (the same for all lanes)
+            const float d0 = (float)(32 * step + 8 * c - pos);
+#pragma unroll
+            for (int i = 0; i < TS_HEADS; ++i) {
+                if (i < heads) {
+                    float x[8], top = m[i];
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) x[e] = fmaf(sc[i][e / 4][e % 4], scale, slope[i] * (d0 + (float)e));
+                    if (!open) {
+#pragma unroll
+                        for (int e = 0; e < 8; ++e) {
+                            const int j = 32 * step + 8 * c + e;
+                            if (j < lo || j > pos) x[e] = NEG_BIG;
+                        }
+                    }
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) top = fmaxf(top, x[e]);
+                    const float base = top <= NEG_BIG ? 0.f : top;
+                    float sum = 0.f;
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) sum += __builtin_amdgcn_exp2f(x[e] - base);
+                    l[i] = l[i] * __builtin_amdgcn_exp2f(m[i] - base) + sum;
+                    m[i] = top;
+                }
+            }
+        }
+        __syncthreads();  // (the round before has been read)
+#pragma unroll
+        for (int i = 0; i < TS_HEADS; ++i) {
+            float top = fmaxf(m[i], __shfl_xor(m[i], 16, LLE_WAVE));
+            top = fmaxf(top, __shfl_xor(top, 32, LLE_WAVE));
+            const float base = top <= NEG_BIG ? 0.f : top;
+            float sum = l[i] * __builtin_amdgcn_exp2f(m[i] - base);
+            sum += __shfl_xor(sum, 16, LLE_WAVE);
+            sum += __shfl_xor(sum, 32, LLE_WAVE);
+            if (c == 0) {
+                s_m[wave][i][r16] = top;
+                s_l[wave][i][r16] = sum;
+            }
+        }
+        __syncthreads();
+        if (threadIdx.x < TS_HEADS * 16) {
+            const int i = threadIdx.x / 16, r = threadIdx.x % 16;
+            if (i < heads && t0 + r <= last) {
+                float top = s_m[0][i][r];
+#pragma unroll
+                for (int w = 1; w < 4; ++w) top = fmaxf(top, s_m[w][i][r]);
+                float sum = 0.f;  // (a row sees a key: itself)
+#pragma unroll
+                for (int w = 0; w < 4; ++w) sum += s_l[w][i][r] * __builtin_amdgcn_exp2f(s_m[w][i][r] - top);
+                ws[(int64_t)(q_start + t0 + r) * a.H + kvh * group + g0 + i] = top + log2f(sum);
+            }
+        }
+    }
+}
+
+// Portions, second launch.  grid = (output splits, blocks of 16 tokens, requests), eight wavefronts.  A wavefront makes the
+// scores of HW heads (all of the model's heads over the eight), one query token a lane column.  Three things happen in
+// step i, each to another 32 keys, with one barrier a step between them:
+//   keys i      scores, weights (divided by their sum already) into LDS as bfloat16 pairs (high and low part: 16 bits of
+//               mantissa), [key][token][head];
+//   keys i - 1  mixed on the matrix cores ([4 tokens x 4 keys] x heads times heads x 16 heads of this workgroup's
+//               split), [token][head][key] into LDS as bfloat16;
+//   keys i - 2  O^T += V^T W^T for the OW heads of the wavefront.
+// Both LDS buffers are there twice.  A split computes all scores and the sums of 8 OW output heads: OW bounds the
+// accumulators.  LDS rows of 64 bytes are cut into four 16-byte pieces whose order is swizzled so that neither the writes nor
+// the reads of the two exchanges meet in a bank.
 template <int HW>
 struct TalkTile {
     static constexpr int KT = HW == 4 ? 2 : 1;  // up to 16 heads: high and low parts share a row; up to 32: a row each
-    static constexpr int P_BYTES = KT * 512 * 64, W_BYTES = 16 * 17 * 64;
+    static constexpr int P_BYTES = KT * 512 * 64, W_BYTES = 16 * 16 * 64;
 };
 __device__ __forceinline__ int talk_p_at(int key, int q, int piece) {  // byte offset of a 16-byte piece of a weight row
     return (key * 16 + q) * 64 + ((piece ^ (q >> 2) ^ key) & 3) * 16;
 }
 __device__ __forceinline__ int talk_w_at(int q, int h, int piece) {  // of a mixed-weight row (32 keys)
-    return (q * 17 + h) * 64 + ((piece ^ (q >> 2) ^ (h >> 2)) & 3) * 16;
+    const int row = h ^ q;
+    return (q * 16 + row) * 64 + ((piece ^ (row >> 2)) & 3) * 16;
 }
 
 template <int DK, int HW, int OW>
-__global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a) {
+__global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a, const float* __restrict__ sums) {
     constexpr int D = DK * 32;
-    constexpr int KT = TalkTile<HW>::KT;
+    constexpr int KT = TalkTile<HW>::KT, P_BYTES = TalkTile<HW>::P_BYTES, W_BYTES = TalkTile<HW>::W_BYTES;
     extern __shared__ __attribute__((aligned(16))) char smem[];
     char* s_p = smem;
-    char* s_w = smem + TalkTile<HW>::P_BYTES;
-    const int s = blockIdx.z, out0 = blockIdx.y * 8 * OW;
+    char* s_w = smem + 2 * P_BYTES;
+    const int s = blockIdx.z, out0 = blockIdx.x * 8 * OW;
     const int q_start = a.cu_tokens[s], q_len = a.cu_tokens[s + 1] - q_start;
-    const int t0 = blockIdx.x * 16;
-    if (q_len <= 1 || t0 >= q_len) return;
+    const int blocks = (q_len + 15) / 16;
+    if (q_len <= 1 || (int)blockIdx.y >= blocks) return;
+    const int t0 = (blocks - 1 - (int)blockIdx.y) * 16;
     const int past = a.kv_lens[s] - q_len;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / LLE_WAVE), lane = threadIdx.x % LLE_WAVE;
     const int c = lane / 16, r16 = lane % 16;
@@ -349,110 +491,49 @@ __global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a) {
     const int pos = exists ? past + t0 + r16 : -1;
     const int lo = exists && a.chunk > 0 ? pos / a.chunk * a.chunk : 0;
     const int key_lo = a.chunk > 0 ? (past + t0) / a.chunk * a.chunk : 0, key_hi = past + last;  // of all rows
-    const int first_step = key_lo / 32, end_step = key_hi / 32 + 1;
+    const int open_lo = a.chunk > 0 ? key_hi / a.chunk * a.chunk : 0, open_hi = exists ? past + t0 : -1;
+    const int first_step = key_lo / 32, steps = key_hi / 32 + 1 - first_step;
     const int half_lo = key_lo / 16, half_hi = key_hi / 16;  // 16-key halves that hold keys: others may have no page
     const int h0 = wave * HW;
     const int heads_here = max(0, min(HW, a.H - h0));  // (the same for the whole wavefront)
+    const bool all_rows = last - t0 == 15;
 
     // weights of heads that do not exist stay zero
-    for (int i = threadIdx.x; i < TalkTile<HW>::P_BYTES / 16; i += 512) ((uint4*)s_p)[i] = make_uint4(0, 0, 0, 0);
+    for (int i = threadIdx.x; i < 2 * P_BYTES / 16; i += 512) ((uint4*)s_p)[i] = make_uint4(0, 0, 0, 0);
 
     bf16x8 qv[HW][DK];
-    float slope[HW];
+    float slope[HW], sum[HW];
 #pragma unroll
     for (int i = 0; i < HW; ++i) {
         const int h = min(h0 + i, a.H - 1);
-        const bf16_t* q = (const bf16_t*)a.q + ((int64_t)(q_start + min(t0 + r16, last)) * a.H + h) * D + 8 * c;
+        const int64_t tok = q_start + min(t0 + r16, last);
+        const bf16_t* q = (const bf16_t*)a.q + (tok * a.H + h) * D + 8 * c;
 #pragma unroll
         for (int ks = 0; ks < DK; ++ks) qv[i][ks] = *(const bf16x8*)(q + 32 * ks);
         slope[i] = a.slopes ? a.slopes[h] * LOG2E : 0.f;
+        sum[i] = sums[tok * a.H + h];
     }
     const float scale = a.scale * LOG2E;
 
-    // a step's two 16-key halves lie in one page each
-    auto half_page = [&](int half) {
-        const int j = min(max(half, half_lo), half_hi) * 16;
-        const int lp = j / P;
-        return kv + (int64_t)table[lp] * a.page_stride;
-    };
-    auto half_off = [&](int half) {
-        const int j = min(max(half, half_lo), half_hi) * 16;
-        return j - j / P * P;
-    };
+    // a step's two 16-key halves lie in one page each; a lane's keys lie in half r16 / 8, its values' keys in half c / 2
+    const int k_half = r16 / 8, v_half = c / 2;
+    auto key_of = [&](int i, int half) { return min(max(2 * (first_step + i) + half, half_lo), half_hi) * 16; };
+    auto page_of = [&](int i, int half) { return table[key_of(i, half) / P]; };
     bf16x8 kreg[2][DK], vreg[2 * DK];
-    auto load_k = [&](int step, int kvh) {
-        const int half = 2 * step + r16 / 8;
-        const bf16_t* k = half_page(half) + ((int64_t)kvh * P + half_off(half)) * D + 8 * c;
+    auto load_k = [&](int i, int page, int kvh) {
+        const int j = key_of(i, k_half);
+        const bf16_t* k = kv + (int64_t)page * a.page_stride + ((int64_t)kvh * P + (j - j / P * P)) * D + 8 * c;
 #pragma unroll
         for (int x = 0; x < 2; ++x)
 #pragma unroll
             for (int ks = 0; ks < DK; ++ks) kreg[x][ks] = *(const bf16x8*)(k + (int64_t)(KEY_OF_ROW(r16, x) % 16) * D + 32 * ks);
     };
-    auto load_v = [&](int step, int kvh) {
-        const int half = 2 * step + c / 2;
-        const bf16_t* v = half_page(half) + ((int64_t)a.G + kvh) * P * D + (int64_t)r16 * P + half_off(half) + 8 * (c % 2);
+    auto load_v = [&](int i, int page, int kvh) {
+        const int j = key_of(i, v_half);
+        const bf16_t* v = kv + (int64_t)page * a.page_stride + ((int64_t)a.G + kvh) * P * D + (int64_t)r16 * P + (j - j / P * P) + 8 * (c % 2);
 #pragma unroll
         for (int n = 0; n < 2 * DK; ++n) vreg[n] = *(const bf16x8*)(v + (int64_t)16 * n * P);
     };
-    // the lane's eight base-2 scores of head h0 + i: keys 32 step + 8 c .. + 7 of the row's token
-    auto scores = [&](int step, int i, float (&x)[8]) {
-        f32x4 sc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
-#pragma unroll
-        for (int t = 0; t < 2; ++t)
-#pragma unroll
-            for (int ks = 0; ks < DK; ++ks) sc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kreg[t][ks], qv[i][ks], sc[t], 0, 0, 0);
-        const int j0 = 32 * step + 8 * c;
-#pragma unroll
-        for (int e = 0; e < 8; ++e) {
-            const int j = j0 + e;
-            x[e] = j < lo || j > pos ? NEG_BIG : fmaf(sc[e / 4][e % 4], scale, slope[i] * (float)(j - pos));
-        }
-    };
-    const int first_kvh = min(h0, a.H - 1) / group;
-
-    // pass 1: every lane keeps the maximum and the sum of its own keys; the four lanes of a row meet at the end
-    float m[HW], l[HW];
-#pragma unroll
-    for (int i = 0; i < HW; ++i) {
-        m[i] = NEG_BIG;
-        l[i] = 0.f;
-    }
-    if (heads_here > 0) {
-        int kvh = first_kvh;
-        load_k(first_step, kvh);
-        for (int step = first_step; step < end_step; ++step) {
-#pragma unroll
-            for (int i = 0; i < HW; ++i) {
-                if (i < heads_here) {
-                    const int own = (h0 + i) / group;
-                    if (own != kvh) load_k(step, kvh = own);
-                    float x[8];
-                    scores(step, i, x);
-                    float top = m[i];
-#pragma unroll
-                    for (int e = 0; e < 8; ++e) top = fmaxf(top, x[e]);
-                    const float base = top <= NEG_BIG ? 0.f : top;
-                    float sum = 0.f;
-#pragma unroll
-                    for (int e = 0; e < 8; ++e) sum += __builtin_amdgcn_exp2f(x[e] - base);
-                    l[i] = l[i] * __builtin_amdgcn_exp2f(m[i] - base) + sum;
-                    m[i] = top;
-                }
-            }
-            load_k(min(step + 1, end_step - 1), kvh = first_kvh);
-        }
-#pragma unroll
-        for (int i = 0; i < HW; ++i) {
-            float top = fmaxf(m[i], __shfl_xor(m[i], 16, LLE_WAVE));
-            top = fmaxf(top, __shfl_xor(top, 32, LLE_WAVE));
-            const float base = top <= NEG_BIG ? 0.f : top;
-            float sum = l[i] * __builtin_amdgcn_exp2f(m[i] - base);
-            sum += __shfl_xor(sum, 16, LLE_WAVE);
-            sum += __shfl_xor(sum, 32, LLE_WAVE);
-            m[i] = base;
-            l[i] = sum > 0.f ? 1.0f / sum : 0.f;  // (a row that does not exist has seen no key)
-        }
-    }
 
     // talk's rows of this split's heads: element e of lane (c, r16) is talk[out0 + r16][8 c + e] (KT = 1: both halves of
     // the contraction are the heads 0 .. 15)
@@ -464,44 +545,65 @@ __global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a) {
     }
     const int oh0 = out0 + wave * OW;
     const int outs_here = max(0, min(OW, a.H - oh0));
-    const int first_vkv = min(oh0, a.H - 1) / group;
+    const int first_kvh = min(h0, a.H - 1) / group, first_vkv = min(oh0, a.H - 1) / group;
     f32x4 o[OW][2 * DK];
 #pragma unroll
     for (int i = 0; i < OW; ++i)
 #pragma unroll
         for (int n = 0; n < 2 * DK; ++n) o[i][n] = f32x4{0.f, 0.f, 0.f, 0.f};
 
-    load_k(first_step, first_kvh);
+    // a page is looked up one step before its keys or values are asked for, these one step before they are used
+    int k_page = page_of(0, k_half), k_page_now = k_page, v_page = page_of(0, v_half), v_page_now = v_page;
+    load_k(0, k_page, first_kvh);
+    k_page = page_of(1, k_half);
     __syncthreads();  // (the zeros are there)
-    for (int step = first_step; step < end_step; ++step) {
-        load_v(step, first_vkv);  // used behind the second barrier
-        int kvh = first_kvh;
-        if (heads_here > 0) {
+    for (int i = 0; i < steps + 2; ++i) {
+        if (i < steps && heads_here > 0) {
+            const int step = first_step + i;
             bf16_t hi[8][HW], low[8][HW];
+            int kvh = first_kvh;
+            const bool open = all_rows && 32 * step >= open_lo && 32 * step + 31 <= past + t0;  // (the same for all lanes)
+            const float d0 = (float)(32 * step + 8 * c - pos);
 #pragma unroll
-            for (int i = 0; i < HW; ++i) {
-                if (i < heads_here) {
-                    const int own = (h0 + i) / group;
-                    if (own != kvh) load_k(step, kvh = own);
+            for (int n = 0; n < HW; ++n) {
+                if (n < heads_here) {
+                    const int own = (h0 + n) / group;
+                    if (own != kvh) load_k(i, k_page_now, kvh = own);
+                    f32x4 sc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+                    for (int t = 0; t < 2; ++t)
+#pragma unroll
+                        for (int ks = 0; ks < DK; ++ks) sc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kreg[t][ks], qv[n][ks], sc[t], 0, 0, 0);
                     float x[8];
-                    scores(step, i, x);
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) x[e] = fmaf(sc[e / 4][e % 4], scale, fmaf(slope[n], d0 + (float)e, -sum[n]));
+                    if (!open) {
+#pragma unroll
+                        for (int e = 0; e < 8; ++e) {
+                            const int j = 32 * step + 8 * c + e;
+                            if (j < lo || j > pos) x[e] = NEG_BIG;
+                        }
+                    }
 #pragma unroll
                     for (int e = 0; e < 8; ++e) {
-                        const float p = __builtin_amdgcn_exp2f(x[e] - m[i]) * l[i];
-                        hi[e][i] = (bf16_t)p;
-                        low[e][i] = (bf16_t)(p - (float)hi[e][i]);
+                        const float p = __builtin_amdgcn_exp2f(x[e]);
+                        hi[e][n] = (bf16_t)p;
+                        low[e][n] = (bf16_t)(p - (float)hi[e][n]);
                     }
                 } else {
 #pragma unroll
-                    for (int e = 0; e < 8; ++e) hi[e][i] = low[e][i] = (bf16_t)0.f;
+                    for (int e = 0; e < 8; ++e) hi[e][n] = low[e][n] = (bf16_t)0.f;
                 }
             }
-            load_k(min(step + 1, end_step - 1), first_kvh);
+            load_k(i + 1, k_page, first_kvh);
+            k_page_now = k_page;
+            k_page = page_of(i + 2, k_half);
+            char* buf = s_p + (i & 1) * P_BYTES;
 #pragma unroll
             for (int e = 0; e < 8; ++e) {
                 const int key = 8 * c + e;
-                char* at_hi = s_p + talk_p_at(key, r16, h0 / 8) + (h0 % 8) * 2;
-                char* at_lo = KT == 1 ? s_p + talk_p_at(key, r16, 2 + h0 / 8) + (h0 % 8) * 2 : at_hi + 512 * 64;
+                char* at_hi = buf + talk_p_at(key, r16, h0 / 8) + (h0 % 8) * 2;
+                char* at_lo = KT == 1 ? buf + talk_p_at(key, r16, 2 + h0 / 8) + (h0 % 8) * 2 : at_hi + 512 * 64;
                 if constexpr (HW == 1) {
                     *(bf16_t*)at_hi = hi[e][0];
                     *(bf16_t*)at_lo = low[e][0];
@@ -514,32 +616,45 @@ __global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a) {
                 }
             }
         }
-        __syncthreads();
-        // 32 tiles of (4 tokens x 4 keys), four a wavefront: row r of a tile is token 4 qa + r / 4, key 4 kq + r % 4
+        if (i >= 1 && i - 1 < steps) {
+            // 32 tiles of (4 tokens x 4 keys), four a wavefront: row r of a tile is token 4 qa + r / 4, key 4 kq + r % 4
+            const char* from = s_p + ((i - 1) & 1) * P_BYTES;
+            char* to = s_w + ((i - 1) & 1) * W_BYTES;
 #pragma unroll
-        for (int t = 0; t < 4; ++t) {
-            const int tile = wave * 4 + t, qa = tile % 4, kq = tile / 4;
-            f32x4 w = {0.f, 0.f, 0.f, 0.f};
+            for (int t = 0; t < 4; ++t) {
+                const int tile = wave * 4 + t, qa = tile % 4, kq = tile / 4;
+                f32x4 w = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-            for (int kt = 0; kt < KT; ++kt) {
-                const bf16x8 p = *(const bf16x8*)(s_p + kt * 512 * 64 + talk_p_at(4 * kq + r16 % 4, 4 * qa + r16 / 4, c));
-                w = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p, talk, w, 0, 0, 0);
-            }
-            // lane (c, r16): head r16 of the split, token 4 qa + c, keys 4 kq .. + 3
-            *(bf16x4*)(s_w + talk_w_at(4 * qa + c, r16, kq / 2) + (kq % 2) * 8) = bf16x4{(bf16_t)w[0], (bf16_t)w[1], (bf16_t)w[2], (bf16_t)w[3]};
-        }
-        __syncthreads();
-        int vkv = first_vkv;
-#pragma unroll
-        for (int i = 0; i < OW; ++i) {
-            if (i < outs_here) {
-                const int own = (oh0 + i) / group;
-                if (own != vkv) load_v(step, vkv = own);
-                const bf16x8 w = *(const bf16x8*)(s_w + talk_w_at(r16, wave * OW + i, c));
-#pragma unroll
-                for (int n = 0; n < 2 * DK; ++n) o[i][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vreg[n], w, o[i][n], 0, 0, 0);
+                for (int kt = 0; kt < KT; ++kt) {
+                    const bf16x8 p = *(const bf16x8*)(from + kt * 512 * 64 + talk_p_at(4 * kq + r16 % 4, 4 * qa + r16 / 4, c));
+                    w = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p, talk, w, 0, 0, 0);
+                }
+                // lane (c, r16): head r16 of the split, token 4 qa + c, keys 4 kq .. + 3
+                *(bf16x4*)(to + talk_w_at(4 * qa + c, r16, kq / 2) + (kq % 2) * 8) = bf16x4{(bf16_t)w[0], (bf16_t)w[1], (bf16_t)w[2], (bf16_t)w[3]};
             }
         }
+        if (outs_here > 0) {
+            if (i >= 2) {
+                const char* from = s_w + (i & 1) * W_BYTES;
+                int vkv = first_vkv;
+#pragma unroll
+                for (int n = 0; n < OW; ++n) {
+                    if (n < outs_here) {
+                        const int own = (oh0 + n) / group;
+                        if (own != vkv) load_v(i - 2, v_page_now, vkv = own);
+                        const bf16x8 w = *(const bf16x8*)(from + talk_w_at(r16, wave * OW + n, c));
+#pragma unroll
+                        for (int m = 0; m < 2 * DK; ++m) o[n][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vreg[m], w, o[n][m], 0, 0, 0);
+                    }
+                }
+            }
+            if (i >= 1) {
+                load_v(i - 1, v_page, first_vkv);  // used in the next step
+                v_page_now = v_page;
+                v_page = page_of(i, v_half);
+            }
+        }
+        __syncthreads();
     }
     if (!exists) return;
 #pragma unroll
@@ -554,64 +669,77 @@ __global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a) {
 }
 
 template <int DK, int HW, int OW>
-static int talk_prefill_launch(const TalkArgs& a, int S, int max_q_len, hipStream_t stream) {
-    const size_t smem = TalkTile<HW>::P_BYTES + TalkTile<HW>::W_BYTES;
+static int talk_prefill_launch(const TalkArgs& a, int S, int max_q_len, const float* sums, hipStream_t stream) {
+    const size_t smem = 2 * (TalkTile<HW>::P_BYTES + TalkTile<HW>::W_BYTES);
     if (smem > 64 * 1024) {
         hipError_t e = hipFuncSetAttribute((const void*)talking_prefill_kernel<DK, HW, OW>,
                                            hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
         if (e != hipSuccess) return (int)e;
     }
     const int splits = (a.H + 8 * OW - 1) / (8 * OW);
-    talking_prefill_kernel<DK, HW, OW><<<dim3((max_q_len + 15) / 16, splits, S), 512, smem, stream>>>(a);
+    talking_prefill_kernel<DK, HW, OW><<<dim3(splits, (max_q_len + 15) / 16, S), 512, smem, stream>>>(a, sums);
     return (int)hipGetLastError();
 }
 
 template <int DK>
 static int talk_launch(const TalkArgs& a, int S, int run_decode, int splits, int K, float* ws_s, float2* ws_ml, int run_prefill,
-                       int max_q_len, int out_heads, hipStream_t stream) {
+                       int max_q_len, int out_heads, float* ws_sums, hipStream_t stream) {
     if (run_decode) {
-        const size_t smem = (size_t)(a.H + 16 * a.H + 4) * sizeof(float) + 16 * (TV_KEYS + 8) * sizeof(bf16_t);
-        if (smem > 64 * 1024) return (int)hipErrorInvalidValue;
         talking_scores_kernel<DK><<<dim3(S, a.G, splits), 256, 0, stream>>>(a, ws_s, ws_ml, K);
         hipError_t e = hipGetLastError();
         if (e != hipSuccess) return (int)e;
-        talking_values_kernel<<<dim3(S, a.G, (a.D + 63) / 64), 256, smem, stream>>>(a, ws_s, ws_ml, K);
-        e = hipGetLastError();
+        const int group = a.H / a.G;
+        const dim3 grid(S, a.G, (a.D + 63) / 64);
+        auto values = [&](auto kernel, int cnt) {
+            const size_t smem = (size_t)cnt * TV_ROW * sizeof(bf16_t) + (size_t)a.H * (1 + cnt) * sizeof(float);
+            if (smem > 64 * 1024) return hipErrorInvalidValue;
+            kernel<<<grid, 1024, smem, stream>>>(a, (const float*)ws_s, (const float2*)ws_ml, K);
+            return hipGetLastError();
+        };
+        if (group == 1) e = values(talking_values_kernel<1>, 1);
+        else if (group == 2) e = values(talking_values_kernel<2>, 2);
+        else if (group <= 4) e = values(talking_values_kernel<4>, 4);
+        else if (group <= 8) e = values(talking_values_kernel<8>, 8);
+        else e = values(talking_values_kernel<16>, 16);
         if (e != hipSuccess) return (int)e;
     }
     if (run_prefill) {
-        if (a.H <= 8) return talk_prefill_launch<DK, 1, 1>(a, S, max_q_len, stream);
+        talking_sums_kernel<DK><<<dim3((max_q_len + 15) / 16, a.G, S), 256, 0, stream>>>(a, ws_sums);
+        const hipError_t e = hipGetLastError();
+        if (e != hipSuccess) return (int)e;
+        if (a.H <= 8) return talk_prefill_launch<DK, 1, 1>(a, S, max_q_len, ws_sums, stream);
         if (a.H <= 16)
-            return out_heads == 1 ? talk_prefill_launch<DK, 2, 1>(a, S, max_q_len, stream)
-                                  : talk_prefill_launch<DK, 2, 2>(a, S, max_q_len, stream);
-        return out_heads == 1 ? talk_prefill_launch<DK, 4, 1>(a, S, max_q_len, stream)
-                              : talk_prefill_launch<DK, 4, 2>(a, S, max_q_len, stream);
+            return out_heads == 1 ? talk_prefill_launch<DK, 2, 1>(a, S, max_q_len, ws_sums, stream)
+                                  : talk_prefill_launch<DK, 2, 2>(a, S, max_q_len, ws_sums, stream);
+        return out_heads == 1 ? talk_prefill_launch<DK, 4, 1>(a, S, max_q_len, ws_sums, stream)
+                              : talk_prefill_launch<DK, 4, 2>(a, S, max_q_len, ws_sums, stream);
     }
     return 0;
 }
 
 // bfloat16, D 32, 64, 96 or 128, pages of a multiple of 16 keys; with run_prefill up to 32 heads.  run_decode: the batch
 // holds requests of one token (ws_s float32 [S H K], ws_ml float32 [S H K / 8]; K a multiple of 16, at least 15 more than
-// the keys that a query sees); run_prefill: it holds longer ones.  out_heads: output heads a wavefront sums up, 1 or 2.
+// the keys that a query sees); run_prefill: it holds longer ones.  ws_sums float32
+// [N H].  out_heads: output heads a wavefront sums up, 1 or 2.
 extern "C" int lle_talking_mfma(const void* q, const void* kv, const void* block_tables, const void* seq_slots,
                                 const void* cu_tokens, const void* kv_lens, const void* token_seq, void* out, int S, int H, int G,
                                 int D, int P, int64_t page_stride, int max_pages, int chunk, float scale, const void* slopes,
                                 const void* talk, int run_decode, int splits, int K, void* ws_s, void* ws_ml, int run_prefill,
-                                int max_q_len, int out_heads, hipStream_t stream) {
+                                int max_q_len, int out_heads, void* ws_sums, hipStream_t stream) {
     if (S <= 0) return 0;
     if (H <= 0 || G <= 0 || H % G != 0 || D % 32 != 0 || D <= 0 || D > 128 || P % 16 != 0 || P <= 0 || chunk < 0 || !talk ||
         S > 65535 || G > 65535)
         return (int)hipErrorInvalidValue;
     if (run_decode && (!ws_s || !ws_ml || K % 16 != 0 || K < 16 || splits < 1 || splits > 65535)) return (int)hipErrorInvalidValue;
-    if (run_prefill && (H > 32 || max_q_len < 2)) return (int)hipErrorInvalidValue;
+    if (run_prefill && (H > 32 || max_q_len < 2 || !ws_sums || (max_q_len + 15) / 16 > 65535)) return (int)hipErrorInvalidValue;
     const TalkArgs a{q, kv, (const int32_t*)block_tables, (const int32_t*)seq_slots, (const int32_t*)cu_tokens,
                      (const int32_t*)kv_lens, (const int32_t*)token_seq, out, H, G, D, P, max_pages, chunk, page_stride, scale,
                      (const float*)slopes, (const float*)talk};
     switch (D / 32) {
-        case 1: return talk_launch<1>(a, S, run_decode, splits, K, (float*)ws_s, (float2*)ws_ml, run_prefill, max_q_len, out_heads, stream);
-        case 2: return talk_launch<2>(a, S, run_decode, splits, K, (float*)ws_s, (float2*)ws_ml, run_prefill, max_q_len, out_heads, stream);
-        case 3: return talk_launch<3>(a, S, run_decode, splits, K, (float*)ws_s, (float2*)ws_ml, run_prefill, max_q_len, out_heads, stream);
-        case 4: return talk_launch<4>(a, S, run_decode, splits, K, (float*)ws_s, (float2*)ws_ml, run_prefill, max_q_len, out_heads, stream);
+        case 1: return talk_launch<1>(a, S, run_decode, splits, K, (float*)ws_s, (float2*)ws_ml, run_prefill, max_q_len, out_heads, (float*)ws_sums, stream);
+        case 2: return talk_launch<2>(a, S, run_decode, splits, K, (float*)ws_s, (float2*)ws_ml, run_prefill, max_q_len, out_heads, (float*)ws_sums, stream);
+        case 3: return talk_launch<3>(a, S, run_decode, splits, K, (float*)ws_s, (float2*)ws_ml, run_prefill, max_q_len, out_heads, (float*)ws_sums, stream);
+        case 4: return talk_launch<4>(a, S, run_decode, splits, K, (float*)ws_s, (float2*)ws_ml, run_prefill, max_q_len, out_heads, (float*)ws_sums, stream);
     }
     return (int)hipErrorInvalidValue;
 }
