@@ -13,7 +13,8 @@
 //
 // The state is linear in what came before: S_out = diag(A) S_in + B, A the product of a stretch's decays.  A long
 // portion is therefore cut into pieces that are walked side by side:
-//   pass 1  every piece but a request's last, from a zero state: A and B                (no outputs)
+//   pass 1  every piece but a request's last, from a zero state: A, and B = sum_t (k_t times the decays behind t) v_t^T, a
+//           product on the 32-bit matrix instruction (products of decays never grow, so nothing is ever divided)
 //   carry   a short walk over the pieces leaves every piece's entry state
 //   pass 2  every piece again from its entry state, with outputs; the last writes the state back
 // A step of single tokens, or of short portions, is one launch from the state itself.
@@ -25,7 +26,12 @@ LLE_DEFINE_ERROR_STRING()
 // grid = (blocks of 256 channels, runs of GD_TOKENS tokens): a thread reads its column of a2 once for the run.
 #define GD_TOKENS 8
 __device__ __forceinline__ float gla_decay_of(float z, float inv_tau) {
-    return expf((fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau);  // log(sigmoid(z)), both ends without overflow
+    // log2(sigmoid(z)) = min(z, 0) log2 e - log2(1 + x), x = e^-|z|: no overflow at either end; a small x takes the
+    // first terms of the series (1 + x would round them away)
+    const float x = __builtin_amdgcn_exp2f(-fabsf(z) * 1.44269504088896340736f);
+    const float series = x * (1.f - x * (0.5f - x * 0.33333333333f)) * 1.44269504088896340736f;
+    const float log2_1px = x < 0.01f ? series : __builtin_amdgcn_logf(1.0f + x);
+    return __builtin_amdgcn_exp2f((fminf(z, 0.f) * 1.44269504088896340736f - log2_1px) * inv_tau);
 }
 
 __global__ __launch_bounds__(256) void gla_decay_kernel(const float* __restrict__ low, const float* __restrict__ a2,
@@ -37,6 +43,7 @@ __global__ __launch_bounds__(256) void gla_decay_kernel(const float* __restrict_
     float z[GD_TOKENS];
 #pragma unroll
     for (int t = 0; t < GD_TOKENS; ++t) z[t] = b[c];
+#pragma unroll 8
     for (int r = 0; r < R; ++r) {
         const float w = a2[(int64_t)r * C + c];
 #pragma unroll
@@ -71,14 +78,13 @@ struct GlaArgs {
     const int32_t* cu_tokens;
     void* out;  // [N, H vdim], activation type
     int H, dim, vdim;
-    int jt;  // threads of a group: 64, 128 or 256, at least vdim
+    int jt_log2;  // log2 of a group's threads: 64, 128 or 256, at least vdim
     int pieces, piece_len;
     float* part;  // [S, pieces, H, dim * vdim + dim]: B (then the entry state) and A of every piece
 };
 
 #define GLA_FROM_STATE 0  // one walk over a request's tokens
-#define GLA_SUMMARY 1     // pass 1
-#define GLA_FROM_ENTRY 2  // pass 2
+#define GLA_FROM_ENTRY 1  // pass 2
 #define GLA_TC 8          // tokens staged at a time
 #define GLA_IG 4          // groups of threads that share a value channel's key channels
 
@@ -88,21 +94,19 @@ struct GlaArgs {
 // MAXT: the most threads of a workgroup (wide heads take 512 where these are enough: twice the registers a thread).
 template <int KD, typename T, int MODE, int MAXT>
 __global__ __launch_bounds__(MAXT) void gla_scan_kernel(GlaArgs a) {
-    constexpr bool OUT = MODE != GLA_SUMMARY;
     constexpr int KI = KD / GLA_IG;
     static_assert(KD % GLA_IG == 0, "the key channels are dealt to the groups in equal shares");
     __shared__ float s_q[GLA_TC][KD], s_k[GLA_TC][KD], s_w[GLA_TC][KD];
     __shared__ float s_inv[GLA_TC];
     extern __shared__ float s_o[];
-    const int dim = a.dim, vdim = a.vdim, HK = a.H * dim, HV = a.H * vdim, jt = a.jt;
+    const int dim = a.dim, vdim = a.vdim, HK = a.H * dim, HV = a.H * vdim, jt = 1 << a.jt_log2;
     const int s = blockIdx.x / a.pieces, piece = blockIdx.x % a.pieces;
     const int h = blockIdx.y;
     const int tid = threadIdx.x;
-    const int j = tid & (jt - 1), ig = tid / jt, i0 = ig * KI;
+    const int j = tid & (jt - 1), ig = tid >> a.jt_log2, i0 = ig * KI;
     const int q0 = a.cu_tokens[s], q1 = a.cu_tokens[s + 1];
     const int live = (q1 - q0 + a.piece_len - 1) / a.piece_len;  // pieces of this request that hold tokens
     if (piece >= live) return;
-    if (MODE == GLA_SUMMARY && piece == live - 1) return;  // nobody comes after the last piece
     const int t0 = q0 + piece * a.piece_len, t1 = min(q1, t0 + a.piece_len);
     float* srow = a.state + (int64_t)a.seq_slots[s] * a.state_stride + (int64_t)h * dim * vdim;
     float* prow = a.part ? a.part + ((int64_t)(s * a.pieces + piece) * a.H + h) * (dim * vdim + dim) : nullptr;
@@ -117,8 +121,6 @@ __global__ __launch_bounds__(MAXT) void gla_scan_kernel(GlaArgs a) {
         if (MODE == GLA_FROM_ENTRY && i < dim && j < vdim) x = prow[i * vdim + j];
         S[ii] = x;
     }
-    float A = 1.0f;  // (threads tid < KD: the product of the piece's decays of key channel tid)
-
     for (int c0 = t0; c0 < t1; c0 += GLA_TC) {
         const int nt = min(GLA_TC, t1 - c0);
         __syncthreads();  // (the chunk before has been read)
@@ -128,11 +130,11 @@ __global__ __launch_bounds__(MAXT) void gla_scan_kernel(GlaArgs a) {
             float qq = 0.f, kk = 0.f, ww = 1.0f;
             if (t < nt && i < dim) {
                 const T* row = u + (int64_t)(c0 + t) * a.cols + h * dim + i;
-                if (OUT) qq = to_f32<T>(row[0]) * a.q_scale;
+                qq = to_f32<T>(row[0]) * a.q_scale;
                 kk = to_f32<T>(row[HK]);
                 ww = a.decay[(int64_t)(c0 + t) * HK + h * dim + i];
             }
-            if (OUT) s_q[t][i] = qq;
+            s_q[t][i] = qq;
             s_k[t][i] = kk;
             s_w[t][i] = ww;
         }
@@ -151,55 +153,107 @@ __global__ __launch_bounds__(MAXT) void gla_scan_kernel(GlaArgs a) {
                 for (int ii = 0; ii < KI; ++ii) {
                     const int i = i0 + ii;
                     S[ii] = fmaf(s_w[t][i], S[ii], s_k[t][i] * vv[t]);
-                    if (OUT) o = fmaf(s_q[t][i], S[ii], o);
+                    o = fmaf(s_q[t][i], S[ii], o);
                 }
-                if (OUT) s_o[(ig * GLA_TC + t) * jt + j] = o;
+                s_o[(ig * GLA_TC + t) * jt + j] = o;
             }
         }
-        if (!OUT && tid < KD) {
+        __syncthreads();
+        // the groups' shares are added up, and every token's head is divided by its own root mean square:
+        // a wavefront per token
+        const int wave = tid / LLE_WAVE, lane = tid % LLE_WAVE, waves = blockDim.x / LLE_WAVE;
+        for (int t = wave; t < nt; t += waves) {
+            float ss = 0.f;
+            for (int e = lane; e < vdim; e += LLE_WAVE) {
+                float o = s_o[t * jt + e];
 #pragma unroll
-            for (int t = 0; t < GLA_TC; ++t) A *= s_w[t][tid];
-        }
-        if (OUT) {
-            __syncthreads();
-            // the groups' shares are added up, and every token's head is divided by its own root mean square:
-            // a wavefront per token
-            const int wave = tid / LLE_WAVE, lane = tid % LLE_WAVE, waves = blockDim.x / LLE_WAVE;
-            for (int t = wave; t < nt; t += waves) {
-                float ss = 0.f;
-                for (int e = lane; e < vdim; e += LLE_WAVE) {
-                    float o = s_o[t * jt + e];
-#pragma unroll
-                    for (int g2 = 1; g2 < GLA_IG; ++g2) o += s_o[(g2 * GLA_TC + t) * jt + e];
-                    s_o[t * jt + e] = o;
-                    ss += o * o;
-                }
-                ss = wave_sum(ss);
-                if (lane == 0) s_inv[t] = 1.0f / sqrtf(ss / (float)vdim + a.eps);
+                for (int g2 = 1; g2 < GLA_IG; ++g2) o += s_o[(g2 * GLA_TC + t) * jt + e];
+                s_o[t * jt + e] = o;
+                ss += o * o;
             }
-            __syncthreads();
-            for (int idx = tid; idx < nt * vdim; idx += blockDim.x) {
-                const int t = idx / vdim, e = idx - t * vdim;
-                const float gate = to_f32<T>(u[(int64_t)(c0 + t) * a.cols + 2 * HK + HV + h * vdim + e]);
-                const float y = s_o[t * jt + e] * s_inv[t] * a.norm_w[e] * (gate / (1.0f + expf(-gate)));
-                ((T*)a.out)[(int64_t)(c0 + t) * HV + h * vdim + e] = from_f32<T>(y);
+            ss = wave_sum(ss);
+            if (lane == 0) s_inv[t] = 1.0f / sqrtf(ss / (float)vdim + a.eps);
+        }
+        __syncthreads();
+        for (int t = ig; t < nt; t += GLA_IG) {
+            if (j < vdim) {
+                const float gate = to_f32<T>(u[(int64_t)(c0 + t) * a.cols + 2 * HK + HV + h * vdim + j]);
+                const float y = s_o[t * jt + j] * s_inv[t] * a.norm_w[j] * (gate / (1.0f + expf(-gate)));
+                ((T*)a.out)[(int64_t)(c0 + t) * HV + h * vdim + j] = from_f32<T>(y);
             }
         }
-    }
-    if (MODE == GLA_SUMMARY) {
-        if (j < vdim) {
-#pragma unroll
-            for (int ii = 0; ii < KI; ++ii)
-                if (i0 + ii < dim) prow[(i0 + ii) * vdim + j] = S[ii];
-        }
-        if (tid < dim) prow[dim * vdim + tid] = A;
-        return;
     }
     if (piece != live - 1) return;
     if (j < vdim) {
 #pragma unroll
         for (int ii = 0; ii < KI; ++ii)
             if (i0 + ii < dim) srow[(i0 + ii) * vdim + j] = S[ii];
+    }
+}
+
+// Pass 1: grid = (requests x pieces, heads), 256 threads.  A piece has at most GLA_PIECE_MAX tokens.  The decays behind a
+// token are multiplied up in four groups of tokens side by side; k times them (float32) and v wait in LDS, and
+// B [dim, vdim] = sum over the tokens is taken in 16 x 16 tiles, four tokens an instruction.
+// LDS: k [tokens][KS], v [tokens][VS] (row strides of 16 modulo 64: the operands' rows lie in different banks), the
+// groups' products [4][dim].
+#define GLA_PIECE_MAX 64
+typedef float gla_f32x4 __attribute__((ext_vector_type(4)));
+template <typename T>
+__global__ __launch_bounds__(256) void gla_piece_kernel(GlaArgs a) {
+    extern __shared__ float lds[];
+    const int dim = a.dim, vdim = a.vdim, HK = a.H * dim;
+    const int KS = (dim + 63) / 64 * 64 + 16, VS = (vdim + 63) / 64 * 64 + 16;
+    const int s = blockIdx.x / a.pieces, piece = blockIdx.x % a.pieces, h = blockIdx.y;
+    const int q0 = a.cu_tokens[s], q1 = a.cu_tokens[s + 1];
+    const int live = (q1 - q0 + a.piece_len - 1) / a.piece_len;
+    if (piece >= live - 1) return;  // nobody comes after the last piece: the others are whole
+    const int t0 = q0 + piece * a.piece_len, L = a.piece_len, quarter = L / 4;
+    float* s_k = lds;
+    float* s_v = s_k + L * KS;
+    float* s_g = s_v + L * VS;
+    float* prow = a.part + ((int64_t)(s * a.pieces + piece) * a.H + h) * (dim * vdim + dim);
+    const T* u = (const T*)a.u;
+    for (int t = threadIdx.x / LLE_WAVE; t < L; t += 4)
+        for (int j = threadIdx.x % LLE_WAVE; j < VS - 16; j += LLE_WAVE)
+            s_v[t * VS + j] = j < vdim ? to_f32<T>(u[(int64_t)(t0 + t) * a.cols + 2 * HK + h * vdim + j]) : 0.f;
+    for (int idx = threadIdx.x; idx < 4 * dim; idx += 256) {
+        const int g = idx / dim, i = idx - g * dim;
+        const float* w = a.decay + (int64_t)(t0 + g * quarter) * HK + h * dim + i;
+        float p = 1.f;
+#pragma unroll 16
+        for (int t = 0; t < quarter; ++t) p *= w[(int64_t)t * HK];
+        s_g[idx] = p;
+    }
+    __syncthreads();
+    for (int idx = threadIdx.x; idx < 4 * (KS - 16); idx += 256) {
+        const int g = idx / (KS - 16), i = idx - g * (KS - 16);
+        if (i >= dim) {  // channels that fill the last tile of sixteen
+            for (int t = 0; t < quarter; ++t) s_k[(g * quarter + t) * KS + i] = 0.f;
+            continue;
+        }
+        float run = 1.f;
+        for (int later = g + 1; later < 4; ++later) run *= s_g[later * dim + i];
+        const float* w = a.decay + (int64_t)(t0 + g * quarter) * HK + h * dim + i;
+        const T* k = u + (int64_t)(t0 + g * quarter) * a.cols + HK + h * dim + i;
+#pragma unroll 16
+        for (int t = quarter - 1; t >= 0; --t) {
+            s_k[(g * quarter + t) * KS + i] = to_f32<T>(k[(int64_t)t * a.cols]) * run;
+            run *= w[(int64_t)t * HK];
+        }
+        if (g == 0) prow[dim * vdim + i] = run;
+    }
+    __syncthreads();
+    const int wave = threadIdx.x / LLE_WAVE, lane = threadIdx.x % LLE_WAVE, c = lane / 16, r = lane % 16;
+    const int row_tiles = (dim + 15) / 16, col_tiles = (vdim + 15) / 16;
+    for (int tile = wave; tile < row_tiles * col_tiles; tile += 4) {
+        const int i0 = tile / col_tiles * 16, j0 = (tile - tile / col_tiles * col_tiles) * 16;
+        gla_f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 8
+        for (int t = 0; t < L; t += 4)
+            acc = __builtin_amdgcn_mfma_f32_16x16x4f32(s_k[(t + c) * KS + i0 + r], s_v[(t + c) * VS + j0 + r], acc, 0, 0, 0);
+#pragma unroll
+        for (int n = 0; n < 4; ++n)
+            if (i0 + 4 * c + n < dim && j0 + r < vdim) prow[(i0 + 4 * c + n) * vdim + j0 + r] = acc[n];
     }
 }
 
@@ -237,15 +291,21 @@ __global__ __launch_bounds__(256) void gla_carry_kernel(GlaArgs a) {
 
 template <int KD, typename T, int MAXT>
 static int gla_launch_of(const GlaArgs& a, int S, hipStream_t stream) {
-    const int threads = a.jt * GLA_IG;
-    const size_t smem = (size_t)GLA_IG * GLA_TC * a.jt * sizeof(float);
+    const int threads = GLA_IG << a.jt_log2;
+    const size_t smem = (size_t)GLA_TC * threads * sizeof(float);
     const dim3 grid(S * a.pieces, a.H);
     if (a.pieces == 1) {
         gla_scan_kernel<KD, T, GLA_FROM_STATE, MAXT><<<grid, threads, smem, stream>>>(a);
         return (int)hipGetLastError();
     }
-    gla_scan_kernel<KD, T, GLA_SUMMARY, MAXT><<<grid, threads, 0, stream>>>(a);
-    hipError_t e = hipGetLastError();
+    const int KS = (a.dim + 63) / 64 * 64 + 16, VS = (a.vdim + 63) / 64 * 64 + 16;
+    const size_t piece_smem = ((size_t)a.piece_len * (KS + VS) + 4 * a.dim) * sizeof(float);
+    hipError_t e = hipSuccess;
+    if (piece_smem > 64 * 1024)
+        e = hipFuncSetAttribute((const void*)gla_piece_kernel<T>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)piece_smem);
+    if (e != hipSuccess) return (int)e;
+    gla_piece_kernel<T><<<grid, 256, piece_smem, stream>>>(a);
+    e = hipGetLastError();
     if (e != hipSuccess) return (int)e;
     gla_carry_kernel<<<dim3(S, a.H, (a.dim * a.vdim + 255) / 256), 256, 0, stream>>>(a);
     e = hipGetLastError();
@@ -257,7 +317,7 @@ static int gla_launch_of(const GlaArgs& a, int S, hipStream_t stream) {
 template <int KD, typename T>
 static int gla_launch(const GlaArgs& a, int S, hipStream_t stream) {
     if constexpr (KD >= 96) {
-        if (a.jt * GLA_IG <= 512) return gla_launch_of<KD, T, 512>(a, S, stream);
+        if (GLA_IG << a.jt_log2 <= 512) return gla_launch_of<KD, T, 512>(a, S, stream);
     }
     return gla_launch_of<KD, T, 1024>(a, S, stream);
 }
@@ -266,19 +326,19 @@ extern "C" int lle_gla_max_dim(void) { return 256; }
 
 // u [N, cols] in `dtype`: q, k, v, g in this order; decay float32 [N, H dim]; state float32 rows of `state_stride` floats
 // that begin with H dim vdim of the matrix state.  `pieces` > 1 needs `part`, float32 [S pieces H (dim vdim + dim)]; every
-// request has at most pieces * piece_len tokens.
+// request has at most pieces * piece_len tokens, and a piece a multiple of 4 and at most 64 of them.
 extern "C" int lle_gla_scan(const void* u, int cols, const void* decay, float q_scale, const void* norm_w, float eps, void* state,
                             int64_t state_stride, const void* seq_slots, const void* cu_tokens, void* out, int S, int H, int dim,
                             int vdim, int pieces, int piece_len, void* part, int dtype, hipStream_t stream) {
     if (S <= 0 || H <= 0) return 0;
-    if (dim <= 0 || dim > 256 || vdim <= 0 || vdim > 256 || pieces < 1 || piece_len < 1 || (pieces > 1 && part == nullptr) ||
+    if (dim <= 0 || dim > 256 || vdim <= 0 || vdim > 256 || pieces < 1 || piece_len < 1 ||
+        (pieces > 1 && (part == nullptr || piece_len > GLA_PIECE_MAX || piece_len % 4)) ||
         H > 65535 || (int64_t)S * pieces > 0x7fffffff || cols < 2 * H * (dim + vdim))
         return (int)hipErrorInvalidValue;
-    // a group has as many threads as there are value channels, and the groups together as many as key channels
-    // (so that pass 1 finds a thread for every channel's product of decays)
-    const int jt = vdim <= 64 ? 64 : vdim <= 128 ? 128 : 256;
+    // a group has as many threads as there are value channels
+    const int jt_log2 = vdim <= 64 ? 6 : vdim <= 128 ? 7 : 8;
     const GlaArgs a{u, cols, (const float*)decay, q_scale, (const float*)norm_w, eps, (float*)state, state_stride,
-                    (const int32_t*)seq_slots, (const int32_t*)cu_tokens, out, H, dim, vdim, jt, pieces, piece_len,
+                    (const int32_t*)seq_slots, (const int32_t*)cu_tokens, out, H, dim, vdim, jt_log2, pieces, piece_len,
                     (float*)part};
 #define GLA_CASE(KD)                                                                    \
     if (dim <= KD)                                                                      \

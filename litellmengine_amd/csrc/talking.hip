@@ -30,11 +30,21 @@ struct TalkArgs {
     const int32_t* token_seq;
     void* out;         // [N, H, D]
     int H, G, D, P, max_pages, chunk;
+    int P_log2;  // -1: the page size is no power of two
     int64_t page_stride;
     float scale;
     const float* slopes;  // [H] or null
     const float* talk;    // [H, H]
 };
+
+static int log2_or_minus_one(int n) {
+    for (int i = 0; i < 31; ++i)
+        if (n == 1 << i) return i;
+    return -1;
+}
+
+// the page that key j lies in (pages of a power of two, the usual case, cost a shift instead of a division)
+__device__ __forceinline__ int page_index(const TalkArgs& a, int j) { return a.P_log2 >= 0 ? j >> a.P_log2 : j / a.P; }
 
 #define TK_KEYS 64
 
@@ -147,7 +157,7 @@ extern "C" int lle_talking_generic(const void* q, const void* kv, const void* bl
     const int64_t smem = lle_talking_generic_lds(H, D);
     if (H <= 0 || G <= 0 || H % G != 0 || D <= 0 || P <= 0 || chunk < 0 || !talk || smem > 160 * 1024) return (int)hipErrorInvalidValue;
     const TalkArgs a{q, kv, (const int32_t*)block_tables, (const int32_t*)seq_slots, (const int32_t*)cu_tokens,
-                     (const int32_t*)kv_lens, (const int32_t*)token_seq, out, H, G, D, P, max_pages, chunk, page_stride, scale,
+                     (const int32_t*)kv_lens, (const int32_t*)token_seq, out, H, G, D, P, max_pages, chunk, log2_or_minus_one(P), page_stride, scale,
                      (const float*)slopes, (const float*)talk};
     const void* fn = dtype == LLE_F32 ? (const void*)talking_generic_kernel<float> : (const void*)talking_generic_kernel<bf16_t>;
     if (smem > 64 * 1024) {
@@ -164,7 +174,9 @@ extern "C" int lle_talking_generic(const void* q, const void* kv, const void* bl
 // ---------------------------------------------------------------------------------
 typedef bf16_t bf16x8 __attribute__((ext_vector_type(8)));
 typedef bf16_t bf16x4 __attribute__((ext_vector_type(4)));
-typedef bf16_t bf16x2 __attribute__((ext_vector_type(2)));
+typedef _Float16 f16x8 __attribute__((ext_vector_type(8)));
+typedef _Float16 f16x4 __attribute__((ext_vector_type(4)));
+typedef _Float16 f16x2 __attribute__((ext_vector_type(2)));
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 
 #define NEG_BIG (-1.0e30f)
@@ -198,7 +210,7 @@ __global__ __launch_bounds__(256) void talking_scores_kernel(TalkArgs a, float* 
         const float slope = a.slopes && exists ? a.slopes[h] * LOG2E : 0.f;
         for (int tile = blockIdx.z * 4 + wave; tile < tiles; tile += 4 * gridDim.z) {
             const int j0 = lo16 + 16 * tile;
-            const int lp = j0 / a.P, off = j0 - lp * a.P;
+            const int lp = page_index(a, j0), off = j0 - lp * a.P;
             const bf16_t* k = kv + (int64_t)table[__builtin_amdgcn_readfirstlane(lp)] * a.page_stride +
                               ((int64_t)kvh * a.P + off + r16) * D + 8 * c;
             f32x4 sc = {0.f, 0.f, 0.f, 0.f};
@@ -253,8 +265,18 @@ __global__ __launch_bounds__(1024) void talking_values_kernel(TalkArgs a, const 
     const bool has_values = e0 < a.D;  // (the same for the whole wavefront)
     const bf16_t* v_base = (const bf16_t*)a.kv + ((int64_t)a.G + kvh) * a.P * a.D + (int64_t)(has_values ? e0 + r16 : 0) * a.P;
     const float* s_row = ws_s + (int64_t)s * a.H * K;
+    bf16x8 vv[8];
+    auto load_v = [&](int b0) {
+#pragma unroll
+        for (int st = 0; st < 8; ++st) {  // keys past the last one read again: their weights are 0
+            const int j = min(lo16 + b0 + 256 * part + 32 * st + 16 * (c / 2), lo16 + 16 * (tiles - 1));
+            const int lp = page_index(a, j), off = j - lp * a.P;
+            vv[st] = *(const bf16x8*)(v_base + (int64_t)table[lp] * a.page_stride + off + 8 * (c % 2));
+        }
+    };
     for (int g0 = 0; g0 < group; g0 += CNT) {
         const int count = min(CNT, group - g0);
+        load_v(0);
         __syncthreads();
         for (int h = wave; h < a.H; h += 16) {
             const float2* ml = ws_ml + ((int64_t)s * a.H + h) * (K / 16);
@@ -270,19 +292,12 @@ __global__ __launch_bounds__(1024) void talking_values_kernel(TalkArgs a, const 
         __syncthreads();
         f32x4 acc = {0.f, 0.f, 0.f, 0.f};
         for (int b0 = 0; b0 < 16 * tiles; b0 += TV_KEYS) {
-            bf16x8 vv[8];
-#pragma unroll
-            for (int st = 0; st < 8; ++st) {  // keys past the last one read again: their weights are 0
-                const int j = min(lo16 + b0 + 256 * part + 32 * st + 16 * (c / 2), lo16 + 16 * (tiles - 1));
-                const int lp = j / a.P, off = j - lp * a.P;
-                vv[st] = *(const bf16x8*)(v_base + (int64_t)table[lp] * a.page_stride + off + 8 * (c % 2));
-            }
             const int key = b0 + threadIdx.x;
             float w[CNT];
 #pragma unroll
             for (int i = 0; i < CNT; ++i) w[i] = 0.f;
             if (key < 16 * tiles) {
-#pragma unroll 8
+#pragma unroll(CNT <= 4 ? 16 : 8)
                 for (int g = 0; g < a.H; ++g) {
                     const float p = __builtin_amdgcn_exp2f(s_row[(int64_t)g * K + key] - s_m[g]);
 #pragma unroll
@@ -298,6 +313,7 @@ __global__ __launch_bounds__(1024) void talking_values_kernel(TalkArgs a, const 
                 const bf16x8 p = *(const bf16x8*)(s_w + (r16 % CNT) * TV_ROW + 256 * part + 32 * st + 8 * c);
                 acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv[st], p, acc, 0, 0, 0);
             }
+            if (b0 + TV_KEYS < 16 * tiles) load_v(b0 + TV_KEYS);
         }
         __syncthreads();
         float* s_o = lds;  // [4][CNT][64]
@@ -315,19 +331,45 @@ __global__ __launch_bounds__(1024) void talking_values_kernel(TalkArgs a, const 
     }
 }
 
+// The tiles of 16 tokens in the order of their work, largest first: a tile's keys begin at its chunk's first, so the last
+// tiles of all chunks come first.  `count` indices, some of them past the last tile (tile_order_count).
+__host__ __device__ __forceinline__ int tile_order_count(int tiles, int chunk) {
+    const int per = chunk > 0 ? (chunk + 15) / 16 : tiles;
+    return per >= tiles ? tiles : (tiles + per - 1) / per * per;
+}
+__device__ __forceinline__ int tile_in_order(int k, int tiles, int chunk) {
+    const int per = chunk > 0 ? (chunk + 15) / 16 : tiles;
+    if (per >= tiles) return tiles - 1 - k;
+    const int chunks = (tiles + per - 1) / per;
+    return k % chunks * per + per - 1 - k / chunks;
+}
+
+// A barrier that waits for this wavefront's LDS traffic only: loads from memory stay on their way across it.
+__device__ __forceinline__ void lds_barrier() {
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
+    __builtin_amdgcn_s_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
+}
+
 // Portions, first launch: the base-2 log of every row's sum, ws [N][H].  grid = (blocks of 16 tokens, G, requests), four
 // wavefronts that take every fourth 32-key step; a wavefront makes the scores of four of the key/value head's query heads
 // with the keys in its registers (the other four and so on in further rounds).
 #define TS_HEADS 4
+#define TS_WAVES 4
 template <int DK>
-__global__ __launch_bounds__(256) void talking_sums_kernel(TalkArgs a, float* __restrict__ ws) {
+__global__ __launch_bounds__(TS_WAVES* LLE_WAVE) void talking_sums_kernel(TalkArgs a, float* __restrict__ ws) {
     constexpr int D = DK * 32;
-    __shared__ float s_m[4][TS_HEADS][16], s_l[4][TS_HEADS][16];
+    __shared__ float s_m[TS_WAVES][TS_HEADS][16], s_l[TS_WAVES][TS_HEADS][16];
     const int s = blockIdx.z, kvh = blockIdx.y;
     const int q_start = a.cu_tokens[s], q_len = a.cu_tokens[s + 1] - q_start;
-    const int blocks = (q_len + 15) / 16;
-    if (q_len <= 1 || (int)blockIdx.x >= blocks) return;
-    const int t0 = (blocks - 1 - (int)blockIdx.x) * 16;
+    if (q_len <= 1) return;
+    const int tiles = (q_len + 15) / 16, order = tile_order_count(tiles, a.chunk);
+    // (launches that are resident at once come two workgroups to a CU, halves of the launch side by side: the second half
+    // takes its tiles the other way round)
+    const int at = blockIdx.y < gridDim.y / 2 ? (int)blockIdx.x : order - 1 - (int)blockIdx.x;
+    if (at < 0 || at >= order) return;
+    const int t0 = tile_in_order(at, tiles, a.chunk) * 16;
+    if (t0 >= q_len) return;
     const int past = a.kv_lens[s] - q_len;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / LLE_WAVE), lane = threadIdx.x % LLE_WAVE;
     const int c = lane / 16, r16 = lane % 16;
@@ -346,11 +388,11 @@ __global__ __launch_bounds__(256) void talking_sums_kernel(TalkArgs a, float* __
     bf16x8 kreg[2][DK];
     auto page_of = [&](int step) {
         const int j = min(max(2 * step + r16 / 8, half_lo), half_hi) * 16;
-        return table[j / P];
+        return table[page_index(a, j)];
     };
     auto load_k = [&](int step, int page) {
         const int j = min(max(2 * step + r16 / 8, half_lo), half_hi) * 16;
-        const bf16_t* k = kv + (int64_t)page * a.page_stride + ((int64_t)kvh * P + (j - j / P * P)) * D + 8 * c;
+        const bf16_t* k = kv + (int64_t)page * a.page_stride + ((int64_t)kvh * P + (j - page_index(a, j) * P)) * D + 8 * c;
 #pragma unroll
         for (int x = 0; x < 2; ++x)
 #pragma unroll
@@ -372,8 +414,8 @@ __global__ __launch_bounds__(256) void talking_sums_kernel(TalkArgs a, float* __
         const int heads = min(TS_HEADS, group - g0);
         int page = page_of(first_step + wave);
         load_k(first_step + wave, page);
-        page = page_of(first_step + wave + 4);
-        for (int step = first_step + wave; step < end_step; step += 4) {
+        page = page_of(first_step + wave + TS_WAVES);
+        for (int step = first_step + wave; step < end_step; step += TS_WAVES) {
             f32x4 sc[TS_HEADS][2];
 #pragma unroll
             for (int i = 0; i < TS_HEADS; ++i) {
@@ -386,8 +428,8 @@ __global__ __launch_bounds__(256) void talking_sums_kernel(TalkArgs a, float* __
                             sc[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kreg[t][ks], qv[i][ks], sc[i][t], 0, 0, 0);
                 }
             }
-            load_k(step + 4, page);  // (past the last step: keys that are there)
-            page = page_of(step + 8);
+            load_k(step + TS_WAVES, page);  // (past the last step: keys that are there)
+            page = page_of(step + 2 * TS_WAVES);
             const bool open = 32 * step >= open_lo && 32 * step + 31 <= open_hi;  // (the same for all lanes)
             const float d0 = (float)(32 * step + 8 * c - pos);
 #pragma unroll
@@ -434,10 +476,10 @@ __global__ __launch_bounds__(256) void talking_sums_kernel(TalkArgs a, float* __
             if (i < heads && t0 + r <= last) {
                 float top = s_m[0][i][r];
 #pragma unroll
-                for (int w = 1; w < 4; ++w) top = fmaxf(top, s_m[w][i][r]);
+                for (int w = 1; w < TS_WAVES; ++w) top = fmaxf(top, s_m[w][i][r]);
                 float sum = 0.f;  // (a row sees a key: itself)
 #pragma unroll
-                for (int w = 0; w < 4; ++w) sum += s_l[w][i][r] * __builtin_amdgcn_exp2f(s_m[w][i][r] - top);
+                for (int w = 0; w < TS_WAVES; ++w) sum += s_l[w][i][r] * __builtin_amdgcn_exp2f(s_m[w][i][r] - top);
                 ws[(int64_t)(q_start + t0 + r) * a.H + kvh * group + g0 + i] = top + log2f(sum);
             }
         }
@@ -447,19 +489,17 @@ __global__ __launch_bounds__(256) void talking_sums_kernel(TalkArgs a, float* __
 // Portions, second launch.  grid = (output splits, blocks of 16 tokens, requests), eight wavefronts.  A wavefront makes the
 // scores of HW heads (all of the model's heads over the eight), one query token a lane column.  Three things happen in
 // step i, each to another 32 keys, with one barrier a step between them:
-//   keys i      scores, weights (divided by their sum already) into LDS as bfloat16 pairs (high and low part: 16 bits of
-//               mantissa), [key][token][head];
+//   keys i      scores, weights (divided by their sum already, so between 0 and 1) into LDS in half precision (11 bits of
+//               mantissa, three more than the mixed weights keep), [key][token][head];
 //   keys i - 1  mixed on the matrix cores ([4 tokens x 4 keys] x heads times heads x 16 heads of this workgroup's
-//               split), [token][head][key] into LDS as bfloat16;
+//               split; talk in half precision holds a bfloat16 number as it is), summed in 32-bit, [token][head][key] into
+//               LDS as bfloat16;
 //   keys i - 2  O^T += V^T W^T for the OW heads of the wavefront.
 // Both LDS buffers are there twice.  A split computes all scores and the sums of 8 OW output heads: OW bounds the
 // accumulators.  LDS rows of 64 bytes are cut into four 16-byte pieces whose order is swizzled so that neither the writes nor
 // the reads of the two exchanges meet in a bank.
-template <int HW>
-struct TalkTile {
-    static constexpr int KT = HW == 4 ? 2 : 1;  // up to 16 heads: high and low parts share a row; up to 32: a row each
-    static constexpr int P_BYTES = KT * 512 * 64, W_BYTES = 16 * 16 * 64;
-};
+#define TALK_P_BYTES (512 * 64)      // 32 keys x 16 tokens, rows of 32 heads
+#define TALK_W_BYTES (16 * 16 * 64)  // 16 tokens x 16 heads, rows of 32 keys
 __device__ __forceinline__ int talk_p_at(int key, int q, int piece) {  // byte offset of a 16-byte piece of a weight row
     return (key * 16 + q) * 64 + ((piece ^ (q >> 2) ^ key) & 3) * 16;
 }
@@ -468,18 +508,23 @@ __device__ __forceinline__ int talk_w_at(int q, int h, int piece) {  // of a mix
     return (q * 16 + row) * 64 + ((piece ^ (row >> 2)) & 3) * 16;
 }
 
-template <int DK, int HW, int OW>
+// ONE: the HW heads of a wavefront, and the OW, share a key/value head (a load under a condition makes the compiler wait for
+// every load on its way where the paths meet again, so the usual case has none; loads past the last step ask for keys that
+// are there).
+template <int DK, int HW, int OW, bool ONE>
 __global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a, const float* __restrict__ sums) {
     constexpr int D = DK * 32;
-    constexpr int KT = TalkTile<HW>::KT, P_BYTES = TalkTile<HW>::P_BYTES, W_BYTES = TalkTile<HW>::W_BYTES;
+    constexpr int P_BYTES = TALK_P_BYTES, W_BYTES = TALK_W_BYTES;
     extern __shared__ __attribute__((aligned(16))) char smem[];
     char* s_p = smem;
     char* s_w = smem + 2 * P_BYTES;
     const int s = blockIdx.z, out0 = blockIdx.x * 8 * OW;
     const int q_start = a.cu_tokens[s], q_len = a.cu_tokens[s + 1] - q_start;
-    const int blocks = (q_len + 15) / 16;
-    if (q_len <= 1 || (int)blockIdx.y >= blocks) return;
-    const int t0 = (blocks - 1 - (int)blockIdx.y) * 16;
+    if (q_len <= 1) return;
+    const int tiles = (q_len + 15) / 16;
+    if ((int)blockIdx.y >= tile_order_count(tiles, a.chunk)) return;
+    const int t0 = tile_in_order(blockIdx.y, tiles, a.chunk) * 16;
+    if (t0 >= q_len) return;
     const int past = a.kv_lens[s] - q_len;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / LLE_WAVE), lane = threadIdx.x % LLE_WAVE;
     const int c = lane / 16, r16 = lane % 16;
@@ -518,11 +563,11 @@ __global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a, const 
     // a step's two 16-key halves lie in one page each; a lane's keys lie in half r16 / 8, its values' keys in half c / 2
     const int k_half = r16 / 8, v_half = c / 2;
     auto key_of = [&](int i, int half) { return min(max(2 * (first_step + i) + half, half_lo), half_hi) * 16; };
-    auto page_of = [&](int i, int half) { return table[key_of(i, half) / P]; };
+    auto page_of = [&](int i, int half) { return table[page_index(a, key_of(i, half))]; };
     bf16x8 kreg[2][DK], vreg[2 * DK];
     auto load_k = [&](int i, int page, int kvh) {
         const int j = key_of(i, k_half);
-        const bf16_t* k = kv + (int64_t)page * a.page_stride + ((int64_t)kvh * P + (j - j / P * P)) * D + 8 * c;
+        const bf16_t* k = kv + (int64_t)page * a.page_stride + ((int64_t)kvh * P + (j - page_index(a, j) * P)) * D + 8 * c;
 #pragma unroll
         for (int x = 0; x < 2; ++x)
 #pragma unroll
@@ -530,18 +575,17 @@ __global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a, const 
     };
     auto load_v = [&](int i, int page, int kvh) {
         const int j = key_of(i, v_half);
-        const bf16_t* v = kv + (int64_t)page * a.page_stride + ((int64_t)a.G + kvh) * P * D + (int64_t)r16 * P + (j - j / P * P) + 8 * (c % 2);
+        const bf16_t* v = kv + (int64_t)page * a.page_stride + ((int64_t)a.G + kvh) * P * D + (int64_t)r16 * P + (j - page_index(a, j) * P) + 8 * (c % 2);
 #pragma unroll
         for (int n = 0; n < 2 * DK; ++n) vreg[n] = *(const bf16x8*)(v + (int64_t)16 * n * P);
     };
 
-    // talk's rows of this split's heads: element e of lane (c, r16) is talk[out0 + r16][8 c + e] (KT = 1: both halves of
-    // the contraction are the heads 0 .. 15)
-    bf16x8 talk;
+    // talk's rows of this split's heads: element e of lane (c, r16) is talk[out0 + r16][8 c + e]
+    f16x8 talk;
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
-        const int g = KT == 1 ? (8 * c + e) % 16 : 8 * c + e, h = out0 + r16;
-        talk[e] = (bf16_t)(r16 < 8 * OW && h < a.H && g < a.H ? a.talk[h * a.H + g] : 0.f);
+        const int g = 8 * c + e, h = out0 + r16;
+        talk[e] = (_Float16)(r16 < 8 * OW && h < a.H && g < a.H ? a.talk[h * a.H + g] : 0.f);
     }
     const int oh0 = out0 + wave * OW;
     const int outs_here = max(0, min(OW, a.H - oh0));
@@ -560,15 +604,17 @@ __global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a, const 
     for (int i = 0; i < steps + 2; ++i) {
         if (i < steps && heads_here > 0) {
             const int step = first_step + i;
-            bf16_t hi[8][HW], low[8][HW];
-            int kvh = first_kvh;
+            _Float16 p[8][HW];
+            [[maybe_unused]] int kvh = first_kvh;
             const bool open = all_rows && 32 * step >= open_lo && 32 * step + 31 <= past + t0;  // (the same for all lanes)
             const float d0 = (float)(32 * step + 8 * c - pos);
 #pragma unroll
             for (int n = 0; n < HW; ++n) {
                 if (n < heads_here) {
-                    const int own = (h0 + n) / group;
-                    if (own != kvh) load_k(i, k_page_now, kvh = own);
+                    if constexpr (!ONE) {
+                        const int own = (h0 + n) / group;
+                        if (own != kvh) load_k(i, k_page_now, kvh = own);
+                    }
                     f32x4 sc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
                     for (int t = 0; t < 2; ++t)
@@ -585,37 +631,24 @@ __global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a, const 
                         }
                     }
 #pragma unroll
-                    for (int e = 0; e < 8; ++e) {
-                        const float p = __builtin_amdgcn_exp2f(x[e]);
-                        hi[e][n] = (bf16_t)p;
-                        low[e][n] = (bf16_t)(p - (float)hi[e][n]);
-                    }
+                    for (int e = 0; e < 8; ++e) p[e][n] = (_Float16)__builtin_amdgcn_exp2f(x[e]);
                 } else {
 #pragma unroll
-                    for (int e = 0; e < 8; ++e) hi[e][n] = low[e][n] = (bf16_t)0.f;
+                    for (int e = 0; e < 8; ++e) p[e][n] = (_Float16)0.f;
                 }
             }
-            load_k(i + 1, k_page, first_kvh);
-            k_page_now = k_page;
-            k_page = page_of(i + 2, k_half);
             char* buf = s_p + (i & 1) * P_BYTES;
 #pragma unroll
             for (int e = 0; e < 8; ++e) {
-                const int key = 8 * c + e;
-                char* at_hi = buf + talk_p_at(key, r16, h0 / 8) + (h0 % 8) * 2;
-                char* at_lo = KT == 1 ? buf + talk_p_at(key, r16, 2 + h0 / 8) + (h0 % 8) * 2 : at_hi + 512 * 64;
-                if constexpr (HW == 1) {
-                    *(bf16_t*)at_hi = hi[e][0];
-                    *(bf16_t*)at_lo = low[e][0];
-                } else if constexpr (HW == 2) {
-                    *(bf16x2*)at_hi = bf16x2{hi[e][0], hi[e][1]};
-                    *(bf16x2*)at_lo = bf16x2{low[e][0], low[e][1]};
-                } else {
-                    *(bf16x4*)at_hi = bf16x4{hi[e][0], hi[e][1], hi[e][2], hi[e][3]};
-                    *(bf16x4*)at_lo = bf16x4{low[e][0], low[e][1], low[e][2], low[e][3]};
-                }
+                char* at = buf + talk_p_at(8 * c + e, r16, h0 / 8) + (h0 % 8) * 2;
+                if constexpr (HW == 1) *(_Float16*)at = p[e][0];
+                else if constexpr (HW == 2) *(f16x2*)at = f16x2{p[e][0], p[e][1]};
+                else *(f16x4*)at = f16x4{p[e][0], p[e][1], p[e][2], p[e][3]};
             }
         }
+        load_k(i + 1, k_page, first_kvh);
+        k_page_now = k_page;
+        k_page = page_of(i + 2, k_half);
         if (i >= 1 && i - 1 < steps) {
             // 32 tiles of (4 tokens x 4 keys), four a wavefront: row r of a tile is token 4 qa + r / 4, key 4 kq + r % 4
             const char* from = s_p + ((i - 1) & 1) * P_BYTES;
@@ -623,38 +656,32 @@ __global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a, const 
 #pragma unroll
             for (int t = 0; t < 4; ++t) {
                 const int tile = wave * 4 + t, qa = tile % 4, kq = tile / 4;
-                f32x4 w = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-                for (int kt = 0; kt < KT; ++kt) {
-                    const bf16x8 p = *(const bf16x8*)(from + kt * 512 * 64 + talk_p_at(4 * kq + r16 % 4, 4 * qa + r16 / 4, c));
-                    w = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p, talk, w, 0, 0, 0);
-                }
+                const f16x8 p = *(const f16x8*)(from + talk_p_at(4 * kq + r16 % 4, 4 * qa + r16 / 4, c));
+                const f32x4 w = __builtin_amdgcn_mfma_f32_16x16x32_f16(p, talk, f32x4{0.f, 0.f, 0.f, 0.f}, 0, 0, 0);
                 // lane (c, r16): head r16 of the split, token 4 qa + c, keys 4 kq .. + 3
                 *(bf16x4*)(to + talk_w_at(4 * qa + c, r16, kq / 2) + (kq % 2) * 8) = bf16x4{(bf16_t)w[0], (bf16_t)w[1], (bf16_t)w[2], (bf16_t)w[3]};
             }
         }
-        if (outs_here > 0) {
-            if (i >= 2) {
-                const char* from = s_w + (i & 1) * W_BYTES;
-                int vkv = first_vkv;
+        if (i >= 2 && outs_here > 0) {
+            const char* from = s_w + (i & 1) * W_BYTES;
+            [[maybe_unused]] int vkv = first_vkv;
 #pragma unroll
-                for (int n = 0; n < OW; ++n) {
-                    if (n < outs_here) {
+            for (int n = 0; n < OW; ++n) {
+                if (n < outs_here) {
+                    if constexpr (!ONE) {
                         const int own = (oh0 + n) / group;
                         if (own != vkv) load_v(i - 2, v_page_now, vkv = own);
-                        const bf16x8 w = *(const bf16x8*)(from + talk_w_at(r16, wave * OW + n, c));
-#pragma unroll
-                        for (int m = 0; m < 2 * DK; ++m) o[n][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vreg[m], w, o[n][m], 0, 0, 0);
                     }
+                    const bf16x8 w = *(const bf16x8*)(from + talk_w_at(r16, wave * OW + n, c));
+#pragma unroll
+                    for (int m = 0; m < 2 * DK; ++m) o[n][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vreg[m], w, o[n][m], 0, 0, 0);
                 }
             }
-            if (i >= 1) {
-                load_v(i - 1, v_page, first_vkv);  // used in the next step
-                v_page_now = v_page;
-                v_page = page_of(i, v_half);
-            }
         }
-        __syncthreads();
+        load_v(i - 1, v_page, first_vkv);  // used in the next step
+        v_page_now = v_page;
+        v_page = page_of(i, v_half);
+        lds_barrier();
     }
     if (!exists) return;
 #pragma unroll
@@ -668,17 +695,24 @@ __global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a, const 
     }
 }
 
-template <int DK, int HW, int OW>
-static int talk_prefill_launch(const TalkArgs& a, int S, int max_q_len, const float* sums, hipStream_t stream) {
-    const size_t smem = 2 * (TalkTile<HW>::P_BYTES + TalkTile<HW>::W_BYTES);
+template <int DK, int HW, int OW, bool ONE>
+static int talk_prefill_launch_of(const TalkArgs& a, int S, int max_q_len, const float* sums, hipStream_t stream) {
+    const size_t smem = 2 * (TALK_P_BYTES + TALK_W_BYTES);
     if (smem > 64 * 1024) {
-        hipError_t e = hipFuncSetAttribute((const void*)talking_prefill_kernel<DK, HW, OW>,
+        hipError_t e = hipFuncSetAttribute((const void*)talking_prefill_kernel<DK, HW, OW, ONE>,
                                            hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
         if (e != hipSuccess) return (int)e;
     }
     const int splits = (a.H + 8 * OW - 1) / (8 * OW);
-    talking_prefill_kernel<DK, HW, OW><<<dim3(splits, (max_q_len + 15) / 16, S), 512, smem, stream>>>(a, sums);
+    talking_prefill_kernel<DK, HW, OW, ONE><<<dim3(splits, tile_order_count((max_q_len + 15) / 16, a.chunk), S), 512, smem, stream>>>(a, sums);
     return (int)hipGetLastError();
+}
+
+template <int DK, int HW, int OW>
+static int talk_prefill_launch(const TalkArgs& a, int S, int max_q_len, const float* sums, hipStream_t stream) {
+    const int group = a.H / a.G;
+    if (group % HW == 0 && group % OW == 0) return talk_prefill_launch_of<DK, HW, OW, true>(a, S, max_q_len, sums, stream);
+    return talk_prefill_launch_of<DK, HW, OW, false>(a, S, max_q_len, sums, stream);
 }
 
 template <int DK>
@@ -704,7 +738,7 @@ static int talk_launch(const TalkArgs& a, int S, int run_decode, int splits, int
         if (e != hipSuccess) return (int)e;
     }
     if (run_prefill) {
-        talking_sums_kernel<DK><<<dim3((max_q_len + 15) / 16, a.G, S), 256, 0, stream>>>(a, ws_sums);
+        talking_sums_kernel<DK><<<dim3(tile_order_count((max_q_len + 15) / 16, a.chunk), a.G, S), TS_WAVES * LLE_WAVE, 0, stream>>>(a, ws_sums);
         const hipError_t e = hipGetLastError();
         if (e != hipSuccess) return (int)e;
         if (a.H <= 8) return talk_prefill_launch<DK, 1, 1>(a, S, max_q_len, ws_sums, stream);
@@ -731,9 +765,9 @@ extern "C" int lle_talking_mfma(const void* q, const void* kv, const void* block
         S > 65535 || G > 65535)
         return (int)hipErrorInvalidValue;
     if (run_decode && (!ws_s || !ws_ml || K % 16 != 0 || K < 16 || splits < 1 || splits > 65535)) return (int)hipErrorInvalidValue;
-    if (run_prefill && (H > 32 || max_q_len < 2 || !ws_sums || (max_q_len + 15) / 16 > 65535)) return (int)hipErrorInvalidValue;
+    if (run_prefill && (H > 32 || max_q_len < 2 || !ws_sums || tile_order_count((max_q_len + 15) / 16, chunk) > 65535)) return (int)hipErrorInvalidValue;
     const TalkArgs a{q, kv, (const int32_t*)block_tables, (const int32_t*)seq_slots, (const int32_t*)cu_tokens,
-                     (const int32_t*)kv_lens, (const int32_t*)token_seq, out, H, G, D, P, max_pages, chunk, page_stride, scale,
+                     (const int32_t*)kv_lens, (const int32_t*)token_seq, out, H, G, D, P, max_pages, chunk, log2_or_minus_one(P), page_stride, scale,
                      (const float*)slopes, (const float*)talk};
     switch (D / 32) {
         case 1: return talk_launch<1>(a, S, run_decode, splits, K, (float*)ws_s, (float2*)ws_ml, run_prefill, max_q_len, out_heads, (float*)ws_sums, stream);
