@@ -126,7 +126,7 @@ def talking_attention(h, w, p: str, m: dict) -> torch.Tensor:
     k = (h @ w[p + "k"].T).view(T, G, d)
     v = (h @ w[p + "v"].T).view(T, G, vd)
     s = head_scores(q, k, m["scale"]) - distance_bias(T, H, h.dtype)
-    a = softmax_weights(s, chunk_mask(T, m["mask"]["size"]))
+    a = softmax_weights(s, chunk_mask(T, (m.get("mask") or {"size": T})["size"]))  # (no mask: one chunk)
     o = heads_values(mixed_over_heads(a, w[p + "talk"]), v).reshape(T, H * vd)
     return (o * sigmoid(h @ w[p + "g"].T)) @ w[p + "o"].T
 
@@ -171,8 +171,8 @@ def window_attention(h, w, p: str, m: dict, eps: float = 0.0) -> torch.Tensor:
     q = turn_pairs((h @ w[p + "q"].T + w[p + "q.b"]).view(T, H, d), pos, dims, base)
     k = turn_pairs((h @ w[p + "k"].T + w[p + "k.b"]).view(T, G, d), pos, dims, base)
     v = turn_pairs((h @ w[p + "v"].T + w[p + "v.b"]).view(T, G, vd), pos, vd, base)
-    a = softmax_weights(head_scores(q, k, m["scale"]),
-                        kept_window_mask(T, m["mask"]["size"], m["mask"].get("keep_first", 0)), w[p + "sink"])
+    mask = m.get("mask") or {"size": T}  # (no mask: every earlier token)
+    a = softmax_weights(head_scores(q, k, m["scale"]), kept_window_mask(T, mask["size"], mask.get("keep_first", 0)), w[p + "sink"])
     o = turn_pairs(heads_values(a, v), pos, vd, base, sign=-1.0).reshape(T, H * vd)
     return (o * sigmoid(h @ w[p + "g"].T)) @ w[p + "o"].T
 
