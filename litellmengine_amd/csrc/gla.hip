@@ -191,65 +191,80 @@ __global__ __launch_bounds__(MAXT) void gla_scan_kernel(GlaArgs a) {
     }
 }
 
-// Pass 1: grid = (requests x pieces, heads), 256 threads.  A piece has at most GLA_PIECE_MAX tokens.  The decays behind a
-// token are multiplied up in four groups of tokens side by side; k times them (float32) and v wait in LDS, and
-// B [dim, vdim] = sum over the tokens is taken in 16 x 16 tiles, four tokens an instruction.
+// Pass 1: grid = (requests x pieces, heads), 256 threads; every piece but a request's last is whole.  The decays behind a
+// token are multiplied up in four groups of tokens side by side (a thread has sixteen tokens of a channel, NI channels one
+// after the other, everything asked for at once); k times them (float32) and v wait in LDS, and B [dim, vdim] = sum over the
+// tokens is taken in 16 x 16 tiles, four tokens an instruction.
 // LDS: k [tokens][KS], v [tokens][VS] (row strides of 16 modulo 64: the operands' rows lie in different banks), the
 // groups' products [4][dim].
-#define GLA_PIECE_MAX 64
+#define GLA_PIECE 64
+#define GLA_QUARTER (GLA_PIECE / 4)
 typedef float gla_f32x4 __attribute__((ext_vector_type(4)));
-template <typename T>
+template <typename T, int NI>
 __global__ __launch_bounds__(256) void gla_piece_kernel(GlaArgs a) {
     extern __shared__ float lds[];
     const int dim = a.dim, vdim = a.vdim, HK = a.H * dim;
     const int KS = (dim + 63) / 64 * 64 + 16, VS = (vdim + 63) / 64 * 64 + 16;
     const int s = blockIdx.x / a.pieces, piece = blockIdx.x % a.pieces, h = blockIdx.y;
     const int q0 = a.cu_tokens[s], q1 = a.cu_tokens[s + 1];
-    const int live = (q1 - q0 + a.piece_len - 1) / a.piece_len;
-    if (piece >= live - 1) return;  // nobody comes after the last piece: the others are whole
-    const int t0 = q0 + piece * a.piece_len, L = a.piece_len, quarter = L / 4;
+    const int live = (q1 - q0 + GLA_PIECE - 1) / GLA_PIECE;
+    if (piece >= live - 1) return;  // nobody comes after the last piece
+    const int t0 = q0 + piece * GLA_PIECE;
     float* s_k = lds;
-    float* s_v = s_k + L * KS;
-    float* s_g = s_v + L * VS;
+    float* s_v = s_k + GLA_PIECE * KS;
+    float* s_g = s_v + GLA_PIECE * VS;
     float* prow = a.part + ((int64_t)(s * a.pieces + piece) * a.H + h) * (dim * vdim + dim);
     const T* u = (const T*)a.u;
-    for (int t = threadIdx.x / LLE_WAVE; t < L; t += 4)
-        for (int j = threadIdx.x % LLE_WAVE; j < VS - 16; j += LLE_WAVE)
-            s_v[t * VS + j] = j < vdim ? to_f32<T>(u[(int64_t)(t0 + t) * a.cols + 2 * HK + h * vdim + j]) : 0.f;
-    for (int idx = threadIdx.x; idx < 4 * dim; idx += 256) {
-        const int g = idx / dim, i = idx - g * dim;
-        const float* w = a.decay + (int64_t)(t0 + g * quarter) * HK + h * dim + i;
-        float p = 1.f;
-#pragma unroll 16
-        for (int t = 0; t < quarter; ++t) p *= w[(int64_t)t * HK];
-        s_g[idx] = p;
-    }
-    __syncthreads();
-    for (int idx = threadIdx.x; idx < 4 * (KS - 16); idx += 256) {
-        const int g = idx / (KS - 16), i = idx - g * (KS - 16);
-        if (i >= dim) {  // channels that fill the last tile of sixteen
-            for (int t = 0; t < quarter; ++t) s_k[(g * quarter + t) * KS + i] = 0.f;
-            continue;
-        }
-        float run = 1.f;
-        for (int later = g + 1; later < 4; ++later) run *= s_g[later * dim + i];
-        const float* w = a.decay + (int64_t)(t0 + g * quarter) * HK + h * dim + i;
-        const T* k = u + (int64_t)(t0 + g * quarter) * a.cols + HK + h * dim + i;
-#pragma unroll 16
-        for (int t = quarter - 1; t >= 0; --t) {
-            s_k[(g * quarter + t) * KS + i] = to_f32<T>(k[(int64_t)t * a.cols]) * run;
-            run *= w[(int64_t)t * HK];
-        }
-        if (g == 0) prow[dim * vdim + i] = run;
-    }
-    __syncthreads();
     const int wave = threadIdx.x / LLE_WAVE, lane = threadIdx.x % LLE_WAVE, c = lane / 16, r = lane % 16;
+    // wavefront g has the tokens g 16 .. g 16 + 15; lane + 64 n is its channel
+    const int g = wave, first = t0 + g * GLA_QUARTER;
+    float w[NI][GLA_QUARTER], k[NI][GLA_QUARTER];
+#pragma unroll
+    for (int n = 0; n < NI; ++n) {
+        const int i = min(lane + LLE_WAVE * n, dim - 1);
+#pragma unroll
+        for (int t = 0; t < GLA_QUARTER; ++t) {
+            w[n][t] = a.decay[(int64_t)(first + t) * HK + h * dim + i];
+            k[n][t] = to_f32<T>(u[(int64_t)(first + t) * a.cols + HK + h * dim + i]);
+        }
+    }
+    for (int j = lane; j < VS - 16; j += LLE_WAVE) {
+        float v[GLA_QUARTER];
+#pragma unroll
+        for (int t = 0; t < GLA_QUARTER; ++t) v[t] = to_f32<T>(u[(int64_t)(first + t) * a.cols + 2 * HK + h * vdim + min(j, vdim - 1)]);
+#pragma unroll
+        for (int t = 0; t < GLA_QUARTER; ++t) s_v[(g * GLA_QUARTER + t) * VS + j] = j < vdim ? v[t] : 0.f;
+    }
+#pragma unroll
+    for (int n = 0; n < NI; ++n) {
+        const int i = lane + LLE_WAVE * n;
+        float p = 1.f;
+#pragma unroll
+        for (int t = 0; t < GLA_QUARTER; ++t) p *= w[n][t];
+        if (i < dim) s_g[g * dim + i] = p;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int n = 0; n < NI; ++n) {
+        const int i = lane + LLE_WAVE * n;
+        float run = 1.f;
+        if (i < dim)
+            for (int later = g + 1; later < 4; ++later) run *= s_g[later * dim + i];
+#pragma unroll
+        for (int t = GLA_QUARTER - 1; t >= 0; --t) {
+            // (channels past the last one fill the last tile of sixteen with zeros)
+            if (i < KS - 16) s_k[(g * GLA_QUARTER + t) * KS + i] = i < dim ? k[n][t] * run : 0.f;
+            run *= w[n][t];
+        }
+        if (g == 0 && i < dim) prow[dim * vdim + i] = run;
+    }
+    __syncthreads();
     const int row_tiles = (dim + 15) / 16, col_tiles = (vdim + 15) / 16;
     for (int tile = wave; tile < row_tiles * col_tiles; tile += 4) {
         const int i0 = tile / col_tiles * 16, j0 = (tile - tile / col_tiles * col_tiles) * 16;
         gla_f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 8
-        for (int t = 0; t < L; t += 4)
+#pragma unroll
+        for (int t = 0; t < GLA_PIECE; t += 4)
             acc = __builtin_amdgcn_mfma_f32_16x16x4f32(s_k[(t + c) * KS + i0 + r], s_v[(t + c) * VS + j0 + r], acc, 0, 0, 0);
 #pragma unroll
         for (int n = 0; n < 4; ++n)
@@ -299,13 +314,16 @@ static int gla_launch_of(const GlaArgs& a, int S, hipStream_t stream) {
         return (int)hipGetLastError();
     }
     const int KS = (a.dim + 63) / 64 * 64 + 16, VS = (a.vdim + 63) / 64 * 64 + 16;
-    const size_t piece_smem = ((size_t)a.piece_len * (KS + VS) + 4 * a.dim) * sizeof(float);
-    hipError_t e = hipSuccess;
-    if (piece_smem > 64 * 1024)
-        e = hipFuncSetAttribute((const void*)gla_piece_kernel<T>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)piece_smem);
-    if (e != hipSuccess) return (int)e;
-    gla_piece_kernel<T><<<grid, 256, piece_smem, stream>>>(a);
-    e = hipGetLastError();
+    const size_t piece_smem = ((size_t)GLA_PIECE * (KS + VS) + 4 * a.dim) * sizeof(float);
+    auto piece = [&](auto kernel) {
+        if (piece_smem > 64 * 1024) {
+            const hipError_t e = hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)piece_smem);
+            if (e != hipSuccess) return e;
+        }
+        kernel<<<grid, 256, piece_smem, stream>>>(a);
+        return hipGetLastError();
+    };
+    hipError_t e = a.dim <= 64 ? piece(gla_piece_kernel<T, 1>) : a.dim <= 128 ? piece(gla_piece_kernel<T, 2>) : piece(gla_piece_kernel<T, 4>);
     if (e != hipSuccess) return (int)e;
     gla_carry_kernel<<<dim3(S, a.H, (a.dim * a.vdim + 255) / 256), 256, 0, stream>>>(a);
     e = hipGetLastError();
@@ -323,16 +341,17 @@ static int gla_launch(const GlaArgs& a, int S, hipStream_t stream) {
 }
 
 extern "C" int lle_gla_max_dim(void) { return 256; }
+extern "C" int lle_gla_piece(void) { return GLA_PIECE; }
 
 // u [N, cols] in `dtype`: q, k, v, g in this order; decay float32 [N, H dim]; state float32 rows of `state_stride` floats
 // that begin with H dim vdim of the matrix state.  `pieces` > 1 needs `part`, float32 [S pieces H (dim vdim + dim)]; every
-// request has at most pieces * piece_len tokens, and a piece a multiple of 4 and at most 64 of them.
+// request has at most pieces * piece_len tokens: 64 of them in a piece, where there are several.
 extern "C" int lle_gla_scan(const void* u, int cols, const void* decay, float q_scale, const void* norm_w, float eps, void* state,
                             int64_t state_stride, const void* seq_slots, const void* cu_tokens, void* out, int S, int H, int dim,
                             int vdim, int pieces, int piece_len, void* part, int dtype, hipStream_t stream) {
     if (S <= 0 || H <= 0) return 0;
     if (dim <= 0 || dim > 256 || vdim <= 0 || vdim > 256 || pieces < 1 || piece_len < 1 ||
-        (pieces > 1 && (part == nullptr || piece_len > GLA_PIECE_MAX || piece_len % 4)) ||
+        (pieces > 1 && (part == nullptr || piece_len != GLA_PIECE)) ||
         H > 65535 || (int64_t)S * pieces > 0x7fffffff || cols < 2 * H * (dim + vdim))
         return (int)hipErrorInvalidValue;
     // a group has as many threads as there are value channels

@@ -1304,7 +1304,7 @@ class HipOps:
                 ws_ml = torch.empty((S * H * (K // 16) * 2,), dtype=torch.float32, device=q.device)
             ws_sums = torch.empty((N * H,), dtype=torch.float32, device=q.device) if run_prefill else None
             # one output head a wavefront: twice the workgroups, which make all scores again; where the tiles leave CUs idle
-            out_heads = 1 if -(-max_q_len // 16) * S * (2 if H > 16 else 1) * 2 <= self.compute_units() else 2
+            out_heads = 1 if -(-max_q_len // 16) * S * 2 <= self.compute_units() else 2
             self._run("talking", "lle_talking_mfma",
                       [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _L, _I, _I, _F, _P, _P, _I, _I, _I, _P, _P, _I, _I, _I,
                        _P, _P],

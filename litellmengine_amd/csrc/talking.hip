@@ -276,7 +276,6 @@ __global__ __launch_bounds__(1024) void talking_values_kernel(TalkArgs a, const 
     };
     for (int g0 = 0; g0 < group; g0 += CNT) {
         const int count = min(CNT, group - g0);
-        load_v(0);
         __syncthreads();
         for (int h = wave; h < a.H; h += 16) {
             const float2* ml = ws_ml + ((int64_t)s * a.H + h) * (K / 16);
@@ -297,13 +296,14 @@ __global__ __launch_bounds__(1024) void talking_values_kernel(TalkArgs a, const 
 #pragma unroll
             for (int i = 0; i < CNT; ++i) w[i] = 0.f;
             if (key < 16 * tiles) {
-#pragma unroll(CNT <= 4 ? 16 : 8)
+#pragma unroll 8
                 for (int g = 0; g < a.H; ++g) {
                     const float p = __builtin_amdgcn_exp2f(s_row[(int64_t)g * K + key] - s_m[g]);
 #pragma unroll
                     for (int i = 0; i < CNT; ++i) w[i] = fmaf(s_t[g * CNT + i], p, w[i]);  // (the same for all threads)
                 }
             }
+            load_v(b0);
             __syncthreads();  // (the keys before have been multiplied)
 #pragma unroll
             for (int i = 0; i < CNT; ++i) s_w[i * TV_ROW + threadIdx.x] = (bf16_t)w[i];
@@ -313,7 +313,6 @@ __global__ __launch_bounds__(1024) void talking_values_kernel(TalkArgs a, const 
                 const bf16x8 p = *(const bf16x8*)(s_w + (r16 % CNT) * TV_ROW + 256 * part + 32 * st + 8 * c);
                 acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv[st], p, acc, 0, 0, 0);
             }
-            if (b0 + TV_KEYS < 16 * tiles) load_v(b0 + TV_KEYS);
         }
         __syncthreads();
         float* s_o = lds;  // [4][CNT][64]
@@ -352,11 +351,10 @@ __device__ __forceinline__ void lds_barrier() {
 }
 
 // Portions, first launch: the base-2 log of every row's sum, ws [N][H].  grid = (blocks of 16 tokens, G, requests), four
-// wavefronts that take every fourth 32-key step; a wavefront makes the scores of four of the key/value head's query heads
-// with the keys in its registers (the other four and so on in further rounds).
-#define TS_HEADS 4
+// wavefronts that take every fourth 32-key step; a wavefront makes the scores of TS_HEADS (a divisor of the group) of the
+// key/value head's query heads with the keys in its registers, the others in further rounds.
 #define TS_WAVES 4
-template <int DK>
+template <int DK, int TS_HEADS>
 __global__ __launch_bounds__(TS_WAVES* LLE_WAVE) void talking_sums_kernel(TalkArgs a, float* __restrict__ ws) {
     constexpr int D = DK * 32;
     __shared__ float s_m[TS_WAVES][TS_HEADS][16], s_l[TS_WAVES][TS_HEADS][16];
@@ -403,7 +401,7 @@ __global__ __launch_bounds__(TS_WAVES* LLE_WAVE) void talking_sums_kernel(TalkAr
         float slope[TS_HEADS], m[TS_HEADS], l[TS_HEADS];
 #pragma unroll
         for (int i = 0; i < TS_HEADS; ++i) {
-            const int h = kvh * group + min(g0 + i, group - 1);
+            const int h = kvh * group + g0 + i;
             const bf16_t* q = (const bf16_t*)a.q + ((int64_t)(q_start + min(t0 + r16, last)) * a.H + h) * D + 8 * c;
 #pragma unroll
             for (int ks = 0; ks < DK; ++ks) qv[i][ks] = *(const bf16x8*)(q + 32 * ks);
@@ -411,7 +409,6 @@ __global__ __launch_bounds__(TS_WAVES* LLE_WAVE) void talking_sums_kernel(TalkAr
             m[i] = NEG_BIG;
             l[i] = 0.f;
         }
-        const int heads = min(TS_HEADS, group - g0);
         int page = page_of(first_step + wave);
         load_k(first_step + wave, page);
         page = page_of(first_step + wave + TS_WAVES);
@@ -420,40 +417,39 @@ __global__ __launch_bounds__(TS_WAVES* LLE_WAVE) void talking_sums_kernel(TalkAr
 #pragma unroll
             for (int i = 0; i < TS_HEADS; ++i) {
                 sc[i][0] = sc[i][1] = f32x4{0.f, 0.f, 0.f, 0.f};
-                if (i < heads) {
+            }
+            // (products that wait for one another stand apart)
+#pragma unroll
+            for (int ks = 0; ks < DK; ++ks)
+#pragma unroll
+                for (int i = 0; i < TS_HEADS; ++i)
 #pragma unroll
                     for (int t = 0; t < 2; ++t)
-#pragma unroll
-                        for (int ks = 0; ks < DK; ++ks)
-                            sc[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kreg[t][ks], qv[i][ks], sc[i][t], 0, 0, 0);
-                }
-            }
+                        sc[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kreg[t][ks], qv[i][ks], sc[i][t], 0, 0, 0);
             load_k(step + TS_WAVES, page);  // (past the last step: keys that are there)
             page = page_of(step + 2 * TS_WAVES);
             const bool open = 32 * step >= open_lo && 32 * step + 31 <= open_hi;  // (the same for all lanes)
             const float d0 = (float)(32 * step + 8 * c - pos);
 #pragma unroll
             for (int i = 0; i < TS_HEADS; ++i) {
-                if (i < heads) {
-                    float x[8], top = m[i];
+                float x[8], top = m[i];
 #pragma unroll
-                    for (int e = 0; e < 8; ++e) x[e] = fmaf(sc[i][e / 4][e % 4], scale, slope[i] * (d0 + (float)e));
-                    if (!open) {
+                for (int e = 0; e < 8; ++e) x[e] = fmaf(sc[i][e / 4][e % 4], scale, slope[i] * (d0 + (float)e));
+                if (!open) {
 #pragma unroll
-                        for (int e = 0; e < 8; ++e) {
-                            const int j = 32 * step + 8 * c + e;
-                            if (j < lo || j > pos) x[e] = NEG_BIG;
-                        }
+                    for (int e = 0; e < 8; ++e) {
+                        const int j = 32 * step + 8 * c + e;
+                        if (j < lo || j > pos) x[e] = NEG_BIG;
                     }
-#pragma unroll
-                    for (int e = 0; e < 8; ++e) top = fmaxf(top, x[e]);
-                    const float base = top <= NEG_BIG ? 0.f : top;
-                    float sum = 0.f;
-#pragma unroll
-                    for (int e = 0; e < 8; ++e) sum += __builtin_amdgcn_exp2f(x[e] - base);
-                    l[i] = l[i] * __builtin_amdgcn_exp2f(m[i] - base) + sum;
-                    m[i] = top;
                 }
+#pragma unroll
+                for (int e = 0; e < 8; ++e) top = fmaxf(top, x[e]);
+                const float base = top <= NEG_BIG ? 0.f : top;
+                float sum = 0.f;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) sum += __builtin_amdgcn_exp2f(x[e] - base);
+                l[i] = l[i] * __builtin_amdgcn_exp2f(m[i] - base) + sum;
+                m[i] = top;
             }
         }
         __syncthreads();  // (the round before has been read)
@@ -473,7 +469,7 @@ __global__ __launch_bounds__(TS_WAVES* LLE_WAVE) void talking_sums_kernel(TalkAr
         __syncthreads();
         if (threadIdx.x < TS_HEADS * 16) {
             const int i = threadIdx.x / 16, r = threadIdx.x % 16;
-            if (i < heads && t0 + r <= last) {
+            if (t0 + r <= last) {
                 float top = s_m[0][i][r];
 #pragma unroll
                 for (int w = 1; w < TS_WAVES; ++w) top = fmaxf(top, s_m[w][i][r]);
@@ -487,14 +483,16 @@ __global__ __launch_bounds__(TS_WAVES* LLE_WAVE) void talking_sums_kernel(TalkAr
 }
 
 // Portions, second launch.  grid = (output splits, blocks of 16 tokens, requests), eight wavefronts.  A wavefront makes the
-// scores of HW heads (all of the model's heads over the eight), one query token a lane column.  Three things happen in
+// scores of HW heads for XT of a step's two 16-key tiles (all of the model's heads over the eight wavefronts), one query
+// token a lane column, so that with ONE key/value head for the HW heads nobody reads a key twice.  Three things happen in
 // step i, each to another 32 keys, with one barrier a step between them:
 //   keys i      scores, weights (divided by their sum already, so between 0 and 1) into LDS in half precision (11 bits of
 //               mantissa, three more than the mixed weights keep), [key][token][head];
 //   keys i - 1  mixed on the matrix cores ([4 tokens x 4 keys] x heads times heads x 16 heads of this workgroup's
 //               split; talk in half precision holds a bfloat16 number as it is), summed in 32-bit, [token][head][key] into
 //               LDS as bfloat16;
-//   keys i - 2  O^T += V^T W^T for the OW heads of the wavefront.
+//   keys i - 2  O^T += V^T W^T: a wavefront takes BH heads of one key/value head and the value elements of its share (the
+//               wavefronts that have the same heads share the elements, so nobody reads a value twice).
 // Both LDS buffers are there twice.  A split computes all scores and the sums of 8 OW output heads: OW bounds the
 // accumulators.  LDS rows of 64 bytes are cut into four 16-byte pieces whose order is swizzled so that neither the writes nor
 // the reads of the two exchanges meet in a bank.
@@ -508,13 +506,15 @@ __device__ __forceinline__ int talk_w_at(int q, int h, int piece) {  // of a mix
     return (q * 16 + row) * 64 + ((piece ^ (row >> 2)) & 3) * 16;
 }
 
-// ONE: the HW heads of a wavefront, and the OW, share a key/value head (a load under a condition makes the compiler wait for
-// every load on its way where the paths meet again, so the usual case has none; loads past the last step ask for keys that
-// are there).
-template <int DK, int HW, int OW, bool ONE>
+// (ONE: a load under a condition makes the compiler wait for every load on its way where the paths meet again, so the usual
+// case has none; loads past the last step ask for keys that are there.)
+template <int DK, int HW, int XT, int OW, int BH, bool ONE>
 __global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a, const float* __restrict__ sums) {
     constexpr int D = DK * 32;
     constexpr int P_BYTES = TALK_P_BYTES, W_BYTES = TALK_W_BYTES;
+    constexpr int BUNDLES = 4 * XT;                   // of HW heads: eight wavefronts, or four for either key tile
+    constexpr int WB = BH / OW, TN = 2 * DK / WB;     // wavefronts that share BH output heads, and their tiles of value elements
+    static_assert(BH % OW == 0 && 2 * DK % WB == 0, "the value elements are dealt to the wavefronts in equal shares");
     extern __shared__ __attribute__((aligned(16))) char smem[];
     char* s_p = smem;
     char* s_w = smem + 2 * P_BYTES;
@@ -539,7 +539,7 @@ __global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a, const 
     const int open_lo = a.chunk > 0 ? key_hi / a.chunk * a.chunk : 0, open_hi = exists ? past + t0 : -1;
     const int first_step = key_lo / 32, steps = key_hi / 32 + 1 - first_step;
     const int half_lo = key_lo / 16, half_hi = key_hi / 16;  // 16-key halves that hold keys: others may have no page
-    const int h0 = wave * HW;
+    const int h0 = wave % BUNDLES * HW, x0 = XT == 1 ? wave / BUNDLES : 0;  // (x0: the wavefront's first key tile)
     const int heads_here = max(0, min(HW, a.H - h0));  // (the same for the whole wavefront)
     const bool all_rows = last - t0 == 15;
 
@@ -560,24 +560,28 @@ __global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a, const 
     }
     const float scale = a.scale * LOG2E;
 
+    // output heads and value elements of this wavefront (heads of a bundle are all there or none is)
+    const int oh_local = wave / WB * BH, oh0 = out0 + oh_local, v_tile0 = wave % WB * TN;
+    const bool has_outs = oh0 < a.H;
+
     // a step's two 16-key halves lie in one page each; a lane's keys lie in half r16 / 8, its values' keys in half c / 2
     const int k_half = r16 / 8, v_half = c / 2;
     auto key_of = [&](int i, int half) { return min(max(2 * (first_step + i) + half, half_lo), half_hi) * 16; };
     auto page_of = [&](int i, int half) { return table[page_index(a, key_of(i, half))]; };
-    bf16x8 kreg[2][DK], vreg[2 * DK];
+    bf16x8 kreg[XT][DK], vreg[TN];
     auto load_k = [&](int i, int page, int kvh) {
         const int j = key_of(i, k_half);
         const bf16_t* k = kv + (int64_t)page * a.page_stride + ((int64_t)kvh * P + (j - page_index(a, j) * P)) * D + 8 * c;
 #pragma unroll
-        for (int x = 0; x < 2; ++x)
+        for (int x = 0; x < XT; ++x)
 #pragma unroll
-            for (int ks = 0; ks < DK; ++ks) kreg[x][ks] = *(const bf16x8*)(k + (int64_t)(KEY_OF_ROW(r16, x) % 16) * D + 32 * ks);
+            for (int ks = 0; ks < DK; ++ks) kreg[x][ks] = *(const bf16x8*)(k + (int64_t)(KEY_OF_ROW(r16, x0 + x) % 16) * D + 32 * ks);
     };
     auto load_v = [&](int i, int page, int kvh) {
         const int j = key_of(i, v_half);
-        const bf16_t* v = kv + (int64_t)page * a.page_stride + ((int64_t)a.G + kvh) * P * D + (int64_t)r16 * P + (j - page_index(a, j) * P) + 8 * (c % 2);
+        const bf16_t* v = kv + (int64_t)page * a.page_stride + ((int64_t)a.G + kvh) * P * D + (int64_t)(v_tile0 * 16 + r16) * P + (j - page_index(a, j) * P) + 8 * (c % 2);
 #pragma unroll
-        for (int n = 0; n < 2 * DK; ++n) vreg[n] = *(const bf16x8*)(v + (int64_t)16 * n * P);
+        for (int n = 0; n < TN; ++n) vreg[n] = *(const bf16x8*)(v + (int64_t)16 * n * P);
     };
 
     // talk's rows of this split's heads: element e of lane (c, r16) is talk[out0 + r16][8 c + e]
@@ -587,60 +591,64 @@ __global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a, const 
         const int g = 8 * c + e, h = out0 + r16;
         talk[e] = (_Float16)(r16 < 8 * OW && h < a.H && g < a.H ? a.talk[h * a.H + g] : 0.f);
     }
-    const int oh0 = out0 + wave * OW;
-    const int outs_here = max(0, min(OW, a.H - oh0));
     const int first_kvh = min(h0, a.H - 1) / group, first_vkv = min(oh0, a.H - 1) / group;
-    f32x4 o[OW][2 * DK];
+    f32x4 o[BH][TN];
 #pragma unroll
-    for (int i = 0; i < OW; ++i)
+    for (int i = 0; i < BH; ++i)
 #pragma unroll
-        for (int n = 0; n < 2 * DK; ++n) o[i][n] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int n = 0; n < TN; ++n) o[i][n] = f32x4{0.f, 0.f, 0.f, 0.f};
 
     // a page is looked up one step before its keys or values are asked for, these one step before they are used
-    int k_page = page_of(0, k_half), k_page_now = k_page, v_page = page_of(0, v_half), v_page_now = v_page;
+    int k_page = page_of(0, k_half), k_page_now = k_page, v_page = page_of(0, v_half);
     load_k(0, k_page, first_kvh);
     k_page = page_of(1, k_half);
     __syncthreads();  // (the zeros are there)
     for (int i = 0; i < steps + 2; ++i) {
         if (i < steps && heads_here > 0) {
             const int step = first_step + i;
-            _Float16 p[8][HW];
+            _Float16 p[4 * XT][HW];
             [[maybe_unused]] int kvh = first_kvh;
             const bool open = all_rows && 32 * step >= open_lo && 32 * step + 31 <= past + t0;  // (the same for all lanes)
-            const float d0 = (float)(32 * step + 8 * c - pos);
+            const int j0 = 32 * step + 8 * c + 4 * x0;
+            const float d0 = (float)(j0 - pos);
+            // SG heads at a time: products that wait for one another stand apart, and their sums fit the registers
+            constexpr int SG = ONE ? (HW * XT > 4 ? HW / 2 : HW) : 1;
 #pragma unroll
-            for (int n = 0; n < HW; ++n) {
-                if (n < heads_here) {
-                    if constexpr (!ONE) {
-                        const int own = (h0 + n) / group;
-                        if (own != kvh) load_k(i, k_page_now, kvh = own);
-                    }
-                    f32x4 sc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+            for (int n0 = 0; n0 < HW; n0 += SG) {
+                f32x4 sc[SG][XT];
+                if constexpr (!ONE) {
+                    const int own = min(h0 + n0, a.H - 1) / group;
+                    if (own != kvh) load_k(i, k_page_now, kvh = own);
+                }
 #pragma unroll
-                    for (int t = 0; t < 2; ++t)
+                for (int ks = 0; ks < DK; ++ks)
 #pragma unroll
-                        for (int ks = 0; ks < DK; ++ks) sc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kreg[t][ks], qv[n][ks], sc[t], 0, 0, 0);
-                    float x[8];
+                    for (int n = 0; n < SG; ++n)
 #pragma unroll
-                    for (int e = 0; e < 8; ++e) x[e] = fmaf(sc[e / 4][e % 4], scale, fmaf(slope[n], d0 + (float)e, -sum[n]));
+                        for (int t = 0; t < XT; ++t)
+                            sc[n][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                                kreg[t][ks], qv[n0 + n][ks], ks == 0 ? f32x4{0.f, 0.f, 0.f, 0.f} : sc[n][t], 0, 0, 0);
+#pragma unroll
+                for (int n = 0; n < SG; ++n) {
+                    float x[4 * XT];
+#pragma unroll
+                    for (int e = 0; e < 4 * XT; ++e)
+                        x[e] = fmaf(sc[n][e / 4][e % 4], scale, fmaf(slope[n0 + n], d0 + (float)e, -sum[n0 + n]));
                     if (!open) {
 #pragma unroll
-                        for (int e = 0; e < 8; ++e) {
-                            const int j = 32 * step + 8 * c + e;
-                            if (j < lo || j > pos) x[e] = NEG_BIG;
-                        }
+                        for (int e = 0; e < 4 * XT; ++e)
+                            if (j0 + e < lo || j0 + e > pos) x[e] = NEG_BIG;
                     }
+                    // (heads that do not exist leave zeros)
 #pragma unroll
-                    for (int e = 0; e < 8; ++e) p[e][n] = (_Float16)__builtin_amdgcn_exp2f(x[e]);
-                } else {
-#pragma unroll
-                    for (int e = 0; e < 8; ++e) p[e][n] = (_Float16)0.f;
+                    for (int e = 0; e < 4 * XT; ++e)
+                        p[e][n0 + n] = n0 + n < heads_here ? (_Float16)__builtin_amdgcn_exp2f(x[e]) : (_Float16)0.f;
                 }
             }
             char* buf = s_p + (i & 1) * P_BYTES;
 #pragma unroll
-            for (int e = 0; e < 8; ++e) {
-                char* at = buf + talk_p_at(8 * c + e, r16, h0 / 8) + (h0 % 8) * 2;
+            for (int e = 0; e < 4 * XT; ++e) {
+                char* at = buf + talk_p_at(8 * c + 4 * x0 + e, r16, h0 / 8) + (h0 % 8) * 2;
                 if constexpr (HW == 1) *(_Float16*)at = p[e][0];
                 else if constexpr (HW == 2) *(f16x2*)at = f16x2{p[e][0], p[e][1]};
                 else *(f16x4*)at = f16x4{p[e][0], p[e][1], p[e][2], p[e][3]};
@@ -662,57 +670,77 @@ __global__ __launch_bounds__(512) void talking_prefill_kernel(TalkArgs a, const 
                 *(bf16x4*)(to + talk_w_at(4 * qa + c, r16, kq / 2) + (kq % 2) * 8) = bf16x4{(bf16_t)w[0], (bf16_t)w[1], (bf16_t)w[2], (bf16_t)w[3]};
             }
         }
-        if (i >= 2 && outs_here > 0) {
+        if (i >= 2 && has_outs) {
             const char* from = s_w + (i & 1) * W_BYTES;
-            [[maybe_unused]] int vkv = first_vkv;
+            bf16x8 w[BH];
 #pragma unroll
-            for (int n = 0; n < OW; ++n) {
-                if (n < outs_here) {
-                    if constexpr (!ONE) {
-                        const int own = (oh0 + n) / group;
-                        if (own != vkv) load_v(i - 2, v_page_now, vkv = own);
-                    }
-                    const bf16x8 w = *(const bf16x8*)(from + talk_w_at(r16, wave * OW + n, c));
+            for (int n = 0; n < BH; ++n) w[n] = *(const bf16x8*)(from + talk_w_at(r16, oh_local + n, c));
 #pragma unroll
-                    for (int m = 0; m < 2 * DK; ++m) o[n][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vreg[m], w, o[n][m], 0, 0, 0);
-                }
-            }
+            for (int n = 0; n < BH; ++n)
+#pragma unroll
+                for (int m = 0; m < TN; ++m) o[n][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vreg[m], w[n], o[n][m], 0, 0, 0);
         }
         load_v(i - 1, v_page, first_vkv);  // used in the next step
-        v_page_now = v_page;
         v_page = page_of(i, v_half);
         lds_barrier();
     }
-    if (!exists) return;
+    if (!exists || !has_outs) return;
 #pragma unroll
-    for (int i = 0; i < OW; ++i) {
-        if (i < outs_here) {
-            bf16_t* dst = (bf16_t*)a.out + ((int64_t)(q_start + t0 + r16) * a.H + oh0 + i) * D + 4 * c;
+    for (int i = 0; i < BH; ++i) {
+        bf16_t* dst = (bf16_t*)a.out + ((int64_t)(q_start + t0 + r16) * a.H + oh0 + i) * D + 16 * v_tile0 + 4 * c;
 #pragma unroll
-            for (int n = 0; n < 2 * DK; ++n)
-                *(bf16x4*)(dst + 16 * n) = bf16x4{(bf16_t)o[i][n][0], (bf16_t)o[i][n][1], (bf16_t)o[i][n][2], (bf16_t)o[i][n][3]};
-        }
+        for (int n = 0; n < TN; ++n)
+            *(bf16x4*)(dst + 16 * n) = bf16x4{(bf16_t)o[i][n][0], (bf16_t)o[i][n][1], (bf16_t)o[i][n][2], (bf16_t)o[i][n][3]};
     }
 }
 
-template <int DK, int HW, int OW, bool ONE>
-static int talk_prefill_launch_of(const TalkArgs& a, int S, int max_q_len, const float* sums, hipStream_t stream) {
+template <int DK, int HW, int XT, int OW, int BH, bool ONE>
+static int talk_prefill_launch(const TalkArgs& a, int S, int max_q_len, const float* sums, hipStream_t stream) {
     const size_t smem = 2 * (TALK_P_BYTES + TALK_W_BYTES);
     if (smem > 64 * 1024) {
-        hipError_t e = hipFuncSetAttribute((const void*)talking_prefill_kernel<DK, HW, OW, ONE>,
+        hipError_t e = hipFuncSetAttribute((const void*)talking_prefill_kernel<DK, HW, XT, OW, BH, ONE>,
                                            hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
         if (e != hipSuccess) return (int)e;
     }
     const int splits = (a.H + 8 * OW - 1) / (8 * OW);
-    talking_prefill_kernel<DK, HW, OW, ONE><<<dim3(splits, tile_order_count((max_q_len + 15) / 16, a.chunk), S), 512, smem, stream>>>(a, sums);
+    talking_prefill_kernel<DK, HW, XT, OW, BH, ONE><<<dim3(splits, tile_order_count((max_q_len + 15) / 16, a.chunk), S), 512, smem, stream>>>(a, sums);
     return (int)hipGetLastError();
 }
 
-template <int DK, int HW, int OW>
-static int talk_prefill_launch(const TalkArgs& a, int S, int max_q_len, const float* sums, hipStream_t stream) {
+// Which form of the kernel takes a model's heads: how many there are, and how many neighbours share a key/value head.  (More
+// than 16 heads: one output head a wavefront, four splits.  Two of them need more registers than two wavefronts a SIMD have,
+// and what spills costs more than the scores made twice as often: 202 against 113 us for 2048 tokens, 32 heads.)
+template <int DK>
+static int talk_prefill(const TalkArgs& a, int S, int max_q_len, int out_heads, float* sums, hipStream_t stream) {
     const int group = a.H / a.G;
-    if (group % HW == 0 && group % OW == 0) return talk_prefill_launch_of<DK, HW, OW, true>(a, S, max_q_len, sums, stream);
-    return talk_prefill_launch_of<DK, HW, OW, false>(a, S, max_q_len, sums, stream);
+    const dim3 grid(tile_order_count((max_q_len + 15) / 16, a.chunk), a.G, S);
+    if (group % 4 == 0) talking_sums_kernel<DK, 4><<<grid, TS_WAVES * LLE_WAVE, 0, stream>>>(a, sums);
+    else if (group % 2 == 0) talking_sums_kernel<DK, 2><<<grid, TS_WAVES * LLE_WAVE, 0, stream>>>(a, sums);
+    else talking_sums_kernel<DK, 1><<<grid, TS_WAVES * LLE_WAVE, 0, stream>>>(a, sums);
+    const hipError_t e = hipGetLastError();
+    if (e != hipSuccess) return (int)e;
+#define LLE_TALK(HW, XT, OW, BH, ONE) return talk_prefill_launch<DK, HW, XT, OW, BH, ONE>(a, S, max_q_len, sums, stream)
+    if (group % 4 == 0) {
+        constexpr int BH1 = DK % 2 == 0 ? 4 : 2;  // (four heads over four wavefronts: an even number of element blocks)
+        if (a.H <= 8) LLE_TALK(2, 1, 1, BH1, true);
+        if (a.H <= 16) {
+            if (out_heads == 1) LLE_TALK(4, 1, 1, BH1, true);
+            LLE_TALK(4, 1, 2, 4, true);
+        }
+        LLE_TALK(4, 2, 1, BH1, true);
+    }
+    if (group % 2 == 0) {
+        if (a.H <= 8) LLE_TALK(2, 1, 1, 2, true);
+        if (a.H <= 16) {
+            if (out_heads == 1) LLE_TALK(2, 2, 1, 2, true);
+            LLE_TALK(2, 2, 2, 2, true);
+        }
+        LLE_TALK(4, 2, 1, 2, false);
+    }
+    if (a.H <= 8) LLE_TALK(1, 2, 1, 1, true);
+    if (a.H <= 16) LLE_TALK(2, 2, 1, 1, false);
+    LLE_TALK(4, 2, 1, 1, false);
+#undef LLE_TALK
 }
 
 template <int DK>
@@ -738,15 +766,7 @@ static int talk_launch(const TalkArgs& a, int S, int run_decode, int splits, int
         if (e != hipSuccess) return (int)e;
     }
     if (run_prefill) {
-        talking_sums_kernel<DK><<<dim3(tile_order_count((max_q_len + 15) / 16, a.chunk), a.G, S), TS_WAVES * LLE_WAVE, 0, stream>>>(a, ws_sums);
-        const hipError_t e = hipGetLastError();
-        if (e != hipSuccess) return (int)e;
-        if (a.H <= 8) return talk_prefill_launch<DK, 1, 1>(a, S, max_q_len, ws_sums, stream);
-        if (a.H <= 16)
-            return out_heads == 1 ? talk_prefill_launch<DK, 2, 1>(a, S, max_q_len, ws_sums, stream)
-                                  : talk_prefill_launch<DK, 2, 2>(a, S, max_q_len, ws_sums, stream);
-        return out_heads == 1 ? talk_prefill_launch<DK, 4, 1>(a, S, max_q_len, ws_sums, stream)
-                              : talk_prefill_launch<DK, 4, 2>(a, S, max_q_len, ws_sums, stream);
+        return talk_prefill<DK>(a, S, max_q_len, out_heads, ws_sums, stream);
     }
     return 0;
 }
@@ -754,7 +774,7 @@ static int talk_launch(const TalkArgs& a, int S, int run_decode, int splits, int
 // bfloat16, D 32, 64, 96 or 128, pages of a multiple of 16 keys; with run_prefill up to 32 heads.  run_decode: the batch
 // holds requests of one token (ws_s float32 [S H K], ws_ml float32 [S H K / 8]; K a multiple of 16, at least 15 more than
 // the keys that a query sees); run_prefill: it holds longer ones.  ws_sums float32
-// [N H].  out_heads: output heads a wavefront sums up, 1 or 2.
+// [N H].  out_heads: output heads a wavefront sums up where both forms are there (9 to 16 heads), 1 or 2.
 extern "C" int lle_talking_mfma(const void* q, const void* kv, const void* block_tables, const void* seq_slots,
                                 const void* cu_tokens, const void* kv_lens, const void* token_seq, void* out, int S, int H, int G,
                                 int D, int P, int64_t page_stride, int max_pages, int chunk, float scale, const void* slopes,

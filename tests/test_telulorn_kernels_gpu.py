@@ -244,6 +244,9 @@ def test_gla_scan(dtype, H, dim, vdim, q_lens):
         at += n
     assert (torch.cat(rows).double() - got[:n0].double()).abs().max() < tol(dtype, max(1.0, big))
     assert (st[int(slots[0])] - got_state[int(slots[0])]).abs().max() < 2e-4 * float(want_state.abs().max())
+    from litellmengine_amd.csrc import build
+
+    assert build.load_library("gla").lle_gla_piece() == o.GLA_PIECE
 
 
 def test_gla_channels_that_never_forget_and_that_forget_at_once():
