@@ -1301,7 +1301,7 @@ __global__ __launch_bounds__(PRE_WAVES* LLE_WAVE, DK <= 6 ? 2 : 1) void mfma_pre
 // ---------------------------------------------------------------------------------
 #define F32_WAVES 4
 #define F32_KEYS 16
-template <int DQ>
+template <int DQ, bool KEEP>
 __global__ __launch_bounds__(F32_WAVES* LLE_WAVE) void mfma_f32_attention_kernel(
     const float* __restrict__ q, const float* __restrict__ kv_layer, const int32_t* __restrict__ block_tables,
     const int32_t* __restrict__ seq_slots, const int32_t* __restrict__ cu_tokens,
@@ -1345,12 +1345,12 @@ __global__ __launch_bounds__(F32_WAVES* LLE_WAVE) void mfma_f32_attention_kernel
 
     // the keys of this wavefront's tile, in steps of 16, and its share of them
     int step_begin = 0, step_end = 0, step_stride = 1;
-    int kept_end = 0;  // steps of the kept first keys, which are the first split's work
+    [[maybe_unused]] int kept_end = 0;  // steps of the kept first keys, which are the first split's work
     if (wave_has_rows) {
         const int last_row = min(nrows, row0 + 16) - 1;
         const int hi = past + last_row / G;
         const int lo_tile = window > 0 ? max(0, past + row0 / G - window + 1) : 0;
-        if (keep_first > 0 && split == 0) kept_end = (min(keep_first, max(0, hi - window + 1)) + F32_KEYS - 1) / F32_KEYS;
+        if (KEEP && split == 0) kept_end = (min(keep_first, max(0, hi - window + 1)) + F32_KEYS - 1) / F32_KEYS;
         const int first = lo_tile / F32_KEYS, end = hi / F32_KEYS + 1;
         const int per_split = (end - first + nsplit - 1) / nsplit;
         step_begin = first + split * per_split;
@@ -1414,12 +1414,14 @@ __global__ __launch_bounds__(F32_WAVES* LLE_WAVE) void mfma_f32_attention_kernel
             for (int e = 0; e < 4; ++e) o[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(vf[buf][n][e], p[e], o[n], 0, 0, 0);
         }
     };
-    const int w_pos = pos, w_lo = lo, w_begin = step_begin, w_end = step_end;
-    for (int range = kept_end > 0 ? 0 : 1; range < 2; ++range) {
-    pos = range == 0 ? (exists ? min(keep_first, w_lo) - 1 : -1) : w_pos;
-    lo = range == 0 ? 0 : w_lo;
-    step_begin = range == 0 ? (few ? wave : 0) : w_begin;
-    step_end = range == 0 ? kept_end : w_end;
+    [[maybe_unused]] const int w_pos = pos, w_lo = lo, w_begin = step_begin, w_end = step_end;
+    for (int range = KEEP && kept_end > 0 ? 0 : 1; range < 2; ++range) {
+    if constexpr (KEEP) {
+        pos = range == 0 ? (exists ? min(keep_first, w_lo) - 1 : -1) : w_pos;
+        lo = range == 0 ? 0 : w_lo;
+        step_begin = range == 0 ? (few ? wave : 0) : w_begin;
+        step_end = range == 0 ? kept_end : w_end;
+    }
     if constexpr (NBUF == 2) {
         // the operands of the next step are asked for before this one is multiplied
         if (step_begin < step_end) load(0, step_begin);
@@ -1539,17 +1541,22 @@ extern "C" int lle_paged_attention_mfma_f32(const void* q, const void* kv_layer,
     const float scale_log2 = scale * 1.44269504088896340736f;
     const dim3 grid(nkv, row_blocks * nsplit, S);
     const size_t smem = (size_t)(F32_WAVES * 16 * d + 2 * F32_WAVES * 16) * sizeof(float);
-#define LLE_F32_CASE(DQV)                                                                                        \
-    case DQV:                                                                                                    \
-        if (smem > 64 * 1024) {                                                                                  \
-            hipError_t e = hipFuncSetAttribute((const void*)mfma_f32_attention_kernel<DQV>,                       \
-                                               hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);           \
-            if (e != hipSuccess) return (int)e;                                                                  \
-        }                                                                                                        \
-        mfma_f32_attention_kernel<DQV><<<grid, F32_WAVES * LLE_WAVE, smem, stream>>>(                             \
-            (const float*)q, (const float*)kv_layer, (const int32_t*)block_tables, (const int32_t*)seq_slots,     \
-            (const int32_t*)cu_tokens, (const int32_t*)kv_lens, (float*)out, (float*)ws_o, (float*)ws_ml, nsplit, \
-            nq, nkv, page_size, page_stride, max_pages, window, keep_first, scale_log2, (const float*)sinks);    \
+    auto launch = [&](auto kernel) {
+        if (smem > 64 * 1024) {
+            const hipError_t e = hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+            if (e != hipSuccess) return e;
+        }
+        kernel<<<grid, F32_WAVES * LLE_WAVE, smem, stream>>>(
+            (const float*)q, (const float*)kv_layer, (const int32_t*)block_tables, (const int32_t*)seq_slots,
+            (const int32_t*)cu_tokens, (const int32_t*)kv_lens, (float*)out, (float*)ws_o, (float*)ws_ml, nsplit, nq, nkv,
+            page_size, page_stride, max_pages, window, keep_first, scale_log2, (const float*)sinks);
+        return hipGetLastError();
+    };
+    hipError_t launched = hipSuccess;
+#define LLE_F32_CASE(DQV)                                                                \
+    case DQV:                                                                            \
+        launched = keep_first > 0 ? launch(mfma_f32_attention_kernel<DQV, true>)         \
+                                  : launch(mfma_f32_attention_kernel<DQV, false>);       \
         break;
     switch (d / 16) {
         LLE_F32_CASE(1) LLE_F32_CASE(2) LLE_F32_CASE(3) LLE_F32_CASE(4) LLE_F32_CASE(5) LLE_F32_CASE(6)
@@ -1557,6 +1564,7 @@ extern "C" int lle_paged_attention_mfma_f32(const void* q, const void* kv_layer,
         LLE_F32_CASE(13) LLE_F32_CASE(14) LLE_F32_CASE(15) LLE_F32_CASE(16)
     }
 #undef LLE_F32_CASE
+    if (launched != hipSuccess) return (int)launched;
     if (nsplit > 1)
         f32_combine_kernel<<<dim3(N, nq), LLE_WAVE, 0, stream>>>((const float*)ws_o, (const float*)ws_ml, nsplit,
                                                                  (float*)out, nq, d, (const float*)sinks);
