@@ -130,8 +130,8 @@ def read(model_dir: str):
     return plain.load(model_dir)
 
 
-def plain_logits(model_dir: str, requests: Dict[str, List[int]]) -> Dict[str, torch.Tensor]:
-    cfg, w = plain.load(model_dir)
+def plain_logits(model_dir: str, requests: Dict[str, List[int]], dtype=torch.float64) -> Dict[str, torch.Tensor]:
+    cfg, w = plain.load(model_dir, dtype)
     return {rid: plain.forward(cfg, w, tokens) for rid, tokens in requests.items()}
 
 

@@ -53,6 +53,11 @@ def draw(seed: int):
     return spec, page, rng.choice([0.5, 1.0, 2.0]), lengths
 
 
+def relative(got, want) -> float:
+    """The largest error of a row, relative to the row's largest value (and to 1 at least)."""
+    return ((got.double() - want).abs().amax(1) / want.abs().amax(1).clamp(min=1)).max().item()
+
+
 @pytest.mark.parametrize("seed", range(8000, 8000 + int(os.environ.get("LLE_RANDOM_DRAWS", "10"))))
 def test_a_configuration_drawn_at_random(tmp_path, seed):
     from litellmengine_amd.config import TelulornConfig
@@ -80,8 +85,13 @@ def test_a_configuration_drawn_at_random(tmp_path, seed):
         sharpen(model_dir, factor if dtype == "float32" else 0.5, memory=1.4 if dtype == "float32" else 1.0,
                 skip=() if dtype == "float32" else (".g", ".a1", ".a2"))
         want = plain_logits(model_dir, requests)
+        tol = TOL[dtype]
+        if dtype == "float32":
+            # (a draw may multiply rounding: a read-out whose norm divides by next to nothing.  The plain implementation in
+            # 32-bit, which shares nothing with the kernels, says by how much)
+            tol = max(tol, 8 * max(relative(got, want[r]) for r, got in plain_logits(model_dir, requests, torch.float32).items()))
         out = str(tmp_path / dtype)
         model = load_model(model_dir, dtype, device="cuda:0")
         replay(model, out, pool, page, 4, io.StringIO(tb.text()), io.StringIO())
-        said += f" {dtype} {check_dumps(out, tb, want, TOL[dtype]):.2e}"
+        said += f" {dtype} {check_dumps(out, tb, want, tol):.2e}"
     print(said)
