@@ -4,6 +4,7 @@ from .kezasun_config import KezasunConfig
 from .malilorn_config import MalilornConfig
 from .birelix_config import BirelixConfig
 from .telulorn_config import TelulornConfig
+from .rorevik_config import RorevikConfig
 from .registry import (
     Architecture,
     architecture_of,
@@ -22,6 +23,7 @@ __all__ = [
     "MalilornConfig",
     "BirelixConfig",
     "TelulornConfig",
+    "RorevikConfig",
     "FULL_ATTENTION",
     "SLIDING_ATTENTION",
     "architecture_of",

@@ -12,7 +12,7 @@
 //   sees keys lo..p,  lo = max(0, p - window + 1) with a window, else 0, and with `keep_first`
 //   also the first keys, 0 .. min(keep_first, lo) - 1: every kernel walks that range first, with
 //   the same running maximum and sums, then lo..p
-//   score_j = (q . k_j) * scale;  softmax over j streamed in 32-bit (m, l, acc)
+//   score_j = (q . k_j) * scale, with a cap then cap * tanh(score_j / cap);  softmax over j streamed in 32-bit (m, l, acc)
 //   kv head of q head h = h / (nq / nkv)                  (:577-668 for the maths)
 // A cache page holds K as [nkv][page_size][d], then V as [nkv][d][page_size].
 //
@@ -46,7 +46,7 @@ __global__ __launch_bounds__(ATT_WAVES* LLE_WAVE) void paged_attention_generic_k
     const int32_t* __restrict__ seq_slots, const int32_t* __restrict__ cu_tokens,
     const int32_t* __restrict__ kv_lens, const int32_t* __restrict__ token_seq, T* __restrict__ out, int nq,
     int nkv, int d, int page_size, int64_t page_stride, int max_pages, int window, int keep_first, float scale,
-    const float* __restrict__ sinks) {
+    const float* __restrict__ sinks, float softcap) {
     __shared__ float s_m[ATT_WAVES], s_l[ATT_WAVES];
     __shared__ float s_acc[ATT_WAVES][ATT_MAX_R * LLE_WAVE];
 
@@ -131,6 +131,7 @@ __global__ __launch_bounds__(ATT_WAVES* LLE_WAVE) void paged_attention_generic_k
 #pragma unroll
         for (int i = 0; i < ATT_KEYS; ++i) {
             score[i] = wave_sum(dot[i]) * scale;
+            if (softcap > 0.f) score[i] = softcap * tanhf(score[i] / softcap);
             if (j0 + i <= pos) new_m = fmaxf(new_m, score[i]);
         }
         const float alpha = expf(m - new_m);
@@ -177,7 +178,7 @@ extern "C" int lle_paged_attention_generic(const void* q, const void* kv_layer, 
                                            const void* seq_slots, const void* cu_tokens, const void* kv_lens,
                                            const void* token_seq, void* out, int N, int nq, int nkv, int d,
                                            int page_size, int64_t page_stride, int max_pages, int window,
-                                           int keep_first, float scale, int dtype, const void* sinks,
+                                           int keep_first, float scale, int dtype, const void* sinks, float softcap,
                                            hipStream_t stream) {
     if (N <= 0) return 0;
     if (keep_first < 0 || d > ATT_MAX_R * LLE_WAVE) return (int)hipErrorInvalidValue;
@@ -186,12 +187,12 @@ extern "C" int lle_paged_attention_generic(const void* q, const void* kv_layer, 
         paged_attention_generic_kernel<float><<<grid, ATT_WAVES * LLE_WAVE, 0, stream>>>(
             (const float*)q, (const float*)kv_layer, (const int32_t*)block_tables, (const int32_t*)seq_slots,
             (const int32_t*)cu_tokens, (const int32_t*)kv_lens, (const int32_t*)token_seq, (float*)out, nq, nkv, d,
-            page_size, page_stride, max_pages, window, keep_first, scale, (const float*)sinks);
+            page_size, page_stride, max_pages, window, keep_first, scale, (const float*)sinks, softcap);
     else
         paged_attention_generic_kernel<bf16_t><<<grid, ATT_WAVES * LLE_WAVE, 0, stream>>>(
             (const bf16_t*)q, (const bf16_t*)kv_layer, (const int32_t*)block_tables, (const int32_t*)seq_slots,
             (const int32_t*)cu_tokens, (const int32_t*)kv_lens, (const int32_t*)token_seq, (bf16_t*)out, nq, nkv,
-            d, page_size, page_stride, max_pages, window, keep_first, scale, (const float*)sinks);
+            d, page_size, page_stride, max_pages, window, keep_first, scale, (const float*)sinks, softcap);
     LLE_RETURN_LAUNCH_STATUS();
 }
 
@@ -318,9 +319,12 @@ __device__ __forceinline__ float max_of_8(const float (&x)[8]) {
 // One 32-key step for RT tiles of 16 rows.  load_k(x, ks): for lane (c, r16) key
 // KEY_OF_ROW(r16, x) of the step, elements 32 ks + 8 c .. + 7.  load_v(n): value element
 // 16 n + r16, keys 8c..8c+7 of the step.  Each operand is fetched once and used by all row tiles.
-template <int DK, int RT, typename LoadK, typename LoadV>
+// CAP: the scores pass through cap * tanh(score / cap).  In the base-2 domain that is C (1 - 2 / (1 + 2^(s k))) with
+// C = cap log2 e (`cap_log2`) and k = 2 log2 e scale / cap, which the caller hands in for the scale; either end of the
+// exponential's range gives the right limit.
+template <int DK, int RT, bool CAP, typename LoadK, typename LoadV>
 __device__ __forceinline__ void tile_step(RowState<DK, RT>& st, const RowInfo (&row)[RT], LoadK load_k,
-                                          LoadV load_v, int j0, float scale_log2) {
+                                          LoadV load_v, int j0, float scale_log2, float cap_log2) {
     const int c = (threadIdx.x % LLE_WAVE) / 16;
     f32x4 s[RT][2];
 #pragma unroll
@@ -340,6 +344,16 @@ __device__ __forceinline__ void tile_step(RowState<DK, RT>& st, const RowInfo (&
 #pragma unroll
     for (int n = 0; n < 2 * DK; ++n) vv[n] = load_v(n);
     __builtin_amdgcn_sched_barrier(0);
+    if constexpr (CAP) {
+#pragma unroll
+        for (int t = 0; t < RT; ++t)
+#pragma unroll
+            for (int i = 0; i < 8; ++i) {
+                const float e = __builtin_amdgcn_exp2f(s[t][i / 4][i % 4] * scale_log2);
+                s[t][i / 4][i % 4] = fmaf(-2.f * cap_log2, __builtin_amdgcn_rcpf(1.f + e), cap_log2);
+            }
+        scale_log2 = 1.f;
+    }
     // Scores relative to the row's reference m, in the base-2 domain: x = s * scale - m.  The
     // reference only has to be near the row's maximum, not equal to it: while no x exceeds
     // LAZY_MAX the weights are exp2(x) <= 2^LAZY_MAX and nothing else is touched.  Only when
@@ -434,12 +448,14 @@ struct StepOperands {
 // this wavefront reads any key.  `after_first_loads()` runs once the first two steps are asked for.
 // A second range of keys is walked by a call with FIRST = false (the rows' lo and pos are the range's
 // then, what the first call has summed up stays); all calls but the last have LAST = false.
-template <int DK, int RT, bool LOAD_Q = true, bool FIRST = true, bool LAST = true, typename BeforeKeys, typename AfterFirstLoads>
+template <int DK, int RT, bool LOAD_Q = true, bool FIRST = true, bool LAST = true, bool CAP = false, typename BeforeKeys,
+          typename AfterFirstLoads>
 __device__ __forceinline__ void attend_rows(RowState<DK, RT>& st, const RowInfo (&row)[RT],
                                             const bf16_t* kv_layer, const int32_t* __restrict__ table,
                                             int kvh, int nkv, int P, int64_t page_stride, int step_begin,
                                             int step_end, int step_stride, int lo_min, int hi, float scale_log2,
-                                            BeforeKeys before_keys, AfterFirstLoads after_first_loads) {
+                                            BeforeKeys before_keys, AfterFirstLoads after_first_loads,
+                                            float cap_log2 = 0.f) {
     constexpr int D = DK * 32;
     const int lane = threadIdx.x % LLE_WAVE;
     const int c = lane / 16, r16 = lane % 16;
@@ -487,9 +503,9 @@ __device__ __forceinline__ void attend_rows(RowState<DK, RT>& st, const RowInfo 
         lookup();
     };
     auto multiply = [&](const StepOperands<DK>& op, int step) {
-        tile_step<DK, RT>(
+        tile_step<DK, RT, CAP>(
             st, row, [&](int x, int ks) { return op.k[x][ks]; }, [&](int n) { return op.v[n]; }, step * KSTEP,
-            scale_log2);
+            scale_log2, cap_log2);
     };
     StepOperands<DK> even, odd;
     lookup();
@@ -706,14 +722,15 @@ __device__ __forceinline__ void fused_kv_write(const FusedQKV& f, int64_t tok, i
 #ifndef DEC_WAVES
 #define DEC_WAVES 4
 #endif
-template <int DK, bool FUSED, bool KEEP>
+template <int DK, bool FUSED, bool KEEP, bool CAP>
 __global__ __launch_bounds__(DEC_WAVES* LLE_WAVE) void mfma_decode_kernel(
     const bf16_t* __restrict__ q, bf16_t* kv_layer, const int32_t* __restrict__ block_tables,
     const int32_t* __restrict__ seq_slots, const int32_t* __restrict__ cu_tokens,
     const int32_t* __restrict__ kv_lens, bf16_t* __restrict__ out, float* __restrict__ ws_o,
     float* __restrict__ ws_ml, int ws_stride, int nq, int nkv, int P, int64_t page_stride, int max_pages,
-    int window, float scale_log2, FusedQKV fused, const float* __restrict__ sinks, int keep_first) {
-    static_assert(!(FUSED && KEEP), "kept first keys: the launch that reads ready-made queries");
+    int window, float scale_log2, FusedQKV fused, const float* __restrict__ sinks, int keep_first, float cap_log2) {
+    static_assert(!(FUSED && (KEEP || CAP)), "kept first keys, capped scores: the launch that reads ready-made queries");
+    static_assert(!(KEEP && CAP), "kept first keys or capped scores");
     constexpr int D = DK * 32;
     extern __shared__ float smem[];  // [waves][16][D] acc, then [waves][16] m, [waves][16] l
     float* s_o = smem;
@@ -802,9 +819,9 @@ __global__ __launch_bounds__(DEC_WAVES* LLE_WAVE) void mfma_decode_kernel(
             st, row, kv_layer, table, kvh, nkv, P, page_stride, sb + wave, se, DEC_WAVES, lo_min, hi_loads, scale_log2,
             []() {}, []() {});
     } else {
-        attend_rows<DK, 1, true>(
+        attend_rows<DK, 1, true, true, true, CAP>(
             st, row, kv_layer, table, kvh, nkv, P, page_stride, sb + wave, se, DEC_WAVES, lo_min, hi_loads, scale_log2,
-            []() {}, []() {});
+            []() {}, []() {}, cap_log2);
     }
 
     // merge the wavefronts (rows that do not exist are not worth the LDS traffic)
@@ -933,14 +950,14 @@ __global__ __launch_bounds__(LLE_WAVE) void mfma_combine_kernel(const float* __r
 #define PRE_RT_MAX 2
 #endif
 #define PRE_RT_OF(DK) ((DK) <= 4 ? PRE_RT_MAX : 1)
-template <int DK, int PRE_RT, int PRE_WAVES, bool KEEP>
+template <int DK, int PRE_RT, int PRE_WAVES, bool KEEP, bool CAP>
 // (heads over 192 elements need more than the 256 registers a lane that two workgroups a CU leave)
 __global__ __launch_bounds__(PRE_WAVES* LLE_WAVE, DK <= 6 ? 2 : 1) void mfma_prefill_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ kv_layer, const int32_t* __restrict__ block_tables,
     const int32_t* __restrict__ seq_slots, const int32_t* __restrict__ cu_tokens,
     const int32_t* __restrict__ kv_lens, bf16_t* __restrict__ out, float* __restrict__ ws_o,
     float* __restrict__ ws_ml, int ws_stride, int nsplit, int nq, int nkv, int P, int64_t page_stride, int max_pages,
-    int window, float scale_log2, int complement_order, const float* __restrict__ sinks, int keep_first) {
+    int window, float scale_log2, int complement_order, const float* __restrict__ sinks, int keep_first, float cap_log2) {
     constexpr int D = DK * 32;
     static_assert(PRE_RT <= PRE_RT_OF(DK), "the accumulators of two row tiles fit the registers up to heads of 128");
     constexpr int PRE_ROWS = PRE_WAVES * 16 * PRE_RT;
@@ -1094,11 +1111,11 @@ __global__ __launch_bounds__(PRE_WAVES* LLE_WAVE, DK <= 6 ? 2 : 1) void mfma_pre
         if (step >= my_first && step < my_end) {
             const bf16_t* kt = lds + buf * TILE;
             const bf16_t* vt = kt + KSTEP * D;
-            tile_step<DK, PRE_RT>(
+            tile_step<DK, PRE_RT, CAP>(
                 st, row,
                 [&](int x, int ks) { return *(const bf16x8*)(kt + kx[x] * D + (((4 * ks + c) ^ ksw[x]) * 8)); },
                 [&](int n) { return *(const bf16x8*)(vt + (16 * n + r16) * KSTEP + ((c ^ vsw) * 8)); },
-                step * KSTEP, scale_log2);
+                step * KSTEP, scale_log2, cap_log2);
         }
         stash(buf ^ 1, set_c);
         __syncthreads();
@@ -1217,9 +1234,10 @@ __global__ __launch_bounds__(PRE_WAVES* LLE_WAVE, DK <= 6 ? 2 : 1) void mfma_pre
                     kreg[x][ks] = *(const bf16x8*)(kt + kx[x] * D + (((4 * ks + c) ^ ksw[x]) * 8));
             dma(next_buf);  // tile step + 2
             if (step >= my_first && step < my_end) {
-                tile_step<DK, PRE_RT>(
+                tile_step<DK, PRE_RT, CAP>(
                     st, row, [&](int x, int ks) { return kreg[x][ks]; },
-                    [&](int n) { return *(const bf16x8*)(vt + v_read + n * 256); }, step * KSTEP, scale_log2);
+                    [&](int n) { return *(const bf16x8*)(vt + v_read + n * 256); }, step * KSTEP, scale_log2,
+                    cap_log2);
             }
             // the loads just issued may stay in flight; the tile before them has landed
             if constexpr (LOADS == 2)
@@ -1301,13 +1319,13 @@ __global__ __launch_bounds__(PRE_WAVES* LLE_WAVE, DK <= 6 ? 2 : 1) void mfma_pre
 // ---------------------------------------------------------------------------------
 #define F32_WAVES 4
 #define F32_KEYS 16
-template <int DQ, bool KEEP>
+template <int DQ, bool KEEP, bool CAP>
 __global__ __launch_bounds__(F32_WAVES* LLE_WAVE) void mfma_f32_attention_kernel(
     const float* __restrict__ q, const float* __restrict__ kv_layer, const int32_t* __restrict__ block_tables,
     const int32_t* __restrict__ seq_slots, const int32_t* __restrict__ cu_tokens,
     const int32_t* __restrict__ kv_lens, float* __restrict__ out, float* __restrict__ ws_o,
     float* __restrict__ ws_ml, int nsplit, int nq, int nkv, int P, int64_t page_stride, int max_pages, int window,
-    int keep_first, float scale_log2, const float* __restrict__ sinks) {
+    int keep_first, float scale_log2, const float* __restrict__ sinks, float cap_log2) {
     constexpr int D = 16 * DQ;
     extern __shared__ float smem[];  // [waves][16][D] acc, then [waves][16] m, [waves][16] l
     float* s_o = smem;
@@ -1388,7 +1406,8 @@ __global__ __launch_bounds__(F32_WAVES* LLE_WAVE) void mfma_f32_attention_kernel
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
             const int j = j0 + 4 * c + e;
-            x[e] = (j < lo || j > pos) ? NEG_BIG : sc[e] * scale_log2;
+            const float score = CAP ? cap_log2 * tanhf(sc[e] * scale_log2) : sc[e] * scale_log2;  // (CAP: scale / cap)
+            x[e] = (j < lo || j > pos) ? NEG_BIG : score;
         }
         float top = fmaxf(fmaxf(x[0], x[1]), fmaxf(x[2], x[3]));
         top = fmaxf(top, __shfl_xor(top, 16, LLE_WAVE));
@@ -1531,14 +1550,17 @@ extern "C" int lle_paged_attention_mfma_f32(const void* q, const void* kv_layer,
                                             void* out, void* ws_o, void* ws_ml, int N, int S, int nq, int nkv, int d,
                                             int page_size, int64_t page_stride, int max_pages, int window,
                                             int keep_first, float scale, int row_blocks, int nsplit, const void* sinks,
-                                            hipStream_t stream) {
+                                            float softcap, hipStream_t stream) {
     if (N <= 0) return 0;
     if (d % 16 != 0 || d > 256 || d <= 0 || page_size % 16 != 0 || nq % nkv != 0) return (int)hipErrorInvalidValue;
     if (S > 65535 || nkv <= 0 || row_blocks < 1 || nsplit < 1 || nsplit > 64 || (int64_t)row_blocks * nsplit > 65535)
         return (int)hipErrorInvalidValue;
     if (nsplit > 1 && (!ws_o || !ws_ml)) return (int)hipErrorInvalidValue;
     if (keep_first < 0 || (keep_first > 0 && window <= 0)) return (int)hipErrorInvalidValue;
-    const float scale_log2 = scale * 1.44269504088896340736f;
+    if (softcap < 0.f || (softcap > 0.f && keep_first > 0)) return (int)hipErrorInvalidValue;
+    // with a cap: the factor that tanh's argument gets, and the cap in the base-2 domain
+    const float scale_log2 = softcap > 0.f ? scale / softcap : scale * 1.44269504088896340736f;
+    const float cap_log2 = softcap * 1.44269504088896340736f;
     const dim3 grid(nkv, row_blocks * nsplit, S);
     const size_t smem = (size_t)(F32_WAVES * 16 * d + 2 * F32_WAVES * 16) * sizeof(float);
     auto launch = [&](auto kernel) {
@@ -1549,14 +1571,15 @@ extern "C" int lle_paged_attention_mfma_f32(const void* q, const void* kv_layer,
         kernel<<<grid, F32_WAVES * LLE_WAVE, smem, stream>>>(
             (const float*)q, (const float*)kv_layer, (const int32_t*)block_tables, (const int32_t*)seq_slots,
             (const int32_t*)cu_tokens, (const int32_t*)kv_lens, (float*)out, (float*)ws_o, (float*)ws_ml, nsplit, nq, nkv,
-            page_size, page_stride, max_pages, window, keep_first, scale_log2, (const float*)sinks);
+            page_size, page_stride, max_pages, window, keep_first, scale_log2, (const float*)sinks, cap_log2);
         return hipGetLastError();
     };
     hipError_t launched = hipSuccess;
 #define LLE_F32_CASE(DQV)                                                                \
     case DQV:                                                                            \
-        launched = keep_first > 0 ? launch(mfma_f32_attention_kernel<DQV, true>)         \
-                                  : launch(mfma_f32_attention_kernel<DQV, false>);       \
+        launched = keep_first > 0 ? launch(mfma_f32_attention_kernel<DQV, true, false>)  \
+                   : softcap > 0.f ? launch(mfma_f32_attention_kernel<DQV, false, true>) \
+                                   : launch(mfma_f32_attention_kernel<DQV, false, false>); \
         break;
     switch (d / 16) {
         LLE_F32_CASE(1) LLE_F32_CASE(2) LLE_F32_CASE(3) LLE_F32_CASE(4) LLE_F32_CASE(5) LLE_F32_CASE(6)
@@ -1584,22 +1607,22 @@ static int compute_units() {
     return cached[dev];
 }
 
-template <int DK, bool FUSED, bool KEEP>
+template <int DK, bool FUSED, bool KEEP, bool CAP = false>
 static int launch_decode(const bf16_t* q, bf16_t* kv_layer, const int32_t* block_tables, const int32_t* seq_slots,
                          const int32_t* cu_tokens, const int32_t* kv_lens, bf16_t* out, float* ws_o, float* ws_ml,
                          int ws_stride, int S, int nq, int nkv, int P, int64_t page_stride, int max_pages, int window,
                          float scale_log2, int nsplit, const FusedQKV& fused, const float* sinks, int keep_first,
-                         hipStream_t stream) {
+                         float cap_log2, hipStream_t stream) {
     constexpr int D = DK * 32;
     const size_t smem = (size_t)(DEC_WAVES * 16 * D + 2 * DEC_WAVES * 16) * sizeof(float);
     if (smem > 64 * 1024) {
-        hipError_t e = hipFuncSetAttribute((const void*)mfma_decode_kernel<DK, FUSED, KEEP>,
+        hipError_t e = hipFuncSetAttribute((const void*)mfma_decode_kernel<DK, FUSED, KEEP, CAP>,
                                            hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
         if (e != hipSuccess) return (int)e;
     }
-    mfma_decode_kernel<DK, FUSED, KEEP><<<dim3(S, nkv, nsplit), DEC_WAVES * LLE_WAVE, smem, stream>>>(
+    mfma_decode_kernel<DK, FUSED, KEEP, CAP><<<dim3(S, nkv, nsplit), DEC_WAVES * LLE_WAVE, smem, stream>>>(
         q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out, ws_o, ws_ml, ws_stride, nq, nkv, P,
-        page_stride, max_pages, window, scale_log2, fused, sinks, keep_first);
+        page_stride, max_pages, window, scale_log2, fused, sinks, keep_first, cap_log2);
     return 0;
 }
 
@@ -1634,13 +1657,14 @@ static int launch_mfma(const bf16_t* q, bf16_t* kv_layer, const int32_t* block_t
                        const int32_t* token_seq, bf16_t* out, float* ws_o, float* ws_ml, int N, int S, int nq,
                        int nkv, int P, int64_t page_stride, int max_pages, int window, float scale_log2,
                        int run_decode, int nsplit_decode, int run_prefill, int nsplit_prefill, int max_q_len,
-                       int prefill_form, const FusedQKV& fused, const float* sinks, int keep_first, hipStream_t stream) {
+                       int prefill_form, const FusedQKV& fused, const float* sinks, int keep_first, float cap_log2,
+                       hipStream_t stream) {
     constexpr int D = DK * 32;
     const int G = nq / nkv;
     if (!run_decode) nsplit_decode = 1;
     if (!run_prefill) nsplit_prefill = 1;
     const int ws_stride = nsplit_decode > nsplit_prefill ? nsplit_decode : nsplit_prefill;
-    if (fused.qkv && (run_prefill || !run_decode || DK % 2 != 0 || keep_first)) return (int)hipErrorInvalidValue;
+    if (fused.qkv && (run_prefill || !run_decode || DK % 2 != 0 || keep_first || cap_log2 > 0.f)) return (int)hipErrorInvalidValue;
     // both kinds in one batch: the decode kernel goes to the side stream, forked from and joined to `stream`
     SideLane* lane = (run_decode && run_prefill) ? side_lane() : nullptr;
     hipStream_t prefill_stream = stream;
@@ -1654,18 +1678,22 @@ static int launch_mfma(const bf16_t* q, bf16_t* kv_layer, const int32_t* block_t
         if (keep_first > 0) {
             e = launch_decode<DK, false, true>(q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out, ws_o, ws_ml,
                                                ws_stride, S, nq, nkv, P, page_stride, max_pages, window, scale_log2,
-                                               nsplit_decode, fused, sinks, keep_first, stream);
+                                               nsplit_decode, fused, sinks, keep_first, 0.f, stream);
+        } else if (cap_log2 > 0.f) {
+            e = launch_decode<DK, false, false, true>(q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out, ws_o, ws_ml,
+                                                      ws_stride, S, nq, nkv, P, page_stride, max_pages, window, scale_log2,
+                                                      nsplit_decode, fused, sinks, 0, cap_log2, stream);
         } else if constexpr (DK % 2 == 0) {
             e = fused.qkv ? launch_decode<DK, true, false>(q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out, ws_o,
                                                     ws_ml, ws_stride, S, nq, nkv, P, page_stride, max_pages, window,
-                                                    scale_log2, nsplit_decode, fused, sinks, 0, stream)
+                                                    scale_log2, nsplit_decode, fused, sinks, 0, 0.f, stream)
                           : launch_decode<DK, false, false>(q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out,
                                                      ws_o, ws_ml, ws_stride, S, nq, nkv, P, page_stride, max_pages,
-                                                     window, scale_log2, nsplit_decode, fused, sinks, 0, stream);
+                                                     window, scale_log2, nsplit_decode, fused, sinks, 0, 0.f, stream);
         } else {
             e = launch_decode<DK, false, false>(q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out, ws_o, ws_ml,
                                          ws_stride, S, nq, nkv, P, page_stride, max_pages, window, scale_log2,
-                                         nsplit_decode, fused, sinks, 0, stream);
+                                         nsplit_decode, fused, sinks, 0, 0.f, stream);
         }
         if (e != 0) {
             if (lane) (void)hipStreamSynchronize(lane->stream);
@@ -1693,10 +1721,11 @@ static int launch_mfma(const bf16_t* q, bf16_t* kv_layer, const int32_t* block_t
                 kernel<<<dim3(nkv, blocks * nsplit_prefill, S), WAVES * LLE_WAVE, 0, stream>>>(
                     q, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, out, ws_o, ws_ml, ws_stride, nsplit_prefill,
                     nq, nkv, P, page_stride, max_pages, window, scale_log2, workgroups <= 2 * compute_units() ? 1 : 0, sinks,
-                    keep_first);
+                    keep_first, cap_log2);
             };
-            if (keep_first > 0) go(mfma_prefill_kernel<DK, RT, WAVES, true>);
-            else go(mfma_prefill_kernel<DK, RT, WAVES, false>);
+            if (keep_first > 0) go(mfma_prefill_kernel<DK, RT, WAVES, true, false>);
+            else if (cap_log2 > 0.f) go(mfma_prefill_kernel<DK, RT, WAVES, false, true>);
+            else go(mfma_prefill_kernel<DK, RT, WAVES, false, false>);
         };
         using Four = std::integral_constant<int, 4>;
         if (DK == 4 && prefill_form == 3) {
@@ -1730,21 +1759,24 @@ static int paged_attention_mfma(const void* q, void* kv_layer, const void* block
                                 int64_t page_stride, int max_pages, int window, float scale, int run_decode,
                                 int nsplit_decode, int run_prefill, int nsplit_prefill, int max_q_len,
                                 int prefill_form, const FusedQKV& fused, const float* sinks, int keep_first,
-                                hipStream_t stream) {
+                                float softcap, hipStream_t stream) {
     if (N <= 0) return 0;
     if (keep_first < 0 || (keep_first > 0 && window <= 0)) return (int)hipErrorInvalidValue;
     if (d % 32 != 0 || d > 256 || page_size % 16 != 0 || nq % nkv != 0) return (int)hipErrorInvalidValue;
     if (S > 65535 || nkv > 65535 || page_stride < 0 || page_stride >= ((int64_t)1 << 32)) return (int)hipErrorInvalidValue;
     if (nsplit_decode < 1 || nsplit_decode > 64 || nsplit_prefill < 1 || nsplit_prefill > 64)
         return (int)hipErrorInvalidValue;
-    const float scale_log2 = scale * 1.44269504088896340736f;
+    if (softcap < 0.f || (softcap > 0.f && keep_first > 0)) return (int)hipErrorInvalidValue;
+    const float cap_log2 = softcap * 1.44269504088896340736f;
+    const float scale_log2 = softcap > 0.f ? 2.f * scale / softcap * 1.44269504088896340736f : scale * 1.44269504088896340736f;
 #define LLE_ATT_CASE(DKV)                                                                                          \
     case DKV:                                                                                                      \
         return launch_mfma<DKV>((const bf16_t*)q, (bf16_t*)kv_layer, (const int32_t*)block_tables,                  \
                                 (const int32_t*)seq_slots, (const int32_t*)cu_tokens, (const int32_t*)kv_lens,      \
                                 (const int32_t*)token_seq, (bf16_t*)out, (float*)ws_o, (float*)ws_ml, N, S, nq, nkv, \
                                 page_size, page_stride, max_pages, window, scale_log2, run_decode, nsplit_decode,   \
-                                run_prefill, nsplit_prefill, max_q_len, prefill_form, fused, sinks, keep_first, stream);
+                                run_prefill, nsplit_prefill, max_q_len, prefill_form, fused, sinks, keep_first, cap_log2,     \
+                                stream);
     switch (d / 32) {
         LLE_ATT_CASE(1)
         LLE_ATT_CASE(2)
@@ -1765,12 +1797,12 @@ extern "C" int lle_paged_attention_mfma(const void* q, const void* kv_layer, con
                                         int nq, int nkv, int d, int page_size, int64_t page_stride, int max_pages,
                                         int window, float scale, int run_decode, int nsplit_decode, int run_prefill,
                                         int nsplit_prefill, int max_q_len, int prefill_form, const void* sinks,
-                                        int keep_first, hipStream_t stream) {
+                                        int keep_first, float softcap, hipStream_t stream) {
     const FusedQKV none = {};
     return paged_attention_mfma(q, (void*)kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, token_seq, out, ws_o,
                                 ws_ml, N, S, nq, nkv, d, page_size, page_stride, max_pages, window, scale, run_decode,
                                 nsplit_decode, run_prefill, nsplit_prefill, max_q_len, prefill_form, none,
-                                (const float*)sinks, keep_first, stream);
+                                (const float*)sinks, keep_first, softcap, stream);
 }
 
 // Decode steps only (every request has at most 16 / group tokens), head_dim a multiple of 64, a
@@ -1799,5 +1831,5 @@ extern "C" int lle_qk_norm_rope_attention_decode(const void* qkv, const void* sl
     fused.write_kv = write_kv;
     return paged_attention_mfma(nullptr, kv_layer, block_tables, seq_slots, cu_tokens, kv_lens, token_seq, out, ws_o,
                                 ws_ml, N, S, nq, nkv, d, page_size, page_stride, max_pages, window, scale, 1,
-                                nsplit_decode, 0, 1, 1, 0, fused, nullptr, 0, stream);
+                                nsplit_decode, 0, 1, 1, 0, fused, nullptr, 0, 0.f, stream);
 }

@@ -39,6 +39,7 @@ LIBRARIES: Dict[str, List[str]] = {
     "delta": ["delta.hip"],
     "gla": ["gla.hip"],
     "talking": ["talking.hip"],
+    "ssd": ["ssd.hip"],
     "probe": ["probe.hip"],
 }
 # libraries without GPU code: compiled with the host's C++ compiler

@@ -4,7 +4,9 @@
 //   q, k <- every head of c's q and k parts as a unit vector (x / sqrt(sum x^2 + unit_eps)), q times q_scale
 //   beta = sigmoid(b),  g = exp(-exp(A_log) softplus(a + dt_bias))     one of each per token and head         delta_scan
 //   S <- g S;  w = beta (v - S^T k);  S <- S + k w^T;  o = S^T q       S [key, value] float32, per head
-//   y = o / rms(o) * norm_w * silu(gate)  per head, eps inside the root                                       delta_out_norm
+//   y = o / rms(o) * norm_w * act(gate)   per head, eps inside the root, act silu or sigmoid                  delta_out_norm
+// The decay may also be one of every key channel, g = exp(-exp(A_log) softplus(z + dt_bias)) with z and dt_bias
+// [head][channel]: it then acts on the rows of S, S <- diag(g) S, and is made ahead of the walk              low_rank_gates
 //
 // Value head h reads the q and k of head h / (H / G).  Every value channel of a head is a recurrence of its
 // own over a vector of `dim` numbers (the column S[:, j]): a thread owns KI key channels of one column, the
@@ -31,6 +33,8 @@ __device__ __forceinline__ float delta_silu(float x) { return x / (1.0f + expf(-
 // units / 4): a wavefront per unit (a q head, a k head or a v head), a lane keeps up to four elements.
 // `state` rows hold the last J - 1 rows of u of earlier steps, oldest first (float32); zeros at admission
 // stand for the zeros before a request's start.
+// ADVANCE (steps of single tokens only): the kept rows move on by the token in the same launch; every element's
+// rows are read and written by the one lane that owns it.
 // ---------------------------------------------------------------------------------
 template <typename T>
 __global__ __launch_bounds__(256) void delta_conv_kernel(const T* __restrict__ u, int cols, const float* __restrict__ taps,
@@ -91,9 +95,9 @@ __global__ __launch_bounds__(256) void delta_conv_kernel(const T* __restrict__ u
 // J - 1 inputs of its elements in registers, so a token costs one new load per element whatever J (a workgroup a
 // token re-reads J rows and the taps for every token: 61 against 25 us for 2048 tokens of 4096 channels and four
 // taps).  Where the request changes inside a run the window is filled anew.
-template <typename T, int J>
+template <typename T, int J, bool ADVANCE>
 __global__ __launch_bounds__(256) void delta_conv_run_kernel(const T* __restrict__ u, int cols, const float* __restrict__ taps,
-                                                              const float* __restrict__ state, int64_t state_stride,
+                                                              float* state, int64_t state_stride,
                                                               const int32_t* __restrict__ token_seq,
                                                               const int32_t* __restrict__ cu_tokens,
                                                               const int32_t* __restrict__ seq_slots, float* __restrict__ q,
@@ -132,7 +136,7 @@ __global__ __launch_bounds__(256) void delta_conv_run_kernel(const T* __restrict
                 const int e = lane + LLE_WAVE * r;
                 if (e < width) {
 #pragma unroll
-                    for (int m = 0; m < W; ++m) {
+                    for (int m = 0; m < W; ++m) {  // (the rows of earlier steps, then those of this one)
                         const int back = J - 1 - m;
                         win[r][m] = back <= before ? to_f32<T>(u[(int64_t)(n - back) * cols + col0 + e])
                                                    : kept[(int64_t)(J - 1 - (back - before)) * cols + col0 + e];
@@ -155,6 +159,11 @@ __global__ __launch_bounds__(256) void delta_conv_run_kernel(const T* __restrict
 #pragma unroll
                     for (int m = 0; m + 1 < W; ++m) win[r][m] = win[r][m + 1];
                     win[r][W - 1] = x;
+                    if (ADVANCE) {
+                        float* kept = state + (int64_t)seq_slots[seq] * state_stride;
+#pragma unroll
+                        for (int m = 0; m < W; ++m) kept[(int64_t)m * cols + col0 + e] = win[r][m];
+                    }
                 }
                 acc = fmaf(tp[r][J - 1], x, acc);
                 y[r] = delta_silu(acc);
@@ -175,8 +184,8 @@ __global__ __launch_bounds__(256) void delta_conv_run_kernel(const T* __restrict
     }
 }
 
-template <typename T>
-static bool delta_conv_runs(const void* u, int cols, const void* taps, int J, const void* state, int64_t state_stride,
+template <typename T, bool ADVANCE>
+static bool delta_conv_runs(const void* u, int cols, const void* taps, int J, void* state, int64_t state_stride,
                             const void* token_seq, const void* cu_tokens, const void* seq_slots, void* q, void* k, void* v, int N,
                             int G, int dim, int H, int vdim, float unit_eps, float q_scale, hipStream_t stream) {
     const int blocks = (2 * G + H + 3) / 4;
@@ -186,8 +195,8 @@ static bool delta_conv_runs(const void* u, int cols, const void* taps, int J, co
     const dim3 grid((N + run - 1) / run, blocks);
 #define DELTA_CONV_CASE(JJ)                                                                                                   \
     case JJ:                                                                                                                  \
-        delta_conv_run_kernel<T, JJ><<<grid, 256, 0, stream>>>(                                                               \
-            (const T*)u, cols, (const float*)taps, (const float*)state, state_stride, (const int32_t*)token_seq,              \
+        delta_conv_run_kernel<T, JJ, ADVANCE><<<grid, 256, 0, stream>>>(                                                      \
+            (const T*)u, cols, (const float*)taps, (float*)state, state_stride, (const int32_t*)token_seq,                    \
             (const int32_t*)cu_tokens, (const int32_t*)seq_slots, (float*)q, (float*)k, (float*)v, N, run, G, dim, H, vdim,   \
             unit_eps, q_scale);                                                                                               \
         return true;
@@ -205,18 +214,24 @@ static bool delta_conv_runs(const void* u, int cols, const void* taps, int J, co
     return false;  // more taps: a workgroup a token
 }
 
-extern "C" int lle_delta_conv(const void* u, int cols, const void* taps, int J, const void* state, int64_t state_stride,
+extern "C" int lle_delta_conv_max_advance(void) { return 8; }
+
+// `advance` != 0: every request of the step has one token, and its kept rows move on (J up to lle_delta_conv_max_advance)
+extern "C" int lle_delta_conv(const void* u, int cols, const void* taps, int J, void* state, int64_t state_stride,
                               const void* token_seq, const void* cu_tokens, const void* seq_slots, void* q, void* k, void* v,
-                              int N, int G, int dim, int H, int vdim, float unit_eps, float q_scale, int dtype,
+                              int N, int G, int dim, int H, int vdim, float unit_eps, float q_scale, int advance, int dtype,
                               hipStream_t stream) {
     if (N <= 0) return 0;
+    if (advance && J > 8) return (int)hipErrorInvalidValue;
     if (J < 1 || (J > 1 && state == nullptr) || G <= 0 || H <= 0 || dim <= 0 || vdim <= 0 || dim > 4 * LLE_WAVE ||
         vdim > 4 * LLE_WAVE || cols != 2 * G * dim + H * vdim || (2 * G + H + 3) / 4 > 65535)
         return (int)hipErrorInvalidValue;
-    if (dtype == LLE_F32 ? delta_conv_runs<float>(u, cols, taps, J, state, state_stride, token_seq, cu_tokens, seq_slots, q, k, v, N, G,
-                                                  dim, H, vdim, unit_eps, q_scale, stream)
-                         : delta_conv_runs<bf16_t>(u, cols, taps, J, state, state_stride, token_seq, cu_tokens, seq_slots, q, k, v, N, G,
-                                                   dim, H, vdim, unit_eps, q_scale, stream))
+    auto runs = [&](auto kernel) {
+        return kernel(u, cols, taps, J, state, state_stride, token_seq, cu_tokens, seq_slots, q, k, v, N, G, dim, H, vdim, unit_eps,
+                      q_scale, stream);
+    };
+    if (dtype == LLE_F32 ? (advance ? runs(delta_conv_runs<float, true>) : runs(delta_conv_runs<float, false>))
+                         : (advance ? runs(delta_conv_runs<bf16_t, true>) : runs(delta_conv_runs<bf16_t, false>)))
         LLE_RETURN_LAUNCH_STATUS();
     const dim3 grid(N, (2 * G + H + 3) / 4);
     if (dtype == LLE_F32)
@@ -239,7 +254,8 @@ struct DeltaArgs {
     const float* q;        // [N, G dim]
     const float* k;        // [N, G dim]
     const float* v;        // [N, H vdim]
-    const float* ba;       // [N, 2 H]: beta's input of every head, then the decay's
+    const float* ba;       // rows of ba_cols: beta's input of every head, then (one decay per head) the decay's
+    int ba_cols;
     const float* a_log;    // [H]
     const float* dt_bias;  // [H]
     float* state;          // rows of state_stride floats: [H][vdim][dim]
@@ -249,21 +265,22 @@ struct DeltaArgs {
     float* out;            // [N, H vdim]
     int H, G, dim, vdim;
     const float* gates;    // [N, 2 H]: decay and beta of every token and head, made ahead (or null: made in the walk)
+    const float* decay;    // [N, H dim]: the decays of every key channel (or null: one per head, as above)
 };
 
 // decay and beta of every token and head, for the walks of long portions: in the walk itself the exponentials and the
 // logarithm of a chunk's sixteen tokens are one wavefront's work while the other three wait (a ninth of the walk's time)
-__global__ __launch_bounds__(256) void delta_gates_kernel(const float* __restrict__ ba, const float* __restrict__ a_log,
+__global__ __launch_bounds__(256) void delta_gates_kernel(const float* __restrict__ ba, int ba_cols, const float* __restrict__ a_log,
                                                            const float* __restrict__ dt_bias, float* __restrict__ gates,
                                                            int64_t total, int H) {
     const int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (idx >= total) return;
     const int64_t n = idx / H;
     const int h = (int)(idx - n * H);
-    const float x = ba[n * 2 * H + H + h] + dt_bias[h];
+    const float x = ba[n * ba_cols + H + h] + dt_bias[h];
     const float softplus = fmaxf(x, 0.f) + log1pf(expf(-fabsf(x)));
     gates[n * 2 * H + h] = expf(-expf(a_log[h]) * softplus);
-    gates[n * 2 * H + H + h] = 1.0f / (1.0f + expf(-ba[n * 2 * H + h]));
+    gates[n * 2 * H + H + h] = 1.0f / (1.0f + expf(-ba[n * ba_cols + h]));
 }
 
 template <int CTRL>
@@ -280,16 +297,29 @@ __device__ __forceinline__ float delta_row_sum(float x) {
     return x;
 }
 
-// What a thread reads of one staged token: its share of k and q, and the token's decay, beta and k . q.
-template <int KI>
+// What a thread reads of one staged token: its share of k and q (CHANNEL: and of the channels' decays), and the
+// token's decay, beta and k . q.
+template <int KI, bool CHANNEL>
 struct DeltaToken {
-    float kk[KI], qq[KI];
+    float kk[KI], qq[KI], gg[CHANNEL ? KI : 1];
     float g, beta, kq;
 };
 
-template <int KI>
-__device__ __forceinline__ void delta_read(DeltaToken<KI>& d, const float* __restrict__ kt, const float* __restrict__ qt,
-                                           const float4* __restrict__ par) {
+template <int KI, bool CHANNEL>
+__device__ __forceinline__ void delta_read(DeltaToken<KI, CHANNEL>& d, const float* __restrict__ kt, const float* __restrict__ qt,
+                                           const float* __restrict__ gt, const float4* __restrict__ par) {
+    if constexpr (CHANNEL) {
+        if (KI % 4 == 0) {
+#pragma unroll
+            for (int ii = 0; ii < KI; ii += 4) {
+                const float4 a = *(const float4*)(gt + ii);
+                d.gg[ii] = a.x, d.gg[ii + 1] = a.y, d.gg[ii + 2] = a.z, d.gg[ii + 3] = a.w;
+            }
+        } else {
+#pragma unroll
+            for (int ii = 0; ii < KI; ++ii) d.gg[ii] = gt[ii];
+        }
+    }
     if (KI % 4 == 0) {
 #pragma unroll
         for (int ii = 0; ii < KI; ii += 4) {
@@ -310,9 +340,23 @@ __device__ __forceinline__ void delta_read(DeltaToken<KI>& d, const float* __res
 
 // One token of the walk for this thread's share of column j: both sums over the key channels in one pass, the
 // lanes' exchange, the correction; returns the read-out.
-template <int KI>
-__device__ __forceinline__ float delta_token(float (&S)[KI], const DeltaToken<KI>& d, float v) {
+template <int KI, bool CHANNEL>
+__device__ __forceinline__ float delta_token(float (&S)[KI], const DeltaToken<KI, CHANNEL>& d, float v) {
     float p = 0.f, r = 0.f, gS[KI];
+    if constexpr (CHANNEL) {  // the rows of S decay each at their own rate: the sums are taken over the decayed column
+#pragma unroll
+        for (int ii = 0; ii < KI; ++ii) {
+            gS[ii] = d.gg[ii] * S[ii];
+            p = fmaf(gS[ii], d.kk[ii], p);
+            r = fmaf(gS[ii], d.qq[ii], r);
+        }
+        p = delta_row_sum(p);
+        r = delta_row_sum(r);
+        const float w = d.beta * (v - p);
+#pragma unroll
+        for (int ii = 0; ii < KI; ++ii) S[ii] = fmaf(d.kk[ii], w, gS[ii]);
+        return fmaf(w, d.kq, r);
+    }
 #pragma unroll
     for (int ii = 0; ii < KI; ++ii) {
         p = fmaf(S[ii], d.kk[ii], p);
@@ -337,13 +381,14 @@ __device__ __forceinline__ float delta_token(float (&S)[KI], const DeltaToken<KI
 // time 281 us; decays and betas made by a launch ahead of the walk 248 us.  Tried and not kept: all of a chunk's operands in registers before its first token
 // and k . q made in the walk (378 us, and two workgroups no longer share a CU: 194 against 116 us for four
 // requests of 512 tokens).
-template <int KI>
+template <int KI, bool CHANNEL>
 __global__ __launch_bounds__(DELTA_THREADS) void delta_scan_kernel(DeltaArgs a) {
     constexpr int KD = KI * DELTA_IG;
     constexpr int PER = DELTA_TC * KD / DELTA_THREADS;  // elements of q (and of k) of a chunk that a thread fetches
     static_assert(DELTA_TC * KD % DELTA_THREADS == 0, "a chunk's q and k are dealt to the threads in equal shares");
     __shared__ __attribute__((aligned(16))) float s_q[DELTA_TC][KD];
     __shared__ __attribute__((aligned(16))) float s_k[DELTA_TC][KD];
+    __shared__ __attribute__((aligned(16))) float s_g[CHANNEL ? DELTA_TC : 1][CHANNEL ? KD : 4];
     __shared__ float4 s_par[DELTA_TC];  // (decay, beta, k . q, -) of every staged token
     __shared__ float s_o[DELTA_TC][DELTA_VB];
     __shared__ float s_v[DELTA_TC][DELTA_VB];
@@ -352,6 +397,7 @@ __global__ __launch_bounds__(DELTA_THREADS) void delta_scan_kernel(DeltaArgs a) 
     const int j0 = blockIdx.z * DELTA_VB, j = j0 + jl;
     const int dim = a.dim, vdim = a.vdim, H = a.H;
     const int hk = h / (H / a.G), GD = a.G * dim, HV = H * vdim;
+    [[maybe_unused]] const int HD = H * dim;
     const int q0 = a.cu_tokens[s], q1 = a.cu_tokens[s + 1];
     if (q1 <= q0) return;
     float* col = a.state + (int64_t)a.seq_slots[s] * a.state_stride + ((int64_t)h * vdim + j) * dim + ig * KI;
@@ -359,9 +405,9 @@ __global__ __launch_bounds__(DELTA_THREADS) void delta_scan_kernel(DeltaArgs a) 
     float S[KI];
 #pragma unroll
     for (int ii = 0; ii < KI; ++ii) S[ii] = (live && ig * KI + ii < dim) ? col[ii] : 0.f;
-    const float decay_rate = expf(a.a_log[h]), dt_bias = a.dt_bias[h];
+    const float decay_rate = CHANNEL ? 0.f : expf(a.a_log[h]), dt_bias = CHANNEL ? 0.f : a.dt_bias[h];
 
-    float fq[PER], fk[PER], fv = 0.f, fb = 0.f, fa = 0.f;  // the chunk that is on its way
+    float fq[PER], fk[PER], fg[CHANNEL ? PER : 1], fv = 0.f, fb = 0.f, fa = 0.f;  // the chunk that is on its way
     const bool wide = PER % 4 == 0 && dim == KD;  // whole heads of a multiple of 64 channels: 16 bytes a load and a store
     auto fetch = [&](int c0, int nt) {
         if (wide) {
@@ -369,6 +415,11 @@ __global__ __launch_bounds__(DELTA_THREADS) void delta_scan_kernel(DeltaArgs a) 
             for (int r = 0; r + 3 < PER; r += 4) {
                 const int e = (tid + DELTA_THREADS * (r / 4)) * 4, t = e / KD, i = e - t * KD;
                 float4 x = float4{0.f, 0.f, 0.f, 0.f}, y = x;
+                if constexpr (CHANNEL) {
+                    float4 z = x;
+                    if (t < nt) z = *(const float4*)(a.decay + (int64_t)(c0 + t) * HD + h * dim + i);
+                    fg[r] = z.x, fg[r + 1] = z.y, fg[r + 2] = z.z, fg[r + 3] = z.w;
+                }
                 if (t < nt) {
                     const int64_t at = (int64_t)(c0 + t) * GD + hk * dim + i;
                     x = *(const float4*)(a.q + at);
@@ -385,6 +436,7 @@ __global__ __launch_bounds__(DELTA_THREADS) void delta_scan_kernel(DeltaArgs a) 
                 const int64_t at = (int64_t)(c0 + t) * GD + hk * dim + i;
                 fq[r] = there ? a.q[at] : 0.f;
                 fk[r] = there ? a.k[at] : 0.f;
+                if constexpr (CHANNEL) fg[r] = there ? a.decay[(int64_t)(c0 + t) * HD + h * dim + i] : 0.f;
             }
         }
         {  // the chunk's values of the workgroup's columns: one element a thread (one load a lane and token, sixteen
@@ -393,9 +445,13 @@ __global__ __launch_bounds__(DELTA_THREADS) void delta_scan_kernel(DeltaArgs a) 
             fv = (t < nt && j0 + e < vdim) ? a.v[(int64_t)(c0 + t) * HV + h * vdim + j0 + e] : 0.f;
         }
         if (tid < nt) {  // (with gates made ahead: beta, then the decay itself)
-            const float* ba = (a.gates ? a.gates : a.ba) + (int64_t)(c0 + tid) * 2 * H;
-            fb = a.gates ? ba[H + h] : ba[h];
-            fa = a.gates ? ba[h] : ba[H + h];
+            if constexpr (CHANNEL) {
+                fb = a.ba[(int64_t)(c0 + tid) * a.ba_cols + h];
+            } else {
+                const float* ba = a.gates ? a.gates + (int64_t)(c0 + tid) * 2 * H : a.ba + (int64_t)(c0 + tid) * a.ba_cols;
+                fb = a.gates ? ba[H + h] : ba[h];
+                fa = a.gates ? ba[h] : ba[H + h];
+            }
         }
     };
     fetch(q0, min(DELTA_TC, q1 - q0));
@@ -409,6 +465,7 @@ __global__ __launch_bounds__(DELTA_THREADS) void delta_scan_kernel(DeltaArgs a) 
                 const int e = (tid + DELTA_THREADS * (r / 4)) * 4, t = e / KD, i = e - t * KD;
                 *(float4*)&s_q[t][i] = float4{fq[r], fq[r + 1], fq[r + 2], fq[r + 3]};
                 *(float4*)&s_k[t][i] = float4{fk[r], fk[r + 1], fk[r + 2], fk[r + 3]};
+                if constexpr (CHANNEL) *(float4*)&s_g[t][i] = float4{fg[r], fg[r + 1], fg[r + 2], fg[r + 3]};
             }
         } else {
 #pragma unroll
@@ -416,11 +473,14 @@ __global__ __launch_bounds__(DELTA_THREADS) void delta_scan_kernel(DeltaArgs a) 
                 const int e = tid + DELTA_THREADS * r, t = e / KD, i = e - t * KD;
                 s_q[t][i] = fq[r];
                 s_k[t][i] = fk[r];
+                if constexpr (CHANNEL) s_g[t][i] = fg[r];
             }
         }
         if (tid < nt) {
             float* par = (float*)&s_par[tid];
-            if (a.gates) {
+            if (CHANNEL) {
+                par[1] = 1.0f / (1.0f + expf(-fb));
+            } else if (a.gates) {
                 par[0] = fa;
                 par[1] = fb;
             } else {
@@ -445,14 +505,16 @@ __global__ __launch_bounds__(DELTA_THREADS) void delta_scan_kernel(DeltaArgs a) 
         __syncthreads();
         const float* kt = &s_k[0][ig * KI];
         const float* qt = &s_q[0][ig * KI];
+        constexpr int GS = CHANNEL ? KD : 0;
+        const float* gt = CHANNEL ? &s_g[0][ig * KI] : &s_g[0][0];
         float oo[DELTA_TC];
         if (nt == DELTA_TC) {  // a whole chunk: nothing under a condition, every token's operands read a token ahead
-            DeltaToken<KI> cur, nxt;
-            delta_read<KI>(cur, kt, qt, &s_par[0]);
+            DeltaToken<KI, CHANNEL> cur, nxt;
+            delta_read<KI, CHANNEL>(cur, kt, qt, gt, &s_par[0]);
 #pragma unroll
             for (int t = 0; t < DELTA_TC; ++t) {
-                if (t + 1 < DELTA_TC) delta_read<KI>(nxt, kt + (t + 1) * KD, qt + (t + 1) * KD, &s_par[t + 1]);
-                oo[t] = delta_token<KI>(S, cur, vv[t]);
+                if (t + 1 < DELTA_TC) delta_read<KI, CHANNEL>(nxt, kt + (t + 1) * KD, qt + (t + 1) * KD, gt + (t + 1) * GS, &s_par[t + 1]);
+                oo[t] = delta_token<KI, CHANNEL>(S, cur, vv[t]);
                 cur = nxt;
             }
         } else {
@@ -460,9 +522,9 @@ __global__ __launch_bounds__(DELTA_THREADS) void delta_scan_kernel(DeltaArgs a) 
             for (int t = 0; t < DELTA_TC; ++t) {
                 oo[t] = 0.f;
                 if (t < nt) {
-                    DeltaToken<KI> cur;
-                    delta_read<KI>(cur, kt + t * KD, qt + t * KD, &s_par[t]);
-                    oo[t] = delta_token<KI>(S, cur, vv[t]);
+                    DeltaToken<KI, CHANNEL> cur;
+                    delta_read<KI, CHANNEL>(cur, kt + t * KD, qt + t * KD, gt + t * GS, &s_par[t]);
+                    oo[t] = delta_token<KI, CHANNEL>(S, cur, vv[t]);
                 }
             }
         }
@@ -487,25 +549,30 @@ extern "C" int lle_delta_max_dim(void) { return 16 * DELTA_IG; }
 
 // q, k float32 [N, G dim] (unit vectors, q scaled), v float32 [N, H vdim], ba float32 [N, 2 H], a_log and dt_bias
 // float32 [H]; state float32 rows of `state_stride` floats whose first H vdim dim hold the heads' states transposed;
-// out float32 [N, H vdim]; `gates` (or null) scratch float32 [N, 2 H] for the decays and betas made ahead of the walk
-extern "C" int lle_delta_scan(const void* q, const void* k, const void* v, const void* ba, const void* a_log,
-                              const void* dt_bias, void* state, int64_t state_stride, const void* seq_slots,
+// out float32 [N, H vdim]; `gates` (or null) scratch float32 [N, 2 H] for the decays and betas made ahead of the walk.
+// `decay` float32 [N, H dim] (or null): the decays of every key channel; then ba (rows of ba_cols floats) holds beta's
+// inputs alone, and a_log, dt_bias and gates are not used.
+extern "C" int lle_delta_scan(const void* q, const void* k, const void* v, const void* ba, int ba_cols, const void* decay,
+                              const void* a_log, const void* dt_bias, void* state, int64_t state_stride, const void* seq_slots,
                               const void* cu_tokens, void* out, int S, int H, int G, int dim, int vdim, void* gates, int N,
                               hipStream_t stream) {
     if (S <= 0 || H <= 0) return 0;
     if (G <= 0 || H % G || dim <= 0 || dim > 16 * DELTA_IG || vdim <= 0 || H > 65535 || (vdim + DELTA_VB - 1) / DELTA_VB > 65535)
         return (int)hipErrorInvalidValue;
-    DeltaArgs a{(const float*)q, (const float*)k, (const float*)v, (const float*)ba, (const float*)a_log, (const float*)dt_bias,
-                (float*)state, state_stride, (const int32_t*)seq_slots, (const int32_t*)cu_tokens, (float*)out, H, G, dim, vdim, (const float*)gates};
-    if (gates != nullptr) {  // scratch float32 [N, 2 H], given for steps with long portions
+    if (ba_cols < (decay ? H : 2 * H)) return (int)hipErrorInvalidValue;
+    DeltaArgs a{(const float*)q, (const float*)k, (const float*)v, (const float*)ba, ba_cols, (const float*)a_log,
+                (const float*)dt_bias, (float*)state, state_stride, (const int32_t*)seq_slots, (const int32_t*)cu_tokens,
+                (float*)out, H, G, dim, vdim, (const float*)gates, (const float*)decay};
+    if (gates != nullptr && decay == nullptr) {  // scratch float32 [N, 2 H], given for steps with long portions
         const int64_t total = (int64_t)N * H;
-        delta_gates_kernel<<<(int)((total + 255) / 256), 256, 0, stream>>>((const float*)ba, (const float*)a_log,
+        delta_gates_kernel<<<(int)((total + 255) / 256), 256, 0, stream>>>((const float*)ba, ba_cols, (const float*)a_log,
                                                                             (const float*)dt_bias, (float*)gates, total, H);
     }
     const dim3 grid(S, H, (vdim + DELTA_VB - 1) / DELTA_VB);
 #define DELTA_CASE(KI)                                                      \
     if (dim <= KI * DELTA_IG) {                                             \
-        delta_scan_kernel<KI><<<grid, DELTA_THREADS, 0, stream>>>(a);       \
+        if (decay) delta_scan_kernel<KI, true><<<grid, DELTA_THREADS, 0, stream>>>(a);   \
+        else delta_scan_kernel<KI, false><<<grid, DELTA_THREADS, 0, stream>>>(a);        \
         LLE_RETURN_LAUNCH_STATUS();                                         \
     }
     DELTA_CASE(1)
@@ -518,11 +585,110 @@ extern "C" int lle_delta_scan(const void* q, const void* k, const void* v, const
 }
 
 // ---------------------------------------------------------------------------------
-// y[n, h, :] = o / sqrt(mean(o^2) + eps) * norm_w * silu(gate): a wavefront per (token, head);
-// grid = (tokens, heads / 4).  norm_w [vdim] is one weight for all heads.
+// What a delta rule with a decay per key channel makes of two small projections, each through a narrow middle:
+//   decay[n][c] = exp(-exp(a_log[c / dim]) softplus(z + dt_bias[c])),  z = sum_r low[n][a_col + r] a2[c][r]
+//   gate[n][c]  = sum_r low[n][g_col + r] g2[c][r]                     (its sigmoid is taken by the output norm)
+// low float32 [N, low_cols], a2 float32 [CA, RA], g2 float32 [CG, RG]: RA and RG multiples of 16 (weights and the
+// columns of `low` padded with zeros), every row 16-byte aligned.  Everything in 32-bit, on the 32-bit matrix
+// instruction: a wavefront takes 16 tokens and NT tiles of 16 channels.  A lane (c, r) loads four neighbouring
+// elements of the contraction of token r (channel r); element e is slot c of instruction e.  The result tile leaves it
+// with token r and channels 4 c .. 4 c + 3.
 // ---------------------------------------------------------------------------------
-template <typename T>
-__global__ __launch_bounds__(256) void delta_out_norm_kernel(const float* __restrict__ o, const T* __restrict__ gate,
+typedef float delta_f32x4 __attribute__((ext_vector_type(4)));
+
+struct LowRankArgs {
+    const float* low;
+    int low_cols, a_col, g_col;
+    const float* a2;
+    int RA, CA;
+    const float* g2;
+    int RG, CG;
+    const float* a_log;
+    const float* dt_bias;
+    int dim;
+    float* decay;
+    float* gate;
+    int N;
+};
+
+__device__ __forceinline__ float delta_decay_of(float z, float rate) {
+    const float softplus = fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
+    return expf(-rate * softplus);
+}
+
+// grid = (blocks of channels: those of the decays, then those of the gates; tiles of 16 tokens in fours); a wavefront
+// of the four has a token tile of its own
+template <int NT>
+__global__ __launch_bounds__(256) void low_rank_gates_kernel(LowRankArgs a) {
+    const int wave = threadIdx.x / LLE_WAVE, lane = threadIdx.x % LLE_WAVE, c = lane / 16, r = lane % 16;
+    const int n0 = (blockIdx.y * 4 + wave) * 16;
+    if (n0 >= a.N) return;
+    const int a_blocks = (a.CA + 16 * NT - 1) / (16 * NT);
+    const bool decays = (int)blockIdx.x < a_blocks;
+    const int c0 = (decays ? blockIdx.x : blockIdx.x - a_blocks) * 16 * NT;
+    const int R = decays ? a.RA : a.RG, C = decays ? a.CA : a.CG;
+    const float* w = decays ? a.a2 : a.g2;
+    const float* x = a.low + (int64_t)min(n0 + r, a.N - 1) * a.low_cols + (decays ? a.a_col : a.g_col) + 4 * c;
+    const float* wr[NT];
+#pragma unroll
+    for (int n = 0; n < NT; ++n) wr[n] = w + (int64_t)min(c0 + 16 * n + r, C - 1) * R + 4 * c;
+    delta_f32x4 acc[NT];
+#pragma unroll
+    for (int n = 0; n < NT; ++n) acc[n] = delta_f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int k = 0; k < R; k += 16) {
+        const delta_f32x4 xv = *(const delta_f32x4*)(x + k);
+        delta_f32x4 wv[NT];
+#pragma unroll
+        for (int n = 0; n < NT; ++n) wv[n] = *(const delta_f32x4*)(wr[n] + k);
+#pragma unroll
+        for (int n = 0; n < NT; ++n)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) acc[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(wv[n][e], xv[e], acc[n], 0, 0, 0);
+    }
+    if (n0 + r >= a.N) return;
+    float* dst = (decays ? a.decay : a.gate) + (int64_t)(n0 + r) * C;
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+        const int ch = c0 + 16 * n + 4 * c;
+        float y[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            y[e] = acc[n][e];
+            if (decays && ch + e < C) y[e] = delta_decay_of(y[e] + a.dt_bias[ch + e], expf(a.a_log[(ch + e) / a.dim]));
+        }
+        if (C % 4 == 0) {
+            if (ch < C) *(float4*)(dst + ch) = make_float4(y[0], y[1], y[2], y[3]);
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+                if (ch + e < C) dst[ch + e] = y[e];
+        }
+    }
+}
+
+extern "C" int lle_low_rank_gates(const void* low, int low_cols, int a_col, int g_col, const void* a2, int RA, int CA,
+                                  const void* g2, int RG, int CG, const void* a_log, const void* dt_bias, int dim, void* decay,
+                                  void* gate, int N, hipStream_t stream) {
+    if (N <= 0) return 0;
+    if (low_cols % 4 || a_col % 4 || g_col % 4 || RA <= 0 || RA % 16 || RG % 16 || RG < 0 || CA <= 0 || CG < 0 || dim <= 0 ||
+        CA % dim || a_col < 0 || g_col < 0 || a_col + RA > low_cols || g_col + RG > low_cols || (CG > 0 && RG == 0))
+        return (int)hipErrorInvalidValue;
+    const LowRankArgs a{(const float*)low, low_cols, a_col, g_col, (const float*)a2, RA, CA, (const float*)g2, RG, CG,
+                        (const float*)a_log, (const float*)dt_bias, dim, (float*)decay, (float*)gate, N};
+    const int rows = (N + 63) / 64;
+    if (rows > 65535) return (int)hipErrorInvalidValue;
+    // few tokens: a tile of channels a wavefront (more of them); many: four, which share the tokens' operands
+    if (N <= 64) low_rank_gates_kernel<1><<<dim3((CA + 15) / 16 + (CG + 15) / 16, rows), 256, 0, stream>>>(a);
+    else low_rank_gates_kernel<4><<<dim3((CA + 63) / 64 + (CG + 63) / 64, rows), 256, 0, stream>>>(a);
+    LLE_RETURN_LAUNCH_STATUS();
+}
+
+// ---------------------------------------------------------------------------------
+// y[n, h, :] = o / sqrt(mean(o^2) + eps) * norm_w * act(gate): a wavefront per (token, head);
+// grid = (tokens, heads / 4).  norm_w [vdim] is one weight for all heads.  act: silu, or (SIGMOID) the sigmoid.
+// ---------------------------------------------------------------------------------
+template <typename T, typename TG, bool SIGMOID>
+__global__ __launch_bounds__(256) void delta_out_norm_kernel(const float* __restrict__ o, const TG* __restrict__ gate,
                                                               const void* __restrict__ norm_w, int norm_dtype, float eps,
                                                               T* __restrict__ out, int H, int vdim) {
     const int64_t n = blockIdx.x;
@@ -532,20 +698,29 @@ __global__ __launch_bounds__(256) void delta_out_norm_kernel(const float* __rest
     float ss = 0.f;
     for (int e = lane; e < vdim; e += LLE_WAVE) ss = fmaf(o[at + e], o[at + e], ss);
     const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)vdim + eps);
-    for (int e = lane; e < vdim; e += LLE_WAVE)
-        out[at + e] = from_f32<T>(o[at + e] * inv * load_as_f32(norm_w, e, norm_dtype) * delta_silu(to_f32<T>(gate[at + e])));
+    for (int e = lane; e < vdim; e += LLE_WAVE) {
+        const float z = to_f32<TG>(gate[at + e]);
+        const float g = SIGMOID ? 1.0f / (1.0f + expf(-z)) : delta_silu(z);
+        out[at + e] = from_f32<T>(o[at + e] * inv * load_as_f32(norm_w, e, norm_dtype) * g);
+    }
 }
 
-extern "C" int lle_delta_out_norm(const void* o, const void* gate, const void* norm_w, int norm_dtype, float eps, void* out,
-                                  int N, int H, int vdim, int dtype, hipStream_t stream) {
+// `gate_dtype`: the output's type, or float32; `sigmoid` != 0: the gate is its sigmoid, else its silu
+extern "C" int lle_delta_out_norm(const void* o, const void* gate, int gate_dtype, int sigmoid, const void* norm_w, int norm_dtype,
+                                  float eps, void* out, int N, int H, int vdim, int dtype, hipStream_t stream) {
     if (N <= 0 || H <= 0) return 0;
-    if (vdim <= 0 || (H + 3) / 4 > 65535) return (int)hipErrorInvalidValue;
+    if (vdim <= 0 || (H + 3) / 4 > 65535 || (gate_dtype != dtype && gate_dtype != LLE_F32)) return (int)hipErrorInvalidValue;
     const dim3 grid(N, (H + 3) / 4);
-    if (dtype == LLE_F32)
-        delta_out_norm_kernel<float><<<grid, 256, 0, stream>>>((const float*)o, (const float*)gate, norm_w, norm_dtype, eps,
-                                                                (float*)out, H, vdim);
-    else
-        delta_out_norm_kernel<bf16_t><<<grid, 256, 0, stream>>>((const float*)o, (const bf16_t*)gate, norm_w, norm_dtype, eps,
-                                                                 (bf16_t*)out, H, vdim);
+#define DELTA_OUT(T, TG, SIG)                                                                                                \
+    delta_out_norm_kernel<T, TG, SIG><<<grid, 256, 0, stream>>>((const float*)o, (const TG*)gate, norm_w, norm_dtype, eps,   \
+                                                                (T*)out, H, vdim)
+    if (dtype == LLE_F32) {
+        if (sigmoid) DELTA_OUT(float, float, true); else DELTA_OUT(float, float, false);
+    } else if (gate_dtype == LLE_F32) {
+        if (sigmoid) DELTA_OUT(bf16_t, float, true); else DELTA_OUT(bf16_t, float, false);
+    } else {
+        if (sigmoid) DELTA_OUT(bf16_t, bf16_t, true); else DELTA_OUT(bf16_t, bf16_t, false);
+    }
+#undef DELTA_OUT
     LLE_RETURN_LAUNCH_STATUS();
 }

@@ -225,12 +225,14 @@ extern "C" int lle_tanh(void* x, int64_t total, int dtype, hipStream_t stream) {
 //   gated:  out[n, f] = act(z[n, f] + b[f]) * (z[n, F + f] + b[F + f])        z [N, 2 F]
 //   plain:  out[n, f] = act(z[n, f] + b[f])                                   z [N, F]
 // times sigmoid(row_gate[n * gate_stride + gate_col]) where a row gate is given (float32).
-// act: 0 silu, 1 relu, 2 the square of relu, 3 gelu in its tanh form.  `b` may be null.  Everything in 32-bit.
+// act: 0 silu, 1 relu, 2 the square of relu, 3 gelu in its tanh form, 4 (gated only) clamped: with g = min(gate + b, limit)
+// and u = clamp(up + b, -limit, limit) the result is g sigmoid(1.702 g) (u + 1).  `b` may be null.  Everything in 32-bit.
 // ---------------------------------------------------------------------------------
 #define LLE_ACT_SILU 0
 #define LLE_ACT_RELU 1
 #define LLE_ACT_RELU2 2
 #define LLE_ACT_GELU_TANH 3
+#define LLE_ACT_CLAMP 4
 
 __device__ __forceinline__ float apply_act(float x, int kind) {
     if (kind == LLE_ACT_SILU) return x / (1.0f + expf(-x));
@@ -240,10 +242,15 @@ __device__ __forceinline__ float apply_act(float x, int kind) {
     return kind == LLE_ACT_RELU ? r : r * r;
 }
 
+__device__ __forceinline__ float clamped_gate(float gate, float up, float limit) {
+    const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+    return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void bias_act_kernel(const T* __restrict__ z, const T* __restrict__ bias,
                                                         const float* __restrict__ row_gate, int gate_stride, int gate_col,
-                                                        T* __restrict__ out, int N, int F, int gated, int kind) {
+                                                        T* __restrict__ out, int N, int F, int gated, int kind, float limit) {
     const int64_t total = (int64_t)N * F;
     const int in_cols = gated ? 2 * F : F;
     for (int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total;
@@ -251,8 +258,9 @@ __global__ __launch_bounds__(256) void bias_act_kernel(const T* __restrict__ z, 
         const int64_t n = idx / F;
         const int f = (int)(idx - n * F);
         const T* row = z + n * in_cols;
-        float a = apply_act(to_f32<T>(row[f]) + (bias ? to_f32<T>(bias[f]) : 0.f), kind);
-        if (gated) a *= to_f32<T>(row[F + f]) + (bias ? to_f32<T>(bias[F + f]) : 0.f);
+        const float first = to_f32<T>(row[f]) + (bias ? to_f32<T>(bias[f]) : 0.f);
+        const float second = gated ? to_f32<T>(row[F + f]) + (bias ? to_f32<T>(bias[F + f]) : 0.f) : 1.0f;
+        float a = kind == LLE_ACT_CLAMP ? clamped_gate(first, second, limit) : apply_act(first, kind) * second;
         if (row_gate) a *= 1.0f / (1.0f + expf(-row_gate[n * gate_stride + gate_col]));
         out[idx] = from_f32<T>(a);
     }
@@ -263,7 +271,7 @@ template <int GATED, int KIND>
 __global__ __launch_bounds__(256) void bias_act_vec_kernel(const bf16_t* __restrict__ z, const bf16_t* __restrict__ bias,
                                                             const float* __restrict__ row_gate, int gate_stride,
                                                             int gate_col, bf16_t* __restrict__ out, int64_t total8,
-                                                            int F8) {
+                                                            int F8, float limit) {
     for (int64_t idx = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total8;
          idx += (int64_t)gridDim.x * blockDim.x) {
         const int64_t n = idx / F8;
@@ -280,8 +288,14 @@ __global__ __launch_bounds__(256) void bias_act_vec_kernel(const bf16_t* __restr
         ebf16x8 o;
 #pragma unroll
         for (int k = 0; k < 8; ++k) {
-            float a = apply_act((float)g[k] + (bias ? (float)bg[k] : 0.f), KIND);
-            if (GATED) a *= (float)u[k] + (bias ? (float)bu[k] : 0.f);
+            const float first = (float)g[k] + (bias ? (float)bg[k] : 0.f);
+            float a;
+            if constexpr (GATED && KIND == LLE_ACT_CLAMP) {
+                a = clamped_gate(first, (float)u[k] + (bias ? (float)bu[k] : 0.f), limit);
+            } else {
+                a = apply_act(first, KIND);
+                if (GATED) a *= (float)u[k] + (bias ? (float)bu[k] : 0.f);
+            }
             o[k] = (bf16_t)(a * rg);
         }
         *(ebf16x8*)(out + idx * 8) = o;
@@ -290,14 +304,15 @@ __global__ __launch_bounds__(256) void bias_act_vec_kernel(const bf16_t* __restr
 
 template <int GATED>
 static void bias_act_vec(const void* z, const void* bias, const void* row_gate, int gate_stride, int gate_col, void* out,
-                         int64_t total8, int F8, int kind, hipStream_t stream) {
+                         int64_t total8, int F8, int kind, float limit, hipStream_t stream) {
     int64_t blocks = (total8 + 255) / 256;
     if (blocks > 16384) blocks = 16384;
 #define LLE_ACT_CASE(K)                                                                                              \
     bias_act_vec_kernel<GATED, K><<<(int)blocks, 256, 0, stream>>>((const bf16_t*)z, (const bf16_t*)bias,            \
                                                                     (const float*)row_gate, gate_stride, gate_col,  \
-                                                                    (bf16_t*)out, total8, F8)
-    if (kind == LLE_ACT_SILU) LLE_ACT_CASE(LLE_ACT_SILU);
+                                                                    (bf16_t*)out, total8, F8, limit)
+    if (kind == LLE_ACT_CLAMP) LLE_ACT_CASE(LLE_ACT_CLAMP);
+    else if (kind == LLE_ACT_SILU) LLE_ACT_CASE(LLE_ACT_SILU);
     else if (kind == LLE_ACT_RELU) LLE_ACT_CASE(LLE_ACT_RELU);
     else if (kind == LLE_ACT_GELU_TANH) LLE_ACT_CASE(LLE_ACT_GELU_TANH);
     else LLE_ACT_CASE(LLE_ACT_RELU2);
@@ -305,23 +320,23 @@ static void bias_act_vec(const void* z, const void* bias, const void* row_gate, 
 }
 
 extern "C" int lle_bias_act(const void* z, const void* bias, const void* row_gate, int gate_stride, int gate_col,
-                            void* out, int N, int F, int gated, int kind, int dtype, hipStream_t stream) {
+                            void* out, int N, int F, int gated, int kind, float limit, int dtype, hipStream_t stream) {
     if (N <= 0 || F <= 0) return 0;
-    if (kind < 0 || kind > LLE_ACT_GELU_TANH) return (int)hipErrorInvalidValue;
+    if (kind < 0 || kind > LLE_ACT_CLAMP || (kind == LLE_ACT_CLAMP && (!gated || !(limit > 0.f)))) return (int)hipErrorInvalidValue;
     if (dtype == LLE_BF16 && F % 8 == 0) {
-        if (gated) bias_act_vec<1>(z, bias, row_gate, gate_stride, gate_col, out, (int64_t)N * F / 8, F / 8, kind, stream);
-        else bias_act_vec<0>(z, bias, row_gate, gate_stride, gate_col, out, (int64_t)N * F / 8, F / 8, kind, stream);
+        if (gated) bias_act_vec<1>(z, bias, row_gate, gate_stride, gate_col, out, (int64_t)N * F / 8, F / 8, kind, limit, stream);
+        else bias_act_vec<0>(z, bias, row_gate, gate_stride, gate_col, out, (int64_t)N * F / 8, F / 8, kind, limit, stream);
         LLE_RETURN_LAUNCH_STATUS();
     }
     int64_t blocks = ((int64_t)N * F + 255) / 256;
     if (blocks > 65536) blocks = 65536;
     if (dtype == LLE_F32)
         bias_act_kernel<float><<<(int)blocks, 256, 0, stream>>>((const float*)z, (const float*)bias, (const float*)row_gate,
-                                                                 gate_stride, gate_col, (float*)out, N, F, gated, kind);
+                                                                 gate_stride, gate_col, (float*)out, N, F, gated, kind, limit);
     else
         bias_act_kernel<bf16_t><<<(int)blocks, 256, 0, stream>>>((const bf16_t*)z, (const bf16_t*)bias,
                                                                   (const float*)row_gate, gate_stride, gate_col,
-                                                                  (bf16_t*)out, N, F, gated, kind);
+                                                                  (bf16_t*)out, N, F, gated, kind, limit);
     LLE_RETURN_LAUNCH_STATUS();
 }
 

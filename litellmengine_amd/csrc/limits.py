@@ -13,6 +13,8 @@ MAX_WKV_HEAD_DIM = 256
 MAX_DELTA_HEAD_DIM = 256
 # gated linear attention: as the recurrence with a matrix state, key and value channels each
 MAX_GLA_HEAD_DIM = 256
+# Mamba-2's recurrence: state and value channels of a head; a wavefront keeps a token's state channels in registers
+MAX_SSD_DIM = 256
 # heads whose weights are mixed keep a tile of scores, one of weights and their sums in LDS
 MAX_TALKING_LDS = 160 * 1024
 TALKING_KEYS = 64

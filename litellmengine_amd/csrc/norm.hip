@@ -54,7 +54,7 @@ template <> struct Quad<bf16_t> {
     }
 };
 
-__device__ __forceinline__ float4 load_weight4(const void* w, int i, int dtype) {
+__device__ __forceinline__ float4 load_weight4(const void* w, int64_t i, int dtype) {
     return dtype == LLE_F32 ? Quad<float>::load((const float*)w + i) : Quad<bf16_t>::load((const bf16_t*)w + i);
 }
 
@@ -381,7 +381,7 @@ extern "C" int lle_rmsnorm_add(void* hidden, const void* y, int y_dtype, const v
 }
 
 // For arrangements whose sublayers run side by side on one norm's result and whose sum enters the stream
-// times a constant: hidden[r] += mult * (a[r] (+ b[r])) in 32-bit and in place, then out[r] = norm(hidden[r]) * w.
+// times constants: hidden[r] += mult_a * a[r] (+ mult_b * b[r]) in 32-bit and in place, then out[r] = norm(hidden[r]) * w.
 // `a`, `b` hold float32 or bfloat16, each said by its own code.  With `rows` only those rows are read, row
 // rows[r] gives out[r], and `hidden` is left alone.  The new row waits in registers between the sum of
 // squares and the scaling (rows up to 256 x 4 x SA_CHUNKS wide and a multiple of 4; a plain loop otherwise).
@@ -389,7 +389,7 @@ extern "C" int lle_rmsnorm_add(void* hidden, const void* y, int y_dtype, const v
 template <typename TO>
 __global__ __launch_bounds__(256) void scaled_add_rmsnorm_kernel(float* __restrict__ hidden, const void* __restrict__ a,
                                                                   int a_dtype, const void* __restrict__ b, int b_dtype,
-                                                                  float mult, const int32_t* __restrict__ rows,
+                                                                  float mult_a, float mult_b, const int32_t* __restrict__ rows,
                                                                   const void* __restrict__ weight, int weight_dtype,
                                                                   TO* __restrict__ out, int H, float eps) {
     __shared__ float red[16];
@@ -402,16 +402,16 @@ __global__ __launch_bounds__(256) void scaled_add_rmsnorm_kernel(float* __restri
         for (int c = 0; c < SA_CHUNKS; ++c) {
             const int i = (c * 256 + threadIdx.x) * 4;
             if (i < H) {
-                float4 h = *(const float4*)(hidden + at + i);
-                float v[4] = {h.x, h.y, h.z, h.w};
-#pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    float d = load_as_f32(a, at + i + e, a_dtype);
-                    if (b) d += load_as_f32(b, at + i + e, b_dtype);
-                    v[e] += mult * d;
-                    ss += v[e] * v[e];
+                float4 v = *(const float4*)(hidden + at + i);
+                const float4 x = load_weight4(a, at + i, a_dtype);
+                float4 d = make_float4(mult_a * x.x, mult_a * x.y, mult_a * x.z, mult_a * x.w);
+                if (b) {
+                    const float4 y = load_weight4(b, at + i, b_dtype);
+                    d = make_float4(fmaf(mult_b, y.x, d.x), fmaf(mult_b, y.y, d.y), fmaf(mult_b, y.z, d.z), fmaf(mult_b, y.w, d.w));
                 }
-                keep[c] = make_float4(v[0], v[1], v[2], v[3]);
+                v = make_float4(v.x + d.x, v.y + d.y, v.z + d.z, v.w + d.w);
+                ss += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
+                keep[c] = v;
                 if (!rows) *(float4*)(hidden + at + i) = keep[c];
             }
         }
@@ -421,40 +421,40 @@ __global__ __launch_bounds__(256) void scaled_add_rmsnorm_kernel(float* __restri
         for (int c = 0; c < SA_CHUNKS; ++c) {
             const int i = (c * 256 + threadIdx.x) * 4;
             if (i < H) {
-                const float v[4] = {keep[c].x, keep[c].y, keep[c].z, keep[c].w};
-#pragma unroll
-                for (int e = 0; e < 4; ++e) out[to + i + e] = from_f32<TO>(v[e] * inv * load_as_f32(weight, i + e, weight_dtype));
+                const float4 w = load_weight4(weight, i, weight_dtype);
+                Quad<TO>::store(out + to + i, make_float4(keep[c].x * inv * w.x, keep[c].y * inv * w.y, keep[c].z * inv * w.z,
+                                                          keep[c].w * inv * w.w));
             }
         }
         return;
     }
     for (int i = threadIdx.x; i < H; i += blockDim.x) {
-        float d = load_as_f32(a, at + i, a_dtype);
-        if (b) d += load_as_f32(b, at + i, b_dtype);
-        const float v = hidden[at + i] + mult * d;
+        float d = mult_a * load_as_f32(a, at + i, a_dtype);
+        if (b) d = fmaf(mult_b, load_as_f32(b, at + i, b_dtype), d);
+        const float v = hidden[at + i] + d;
         ss += v * v;
     }
     ss = block_sum(ss, red);
     const float inv = 1.0f / sqrtf(ss / (float)H + eps);
     for (int i = threadIdx.x; i < H; i += blockDim.x) {
-        float d = load_as_f32(a, at + i, a_dtype);
-        if (b) d += load_as_f32(b, at + i, b_dtype);
-        const float v = hidden[at + i] + mult * d;
+        float d = mult_a * load_as_f32(a, at + i, a_dtype);
+        if (b) d = fmaf(mult_b, load_as_f32(b, at + i, b_dtype), d);
+        const float v = hidden[at + i] + d;
         if (!rows) hidden[at + i] = v;
         out[to + i] = from_f32<TO>(v * inv * load_as_f32(weight, i, weight_dtype));
     }
 }
 
 // R = number of rows of `out` (all rows of `hidden`, or the length of `rows`)
-extern "C" int lle_scaled_add_rmsnorm(void* hidden, const void* a, int a_dtype, const void* b, int b_dtype, float mult,
-                                      const void* rows, const void* weight, int weight_dtype, void* out, int R, int H,
+extern "C" int lle_scaled_add_rmsnorm(void* hidden, const void* a, int a_dtype, const void* b, int b_dtype, float mult_a,
+                                      float mult_b, const void* rows, const void* weight, int weight_dtype, void* out, int R, int H,
                                       float eps, int out_dtype, hipStream_t stream) {
     if (R <= 0) return 0;
     if (out_dtype == LLE_F32)
-        scaled_add_rmsnorm_kernel<float><<<R, 256, 0, stream>>>((float*)hidden, a, a_dtype, b, b_dtype, mult,
+        scaled_add_rmsnorm_kernel<float><<<R, 256, 0, stream>>>((float*)hidden, a, a_dtype, b, b_dtype, mult_a, mult_b,
                                                                  (const int32_t*)rows, weight, weight_dtype, (float*)out, H, eps);
     else
-        scaled_add_rmsnorm_kernel<bf16_t><<<R, 256, 0, stream>>>((float*)hidden, a, a_dtype, b, b_dtype, mult,
+        scaled_add_rmsnorm_kernel<bf16_t><<<R, 256, 0, stream>>>((float*)hidden, a, a_dtype, b, b_dtype, mult_a, mult_b,
                                                                   (const int32_t*)rows, weight, weight_dtype, (bf16_t*)out, H,
                                                                   eps);
     LLE_RETURN_LAUNCH_STATUS();
@@ -548,7 +548,8 @@ extern "C" int lle_rmsnorm_add_rmsnorm(void* hidden, const void* y, int y_dtype,
 // 32-bit and in place, then out[n] = norm(hidden[n]) * w, one launch.  `a` (float32 or bfloat16, null: nothing is left
 // to be added) may come as `slices` partial sums, `slice_stride` elements apart, added in slice order; `b` (or null)
 // is another summand of a's kind with a type of its own; `vec` float32 [H] or null; `table` [V, H] or null: the
-// embedding's rows once more, ids as in the embedding kernel.  The new row waits in registers where rows are no wider
+// embedding's rows once more, ids as in the embedding kernel.  With `rows` only those rows are read, row rows[r] gives
+// row r of the result, and `hidden` is left alone.  The new row waits in registers where rows are no wider
 // than 256 x 4 x NORM_CHUNKS and a multiple of 4 (a plain loop otherwise).
 struct InjectArgs {
     float* hidden;
@@ -563,6 +564,7 @@ struct InjectArgs {
     int table_dtype;
     float scale;
     const int32_t *feedback, *token_seq, *seq_slots;
+    const int32_t* rows;
     const void* weight;
     int weight_dtype;
     void* out;
@@ -583,7 +585,7 @@ __device__ __forceinline__ void add_quad(float4& v, float4 d) {
 template <typename TO>
 __global__ __launch_bounds__(256) void inject_rmsnorm_kernel(InjectArgs x) {
     __shared__ float red[16];
-    const int64_t n = blockIdx.x, at = n * x.H;
+    const int64_t n = x.rows ? x.rows[blockIdx.x] : blockIdx.x, at = n * x.H, to = (int64_t)blockIdx.x * x.H;
     const int H = x.H;
     int64_t row = 0;
     if (x.table) {
@@ -612,7 +614,7 @@ __global__ __launch_bounds__(256) void inject_rmsnorm_kernel(InjectArgs x) {
                     add_quad(v, make_float4(e.x * x.scale, e.y * x.scale, e.z * x.scale, e.w * x.scale));
                 }
                 if (x.vec) add_quad(v, Quad<float>::load(x.vec + i));
-                *(float4*)(x.hidden + at + i) = v;
+                if (!x.rows) *(float4*)(x.hidden + at + i) = v;
                 keep[k] = v;
                 ss += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
             }
@@ -623,12 +625,12 @@ __global__ __launch_bounds__(256) void inject_rmsnorm_kernel(InjectArgs x) {
         for (int k = 0; k < NORM_CHUNKS; ++k) {
             const int i = (k * 256 + threadIdx.x) * 4;
             if (i < H)
-                Quad<TO>::store(out + at + i, make_float4(keep[k].x * inv * wv[k].x, keep[k].y * inv * wv[k].y,
+                Quad<TO>::store(out + to + i, make_float4(keep[k].x * inv * wv[k].x, keep[k].y * inv * wv[k].y,
                                                           keep[k].z * inv * wv[k].z, keep[k].w * inv * wv[k].w));
         }
         return;
     }
-    for (int i = threadIdx.x; i < H; i += blockDim.x) {
+    auto sum_at = [&](int i) {
         float v = x.hidden[at + i];
         if (x.a) {
             float d = load_as_f32(x.a, at + i, x.a_dtype);
@@ -638,28 +640,144 @@ __global__ __launch_bounds__(256) void inject_rmsnorm_kernel(InjectArgs x) {
         }
         if (x.table) v += load_as_f32(x.table, row + i, x.table_dtype) * x.scale;
         if (x.vec) v += x.vec[i];
-        x.hidden[at + i] = v;
+        return v;
+    };
+    for (int i = threadIdx.x; i < H; i += blockDim.x) {
+        const float v = sum_at(i);
         ss += v * v;
     }
     ss = block_sum(ss, red);
     const float inv = 1.0f / sqrtf(ss / (float)H + x.eps);
-    for (int i = threadIdx.x; i < H; i += blockDim.x)  // (each thread reads back the elements that it wrote itself)
-        out[at + i] = from_f32<TO>(x.hidden[at + i] * inv * load_as_f32(x.weight, i, x.weight_dtype));
+    for (int i = threadIdx.x; i < H; i += blockDim.x) {
+        const float v = sum_at(i);
+        if (!x.rows) x.hidden[at + i] = v;
+        out[to + i] = from_f32<TO>(v * inv * load_as_f32(x.weight, i, x.weight_dtype));
+    }
 }
 
 extern "C" int lle_inject_rmsnorm(void* hidden, const void* a, int a_dtype, int slices, int64_t slice_stride, const void* b,
                                   int b_dtype, const void* vec, const void* ids, const void* table, int table_dtype,
                                   float scale, const void* feedback, const void* token_seq, const void* seq_slots,
-                                  const void* weight, int weight_dtype, void* out, int N, int H, float eps, int out_dtype,
-                                  hipStream_t stream) {
+                                  const void* rows, const void* weight, int weight_dtype, void* out, int N, int H, float eps,
+                                  int out_dtype, hipStream_t stream) {
     if (N <= 0 || H <= 0) return 0;
     if (slices < 1 || (b && !a) || (table && !ids) || (feedback != nullptr) != (token_seq != nullptr) ||
         (feedback != nullptr) != (seq_slots != nullptr))
         return (int)hipErrorInvalidValue;
     const InjectArgs x{(float*)hidden, a, a_dtype, slices, slice_stride, b, b_dtype, (const float*)vec, (const int32_t*)ids,
                        table, table_dtype, scale, (const int32_t*)feedback, (const int32_t*)token_seq,
-                       (const int32_t*)seq_slots, weight, weight_dtype, out, H, eps};
+                       (const int32_t*)seq_slots, (const int32_t*)rows, weight, weight_dtype, out, H, eps};
     if (out_dtype == LLE_F32) inject_rmsnorm_kernel<float><<<N, 256, 0, stream>>>(x);
     else inject_rmsnorm_kernel<bf16_t><<<N, 256, 0, stream>>>(x);
+    LLE_RETURN_LAUNCH_STATUS();
+}
+
+// The first rows of the residual stream where they are made of more than the embedding table:
+//   h[n] = RMSNorm(table[id(n)] * scale (+ pos[position n])) * w0 (w0 null: without that norm)
+// and, with `weight`, the first block's norm of the new row in the same launch: out[n] = RMSNorm(h[n]) * weight.  All in
+// 32-bit; h is float32.  Ids as in the embedding kernel; the host has checked ids and positions (a position past the
+// table would read its last row).  A thread keeps its share of the row in registers (rows up to 256 x EN_PER; wider ones
+// are read back from `hidden`, each element by the thread that wrote it).
+#define EN_PER 32
+struct EmbedArgs {
+    const int32_t* ids;
+    const void* table;
+    int table_dtype;
+    float scale;
+    const int32_t *feedback, *token_seq, *seq_slots;
+    const void* pos;
+    int pos_dtype, pos_rows;
+    const int32_t* positions;
+    const void* w0;
+    int w0_dtype;
+    float eps0;
+    float* hidden;
+    const void* weight;
+    int weight_dtype;
+    float eps;
+    void* out;
+    int H;
+};
+
+template <typename TO>
+__global__ __launch_bounds__(256) void embedding_norm_kernel(EmbedArgs x) {
+    __shared__ float red[16];
+    const int64_t n = blockIdx.x;
+    const int H = x.H;
+    int id = x.ids[n];
+    if (id < 0) id = x.feedback ? x.feedback[x.seq_slots[x.token_seq[n]]] : 0;
+    const int64_t row = (int64_t)id * H;
+    const int64_t prow = x.pos ? (int64_t)min(max(x.positions[n], 0), x.pos_rows - 1) * H : 0;
+    float* h = x.hidden + n * H;
+    auto made = [&](int i) {
+        float v = load_as_f32(x.table, row + i, x.table_dtype) * x.scale;
+        if (x.pos) v += load_as_f32(x.pos, prow + i, x.pos_dtype);
+        return v;
+    };
+    const bool fits = H <= 256 * EN_PER;
+    float keep[EN_PER];
+    float ss = 0.f;
+    if (fits) {
+#pragma unroll
+        for (int k = 0; k < EN_PER; ++k) {
+            const int i = k * 256 + threadIdx.x;
+            keep[k] = i < H ? made(i) : 0.f;
+            ss += keep[k] * keep[k];
+        }
+    } else {
+        for (int i = threadIdx.x; i < H; i += blockDim.x) {
+            const float v = made(i);
+            h[i] = v;
+            ss += v * v;
+        }
+    }
+    const float inv0 = x.w0 ? 1.0f / sqrtf(block_sum(ss, red) / (float)H + x.eps0) : 1.0f;
+    ss = 0.f;
+    if (fits) {
+#pragma unroll
+        for (int k = 0; k < EN_PER; ++k) {
+            const int i = k * 256 + threadIdx.x;
+            if (i < H) {
+                if (x.w0) keep[k] *= inv0 * load_as_f32(x.w0, i, x.w0_dtype);
+                h[i] = keep[k];
+                ss += keep[k] * keep[k];
+            }
+        }
+    } else {
+        for (int i = threadIdx.x; i < H; i += blockDim.x) {
+            float v = h[i];
+            if (x.w0) v *= inv0 * load_as_f32(x.w0, i, x.w0_dtype);
+            h[i] = v;
+            ss += v * v;
+        }
+    }
+    if (!x.weight) return;  // (the same for every thread)
+    const float inv = 1.0f / sqrtf(block_sum(ss, red) / (float)H + x.eps);
+    TO* out = (TO*)x.out + n * H;
+    if (fits) {
+#pragma unroll
+        for (int k = 0; k < EN_PER; ++k) {
+            const int i = k * 256 + threadIdx.x;
+            if (i < H) out[i] = from_f32<TO>(keep[k] * inv * load_as_f32(x.weight, i, x.weight_dtype));
+        }
+    } else {
+        for (int i = threadIdx.x; i < H; i += blockDim.x) out[i] = from_f32<TO>(h[i] * inv * load_as_f32(x.weight, i, x.weight_dtype));
+    }
+}
+
+extern "C" int lle_embedding_norm(const void* ids, const void* table, int table_dtype, float scale, const void* feedback,
+                                  const void* token_seq, const void* seq_slots, const void* pos, int pos_dtype, int pos_rows,
+                                  const void* positions, const void* w0, int w0_dtype, float eps0, void* hidden,
+                                  const void* weight, int weight_dtype, float eps, void* out, int N, int H, int out_dtype,
+                                  hipStream_t stream) {
+    if (N <= 0 || H <= 0) return 0;
+    if ((feedback != nullptr) != (token_seq != nullptr) || (feedback != nullptr) != (seq_slots != nullptr) ||
+        (pos && (!positions || pos_rows <= 0)) || (weight && !out))
+        return (int)hipErrorInvalidValue;
+    const EmbedArgs x{(const int32_t*)ids, table, table_dtype, scale, (const int32_t*)feedback, (const int32_t*)token_seq,
+                      (const int32_t*)seq_slots, pos, pos_dtype, pos_rows, (const int32_t*)positions, w0, w0_dtype, eps0,
+                      (float*)hidden, weight, weight_dtype, eps, out, H};
+    if (out_dtype == LLE_F32) embedding_norm_kernel<float><<<N, 256, 0, stream>>>(x);
+    else embedding_norm_kernel<bf16_t><<<N, 256, 0, stream>>>(x);
     LLE_RETURN_LAUNCH_STATUS();
 }

@@ -10,10 +10,11 @@ from typing import Optional
 
 import torch
 
-from ..parts.base import PartialSums, Prenormed, ScaledSum
+from ..parts.base import Injected, PartialSums, Prenormed, ScaledSum
 from . import build
 from .tuning import ProductTuning
-from .limits import MAX_DELTA_HEAD_DIM, MAX_GLA_HEAD_DIM, MAX_HEAD_DIM, MAX_SUMMED_NORM_WIDTH, MAX_WKV_HEAD_DIM
+from .limits import (MAX_DELTA_HEAD_DIM, MAX_GLA_HEAD_DIM, MAX_HEAD_DIM, MAX_SSD_DIM, MAX_SUMMED_NORM_WIDTH,
+                     MAX_WKV_HEAD_DIM)
 
 F32, BF16 = 0, 1
 _P = ctypes.c_void_p
@@ -148,6 +149,42 @@ class HipOps:
                   _ptr(ids), _ptr(table), _ptr(hidden), _ptr(weight), dtype_code(weight.dtype), _ptr(out), N, H,
                   float(eps), dtype_code(table.dtype), _ptr(feedback),
                   _ptr(token_seq) if feedback is not None else None, _ptr(seq_slots) if feedback is not None else None)
+        return hidden, out
+
+    def embedding_norm(self, ids, table, scale: float, positions, pos_table, weight, eps: float, next_weight, next_eps: float,
+                       out_dtype, feedback=None, token_seq=None, seq_slots=None):
+        """The first rows of the residual stream where they are more than the embedding's: float32 [N, H]
+        h[n] = RMSNorm(table[ids[n]] * scale + pos_table[positions[n]]) * weight (`pos_table` None: no position vectors;
+        `weight` None: without that norm), and RMSNorm(h) * next_weight in `out_dtype` from the same launch (None where
+        `next_weight` is None).  The caller has checked ids and positions."""
+        _dev(ids, "ids", torch.int32)
+        _dev(table, "embedding table")
+        _need(ids.dim() == 1 and table.dim() == 2, "embedding wants ids [N] and a table [V, H]")
+        N, H = ids.shape[0], table.shape[1]
+        if pos_table is not None:
+            _dev(pos_table, "position table")
+            _dev(positions, "positions", torch.int32)
+            _need(pos_table.dim() == 2 and pos_table.shape[1] == H and pos_table.shape[0] > 0, f"the position table must be [P, {H}]")
+            _need(positions.shape == (N,), "positions must be [N]")
+        for t, name in ((weight, "norm weight"), (next_weight, "next norm weight")):
+            if t is not None:
+                _dev(t, name)
+                _need(t.shape == (H,), f"{name} must be [{H}]")
+        if feedback is not None:
+            for t, name in ((feedback, "feedback"), (token_seq, "token_seq"), (seq_slots, "seq_slots")):
+                _need(t is not None, "feedback, token_seq and seq_slots come together")
+                _dev(t, name, torch.int32)
+            _need(token_seq.shape == (N,), "token_seq must be [N]")
+        hidden = torch.empty((N, H), dtype=torch.float32, device=table.device)
+        out = torch.empty((N, H), dtype=out_dtype, device=table.device) if next_weight is not None else None
+        code = lambda t: F32 if t is None else dtype_code(t.dtype)
+        self._run("norm", "lle_embedding_norm",
+                  [_P, _P, _I, _F, _P, _P, _P, _P, _I, _I, _P, _P, _I, _F, _P, _P, _I, _F, _P, _I, _I, _I, _P],
+                  _ptr(ids), _ptr(table), dtype_code(table.dtype), float(scale), _ptr(feedback),
+                  _ptr(token_seq) if feedback is not None else None, _ptr(seq_slots) if feedback is not None else None,
+                  _ptr(pos_table), code(pos_table), pos_table.shape[0] if pos_table is not None else 0,
+                  _ptr(positions) if pos_table is not None else None, _ptr(weight), code(weight), float(eps), _ptr(hidden),
+                  _ptr(next_weight), code(next_weight), float(next_eps), _ptr(out), N, H, dtype_code(out_dtype))
         return hidden, out
 
     # -- norms ---------------------------------------------------------------
@@ -441,8 +478,9 @@ class HipOps:
 
     def paged_attention(self, q, kv_layer, block_table, seq_slots, cu_tokens, kv_lens, token_seq,
                         window: Optional[int], scale: float, min_q_len: int = 0, max_q_len: int = 0,
-                        max_kv_len: int = 0, sinks=None, keep_first: int = 0) -> torch.Tensor:
-        """q [N, nq, d] against the pages -> [N, nq * d].  `keep_first`: beside a window the first so many keys stay
+                        max_kv_len: int = 0, sinks=None, keep_first: int = 0, softcap: Optional[float] = None) -> torch.Tensor:
+        """q [N, nq, d] against the pages -> [N, nq * d].  `softcap`: the scores pass through
+        softcap * tanh(score / softcap) (None: not).  `keep_first`: beside a window the first so many keys stay
         in sight too.  `sinks` (float32 [nq], or None): every head's
         softmax has one more place, with that score and no value: p_j = exp(s_j) / (exp(sink) + sum exp(s_j)).
         `min_q_len`, `max_q_len`
@@ -471,11 +509,14 @@ class HipOps:
         win = int(window) if window else 0
         keep = int(keep_first) if win else 0
         _need(keep >= 0, "keep_first must not be negative")
+        cap = float(softcap) if softcap else 0.0
+        _need(cap >= 0.0, "a cap must be positive")
+        both = keep > 0 and cap > 0.0  # (only the generic kernel knows kept keys and capped scores together)
         mfma = (q.dtype == torch.bfloat16 and d % 32 == 0 and page_size % 16 == 0 and max_q_len > 0
-                and max_kv_len > 0 and S <= 65535 and not self.force_generic_attention)
+                and max_kv_len > 0 and S <= 65535 and not both and not self.force_generic_attention)
         group = nq // nkv
         if (q.dtype == torch.float32 and d % 16 == 0 and page_size % 16 == 0 and max_q_len > 0 and max_kv_len > 0
-                and S <= 65535 and not self.force_generic_attention):
+                and S <= 65535 and not both and not self.force_generic_attention):
             # float32 on the matrix cores (float32 operands, products and sums)
             rows = max_q_len * group
             row_blocks = 1 if rows <= 16 else -(-rows // 64)
@@ -485,17 +526,17 @@ class HipOps:
                 ws_o = torch.empty((N * nq * ns * d,), dtype=torch.float32, device=q.device)
                 ws_ml = torch.empty((N * nq * ns * 2,), dtype=torch.float32, device=q.device)
             self._run("attention", "lle_paged_attention_mfma_f32",
-                      [_P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _L, _I, _I, _I, _F, _I, _I, _P, _P],
+                      [_P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _L, _I, _I, _I, _F, _I, _I, _P, _F, _P],
                       _ptr(q), _ptr(kv_layer), _ptr(block_table), _ptr(seq_slots), _ptr(cu_tokens), _ptr(kv_lens),
                       _ptr(out), _ptr(ws_o), _ptr(ws_ml), N, S, nq, nkv, d, page_size, kv_layer.stride(0),
-                      block_table.shape[1], win, keep, float(scale), row_blocks, ns, _ptr(sinks))
+                      block_table.shape[1], win, keep, float(scale), row_blocks, ns, _ptr(sinks), cap)
             return out
         if not mfma:
             self._run("attention", "lle_paged_attention_generic",
-                      [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _L, _I, _I, _I, _F, _I, _P, _P],
+                      [_P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _L, _I, _I, _I, _F, _I, _P, _F, _P],
                       _ptr(q), _ptr(kv_layer), _ptr(block_table), _ptr(seq_slots), _ptr(cu_tokens), _ptr(kv_lens),
                       _ptr(token_seq), _ptr(out), N, nq, nkv, d, page_size, kv_layer.stride(0), block_table.shape[1],
-                      win, keep, float(scale), dtype_code(q.dtype), _ptr(sinks))
+                      win, keep, float(scale), dtype_code(q.dtype), _ptr(sinks), cap)
             return out
         min_q_len = min_q_len or 1
         run_decode = min_q_len * group <= 16
@@ -511,11 +552,11 @@ class HipOps:
             ws_ml = torch.empty((N * nq * ns * 2,), dtype=torch.float32, device=q.device)
         self._run("attention", "lle_paged_attention_mfma",
                   [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _L, _I, _I, _F, _I, _I, _I, _I, _I, _I,
-                   _P, _I, _P],
+                   _P, _I, _F, _P],
                   _ptr(q), _ptr(kv_layer), _ptr(block_table), _ptr(seq_slots), _ptr(cu_tokens), _ptr(kv_lens),
                   _ptr(token_seq), _ptr(out), _ptr(ws_o), _ptr(ws_ml), N, S, nq, nkv, d, page_size,
                   kv_layer.stride(0), block_table.shape[1], win, float(scale), int(run_decode), ns_decode,
-                  int(run_prefill), ns_prefill, max_q_len, row_tiles, _ptr(sinks), keep)
+                  int(run_prefill), ns_prefill, max_q_len, row_tiles, _ptr(sinks), keep, cap)
         return out
 
     def can_fuse_rope_attention(self, dtype, head_dim: int, rotary_dim: int, page_size: int, group: int,
@@ -1072,9 +1113,10 @@ class HipOps:
         self._run("elementwise", "lle_tanh", [_P, _L, _I, _P], _ptr(x), x.numel(), dtype_code(x.dtype))
         return x
 
-    def scaled_add_rmsnorm(self, hidden, a, b, mult: float, weight, eps: float, out_dtype, rows=None) -> torch.Tensor:
-        """hidden float32 [N, H] += mult * (a + b) in 32-bit and in place (`b` may be None; a, b [N, H],
-        float32 or bfloat16 each), then RMSNorm(hidden) * weight in `out_dtype`.  With `rows` (int32 [R]) only
+    def scaled_add_rmsnorm(self, hidden, a, b, mult: float, weight, eps: float, out_dtype, rows=None,
+                           mult_b: Optional[float] = None) -> torch.Tensor:
+        """hidden float32 [N, H] += mult * a + mult_b * b in 32-bit and in place (`b` may be None; a, b [N, H],
+        float32 or bfloat16 each; `mult_b` None: mult), then RMSNorm(hidden) * weight in `out_dtype`.  With `rows` (int32 [R]) only
         those rows are read, row rows[r] gives row r of the result, and `hidden` is left alone."""
         _dev(hidden, "hidden", torch.float32)
         _dev(weight, "norm weight")
@@ -1089,9 +1131,9 @@ class HipOps:
             _dev(rows, "rows", torch.int32)
             R = rows.shape[0]
         out = torch.empty((R, H), dtype=out_dtype, device=hidden.device)
-        self._run("norm", "lle_scaled_add_rmsnorm", [_P, _P, _I, _P, _I, _F, _P, _P, _I, _P, _I, _I, _F, _I, _P],
+        self._run("norm", "lle_scaled_add_rmsnorm", [_P, _P, _I, _P, _I, _F, _F, _P, _P, _I, _P, _I, _I, _F, _I, _P],
                   _ptr(hidden), _ptr(a), dtype_code(a.dtype), _ptr(b), dtype_code(b.dtype) if b is not None else 0,
-                  float(mult), _ptr(rows), _ptr(weight), dtype_code(weight.dtype), _ptr(out), R, H, float(eps),
+                  float(mult), float(mult if mult_b is None else mult_b), _ptr(rows), _ptr(weight), dtype_code(weight.dtype), _ptr(out), R, H, float(eps),
                   dtype_code(out_dtype))
         return out
 
@@ -1158,10 +1200,12 @@ class HipOps:
         return out
 
     # -- what enters the stream between two blocks ------------------------------------------------
-    def inject_rmsnorm(self, hidden, delta, vector, again, weight, eps: float, out_dtype) -> torch.Tensor:
+    def inject_rmsnorm(self, hidden, delta, vector, again, weight, eps: float, out_dtype, rows=None) -> torch.Tensor:
         """hidden float32 [N, H] += delta + vector + the embedding's rows, in 32-bit and in place, then
         RMSNorm(hidden) * weight in `out_dtype`.  `delta`: [N, H] in either type, PartialSums, a ScaledSum with a
-        factor of one, or None; `vector` float32 [H] or None; `again` a parts.base.EmbeddedRows or None."""
+        factor of one, or None (any other delta is added up first); `vector` float32 [H] or None; `again` a
+        parts.base.EmbeddedRows or None.  With `rows` (int32 [R]) only those rows are read, row rows[r] gives row r of
+        the result, and `hidden` is left alone."""
         _dev(hidden, "hidden", torch.float32)
         _dev(weight, "norm weight")
         N, H = hidden.shape
@@ -1174,8 +1218,10 @@ class HipOps:
             _need(a.dim() == 3 and a.shape[1:] == hidden.shape, "partial sums must be [slices, N, H]")
         elif isinstance(delta, ScaledSum):
             a, b = delta.a, delta.b
-            if delta.mult != 1.0:
+            if delta.mult != 1.0 or (delta.b is not None and delta.mult_b not in (None, 1.0)):
                 a, b = delta.total(), None
+        elif isinstance(delta, Injected):
+            a = delta.total()
         if a is not None and not isinstance(delta, PartialSums):
             for t, name in ((a, "delta"), (b, "delta's second summand")):
                 if t is not None:
@@ -1197,14 +1243,18 @@ class HipOps:
                     _need(t is not None, "feedback, token_seq and seq_slots come together")
                     _dev(t, name, torch.int32)
                 _need(token_seq.shape == (N,), "token_seq must be [N]")
-        out = torch.empty((N, H), dtype=out_dtype, device=hidden.device)
+        R = N
+        if rows is not None:
+            _dev(rows, "rows", torch.int32)
+            R = rows.shape[0]
+        out = torch.empty((R, H), dtype=out_dtype, device=hidden.device)
         code = lambda t: 0 if t is None else dtype_code(t.dtype)
         self._run("norm", "lle_inject_rmsnorm",
-                  [_P, _P, _I, _I, _L, _P, _I, _P, _P, _P, _I, _F, _P, _P, _P, _P, _I, _P, _I, _I, _F, _I, _P],
+                  [_P, _P, _I, _I, _L, _P, _I, _P, _P, _P, _I, _F, _P, _P, _P, _P, _P, _I, _P, _I, _I, _F, _I, _P],
                   _ptr(hidden), _ptr(a), code(a), slices, stride, _ptr(b), code(b), _ptr(vector), _ptr(ids), _ptr(table),
                   code(table), scale, _ptr(feedback), _ptr(token_seq) if feedback is not None else None,
-                  _ptr(seq_slots) if feedback is not None else None, _ptr(weight), dtype_code(weight.dtype), _ptr(out), N, H,
-                  float(eps), dtype_code(out_dtype))
+                  _ptr(seq_slots) if feedback is not None else None, _ptr(rows), _ptr(weight), dtype_code(weight.dtype),
+                  _ptr(out), R, H, float(eps), dtype_code(out_dtype))
         return out
 
     # -- attention gated element by element, heads' weights mixed ----------------------------------
@@ -1372,16 +1422,18 @@ class HipOps:
         return out
 
     # -- activations, caps, chained norms ---------------------------------------------------------
-    ACT_CODES = {"silu": 0, "relu": 1, "relu2": 2, "gelu_tanh": 3}
+    ACT_CODES = {"silu": 0, "relu": 1, "relu2": 2, "gelu_tanh": 3, "clamp": 4}
 
-    def bias_act(self, z, kind: str, gated: bool, bias=None, row_gate=None) -> torch.Tensor:
+    def bias_act(self, z, kind: str, gated: bool, bias=None, row_gate=None, limit: float = 0.0) -> torch.Tensor:
         """gated: z [N, 2 F] (gate columns first) -> act(gate + b) * (up + b), [N, F]; else z [N, F] -> act(z + b).
-        `kind`: silu, relu, relu2 (the square of relu), gelu_tanh (gelu in its tanh form); `bias` (or None) covers z's row; `row_gate` = (t, col), t
+        `kind`: silu, relu, relu2 (the square of relu), gelu_tanh (gelu in its tanh form), or, gated only, clamp: with
+        g = min(gate + b, limit) and u = clamp(up + b, -limit, limit) the result is g sigmoid(1.702 g) (u + 1); `bias` (or None) covers z's row; `row_gate` = (t, col), t
         float32 [N, any]: row n is multiplied by sigmoid(t[n, col]).  Everything in 32-bit."""
         _dev(z, "z")
         _need(kind in self.ACT_CODES, f"unknown activation {kind!r}")
         N, cols = z.shape
         _need(not gated or cols % 2 == 0, "a gated input has an even width")
+        _need(kind != "clamp" or (gated and limit > 0.0), "a clamped activation is gated and has a positive limit")
         F = cols // 2 if gated else cols
         if bias is not None:
             _dev(bias, "bias", z.dtype)
@@ -1393,9 +1445,9 @@ class HipOps:
             _need(gate_t.dim() == 2 and gate_t.shape[0] == N and 0 <= col < gate_t.shape[1], "row gate [N, > col]")
             stride = gate_t.shape[1]
         out = torch.empty((N, F), dtype=z.dtype, device=z.device)
-        self._run("elementwise", "lle_bias_act", [_P, _P, _P, _I, _I, _P, _I, _I, _I, _I, _I, _P], _ptr(z), _ptr(bias),
+        self._run("elementwise", "lle_bias_act", [_P, _P, _P, _I, _I, _P, _I, _I, _I, _I, _F, _I, _P], _ptr(z), _ptr(bias),
                   _ptr(gate_t), stride, int(col), _ptr(out), N, F, 1 if gated else 0, self.ACT_CODES[kind],
-                  dtype_code(z.dtype))
+                  float(limit), dtype_code(z.dtype))
         return out
 
     def softcap_(self, x, cap: float) -> torch.Tensor:
@@ -1490,16 +1542,17 @@ class HipOps:
 
     # -- the gated delta rule --------------------------------------------------------------
     DELTA_MAX_DIM = MAX_DELTA_HEAD_DIM
+    DELTA_MAX_ADVANCE = 8  # (lle_delta_conv_max_advance)
 
     def delta_conv(self, u, taps, state, token_seq, cu_tokens, seq_slots, kv_heads: int, dim: int, heads: int, vdim: int,
-                   unit_eps: float, q_scale: float):
+                   unit_eps: float, q_scale: float, advance: bool = False):
         """A row of u holds q [G dim], k [G dim], v [H vdim] of one token (G = kv_heads, H = heads).  Every channel is
         convolved over time with its J taps (float32 [cols, J]; the last tap meets the token itself), reading the
         rows of the same request ahead of it in this step and, before those, the request's state row (float32
         [slots + 1, >= (J - 1) cols], the last J - 1 rows of u that earlier steps brought, oldest first; None for
         J = 1), then passes silu; every head of q and k becomes x / sqrt(sum x^2 + unit_eps), q times q_scale.
-        Returns float32 q [N, G dim], k [N, G dim], v [N, H vdim].  The state is left as it is: conv_state_update
-        advances it."""
+        Returns float32 q [N, G dim], k [N, G dim], v [N, H vdim].  The state is left as it is (conv_state_update
+        advances it), or with `advance` moves on in the same launch (see can_advance_conv)."""
         _dev(u, "u")
         _dev(taps, "taps", torch.float32)
         for t, name in ((token_seq, "token_seq"), (cu_tokens, "cu_tokens"), (seq_slots, "seq_slots")):
@@ -1520,23 +1573,53 @@ class HipOps:
         q = torch.empty((N, G * dim), dtype=torch.float32, device=u.device)
         k = torch.empty((N, G * dim), dtype=torch.float32, device=u.device)
         v = torch.empty((N, H * vdim), dtype=torch.float32, device=u.device)
-        self._run("delta", "lle_delta_conv", [_P, _I, _P, _I, _P, _L, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _F, _I, _P],
+        _need(not advance or (1 < J <= self.DELTA_MAX_ADVANCE and N == S), "the state moves on in this launch for single tokens")
+        self._run("delta", "lle_delta_conv", [_P, _I, _P, _I, _P, _L, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _F, _I, _I, _P],
                   _ptr(u), cols, _ptr(taps), J, _ptr(state) if J > 1 else None, state.stride(0) if J > 1 else 0,
                   _ptr(token_seq), _ptr(cu_tokens), _ptr(seq_slots), _ptr(q), _ptr(k), _ptr(v), N, G, dim, H, vdim,
-                  float(unit_eps), float(q_scale), dtype_code(u.dtype))
+                  float(unit_eps), float(q_scale), int(advance), dtype_code(u.dtype))
         return q, k, v
+
+    def can_advance_conv(self, taps: int, max_q_len: int) -> bool:
+        """Whether delta_conv can move the kept rows on itself: a step of single tokens, few taps."""
+        return max_q_len == 1 and 1 < taps <= self.DELTA_MAX_ADVANCE
+
+    def low_rank_gates(self, low, a_col: int, a2, a_log, dt_bias, dim: int, g_col: int = 0, g2=None):
+        """low float32 [N, cols], a2 float32 [CA, RA], a_log float32 [CA / dim], dt_bias float32 [CA] ->
+        decay float32 [N, CA]: exp(-exp(a_log[c // dim]) softplus(low[:, a_col : a_col + RA] @ a2[c] + dt_bias[c])); and with
+        g2 [CG, RG] gate float32 [N, CG] = low[:, g_col : g_col + RG] @ g2^T (else None).  RA and RG are multiples of 16 (pad
+        weights and columns with zeros), columns start at multiples of 4."""
+        for t, name in ((low, "low"), (a2, "a2"), (a_log, "a_log"), (dt_bias, "dt_bias")):
+            _dev(t, name, torch.float32)
+        N, cols = low.shape
+        CA, RA = a2.shape
+        CG, RG = (0, 0) if g2 is None else g2.shape
+        if g2 is not None:
+            _dev(g2, "g2", torch.float32)
+        _need(CA % dim == 0 and a_log.shape == (CA // dim,) and dt_bias.shape == (CA,), "a2 [heads * dim, R], a_log [heads], dt_bias [heads * dim]")
+        _need(RA % 16 == 0 and RG % 16 == 0 and cols % 4 == 0 and a_col % 4 == 0 and g_col % 4 == 0, "ranks are multiples of 16, columns start at multiples of 4")
+        _need(0 <= a_col and a_col + RA <= cols and 0 <= g_col and g_col + RG <= cols, "low has too few columns")
+        decay = torch.empty((N, CA), dtype=torch.float32, device=low.device)
+        gate = torch.empty((N, CG), dtype=torch.float32, device=low.device) if g2 is not None else None
+        self._run("delta", "lle_low_rank_gates", [_P, _I, _I, _I, _P, _I, _I, _P, _I, _I, _P, _P, _I, _P, _P, _I, _P],
+                  _ptr(low), cols, int(a_col), int(g_col), _ptr(a2), RA, CA, _ptr(g2), RG, CG, _ptr(a_log), _ptr(dt_bias), int(dim),
+                  _ptr(decay), _ptr(gate), N)
+        return decay, gate
 
     DELTA_GATES_AHEAD = 64  # tokens of a step from which decays and betas are made by a launch of their own
 
     def delta_scan(self, q, k, v, ba, a_log, dt_bias, state, heads: int, kv_heads: int, dim: int, vdim: int, seq_slots,
-                   cu_tokens) -> torch.Tensor:
+                   cu_tokens, decay=None) -> torch.Tensor:
         """Per head h, with the matrix state S [dim, vdim] of the request (float32; `state[slot]` holds the heads'
         states transposed, [heads][vdim][dim]) and the q, k of head h // (heads // kv_heads), token by token:
             beta = sigmoid(ba[t, h]);  g = exp(-exp(a_log[h]) softplus(ba[t, heads + h] + dt_bias[h]))
             S <- g S;  w = beta (v_t - S^T k_t);  S <- S + k_t w^T;  o_t = S^T q_t
         q, k float32 [N, kv_heads dim]; v float32 [N, heads vdim]; ba float32 [N, 2 heads]; a_log, dt_bias float32
-        [heads].  Returns o float32 [N, heads vdim]; the states are advanced in place."""
-        for t, name in ((q, "q"), (k, "k"), (v, "v"), (ba, "ba"), (a_log, "a_log"), (dt_bias, "dt_bias")):
+        [heads].  With `decay` (float32 [N, heads dim], one of every key channel) S <- diag(decay_t) S instead; ba
+        [N, >= heads] then begins with beta's inputs, and a_log and dt_bias are not used (None).
+        Returns o float32 [N, heads vdim]; the states are advanced in place."""
+        for t, name in ((q, "q"), (k, "k"), (v, "v"), (ba, "ba")) + (((a_log, "a_log"), (dt_bias, "dt_bias")) if decay is None
+                                                                      else ((decay, "decay"),)):
             _dev(t, name, torch.float32)
         _rows(state, "state", torch.float32)
         _dev(seq_slots, "seq_slots", torch.int32)
@@ -1546,33 +1629,134 @@ class HipOps:
         H, G = int(heads), int(kv_heads)
         _need(G > 0 and H % G == 0, "the value heads are a multiple of the query/key heads")
         _need(0 < dim <= self.DELTA_MAX_DIM, f"a head of the delta rule holds at most {self.DELTA_MAX_DIM} key channels")
-        _need(q.shape == (N, G * dim) and k.shape == (N, G * dim) and v.shape == (N, H * vdim) and ba.shape == (N, 2 * H),
-              "q, k [N, kv_heads dim]; v [N, heads vdim]; ba [N, 2 heads]")
-        _need(a_log.shape == (H,) and dt_bias.shape == (H,), "a_log and dt_bias must be [heads]")
+        _need(q.shape == (N, G * dim) and k.shape == (N, G * dim) and v.shape == (N, H * vdim),
+              "q, k [N, kv_heads dim]; v [N, heads vdim]")
+        if decay is None:
+            _need(ba.shape == (N, 2 * H), "ba must be [N, 2 heads]")
+            _need(a_log.shape == (H,) and dt_bias.shape == (H,), "a_log and dt_bias must be [heads]")
+        else:
+            _need(ba.dim() == 2 and ba.shape[0] == N and ba.shape[1] >= H and decay.shape == (N, H * dim),
+                  "ba [N, >= heads]; decay [N, heads dim]")
         _need(state.shape[1] >= H * vdim * dim, "a state row holds heads * vdim * dim floats")
         _need(cu_tokens.shape == (S + 1,), "cu_tokens must be [S + 1]")
         out = torch.empty((N, H * vdim), dtype=torch.float32, device=v.device)
         # steps with portions: the exponentials of decay and beta leave the walk (a step of single tokens keeps them there:
         # one launch less).  The number of tokens is known on the host and fixed inside a graph.
-        gates = torch.empty((N, 2 * H), dtype=torch.float32, device=v.device) if N >= max(self.DELTA_GATES_AHEAD, 2 * S) else None
-        self._run("delta", "lle_delta_scan", [_P, _P, _P, _P, _P, _P, _P, _L, _P, _P, _P, _I, _I, _I, _I, _I, _P, _I, _P],
-                  _ptr(q), _ptr(k), _ptr(v), _ptr(ba), _ptr(a_log), _ptr(dt_bias), _ptr(state), state.stride(0),
+        gates = torch.empty((N, 2 * H), dtype=torch.float32, device=v.device) if decay is None and N >= max(self.DELTA_GATES_AHEAD, 2 * S) else None
+        self._run("delta", "lle_delta_scan", [_P, _P, _P, _P, _I, _P, _P, _P, _P, _L, _P, _P, _P, _I, _I, _I, _I, _I, _P, _I, _P],
+                  _ptr(q), _ptr(k), _ptr(v), _ptr(ba), ba.shape[1], _ptr(decay), _ptr(a_log), _ptr(dt_bias), _ptr(state), state.stride(0),
                   _ptr(seq_slots), _ptr(cu_tokens), _ptr(out), S, H, G, dim, vdim, _ptr(gates), N)
         return out
 
-    def delta_out_norm(self, o, gate, norm_w, eps: float, heads: int, vdim: int) -> torch.Tensor:
-        """o float32 [N, heads vdim], gate [N, heads vdim] in the activation type -> every head of o divided by its
-        root mean square (eps inside the root) times norm_w [vdim] times silu(gate), in the gate's type."""
+    def delta_out_norm(self, o, gate, norm_w, eps: float, heads: int, vdim: int, act: str = "silu", out_dtype=None) -> torch.Tensor:
+        """o float32 [N, heads vdim], gate [N, heads vdim] in the activation type (or float32, with `out_dtype` saying
+        the activation type) -> every head of o divided by its root mean square (eps inside the root) times norm_w [vdim]
+        times act(gate), act silu or sigmoid."""
         _dev(o, "o", torch.float32)
         _dev(gate, "gate")
         _dev(norm_w, "norm weight")
+        _need(act in ("silu", "sigmoid"), f"a gate's activation is silu or sigmoid, not {act!r}")
         N = o.shape[0]
         _need(o.shape == (N, heads * vdim) and gate.shape == o.shape and norm_w.shape == (vdim,),
               "o and gate [N, heads vdim]; norm weight [vdim]")
-        out = torch.empty_like(gate)
-        self._run("delta", "lle_delta_out_norm", [_P, _P, _P, _I, _F, _P, _I, _I, _I, _I, _P], _ptr(o), _ptr(gate),
-                  _ptr(norm_w), dtype_code(norm_w.dtype), float(eps), _ptr(out), N, int(heads), int(vdim),
-                  dtype_code(gate.dtype))
+        out = torch.empty(o.shape, dtype=out_dtype or gate.dtype, device=o.device)
+        _need(gate.dtype in (torch.float32, out.dtype), "the gate is float32 or of the result's type")
+        self._run("delta", "lle_delta_out_norm", [_P, _P, _I, _I, _P, _I, _F, _P, _I, _I, _I, _I, _P], _ptr(o), _ptr(gate),
+                  dtype_code(gate.dtype), 1 if act == "sigmoid" else 0, _ptr(norm_w), dtype_code(norm_w.dtype), float(eps),
+                  _ptr(out), N, int(heads), int(vdim), dtype_code(out.dtype))
+        return out
+
+    # -- the state-space recurrence of Mamba-2 ----------------------------------------------------
+    SSD_MAX_DIM = MAX_SSD_DIM
+    SSD_CHUNK = 64  # tokens of a chunk (lle_ssd_chunk)
+    SSD_WALK = 32  # most tokens of a request that are walked one by one (lle_ssd_walk)
+
+    def ssd_conv(self, u, col0: int, taps, bias, state, token_seq, cu_tokens, seq_slots, single: bool = False) -> torch.Tensor:
+        """The columns col0 .. col0 + C - 1 of u [N, cols] convolved over time channel by channel with J taps (float32
+        [C, J]; the last tap meets the token itself) + bias (float32 [C] or None), then silu -> float32 [N, C].  Tokens
+        ahead of the step come from the request's state row (float32 [slots + 1, >= (J - 1) C]: the last J - 1 inputs of
+        earlier steps, oldest first; None for J = 1), which moves on by the step's tokens.  `single`: every request of the
+        step has one token (the row then moves on in the same launch)."""
+        _dev(u, "u")
+        _dev(taps, "taps", torch.float32)
+        for t, name in ((token_seq, "token_seq"), (cu_tokens, "cu_tokens"), (seq_slots, "seq_slots")):
+            _dev(t, name, torch.int32)
+        N, cols = u.shape
+        C, J = taps.shape
+        S = seq_slots.shape[0]
+        _need(0 <= col0 and col0 + C <= cols and J >= 1, "u has too few columns")
+        _need(token_seq.shape == (N,) and cu_tokens.shape == (S + 1,), "token_seq [N]; cu_tokens [S + 1]")
+        if bias is not None:
+            _dev(bias, "bias", torch.float32)
+            _need(bias.shape == (C,), "the convolution's bias must be [C]")
+        if J > 1:
+            _need(state is not None, "a convolution of several taps needs the requests' state rows")
+            _rows(state, "state", torch.float32)
+            _need(state.shape[1] >= (J - 1) * C, "a state row holds J - 1 inputs")
+        out = torch.empty((N, C), dtype=torch.float32, device=u.device)
+        self._run("ssd", "lle_ssd_conv", [_P, _I, _I, _P, _I, _P, _P, _L, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P],
+                  _ptr(u), cols, int(col0), _ptr(taps), J, _ptr(bias), _ptr(state) if J > 1 else None,
+                  state.stride(0) if J > 1 else 0, _ptr(token_seq), _ptr(cu_tokens), _ptr(seq_slots), _ptr(out), N, S, C,
+                  1 if single else 0, dtype_code(u.dtype))
+        return out
+
+    def ssd_heads_a_group(self, heads: int, groups: int, chunks: int) -> int:
+        """Heads of a group that one workgroup of the chunks' second pass takes (they share C . B): as many as leave
+        two workgroups for every CU."""
+        most, share = max(1, heads * chunks // (2 * self.compute_units())), heads // groups
+        return max(k for k in range(1, share + 1) if share % k == 0 and (k <= most or k == 1))
+
+    def ssd_scan(self, c, dt_in, dt_bias, a_log, D, state, heads: int, groups: int, vdim: int, n: int, seq_slots, cu_tokens,
+                 min_q_len: int = 0, max_q_len: int = 0) -> torch.Tensor:
+        """Per head h, with the matrix state S [n, vdim] of the request (float32; `state[slot]` begins with the heads'
+        states transposed, [heads][vdim][n]) and the B, C of group h // (heads // groups), token by token:
+            dt = softplus(dt_in[t, h] + dt_bias[h]);  S <- exp(-exp(a_log[h]) dt) S + dt B_t x_t^T;  y_t = S^T C_t + D[h] x_t
+        A row of c (float32) holds x [heads vdim], B [groups n], C [groups n]; dt_in float32 [N, >= heads].  Returns y float32
+        [N, heads vdim]; the states are advanced in place.  `min_q_len` and `max_q_len` are host-side bounds of the
+        requests' tokens in this step (0: not known); they choose kernels, never results."""
+        for t, name in ((c, "c"), (dt_in, "dt_in"), (dt_bias, "dt_bias"), (a_log, "a_log"), (D, "D")):
+            _dev(t, name, torch.float32)
+        _rows(state, "state", torch.float32)
+        _dev(seq_slots, "seq_slots", torch.int32)
+        _dev(cu_tokens, "cu_tokens", torch.int32)
+        N, CC = c.shape
+        S = seq_slots.shape[0]
+        H, G = int(heads), int(groups)
+        _need(G > 0 and H % G == 0, "the heads are a multiple of the groups")
+        _need(0 < vdim <= self.SSD_MAX_DIM and 0 < n <= self.SSD_MAX_DIM, f"a head of the recurrence holds at most {self.SSD_MAX_DIM} channels")
+        _need(CC == H * vdim + 2 * G * n, "a row of c holds x, B and C")
+        _need(dt_in.dim() == 2 and dt_in.shape[0] == N and dt_in.shape[1] >= H, "dt_in must be [N, >= heads]")
+        _need(dt_bias.shape == (H,) and a_log.shape == (H,) and D.shape == (H,), "dt_bias, a_log and D must be [heads]")
+        _need(state.shape[1] >= H * vdim * n and cu_tokens.shape == (S + 1,), "a state row holds heads * vdim * n floats")
+        longest = min(max_q_len or N, N)
+        pieces = -(-longest // self.SSD_CHUNK) if longest > self.SSD_WALK else 0
+        y = torch.empty((N, H * vdim), dtype=torch.float32, device=c.device)
+        part = part_decay = None
+        together = 1
+        if pieces:
+            slots = N // self.SSD_CHUNK + S
+            part = torch.empty((slots * H * vdim * n,), dtype=torch.float32, device=c.device)
+            part_decay = torch.empty((slots * H,), dtype=torch.float32, device=c.device)
+            together = self.ssd_heads_a_group(H, G, -(-N // self.SSD_CHUNK))
+        self._run("ssd", "lle_ssd_scan",
+                  [_P, _I, _P, _I, _P, _P, _P, _P, _L, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P, _P, _P],
+                  _ptr(c), CC, _ptr(dt_in), dt_in.shape[1], _ptr(dt_bias), _ptr(a_log), _ptr(D), _ptr(state), state.stride(0),
+                  _ptr(seq_slots), _ptr(cu_tokens), _ptr(y), S, H, G, int(vdim), int(n),
+                  1 if (min_q_len or 1) <= self.SSD_WALK else 0, pieces, together, _ptr(part), _ptr(part_decay))
+        return y
+
+    def ssd_gate_norm(self, y, u, z_col: int, norm_w, eps: float, groups: int) -> torch.Tensor:
+        """y float32 [N, inner], z = u[:, z_col : z_col + inner] -> y * silu(z), every one of `groups` equal parts of a row
+        divided by its own root mean square (eps inside the root), times norm_w (float32 [inner]), in u's type."""
+        _dev(y, "y", torch.float32)
+        _dev(u, "u")
+        _dev(norm_w, "norm weight", torch.float32)
+        N, inner = y.shape
+        _need(u.shape[0] == N and 0 <= z_col and z_col + inner <= u.shape[1], "u has too few columns")
+        _need(norm_w.shape == (inner,) and groups > 0 and inner % groups == 0, "the norm weight must be [inner], cut into equal parts")
+        out = torch.empty((N, inner), dtype=u.dtype, device=u.device)
+        self._run("ssd", "lle_ssd_gate_norm", [_P, _P, _I, _I, _P, _F, _P, _I, _I, _I, _I, _P], _ptr(y), _ptr(u), u.shape[1],
+                  int(z_col), _ptr(norm_w), float(eps), _ptr(out), N, inner, int(groups), dtype_code(u.dtype))
         return out
 
     # -- picking tokens --------------------------------------------------------------

@@ -37,7 +37,8 @@ class LLMEngine:
         self.runner = ModelRunner(model, self.cache, pick_tokens=self.run_ahead)
         self._ahead = None  # (plan, PendingTokens) of a step that is on its way
         self.num_steps_ahead = 0  # steps that were launched before the step before them had been read
-        self.scheduler = Scheduler(self.cache, max_tokens_per_step, prefill_chunk)
+        self.scheduler = Scheduler(self.cache, max_tokens_per_step, prefill_chunk,
+                                   max_positions=getattr(model, "max_positions", None))
         self.sampler = Sampler(ctx.ops, ctx.device)
         self.verbose = verbose
         self.num_steps = 0

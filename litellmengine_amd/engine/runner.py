@@ -67,6 +67,7 @@ class ModelRunner:
         self.cache = cache
         self.device = cache.device
         self.vocab_size = model.vocab_size
+        self.max_positions = getattr(model, "max_positions", None)  # most tokens of a request (None: no bound of the model's own)
         self.last_step: Optional[StepState] = None
         self.pick_tokens = bool(pick_tokens)
         # by request slot (and the spare one of padding rows): the token picked for it last
@@ -182,6 +183,8 @@ class ModelRunner:
         cache = self.cache
         before = [(e.slot, cache.length(e.slot)) for e in entries]
         wants = [(slot, length + len(e.tokens)) for (slot, length), e in zip(before, entries)]
+        if self.max_positions is not None and any(n > self.max_positions for _, n in wants):
+            raise ValueError(f"a request would hold more tokens than the model has positions ({self.max_positions})")
         self.check_tokens(entries, allow_deferred=ahead)
         cache.extend_many(wants)
         picks = None

@@ -51,12 +51,15 @@ class Portion(NamedTuple):
 
 
 class Scheduler:
-    def __init__(self, cache: CacheManager, max_tokens_per_step: int = 2048, prefill_chunk: Optional[int] = None):
+    def __init__(self, cache: CacheManager, max_tokens_per_step: int = 2048, prefill_chunk: Optional[int] = None,
+                 max_positions: Optional[int] = None):
+        """`max_positions`: most tokens of a request that the model can place (None: any number)."""
         if max_tokens_per_step <= 0:
             raise ValueError("max_tokens_per_step must be positive")
         if prefill_chunk is not None and prefill_chunk <= 0:
             raise ValueError("prefill_chunk must be positive")
         self.cache = cache
+        self.max_positions = max_positions
         self.max_tokens_per_step = max_tokens_per_step
         self.prefill_chunk = prefill_chunk or max_tokens_per_step
         self.waiting: Deque[Request] = collections.deque()
@@ -94,6 +97,9 @@ class Scheduler:
 
     def _check_fits(self, prompt_len: int, max_new_tokens: int) -> None:
         longest = prompt_len + max_new_tokens - 1  # the last token drawn is never cached
+        if self.max_positions is not None and longest > self.max_positions:
+            raise ValueError(f"request of {prompt_len} prompt + {max_new_tokens} new tokens is longer than the model's "
+                             f"{self.max_positions} positions")
         for group in self.cache.groups:
             pages = group.pages_for(longest)
             if not group.forgets and pages > group.pool.num_pages:

@@ -4,6 +4,7 @@ from . import kezasun  # noqa: F401  (registers Kezasun)
 from . import malilorn  # noqa: F401  (registers Malilorn)
 from . import birelix  # noqa: F401  (registers Birelix)
 from . import telulorn  # noqa: F401  (registers Telulorn)
+from . import rorevik  # noqa: F401  (registers Rorevik)
 from .build import expected_tensors, load_model, make_context, parse_dtype, random_model
 from .decoder import DecoderLM, Inject, PlanEntry, looped_plan
 

@@ -45,14 +45,15 @@ class PlanEntry:
     inject: Optional[Inject] = None
 
 
-def looped_plan(blocks: int, start: int, stop: int, times: int) -> List[PlanEntry]:
+def looped_plan(blocks: int, start: int, stop: int, times: int, inject: bool = True) -> List[PlanEntry]:
     """Blocks start .. stop - 1 run `times` times in a row (each time with caches and states of their own), the
-    others once.  Ahead of pass t the stream gets pass vector t, and from the second pass on also the embedding's rows."""
+    others once.  Ahead of pass t the stream gets pass vector t, and from the second pass on also the embedding's rows
+    (`inject=False`: nothing enters the stream between passes)."""
     if not 0 <= start < stop <= blocks or times < 1:
         raise ValueError(f"a loop over blocks {start} .. {stop - 1}, {times} times, does not fit {blocks} blocks")
     plan = [PlanEntry(i) for i in range(start)]
     for t in range(times):
-        plan += [PlanEntry(i, inject=Inject(t, t > 0) if i == start else None) for i in range(start, stop)]
+        plan += [PlanEntry(i, inject=Inject(t, t > 0) if inject and i == start else None) for i in range(start, stop)]
     return plan + [PlanEntry(i) for i in range(stop, blocks)]
 
 
@@ -99,6 +100,11 @@ class DecoderLM:
     @property
     def vocab_size(self) -> int:
         return self.embedding.vocab_size
+
+    @property
+    def max_positions(self) -> Optional[int]:
+        """Most tokens of one request, where the model has a bound of its own (a table of position vectors)."""
+        return getattr(self.embedding, "max_positions", None)
 
     def tensor_specs(self) -> Dict[str, TensorSpec]:
         specs: Dict[str, TensorSpec] = dict(self.embedding.tensor_specs())

@@ -15,6 +15,7 @@ from .norm import RMSNorm
 from .position import NoPositionEncoding, RotaryHalfSplit, RotaryInterleaved
 from .recurrent import MinGRU
 from .side_by_side import SideBySideMixer
+from .ssd import StateSpaceMixer
 from .wkv import WKVMixer
 
 __all__ = [
@@ -24,4 +25,5 @@ __all__ = [
     "RotaryHalfSplit", "StateSpec", "GroupLimitedMLP", "ParallelBlock", "ScaledSum", "SinkAttention", "WKVMixer",
     "ConvAttention", "SandwichBlock", "PlainMLP", "ScoreRoutedMLP", "SideBySideMixer", "GatedDeltaMixer",
     "EmbeddedRows", "GatedAttention", "GatedLinearAttention", "Injected", "PassVectors", "geometric_slopes",
+    "StateSpaceMixer",
 ]

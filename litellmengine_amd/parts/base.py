@@ -185,16 +185,21 @@ class PartialSums:
 @dataclasses.dataclass
 class ScaledSum:
     """What a block whose sublayers run side by side leaves to be added to the residual stream:
-    `mult * (a + b)` (`b` may be None; a, b [N, width], each in the activation type or in 32-bit).
+    `mult * a + mult_b * b` (`b` may be None; a, b [N, width], each in the activation type or in 32-bit;
+    `mult_b` None: mult).
     Norm.forward takes it where it takes a delta; `total()` is the plain way to take it."""
 
     a: torch.Tensor
     b: Optional[torch.Tensor]
     mult: float
+    mult_b: Optional[float] = None
 
     def total(self) -> torch.Tensor:
-        t = self.a.float() if self.b is None else self.a.float() + self.b.float()
-        return t * self.mult
+        if self.b is None:
+            return self.a.float() * self.mult
+        if self.mult_b is None or self.mult_b == self.mult:
+            return (self.a.float() + self.b.float()) * self.mult
+        return self.a.float() * self.mult + self.b.float() * self.mult_b
 
 
 @dataclasses.dataclass
@@ -217,9 +222,10 @@ class EmbeddedRows:
 
 @dataclasses.dataclass
 class Injected:
-    """What is left to be added to the residual stream where something enters it between two blocks:
-    `delta` (what the block before has left: a tensor, PartialSums, a ScaledSum or nothing), a `vector`
-    [width] in 32-bit that every row gets (or None), and the embedding's rows once more (`again`, or None).
+    """What is left to be added to the residual stream where something enters it between two blocks, or beside a
+    block's result (the bias of its last projection):
+    `delta` (what the block before has left: a tensor, PartialSums, a ScaledSum, another Injected or nothing), a
+    `vector` [width] in 32-bit that every row gets (or None), and the embedding's rows once more (`again`, or None).
     Norm.forward takes it where it takes a delta; `total()` is the plain way to take it."""
 
     delta: Any

@@ -1,4 +1,4 @@
-"""Grouped-query attention whose result is gated element by element, with what a design may want of the
+"""Grouped-query attention whose result may be gated element by element, with what a design may want of the
 rest given as parameters:
 
     q, k, v = W_q h (+ b_q), W_k h (+ b_k), W_v h (+ b_v)
@@ -6,14 +6,16 @@ rest given as parameters:
     v     <- rotated by its own position over all of its elements, and every head's result turned back by
              the query's position (`value_rotation`): the result depends on distances in the values too
     s_ij   = (q_i . k_j) * scale - slope_h (i - j)                               (`slopes`: a number per head)
+    s_ij  <- cap tanh(s_ij / cap)                                                (`softcap`)
     keys   : `window`: i sees j <= i with i - j < window, or j < keep_first;  `chunk`: i sees j <= i of its
              own chunk of so many positions, counted from the request's first;  neither: every j <= i
     p_ij   = exp(s_ij) / (exp(sink_h) + sum_j exp(s_ij))                         (`sinks`: a learned number per head)
     p_h   <- sum_g T[h, g] p_g                                                   (`talk`: the heads' weights mixed, T [H, H])
-    y      = W_o (out_scale * sigmoid(W_g h) * [heads' sum_j p_ij v_j])
+    y      = W_o (out_scale * sigmoid(W_g h) * [heads' sum_j p_ij v_j])         (`gated=False`: W_o [heads' sum_j p_ij v_j])
 
 Keys may be `dim` wide and values `vdim`: the cache's heads hold `cache_dim` >= both elements (a multiple of
-32, which the matrix-core kernels take), the rest zeros; the gates' kernel drops the padding.  The
+32, which the matrix-core kernels take), the rest zeros; the gates' kernel drops the padding (without gates the
+output projection has zero columns there).  The
 projections are one stacked product; rotations, scores, softmax, sinks, mixing and gates are 32-bit.
 """
 from __future__ import annotations
@@ -42,8 +44,13 @@ class GatedAttention(Mixer):
                  window: Optional[int] = None, keep_first: int = 0, chunk: Optional[int] = None, qkv_bias: bool = False,
                  sinks: bool = False, slopes: Optional[Sequence[float]] = None, talk: bool = False, out_scale: float = 1.0,
                  names: Sequence[str] = ("q", "k", "v", "g", "o"), bias_suffix: str = ".b", sink_name: str = "sink",
-                 talk_name: str = "talk"):
-        """`names`: the checkpoint's names after `prefix` of the query, key, value, gate and output projections."""
+                 talk_name: str = "talk", gated: bool = True, softcap: Optional[float] = None):
+        """`names`: the checkpoint's names after `prefix` of the query, key, value, gate (not with `gated=False`) and
+        output projections."""
+        if not gated and (value_rotation is not None or out_scale != 1.0):
+            raise ValueError("turned-back values and a factor on the result are the gates' kernel's work")
+        if softcap is not None and not softcap > 0:
+            raise ValueError("a cap on the scores must be positive")
         if num_q_heads <= 0 or num_kv_heads <= 0 or num_q_heads % num_kv_heads:
             raise ValueError("num_q_heads must be a multiple of num_kv_heads")
         self.cache_dim = -(-max(dim, vdim) // 32) * 32
@@ -58,8 +65,8 @@ class GatedAttention(Mixer):
             raise ValueError("first tokens are kept beside a window only")
         # chunks and distance biases are known to the kernels that mix the heads' weights (without a mix: by the identity)
         self.talking = bool(talk or slopes is not None or chunk is not None)
-        if self.talking and (sinks or window is not None):
-            raise ValueError("the kernels that mix the heads' weights know chunks and distance biases, no windows and no sinks")
+        if self.talking and (sinks or window is not None or softcap is not None):
+            raise ValueError("the kernels that mix the heads' weights know chunks and distance biases, no windows, sinks or caps")
         if self.talking:
             check_talking_sizes(num_q_heads, self.cache_dim)
         self.prefix, self.hidden = prefix, hidden_size
@@ -67,11 +74,12 @@ class GatedAttention(Mixer):
         self.scale, self.out_scale = float(scale), float(out_scale)
         self.rotation, self.value_rotation = rotation, value_rotation
         self.window, self.keep_first, self.chunk = window, int(keep_first), chunk
-        q, k, v, g, o = (prefix + n for n in names)
+        self.gated, self.softcap = bool(gated), None if softcap is None else float(softcap)
+        q, k, v, g, o = (prefix + n for n in (names if gated or len(names) == 5 else (*names[:3], "", names[3])))
         widths = [num_q_heads * dim, num_kv_heads * dim, num_kv_heads * vdim]
         self.gate_col = sum(widths)
         # one product for q, k, v and the gates' inputs (the gates have no bias)
-        self.qkvg = Linear([q, k, v, g], hidden_size, widths + [num_q_heads * vdim])
+        self.qkvg = Linear([q, k, v] + ([g] if gated else []), hidden_size, widths + ([num_q_heads * vdim] if gated else []))
         self.o = Linear([o], num_q_heads * vdim, [hidden_size])
         self.bias_names = [n + bias_suffix for n in (q, k, v)] if qkv_bias else []
         self.bias_widths = widths
@@ -96,7 +104,12 @@ class GatedAttention(Mixer):
     def bind(self, weights, ctx: BuildContext) -> None:
         self.ctx = ctx
         self.qkvg.bind(weights, ctx)
-        self.o.bind(weights, ctx)
+        if self.gated or self.cache_dim == self.vdim:
+            self.o.bind(weights, ctx)
+        else:  # without gates nothing drops the cache's padding: the output projection gets zero columns there
+            o = weights[self.o.names[0]].to(ctx.dtype).view(self.hidden, self.nq, self.vdim)
+            o = torch.nn.functional.pad(o, (0, self.cache_dim - self.vdim))
+            self.o.bind_tensor(o.reshape(self.hidden, self.nq * self.cache_dim).contiguous(), ctx)
         for p in (self.rotation, self.value_rotation):
             if p is not None:
                 p.bind(weights, ctx)
@@ -125,5 +138,7 @@ class GatedAttention(Mixer):
                                       step.max_q_len, step.max_kv_len)
         else:
             a = ops.paged_attention(q, *where, self.window, self.scale, step.min_q_len, step.max_q_len, step.max_kv_len,
-                                    sinks=self.sinks, keep_first=self.keep_first)
+                                    sinks=self.sinks, keep_first=self.keep_first, softcap=self.softcap)
+        if not self.gated:  # heads of cache_dim elements, zeros past vdim, against zero columns of the weight
+            return self.o.forward(a)
         return self.o.forward(ops.turn_back_gate(a, u, self.gate_col, self.nq, self.vdim, value_turn, self.out_scale))

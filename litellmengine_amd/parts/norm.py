@@ -43,12 +43,12 @@ class RMSNorm(Norm):
         return then.forward(hidden, None)
 
     def forward(self, hidden, delta, rows=None) -> torch.Tensor:
-        if isinstance(delta, Injected) and rows is None:  # everything that enters the stream, and the norm, in one launch
+        if isinstance(delta, Injected):  # everything that enters the stream, and the norm, in one launch
             return self.ctx.ops.inject_rmsnorm(hidden, delta.delta, delta.vector, delta.again, self.weight, self.eps,
-                                               self.ctx.dtype)
+                                               self.ctx.dtype, rows)
         if isinstance(delta, ScaledSum):  # the add, times its constant, and the norm in one launch
             return self.ctx.ops.scaled_add_rmsnorm(hidden, delta.a, delta.b, delta.mult, self.weight, self.eps,
-                                                   self.ctx.dtype, rows)
+                                                   self.ctx.dtype, rows, mult_b=delta.mult_b)
         return self.ctx.ops.add_rmsnorm(hidden, delta, self.weight, self.eps, self.ctx.dtype, rows)
 
     def of_embedding(self, ids, table, step=None):

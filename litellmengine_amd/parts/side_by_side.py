@@ -2,9 +2,11 @@
 
     y = left(h) + right(h)
 
-Each of the two brings its own constant factor (a mixer's `out_scale`), so the sum needs no
-arithmetic of its own: the result is handed on as the pair (left, right), and the norm's kernel that
-takes the mixer's result adds the two in 32-bit (`Norm.add_normed(hidden, y, extra)`).  At most one
+Each of the two may bring its own constant factor (a mixer's `out_scale`): the sum then needs no
+arithmetic of its own, the result is handed on as the pair (left, right), and the norm's kernel that
+takes the mixer's result adds the two in 32-bit (`Norm.add_normed(hidden, y, extra)`).  Or the factors are
+given here (`left_scale`, `right_scale`): the result is then a ScaledSum, and the factors are applied in 32-bit
+by the norm's kernel that adds it into the stream (pre-norm arrangements).  At most one
 of the two may keep a per-token cache; the fixed-size states of both lie one behind the other in
 one state row of the request, and each mixer sees its own columns of it.
 """
@@ -16,12 +18,15 @@ from typing import Dict, Optional
 import torch
 
 from ..weights.spec import TensorSpec
-from .base import BuildContext, CacheSpec, Mixer, StateSpec
+from .base import BuildContext, CacheSpec, Mixer, ScaledSum, StateSpec
 
 
 class SideBySideMixer(Mixer):
-    def __init__(self, left: Mixer, right: Mixer):
+    def __init__(self, left: Mixer, right: Mixer, left_scale: Optional[float] = None, right_scale: Optional[float] = None):
+        if (left_scale is None) != (right_scale is None):
+            raise ValueError("both mixers' factors are given, or neither")
         self.left, self.right = left, right
+        self.scales = None if left_scale is None else (float(left_scale), float(right_scale))
         self.graph_safe = bool(getattr(left, "graph_safe", False) and getattr(right, "graph_safe", False))
         if left.cache_spec() is not None and right.cache_spec() is not None:
             raise ValueError("of two mixers side by side at most one keeps a per-token cache")
@@ -58,5 +63,6 @@ class SideBySideMixer(Mixer):
         return dataclasses.replace(cache, state=state)
 
     def forward(self, x, step, cache):
-        """-> (left's result, right's result): a pair that a norm's kernel adds up."""
-        return self.left.forward(x, step, self._share(cache, 0)), self.right.forward(x, step, self._share(cache, 1))
+        """-> (left's result, right's result): a pair that a norm's kernel adds up; with factors a ScaledSum."""
+        y = self.left.forward(x, step, self._share(cache, 0)), self.right.forward(x, step, self._share(cache, 1))
+        return y if self.scales is None else ScaledSum(*y, *self.scales)

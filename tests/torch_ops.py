@@ -35,6 +35,20 @@ class TorchOps:
         x = x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * weight.to(self.cd)
         return hidden, x.to(table.dtype)
 
+    def embedding_norm(self, ids, table, scale, positions, pos_table, weight, eps, next_weight, next_eps, out_dtype,
+                       feedback=None, token_seq=None, seq_slots=None):
+        ids = ids.long()
+        if feedback is not None:
+            ids = torch.where(ids < 0, feedback.long()[seq_slots.long()[token_seq.long()]], ids)
+        x = table[ids].to(self.cd) * scale
+        if pos_table is not None:
+            x = x + pos_table[positions.long()].to(self.cd)
+        normed = lambda t, w, e: t / torch.sqrt((t * t).mean(-1, keepdim=True) + e) * w.to(self.cd)
+        if weight is not None:
+            x = normed(x, weight, eps)
+        x = x.to(torch.float32)
+        return x, None if next_weight is None else normed(x.to(self.cd), next_weight, next_eps).to(out_dtype)
+
     # the fused and sliced forms are the HIP kernels' own: this stand-in offers none of them
     def can_fold_norm(self, rows, width, dtype):
         return False
@@ -115,7 +129,7 @@ class TorchOps:
         return q.to(qkv.dtype).contiguous()
 
     def paged_attention(self, q, kv_layer, block_table, seq_slots, cu_tokens, kv_lens, token_seq, window, scale,
-                        min_q_len=0, max_q_len=0, max_kv_len=0, sinks=None, keep_first=0):
+                        min_q_len=0, max_q_len=0, max_kv_len=0, sinks=None, keep_first=0, softcap=None):
         N, nq, d = q.shape
         nkv, P = kv_layer.shape[2], kv_layer.shape[3]
         group = nq // nkv
@@ -137,6 +151,8 @@ class TorchOps:
                 keys = keys.repeat_interleave(group, dim=1)
                 vals = vals.repeat_interleave(group, dim=1)
                 sc = torch.einsum("hd,nhd->hn", q[t].to(self.cd), keys) * scale
+                if softcap:
+                    sc = softcap * torch.tanh(sc / softcap)
                 if sinks is None:
                     p = torch.softmax(sc, dim=-1)
                 else:  # one more place in every head's sum, with a score of its own and no value
@@ -330,10 +346,14 @@ class TorchOps:
                 out[n] += y if gain_on_input else g * y
         return out.to(torch.float32)
 
-    def bias_act(self, z, kind, gated, bias=None, row_gate=None):
+    def bias_act(self, z, kind, gated, bias=None, row_gate=None, limit=0.0):
         zz = z.to(self.cd)
         if bias is not None:
             zz = zz + bias.to(self.cd)
+        if kind == "clamp":
+            F = zz.shape[1] // 2
+            g, u = torch.clamp(zz[:, :F], max=limit), torch.clamp(zz[:, F:], min=-limit, max=limit)
+            return (g * torch.sigmoid(1.702 * g) * (u + 1.0)).to(z.dtype)
         act = {"silu": lambda t: t * torch.sigmoid(t), "relu": lambda t: torch.clamp(t, min=0.0),
                "relu2": lambda t: torch.clamp(t, min=0.0) ** 2,
                "gelu_tanh": lambda t: 0.5 * t * (1.0 + torch.tanh(math.sqrt(2.0 / math.pi) * (t + 0.044715 * t ** 3)))}[kind]
@@ -459,7 +479,9 @@ class TorchOps:
         return q.to(qkv.dtype).contiguous()
 
     # -- the gated delta rule ------------------------------------------------------------------
-    def delta_conv(self, u, taps, state, token_seq, cu_tokens, seq_slots, kv_heads, dim, heads, vdim, unit_eps, q_scale):
+    def delta_conv(self, u, taps, state, token_seq, cu_tokens, seq_slots, kv_heads, dim, heads, vdim, unit_eps, q_scale,
+                   advance=False):
+        assert not advance, "this stand-in moves no state on (can_advance_conv says so)"
         N, cols = u.shape
         J = taps.shape[1]
         G, H = kv_heads, heads
@@ -484,13 +506,27 @@ class TorchOps:
         k = unit(y[:, G * dim : 2 * G * dim])
         return q.to(torch.float32), k.to(torch.float32), y[:, 2 * G * dim :].to(torch.float32).contiguous()
 
-    def delta_scan(self, q, k, v, ba, a_log, dt_bias, state, heads, kv_heads, dim, vdim, seq_slots, cu_tokens):
+    def can_advance_conv(self, taps, max_q_len):
+        return False
+
+    def low_rank_gates(self, low, a_col, a2, a_log, dt_bias, dim, g_col=0, g2=None):
+        x = low.to(self.cd)
+        z = x[:, a_col : a_col + a2.shape[1]] @ a2.to(self.cd).t() + dt_bias.to(self.cd)
+        rate = torch.exp(a_log.to(self.cd)).repeat_interleave(dim)
+        decay = torch.exp(-rate * torch.nn.functional.softplus(z)).to(torch.float32)
+        return decay, None if g2 is None else (x[:, g_col : g_col + g2.shape[1]] @ g2.to(self.cd).t()).to(torch.float32)
+
+    def delta_scan(self, q, k, v, ba, a_log, dt_bias, state, heads, kv_heads, dim, vdim, seq_slots, cu_tokens, decay=None):
         N = v.shape[0]
         H, G = heads, kv_heads
         out = torch.zeros((N, H, vdim), dtype=self.cd, device=v.device)
         qq, kk, vv = q.to(self.cd).view(N, G, dim), k.to(self.cd).view(N, G, dim), v.to(self.cd).view(N, H, vdim)
         beta = torch.sigmoid(ba[:, :H].to(self.cd))
-        g = torch.exp(-torch.exp(a_log.to(self.cd)) * torch.nn.functional.softplus(ba[:, H:].to(self.cd) + dt_bias.to(self.cd)))
+        if decay is None:
+            g = torch.exp(-torch.exp(a_log.to(self.cd)) * torch.nn.functional.softplus(ba[:, H:].to(self.cd) + dt_bias.to(self.cd)))
+            g = g[:, :, None].expand(N, H, dim)
+        else:
+            g = decay.to(self.cd).view(N, H, dim)
         for s in range(seq_slots.shape[0]):
             q0, q1 = int(cu_tokens[s]), int(cu_tokens[s + 1])
             if q1 <= q0:
@@ -500,19 +536,65 @@ class TorchOps:
             for t in range(q0, q1):
                 for h in range(H):
                     j = h // (H // G)
-                    S[h] = g[t, h] * S[h]
+                    S[h] = g[t, h][None, :] * S[h]
                     w = beta[t, h] * (vv[t, h] - S[h] @ kk[t, j])
                     S[h] = S[h] + torch.outer(w, kk[t, j])
                     out[t, h] = S[h] @ qq[t, j]
             state[slot, : H * vdim * dim] = S.reshape(-1).to(state.dtype)
         return out.reshape(N, H * vdim).to(torch.float32)
 
-    def delta_out_norm(self, o, gate, norm_w, eps, heads, vdim):
+    def delta_out_norm(self, o, gate, norm_w, eps, heads, vdim, act="silu", out_dtype=None):
         N = o.shape[0]
         x = o.to(self.cd).view(N, heads, vdim)
         x = x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * norm_w.to(self.cd)
         gg = gate.to(self.cd).view(N, heads, vdim)
-        return (x * gg * torch.sigmoid(gg)).reshape(N, heads * vdim).to(gate.dtype)
+        gg = torch.sigmoid(gg) if act == "sigmoid" else gg * torch.sigmoid(gg)
+        return (x * gg).reshape(N, heads * vdim).to(out_dtype or gate.dtype)
+
+    # -- the state-space recurrence of Mamba-2 --------------------------------------------------
+    def ssd_conv(self, u, col0, taps, bias, state, token_seq, cu_tokens, seq_slots, single=False):
+        N, (C, J) = u.shape[0], taps.shape
+        x = u[:, col0 : col0 + C].to(self.cd)
+        y = torch.zeros((N, C), dtype=self.cd, device=u.device)
+        for s in range(seq_slots.shape[0]):
+            q0, q1, slot = int(cu_tokens[s]), int(cu_tokens[s + 1]), int(seq_slots[s])
+            if q1 <= q0:
+                continue
+            rows = x[q0:q1]
+            if J > 1:
+                rows = torch.cat([state[slot, : (J - 1) * C].view(J - 1, C).to(self.cd), rows], dim=0)
+                state[slot, : (J - 1) * C] = rows[-(J - 1):].reshape(-1).to(state.dtype)
+            for j in range(J):
+                y[q0:q1] += rows[j : j + (q1 - q0)] * taps[:, j].to(self.cd)
+        if bias is not None:
+            y = y + bias.to(self.cd)
+        return (y * torch.sigmoid(y)).to(torch.float32)
+
+    def ssd_scan(self, c, dt_in, dt_bias, a_log, D, state, heads, groups, vdim, n, seq_slots, cu_tokens, min_q_len=0, max_q_len=0):
+        N, H, G = c.shape[0], heads, groups
+        x, B, C = c.to(self.cd).split([H * vdim, G * n, G * n], dim=1)
+        x = x.reshape(N, H, vdim)
+        B, C = (t.reshape(N, G, n).repeat_interleave(H // G, dim=1) for t in (B, C))
+        dt = torch.nn.functional.softplus(dt_in[:, :H].to(self.cd) + dt_bias.to(self.cd))
+        g = torch.exp(-torch.exp(a_log.to(self.cd)) * dt)
+        y = torch.zeros((N, H, vdim), dtype=self.cd, device=c.device)
+        for s in range(seq_slots.shape[0]):
+            q0, q1, slot = int(cu_tokens[s]), int(cu_tokens[s + 1]), int(seq_slots[s])
+            if q1 <= q0:
+                continue
+            S = state[slot, : H * vdim * n].view(H, vdim, n).to(self.cd).clone()
+            for t in range(q0, q1):
+                S = g[t][:, None, None] * S + dt[t][:, None, None] * x[t][:, :, None] * B[t][:, None, :]
+                y[t] = (S * C[t][:, None, :]).sum(-1) + D.to(self.cd)[:, None] * x[t]
+            state[slot, : H * vdim * n] = S.reshape(-1).to(state.dtype)
+        return y.reshape(N, H * vdim).to(torch.float32)
+
+    def ssd_gate_norm(self, y, u, z_col, norm_w, eps, groups):
+        N, inner = y.shape
+        z = u[:, z_col : z_col + inner].to(self.cd)
+        a = (y.to(self.cd) * z * torch.sigmoid(z)).view(N, groups, -1)
+        a = a / torch.sqrt((a * a).mean(-1, keepdim=True) + eps)
+        return (a.reshape(N, inner) * norm_w.to(self.cd)).to(u.dtype)
 
     def head_gate(self, a, gates, col0, heads, vdim):
         N = a.shape[0]
@@ -523,8 +605,10 @@ class TorchOps:
         x.copy_(torch.tanh(x.to(self.cd)).to(x.dtype))
         return x
 
-    def scaled_add_rmsnorm(self, hidden, a, b, mult, weight, eps, out_dtype, rows=None):
-        d = a.to(torch.float32) if b is None else a.to(torch.float32) + b.to(torch.float32)
+    def scaled_add_rmsnorm(self, hidden, a, b, mult, weight, eps, out_dtype, rows=None, mult_b=None):
+        d = a.to(torch.float32)
+        if b is not None:
+            d = d + b.to(torch.float32) * ((mult if mult_b is None else mult_b) / mult)
         if rows is None:
             hidden += mult * d
             h = hidden
@@ -534,14 +618,16 @@ class TorchOps:
         return (x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * weight.to(self.cd)).to(out_dtype)
 
     # -- what enters the stream between two blocks -----------------------------------------------
-    def inject_rmsnorm(self, hidden, delta, vector, again, weight, eps, out_dtype):
+    def inject_rmsnorm(self, hidden, delta, vector, again, weight, eps, out_dtype, rows=None):
+        if rows is not None:
+            hidden = hidden.clone()
         if delta is not None:
             hidden += (delta.total() if hasattr(delta, "total") else delta).to(torch.float32)
         if vector is not None:
             hidden += vector
         if again is not None:
             hidden += again.rows(self)
-        return self.add_rmsnorm(hidden, None, weight, eps, out_dtype)
+        return self.add_rmsnorm(hidden, None, weight, eps, out_dtype, rows)
 
     # -- attention gated element by element, heads' weights mixed ---------------------------------
     def _turned(self, t, cos_sin, sign):
