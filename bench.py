@@ -13,6 +13,7 @@
     python bench.py --workload malilorn [--sizes small|mid|wide]  # Malilorn beside Kezasun, kernel by kernel
     python bench.py --workload birelix [--sizes small|mid|wide]   # Birelix beside Kezasun, kernel by kernel
     python bench.py --workload telulorn [--sizes small|mid|wide]  # Telulorn beside Malilorn, kernel by kernel
+    python bench.py --workload rorevik [--sizes small|mid|wide]  # Rorevik beside Telulorn, kernel by kernel
 
 A "step" is one decode step of the whole engine (scheduler, model step over the
 paged cache, sampling) with `batch` live requests whose context ends at
@@ -1331,6 +1332,200 @@ def telulorn_workload(args):
     return 0
 
 
+ROREVIK_SIZES = {
+    # width; attention: q heads, kv heads, dim, rotated, cap; state space: heads, vdim, state, groups, taps, norm parts; delta rule:
+    # value heads, query/key heads, dim, vdim, taps, inner ranks; dense ff, limit
+    "small": (1024, 8, 2, 128, 64, 30.0, 32, 64, 128, 1, 4, 1, 16, 8, 64, 64, 4, 64, 4096, 7.0),
+    "mid": (2048, 16, 4, 128, 64, 30.0, 64, 64, 128, 2, 4, 2, 32, 16, 64, 64, 4, 64, 8192, 7.0),
+    "wide": (4096, 32, 8, 128, 64, 30.0, 128, 64, 128, 8, 4, 8, 64, 32, 64, 64, 4, 64, 12288, 7.0),
+}
+
+
+def rorevik_config(which, groups):
+    from litellmengine_amd.config import RorevikConfig
+
+    W, H, G, dim, rot, cap, SH, svdim, state, SG, staps, parts, DH, DG, ddim, dvdim, dtaps, rank, ff, limit = ROREVIK_SIZES[which]
+    mlp = {"kind": "dense", "ff": ff, "limit": limit}
+    parallel = {"type": "parallel", "mlp": mlp, "mixer": {
+        "left": {"heads": H, "kv_heads": G, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "softcap": cap, "rot": {"base": 5e5, "dims": rot}},
+        "right": {"heads": SH, "vdim": svdim, "state": state, "groups": SG, "conv": staps, "norm_groups": parts},
+        "left_scale": 0.7, "right_scale": 0.8}}
+    delta = {"type": "channel_delta", "mlp": mlp, "mixer": {"heads": DH, "kv_heads": DG, "dim": ddim, "vdim": dvdim, "conv": dtaps,
+                                                            "decay_rank": rank, "gate_rank": rank}}
+    return RorevikConfig.from_dict({"architecture": "Rorevik", "vocab": 32768, "width": W, "max_positions": 8192, "norm": {"eps": 1e-6},
+                                    "embedding": {"scale": W ** 0.5}, "layers": [parallel, delta, parallel, parallel] * groups,
+                                    "loop": {"start": 1, "stop": 3, "times": 2}})
+
+
+def rorevik_kernels(which):
+    """Each kernel of Rorevik's own at two shapes (a 2048-token prompt; 8 decoded tokens after 4096) beside the like kernel
+    of Telulorn (the closest model: two mixers side by side, a recurrence with a matrix state per head, a loop over depth)
+    or of Birelix (the delta rule, its convolution and output norm) at their sizes of the same name, or beside the same
+    kernel without what Rorevik adds to it: microseconds and the share of its roofline."""
+    import torch
+
+    from litellmengine_amd.csrc.ops import default_ops
+
+    ops = default_ops()
+    W, H, G, dim, rot, cap, SH, svdim, state, SG, staps, parts, DH, DG, ddim, dvdim, dtaps, rank, ff, limit = ROREVIK_SIZES[which]
+    _, _, _, _, _, _, _, _, _, LH, ldim, lvdim, lrank, _ = TELULORN_SIZES[which]
+    dev, bf, f32 = "cuda", torch.bfloat16, torch.float32
+    P = PAGE_SIZE
+    rnd = lambda *shape, dtype=bf, scale=1.0: (torch.randn(shape, device=dev) * scale).to(dtype)
+    ints = lambda values: torch.tensor(values, dtype=torch.int32, device=dev)
+    out = {}
+
+    def entry(name, seconds, flops, nbytes, like=None):
+        floor = max(flops / MFMA_PEAK["bf16"], nbytes / HBM_PEAK)
+        e = {"us": round(seconds * 1e6, 1), "roofline_us": round(floor * 1e6, 2), "frac": round(floor / seconds, 4),
+             "bound": "mfma" if flops / MFMA_PEAK["bf16"] > nbytes / HBM_PEAK else "hbm"}
+        if like is not None:
+            e["like"] = like
+            e["times_farther_from_roofline"] = round(like["frac"] / e["frac"], 2) if e["frac"] > 0 else None
+        out[name] = e
+        return e
+
+    for shape, S, q_len, past in (("prefill_2048", 1, 2048, 0), ("decode_b8_ctx4096", 8, 1, 4095)):
+        N, kv = S * q_len, past + q_len
+        pages_each = -(-kv // P)
+        table = torch.arange(S * pages_each, dtype=torch.int32, device=dev).view(S, pages_each).contiguous()
+        seq_slots, cu = ints(list(range(S))), ints([i * q_len for i in range(S + 1)])
+        kv_lens = ints([kv] * S)
+        token_seq = ints([i // q_len for i in range(N)])
+        positions = ints([past + i % q_len for i in range(N)])
+        where = (table, seq_slots, cu, kv_lens, token_seq)
+        # attention with capped scores beside the same without a cap
+        kv_layer = rnd(S * pages_each + 1, 2, G, P, dim)
+        q = rnd(N, H, dim, scale=0.1)
+        seen = S * (q_len * past + q_len * (q_len + 1) / 2)
+        work = (4.0 * H * dim * seen, 2.0 * (S * kv * 2 * G * dim + 2 * N * H * dim))
+        tk = timed_launches(lambda: ops.paged_attention(q, kv_layer, *where, None, 0.1, q_len, q_len, kv))
+        like = dict(entry(f"{shape}/paged_attention (Qwen3)", tk, *work), name="paged_attention")
+        t = timed_launches(lambda: ops.paged_attention(q, kv_layer, *where, None, 0.1, q_len, q_len, kv, softcap=cap))
+        entry(f"{shape}/paged_attention, capped scores", t, *work, like)
+        # Mamba-2's recurrence beside gated linear attention (its decays and walk)
+        gu, low = rnd(N, 2 * LH * (ldim + lvdim), scale=0.5), rnd(N, lrank, dtype=f32)
+        a2, ab = rnd(lrank, LH * ldim, dtype=f32), torch.zeros(LH * ldim, device=dev)
+        gstate, gnw = torch.zeros(S + 1, LH * ldim * lvdim, device=dev), torch.ones(lvdim, device=dev)
+        tk = timed_launches(lambda: ops.gla_scan(gu, ops.gla_decay(low, a2, ab, 16.0), 0.125, gnw, 1e-6, gstate, LH, ldim, lvdim, seq_slots,
+                                                 cu, q_len))
+        like = dict(entry(f"{shape}/gla_decay + gla_scan (Telulorn)", tk, 0, N * (4.0 * LH * (ldim + lvdim) + 4.0 * lrank + 2.0 * LH * lvdim)
+                          + 8.0 * S * LH * ldim * lvdim), name="gla_decay + gla_scan")
+        inner = SH * svdim
+        cc = inner + 2 * SG * state
+        c, dt = rnd(N, cc, dtype=f32), rnd(N, SH, dtype=f32)
+        per_head = [torch.zeros(SH, device=dev) for _ in range(3)]
+        sstate = torch.zeros(S + 1, inner * state, device=dev)
+        t = timed_launches(lambda: ops.ssd_scan(c, dt, *per_head, sstate, SH, SG, svdim, state, seq_slots, cu, q_len, q_len))
+        e = entry(f"{shape}/ssd_scan", t, 0, 4.0 * N * (cc + SH + inner) + 8.0 * S * inner * state, like)
+        e["fp32_flops_T"] = round(6.0 * N * inner * state / t / 1e12, 2)
+        # its convolution beside the delta rule's
+        dcols = 2 * DG * ddim + DH * dvdim
+        du, dtap = rnd(N, dcols), rnd(dcols, dtaps, dtype=f32)
+        dkept = torch.zeros(S + 1, (dtaps - 1) * dcols, device=dev)
+
+        def conv():
+            ops.delta_conv(du, dtap, dkept, token_seq, cu, seq_slots, DG, ddim, DH, dvdim, 1e-6, ddim ** -0.5)
+            ops.conv_state_update(du, dkept, dtaps - 1, cu, seq_slots)
+
+        tk = timed_launches(conv)
+        like = dict(entry(f"{shape}/delta_conv + conv_state_update (Birelix)", tk, 0, N * dcols * (2 + 4.0) + 8.0 * S * (dtaps - 1) * dcols),
+                    name="delta_conv + conv_state_update")
+        u, stap, sbias = rnd(N, inner + cc), rnd(cc, staps, dtype=f32), rnd(cc, dtype=f32)
+        skept = torch.zeros(S + 1, (staps - 1) * cc, device=dev)
+        t = timed_launches(lambda: ops.ssd_conv(u, inner, stap, sbias, skept, token_seq, cu, seq_slots, single=q_len == 1))
+        entry(f"{shape}/ssd_conv", t, 0, N * cc * (2 + 4.0) + 8.0 * S * (staps - 1) * cc, like)
+        if q_len == 1:
+            t = timed_launches(lambda: ops.delta_conv(du, dtap, dkept, token_seq, cu, seq_slots, DG, ddim, DH, dvdim, 1e-6, ddim ** -0.5,
+                                                      advance=True))
+            entry(f"{shape}/delta_conv that moves the state on", t, 0, N * dcols * (2 + 4.0) + 8.0 * S * (dtaps - 1) * dcols, like)
+        # the output norms
+        o, gate, gate32, nw = rnd(N, DH * dvdim, dtype=f32), rnd(N, DH * dvdim), rnd(N, DH * dvdim, dtype=f32), torch.ones(dvdim, device=dev)
+        tk = timed_launches(lambda: ops.delta_out_norm(o, gate, nw, 1e-6, DH, dvdim))
+        like = dict(entry(f"{shape}/delta_out_norm (Birelix)", tk, 0, N * DH * dvdim * (4 + 2 + 2.0)), name="delta_out_norm")
+        t = timed_launches(lambda: ops.delta_out_norm(o, gate32, nw, 1e-6, DH, dvdim, act="sigmoid", out_dtype=bf))
+        entry(f"{shape}/delta_out_norm, 32-bit sigmoid gate", t, 0, N * DH * dvdim * (4 + 4 + 2.0), like)
+        y, sw = rnd(N, inner, dtype=f32), torch.ones(inner, device=dev)
+        t = timed_launches(lambda: ops.ssd_gate_norm(y, u, 0, sw, 1e-6, parts))
+        entry(f"{shape}/ssd_gate_norm", t, 0, N * inner * (4 + 2 + 2.0), like)
+        # the delta rule's walk with a decay per key channel beside the walk with one per head
+        dq, dk = rnd(N, DG * ddim, dtype=f32, scale=ddim ** -0.5), rnd(N, DG * ddim, dtype=f32, scale=ddim ** -0.5)
+        dv, ba = rnd(N, DH * dvdim, dtype=f32), rnd(N, 2 * DH, dtype=f32)
+        zeros, dstate = torch.zeros(DH, device=dev), torch.zeros(S + 1, DH * dvdim * ddim, device=dev)
+        tk = timed_launches(lambda: ops.delta_scan(dq, dk, dv, ba, zeros, zeros, dstate, DH, DG, ddim, dvdim, seq_slots, cu))
+        like = dict(entry(f"{shape}/delta_scan (Birelix)", tk, 0, N * (2 * DG * ddim + 2 * DH * dvdim + 2 * DH) * 4.0
+                          + 8.0 * S * DH * dvdim * ddim), name="delta_scan")
+        decay = torch.rand(N, DH * ddim, device=dev)
+        t = timed_launches(lambda: ops.delta_scan(dq, dk, dv, ba, None, None, dstate, DH, DG, ddim, dvdim, seq_slots, cu, decay=decay))
+        e = entry(f"{shape}/delta_scan, a decay per channel", t, 0, N * (2 * DG * ddim + DH * ddim + 2 * DH * dvdim + DH) * 4.0
+                  + 8.0 * S * DH * dvdim * ddim, like)
+        e["fp32_flops_T"] = round(9.0 * N * DH * dvdim * ddim / t / 1e12, 2)
+        # its decays and gates through narrow middles beside linear attention's decays
+        tk = timed_launches(lambda: ops.gla_decay(low, a2, ab, 16.0))
+        like = dict(entry(f"{shape}/gla_decay (Telulorn)", tk, 0, 4.0 * (N * (lrank + LH * ldim) + lrank * LH * ldim)), name="gla_decay")
+        h4 = -(-DH // 4) * 4
+        dlow, da2, dg2 = rnd(N, h4 + 2 * rank, dtype=f32), rnd(DH * ddim, rank, dtype=f32), rnd(DH * dvdim, rank, dtype=f32)
+        dbias = torch.zeros(DH * ddim, device=dev)
+        t = timed_launches(lambda: ops.low_rank_gates(dlow, h4, da2, zeros, dbias, ddim, h4 + rank, dg2))
+        entry(f"{shape}/low_rank_gates", t, 0, 4.0 * (N * (h4 + 2 * rank + DH * (ddim + dvdim)) + rank * DH * (ddim + dvdim)), like)
+        # the stream's sums and norms
+        hidden, da, db = rnd(N, W, dtype=f32), rnd(N, W), rnd(N, W)
+        w, vec = torch.ones(W, device=dev, dtype=bf), torch.zeros(W, device=dev)
+        tk = timed_launches(lambda: ops.scaled_add_rmsnorm(hidden, da, db, 1.0, w, 1e-6, bf))
+        like = dict(entry(f"{shape}/scaled_add_rmsnorm, one factor (Telulorn)", tk, 0, N * W * (4 + 4 + 2 + 2 + 2.0)), name="scaled_add_rmsnorm")
+        t = timed_launches(lambda: ops.scaled_add_rmsnorm(hidden, da, db, 0.3, w, 1e-6, bf, mult_b=0.2))
+        entry(f"{shape}/scaled_add_rmsnorm, two factors", t, 0, N * W * (4 + 4 + 2 + 2 + 2.0), like)
+        t = timed_launches(lambda: ops.inject_rmsnorm(hidden, da, vec, None, w, 1e-6, bf))
+        entry(f"{shape}/inject_rmsnorm, a bias beside the delta", t, 0, N * W * (4 + 4 + 2 + 2.0), like)
+        ids = torch.randint(0, 32768, (N,), device=dev, dtype=torch.int32)
+        words, pos = rnd(32768, W), rnd(8192, W)
+        tk = timed_launches(lambda: ops.embedding_rmsnorm(ids, words, w, 1e-6))
+        like = dict(entry(f"{shape}/embedding_rmsnorm (Qwen3)", tk, 0, N * W * (2 + 4 + 2.0)), name="embedding_rmsnorm")
+        t = timed_launches(lambda: ops.embedding_norm(ids, words, 2.0, positions, pos, w, 1e-6, w, 1e-6, bf))
+        entry(f"{shape}/embedding_norm", t, 0, N * W * (2 + 2 + 4 + 2.0), like)
+        # the clamped gate with biases beside silu_mul
+        z, zb = rnd(N, 2 * ff), rnd(2 * ff)
+        tk = timed_launches(lambda: ops.silu_mul(z))
+        like = dict(entry(f"{shape}/silu_mul (Qwen3)", tk, 0, 2.0 * N * 3 * ff), name="silu_mul")
+        t = timed_launches(lambda: ops.bias_act(z, "clamp", True, bias=zb, limit=limit))
+        entry(f"{shape}/bias_act, clamped with biases", t, 0, 2.0 * N * 3 * ff, like)
+        del kv_layer, words, pos
+    return out
+
+
+def rorevik_workload(args):
+    import torch
+
+    from litellmengine_amd.models import random_model
+
+    which = args.sizes if args.sizes in ROREVIK_SIZES else "mid"
+    groups = max(1, args.layers // 4) if args.layers != SIZES["num_hidden_layers"] else 1
+    rcfg = rorevik_config(which, groups)
+    tcfg = telulorn_config(which, groups)
+    names = ("width", "heads", "kv_heads", "dim", "rotated", "softcap", "ssd_heads", "ssd_vdim", "ssd_state", "ssd_groups", "ssd_taps",
+             "norm_parts", "delta_heads", "delta_kv_heads", "delta_dim", "delta_vdim", "delta_taps", "inner_ranks", "dense_ff", "limit")
+    line = {"metric": f"Rorevik beside Telulorn at layer sizes of the same name ({which}): prefill tok/s @ 2048 and decode tok/s "
+                      f"@ batch {args.batch}, context {args.context}", "unit": "tok/s", "n_gpus": 1, "dtype": "bf16",
+            "data": "synthetic: seeded random weights, uniform random token ids", "higher_is_better": True,
+            "config": {"sizes": dict(zip(names, ROREVIK_SIZES[which])), "layers": len(rcfg.layers), "layer_runs": len(rcfg.layers) + 2,
+                       "pattern": "parallel, channel_delta, parallel, parallel; the second and third layer run twice",
+                       "beside": "Telulorn: parallel, attention, parallel, parallel; the second and third layer run twice"}}
+    steps, warmup = min(args.steps, 16), min(args.warmup, 4)
+    for name, cfg in (("rorevik", rcfg), ("telulorn", tcfg)):
+        model = random_model(cfg, seed=0, dtype="bfloat16")
+        dt = time_decode(model, cfg, args.batch, args.context, steps, warmup)
+        pt = time_prefill(model, cfg, PREFILL_TOKENS)
+        line[name] = {"decode_tok_s": round(args.batch / dt, 1), "decode_ms_per_step": round(dt * 1e3, 3),
+                      "prefill_tok_s": round(PREFILL_TOKENS / pt, 1), "prefill_ms": round(pt * 1e3, 3)}
+        del model
+        torch.cuda.empty_cache()
+    line["value"] = line["rorevik"]["decode_tok_s"]
+    line["steps"], line["warmup"] = steps, warmup
+    line["kernels"] = rorevik_kernels(which)
+    print(json.dumps(line))
+    return 0
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -1344,12 +1539,13 @@ def main():
     ap.add_argument("--no-more", action="store_true", help="skip the other workloads that the default line carries")
     ap.add_argument("--sizes", default="8b", choices=["8b", "0p6b", "32b", "small", "mid", "wide"],
                     help="layer sizes of the decode workload: Qwen3-8B (default, the headline), Qwen3-0.6B or Qwen3-32B; "
-                         "small, mid or wide: the layer sizes of --workload visadra, kezasun, malilorn, birelix and telulorn")
-    ap.add_argument("--workload", default="decode", choices=["decode", "reference-0p6b", "mixed-32b", "serving", "visadra", "kezasun", "malilorn", "birelix", "telulorn"],
+                         "small, mid or wide: the layer sizes of --workload visadra, kezasun, malilorn, birelix, telulorn and rorevik")
+    ap.add_argument("--workload", default="decode", choices=["decode", "reference-0p6b", "mixed-32b", "serving", "visadra", "kezasun", "malilorn", "birelix", "telulorn", "rorevik"],
                     help="decode (default: the headline line), the reference's own benchmark shape at Qwen3-0.6B "
                          "sizes, a mixed prompt-portion + decode step at Qwen3-32B sizes, requests arriving over time, "
                          "Visadra beside Qwen3 at equal layer sizes with every kernel against its roofline, Kezasun "
-                         "beside Visadra the same way, or Malilorn or Birelix beside Kezasun the same way")
+                         "beside Visadra the same way, Malilorn or Birelix beside Kezasun, Telulorn beside Malilorn or Rorevik beside "
+                         "Telulorn the same way")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py measures one GPU only: --gpus {args.gpus} is not supported")
@@ -1373,6 +1569,8 @@ def main():
             return birelix_workload(args)
         if args.workload == "telulorn":
             return telulorn_workload(args)
+        if args.workload == "rorevik":
+            return rorevik_workload(args)
         args.steps, args.warmup = min(args.steps, 3), min(args.warmup, 1)
         return mixed_workload(args)
 
