@@ -611,9 +611,13 @@ struct LowRankArgs {
     int N;
 };
 
+// exp(-rate softplus(z)) in base 2: softplus(z) log2 e = max(z, 0) log2 e + log2(1 + x), x = e^-|z|; a small x takes the
+// first terms of the series (1 + x would round them away)
 __device__ __forceinline__ float delta_decay_of(float z, float rate) {
-    const float softplus = fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
-    return expf(-rate * softplus);
+    const float x = __builtin_amdgcn_exp2f(-fabsf(z) * 1.44269504088896340736f);
+    const float series = x * (1.f - x * (0.5f - x * 0.33333333333f)) * 1.44269504088896340736f;
+    const float log2_1px = x < 0.01f ? series : __builtin_amdgcn_logf(1.0f + x);
+    return __builtin_amdgcn_exp2f(-rate * fmaf(fmaxf(z, 0.f), 1.44269504088896340736f, log2_1px));
 }
 
 // grid = (blocks of channels: those of the decays, then those of the gates; tiles of 16 tokens in fours); a wavefront
@@ -635,15 +639,23 @@ __global__ __launch_bounds__(256) void low_rank_gates_kernel(LowRankArgs a) {
     delta_f32x4 acc[NT];
 #pragma unroll
     for (int n = 0; n < NT; ++n) acc[n] = delta_f32x4{0.f, 0.f, 0.f, 0.f};
-    for (int k = 0; k < R; k += 16) {
-        const delta_f32x4 xv = *(const delta_f32x4*)(x + k);
-        delta_f32x4 wv[NT];
+    // (the next sixteen of the contraction are asked for before these are multiplied; past the end: the last ones again)
+    delta_f32x4 xv = *(const delta_f32x4*)x, wv[NT];
 #pragma unroll
-        for (int n = 0; n < NT; ++n) wv[n] = *(const delta_f32x4*)(wr[n] + k);
+    for (int n = 0; n < NT; ++n) wv[n] = *(const delta_f32x4*)wr[n];
+    for (int k = 0; k < R; k += 16) {
+        const int next = min(k + 16, R - 16);
+        const delta_f32x4 xn = *(const delta_f32x4*)(x + next);
+        delta_f32x4 wn[NT];
+#pragma unroll
+        for (int n = 0; n < NT; ++n) wn[n] = *(const delta_f32x4*)(wr[n] + next);
 #pragma unroll
         for (int n = 0; n < NT; ++n)
 #pragma unroll
             for (int e = 0; e < 4; ++e) acc[n] = __builtin_amdgcn_mfma_f32_16x16x4f32(wv[n][e], xv[e], acc[n], 0, 0, 0);
+        xv = xn;
+#pragma unroll
+        for (int n = 0; n < NT; ++n) wv[n] = wn[n];
     }
     if (n0 + r >= a.N) return;
     float* dst = (decays ? a.decay : a.gate) + (int64_t)(n0 + r) * C;
@@ -651,10 +663,19 @@ __global__ __launch_bounds__(256) void low_rank_gates_kernel(LowRankArgs a) {
     for (int n = 0; n < NT; ++n) {
         const int ch = c0 + 16 * n + 4 * c;
         float y[4];
+        if (decays) {
+            // four neighbouring channels of one head share its rate
+            const int h = min(ch, C - 1) / a.dim;
+            const float rate = expf(a.a_log[h]);
+            const bool one_head = a.dim % 4 == 0;
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            y[e] = acc[n][e];
-            if (decays && ch + e < C) y[e] = delta_decay_of(y[e] + a.dt_bias[ch + e], expf(a.a_log[(ch + e) / a.dim]));
+            for (int e = 0; e < 4; ++e) {
+                const int at = min(ch + e, C - 1);
+                y[e] = delta_decay_of(acc[n][e] + a.dt_bias[at], one_head ? rate : expf(a.a_log[at / a.dim]));
+            }
+        } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) y[e] = acc[n][e];
         }
         if (C % 4 == 0) {
             if (ch < C) *(float4*)(dst + ch) = make_float4(y[0], y[1], y[2], y[3]);

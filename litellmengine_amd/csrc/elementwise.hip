@@ -291,7 +291,10 @@ __global__ __launch_bounds__(256) void bias_act_vec_kernel(const bf16_t* __restr
             const float first = (float)g[k] + (bias ? (float)bg[k] : 0.f);
             float a;
             if constexpr (GATED && KIND == LLE_ACT_CLAMP) {
-                a = clamped_gate(first, (float)u[k] + (bias ? (float)bu[k] : 0.f), limit);
+                // (clamped_gate with the hardware's exponential and reciprocal: the result is rounded to 16 bits)
+                const float gg = fminf(first, limit), uu = fminf(fmaxf((float)u[k] + (bias ? (float)bu[k] : 0.f), -limit), limit);
+                const float sig = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(gg * (-1.702f * 1.44269504088896340736f)));
+                a = gg * sig * (uu + 1.0f);
             } else {
                 a = apply_act(first, KIND);
                 if (GATED) a *= (float)u[k] + (bias ? (float)bu[k] : 0.f);

@@ -676,9 +676,8 @@ extern "C" int lle_inject_rmsnorm(void* hidden, const void* a, int a_dtype, int 
 //   h[n] = RMSNorm(table[id(n)] * scale (+ pos[position n])) * w0 (w0 null: without that norm)
 // and, with `weight`, the first block's norm of the new row in the same launch: out[n] = RMSNorm(h[n]) * weight.  All in
 // 32-bit; h is float32.  Ids as in the embedding kernel; the host has checked ids and positions (a position past the
-// table would read its last row).  A thread keeps its share of the row in registers (rows up to 256 x EN_PER; wider ones
-// are read back from `hidden`, each element by the thread that wrote it).
-#define EN_PER 32
+// table would read its last row).  A thread keeps its share of the row in registers (rows up to 256 x 4 x NORM_CHUNKS and a
+// multiple of 4; others are read back from `hidden`, each element by the thread that wrote it).
 struct EmbedArgs {
     const int32_t* ids;
     const void* table;
@@ -714,15 +713,21 @@ __global__ __launch_bounds__(256) void embedding_norm_kernel(EmbedArgs x) {
         if (x.pos) v += load_as_f32(x.pos, prow + i, x.pos_dtype);
         return v;
     };
-    const bool fits = H <= 256 * EN_PER;
-    float keep[EN_PER];
+    const bool fits = H % 4 == 0 && H <= 256 * 4 * NORM_CHUNKS;
+    float4 keep[NORM_CHUNKS];
     float ss = 0.f;
+    const auto squares = [](float4 v) { return v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w; };
+    const auto times = [](float4 v, float f, float4 w) { return make_float4(v.x * f * w.x, v.y * f * w.y, v.z * f * w.z, v.w * f * w.w); };
     if (fits) {
 #pragma unroll
-        for (int k = 0; k < EN_PER; ++k) {
-            const int i = k * 256 + threadIdx.x;
-            keep[k] = i < H ? made(i) : 0.f;
-            ss += keep[k] * keep[k];
+        for (int k = 0; k < NORM_CHUNKS; ++k) {
+            const int i = (k * 256 + threadIdx.x) * 4;
+            if (i < H) {
+                const float4 e = load_quad(x.table, row + i, x.table_dtype);
+                keep[k] = make_float4(e.x * x.scale, e.y * x.scale, e.z * x.scale, e.w * x.scale);
+                if (x.pos) add_quad(keep[k], load_quad(x.pos, prow + i, x.pos_dtype));
+                ss += squares(keep[k]);
+            }
         }
     } else {
         for (int i = threadIdx.x; i < H; i += blockDim.x) {
@@ -735,12 +740,12 @@ __global__ __launch_bounds__(256) void embedding_norm_kernel(EmbedArgs x) {
     ss = 0.f;
     if (fits) {
 #pragma unroll
-        for (int k = 0; k < EN_PER; ++k) {
-            const int i = k * 256 + threadIdx.x;
+        for (int k = 0; k < NORM_CHUNKS; ++k) {
+            const int i = (k * 256 + threadIdx.x) * 4;
             if (i < H) {
-                if (x.w0) keep[k] *= inv0 * load_as_f32(x.w0, i, x.w0_dtype);
-                h[i] = keep[k];
-                ss += keep[k] * keep[k];
+                if (x.w0) keep[k] = times(keep[k], inv0, load_quad(x.w0, i, x.w0_dtype));
+                *(float4*)(h + i) = keep[k];
+                ss += squares(keep[k]);
             }
         }
     } else {
@@ -756,9 +761,9 @@ __global__ __launch_bounds__(256) void embedding_norm_kernel(EmbedArgs x) {
     TO* out = (TO*)x.out + n * H;
     if (fits) {
 #pragma unroll
-        for (int k = 0; k < EN_PER; ++k) {
-            const int i = k * 256 + threadIdx.x;
-            if (i < H) out[i] = from_f32<TO>(keep[k] * inv * load_as_f32(x.weight, i, x.weight_dtype));
+        for (int k = 0; k < NORM_CHUNKS; ++k) {
+            const int i = (k * 256 + threadIdx.x) * 4;
+            if (i < H) Quad<TO>::store(out + i, times(keep[k], inv, load_quad(x.weight, i, x.weight_dtype)));
         }
     } else {
         for (int i = threadIdx.x; i < H; i += blockDim.x) out[i] = from_f32<TO>(h[i] * inv * load_as_f32(x.weight, i, x.weight_dtype));

@@ -614,10 +614,10 @@ extern "C" int lle_ssd_scan(const void* c, int CC, const void* dt_in, int dt_col
 // ---------------------------------------------------------------------------------
 // out[n, :] = (y silu(z)) / rms(its part) * w: a row is cut into `groups` equal parts, each divided by its own root mean
 // square.  z: the columns z0 .. of u.  A workgroup of 256 threads a (token, part); a thread keeps its share of the part in
-// registers (parts up to 256 x SSD_PER; wider ones are made twice).
+// registers, in pieces of V elements (parts up to 256 x SSD_PER; wider ones are made twice).
 // ---------------------------------------------------------------------------------
 #define SSD_PER 32
-template <typename T>
+template <typename T, int V>
 __global__ __launch_bounds__(256) void ssd_gate_norm_kernel(const float* __restrict__ y, const T* __restrict__ u, int cols, int z0,
                                                              const float* __restrict__ w, float eps, T* __restrict__ out, int inner,
                                                              int width) {
@@ -627,15 +627,25 @@ __global__ __launch_bounds__(256) void ssd_gate_norm_kernel(const float* __restr
     const float* yr = y + n * inner + p0;
     const T* zr = u + n * cols + z0 + p0;
     T* dst = out + n * inner + p0;
+    typedef T piece_t __attribute__((ext_vector_type(V)));
+    typedef float fpiece_t __attribute__((ext_vector_type(V)));
     float keep[SSD_PER], ss = 0.f;
     const bool fits = width <= 256 * SSD_PER;
     if (fits) {
 #pragma unroll
-        for (int k = 0; k < SSD_PER; ++k) {
-            const int i = k * 256 + threadIdx.x;
+        for (int k = 0; k < SSD_PER; k += V) {
+            const int i = (k / V * 256 + threadIdx.x) * V;
             if (k * 256 >= width) break;  // (the same for every thread)
-            keep[k] = i < width ? yr[i] * ssd_silu(to_f32<T>(zr[i])) : 0.f;
-            ss = fmaf(keep[k], keep[k], ss);
+            if (i < width) {  // (V divides the width and every offset)
+                const fpiece_t yv = *(const fpiece_t*)(yr + i);
+                const piece_t zv = *(const piece_t*)(zr + i);
+#pragma unroll
+                for (int e = 0; e < V; ++e) {
+                    const float z = to_f32<T>(zv[e]);
+                    keep[k + e] = yv[e] * z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(z * -1.44269504088896340736f));
+                    ss = fmaf(keep[k + e], keep[k + e], ss);
+                }
+            }
         }
     } else {
         for (int i = threadIdx.x; i < width; i += 256) {
@@ -646,10 +656,16 @@ __global__ __launch_bounds__(256) void ssd_gate_norm_kernel(const float* __restr
     const float inv = 1.0f / sqrtf(block_sum(ss, red) / (float)width + eps);
     if (fits) {
 #pragma unroll
-        for (int k = 0; k < SSD_PER; ++k) {
-            const int i = k * 256 + threadIdx.x;
+        for (int k = 0; k < SSD_PER; k += V) {
+            const int i = (k / V * 256 + threadIdx.x) * V;
             if (k * 256 >= width) break;
-            if (i < width) dst[i] = from_f32<T>(keep[k] * inv * w[p0 + i]);
+            if (i < width) {
+                const fpiece_t wv = *(const fpiece_t*)(w + p0 + i);
+                piece_t o;
+#pragma unroll
+                for (int e = 0; e < V; ++e) o[e] = from_f32<T>(keep[k + e] * inv * wv[e]);
+                *(piece_t*)(dst + i) = o;
+            }
         }
     } else {
         for (int i = threadIdx.x; i < width; i += 256)
@@ -662,11 +678,15 @@ extern "C" int lle_ssd_gate_norm(const void* y, const void* u, int cols, int z0,
     if (N <= 0 || inner <= 0) return 0;
     if (groups <= 0 || inner % groups || groups > 65535 || z0 < 0 || z0 + inner > cols) return (int)hipErrorInvalidValue;
     const dim3 grid(N, groups);
-    if (dtype == LLE_F32)
-        ssd_gate_norm_kernel<float><<<grid, 256, 0, stream>>>((const float*)y, (const float*)u, cols, z0, (const float*)w, eps, (float*)out,
-                                                               inner, inner / groups);
-    else
-        ssd_gate_norm_kernel<bf16_t><<<grid, 256, 0, stream>>>((const float*)y, (const bf16_t*)u, cols, z0, (const float*)w, eps,
-                                                                (bf16_t*)out, inner, inner / groups);
+    const bool wide = (inner / groups) % 4 == 0 && cols % 4 == 0 && z0 % 4 == 0;
+#define SSD_GATE(T, V)                                                                                                         \
+    ssd_gate_norm_kernel<T, V><<<grid, 256, 0, stream>>>((const float*)y, (const T*)u, cols, z0, (const float*)w, eps, (T*)out, inner, \
+                                                         inner / groups)
+    if (dtype == LLE_F32) {
+        if (wide) SSD_GATE(float, 4); else SSD_GATE(float, 1);
+    } else {
+        if (wide) SSD_GATE(bf16_t, 4); else SSD_GATE(bf16_t, 1);
+    }
+#undef SSD_GATE
     LLE_RETURN_LAUNCH_STATUS();
 }

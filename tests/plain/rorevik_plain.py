@@ -140,8 +140,9 @@ def causal_softmax(scores: torch.Tensor) -> torch.Tensor:
 def capped_attention(h, w, p: str, m: dict) -> torch.Tensor:
     T, H, G, d, vd = h.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
     pos = torch.arange(T)
-    q = turn_pairs((h @ w[p + "q"].T).view(T, H, d), pos, m["rot"]["dims"], m["rot"]["base"])
-    k = turn_pairs((h @ w[p + "k"].T).view(T, G, d), pos, m["rot"]["dims"], m["rot"]["base"])
+    rot = m.get("rot") or {"dims": 0, "base": 1.0}  # (no rotation)
+    q = turn_pairs((h @ w[p + "q"].T).view(T, H, d), pos, rot["dims"], rot["base"])
+    k = turn_pairs((h @ w[p + "k"].T).view(T, G, d), pos, rot["dims"], rot["base"])
     v = (h @ w[p + "v"].T).view(T, G, vd)
     k, v = (x.repeat_interleave(H // G, dim=1) for x in (k, v))
     a = causal_softmax(capped(torch.einsum("ihd,jhd->hij", q, k) * m["scale"], m["softcap"]))
