@@ -192,7 +192,25 @@ struct NormFold {
     const float* ss_in;     // SCALED: [16][parts]
     int parts;              // SCALED
     float eps;              // SCALED
+    // GATED: biases [N] (or null) and with act_limit > 0 the clamped activation instead of silu
+    const bf16_t* act_bias;
+    float act_limit;
 };
+
+// what a gated product makes of a gate's and an up row's sums: silu(g) u, or with a limit, g = min(g, limit) and
+// u = clamp(u, -limit, limit), g sigmoid(1.702 g) (u + 1)
+__device__ __forceinline__ float gated_result(float g, float u, const NormFold& fold, int64_t col, int64_t rows) {
+    if (fold.act_limit > 0.f) {  // (the same for the whole launch)
+        if (fold.act_bias) {
+            g += (float)fold.act_bias[col];
+            u += (float)fold.act_bias[rows + col];
+        }
+        g = fminf(g, fold.act_limit);
+        u = fminf(fmaxf(u, -fold.act_limit), fold.act_limit);
+        return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
+    }
+    return g / (1.0f + expf(-g)) * u;
+}
 
 template <int MT, int NT, bool GATED, bool RESID, bool SCALED, typename TC, int SK_WAVES, int UNROLL>
 // one tile of W and up to 16 rows of X: two workgroups of 16 wavefronts a CU (8 wavefronts a SIMD),
@@ -363,7 +381,7 @@ __global__ __launch_bounds__(SK_WAVES* LLE_WAVE, (MT == 1 && !GATED) ? 8 : 4) vo
                 g *= s_inv[16 * mt + m];
                 u *= s_inv[16 * mt + m];
             }
-            C[row * (N / 2) + col] = from_f32<TC>(g / (1.0f + expf(-g)) * u);
+            C[row * (N / 2) + col] = from_f32<TC>(gated_result(g, u, fold, col, N / 2));
         }
         return;
     }
@@ -720,7 +738,7 @@ __global__ __launch_bounds__(16 * LLE_WAVE, 4) void gemm_skinny_stream_kernel(co
                     g *= s_inv[m];
                     u *= s_inv[m];
                 }
-                C[(int64_t)m * rows + col] = from_f32<TC>(GATED ? g / (1.0f + expf(-g)) * u : g);
+                C[(int64_t)m * rows + col] = from_f32<TC>(GATED ? gated_result(g, u, fold, col, rows) : g);
             }
         }
         // The other half is written next; this one again only after the next tile's barrier,
@@ -862,14 +880,13 @@ extern "C" int lle_gemm_skinny_resid_parts(int N) {
 }
 
 template <typename TC, int NT, bool GATED>
-static int launch_skinny(const bf16_t* X, const bf16_t* W, TC* C, int M, int N, int K, hipStream_t stream) {
+static int launch_skinny(const bf16_t* X, const bf16_t* W, TC* C, int M, int N, int K, hipStream_t stream, const NormFold& none = {}) {
     constexpr int WAVES = 16, UNROLL = 4 / NT;
     const int rows = GATED ? N / 2 : N;
     const int tile_rows = (GATED || NT == 1) ? skinny_tile_rows(rows) : 16;
     const int per_block = (GATED || NT == 1) ? tile_rows : 16 * NT;
     const int blocks = (rows + per_block - 1) / per_block;
     const int mt = (M + 15) / 16;
-    const NormFold none = {};
     switch (mt) {
         case 1: gemm_skinny_kernel<1, NT, GATED, false, false, TC, WAVES, UNROLL><<<blocks, WAVES * LLE_WAVE, 0, stream>>>(X, W, C, M, N, K, tile_rows, none); break;
         case 2: gemm_skinny_kernel<2, NT, GATED, false, false, TC, WAVES, UNROLL><<<blocks, WAVES * LLE_WAVE, 0, stream>>>(X, W, C, M, N, K, tile_rows, none); break;
@@ -909,6 +926,20 @@ extern "C" int lle_gemm_skinny_gated_bf16(const void* X, const void* W, void* C,
     if (launch_skinny_stream<true, false, bf16_t>((const bf16_t*)X, (const bf16_t*)W, (bf16_t*)C, M, N2, K, NormFold{}, stream))
         LLE_RETURN_LAUNCH_STATUS();
     return launch_skinny<bf16_t, 2, true>((const bf16_t*)X, (const bf16_t*)W, (bf16_t*)C, M, N2, K, stream);
+}
+
+// The same with biases [N2] (or null) and the clamped activation: g = min(gate + b, limit), u = clamp(up + b, -limit, limit),
+// C = g sigmoid(1.702 g) (u + 1).
+extern "C" int lle_gemm_skinny_clamped_bf16(const void* X, const void* W, const void* bias, float limit, void* C, int M, int N2, int K,
+                                            hipStream_t stream) {
+    if (M <= 0 || N2 <= 0) return 0;
+    if (M > 32 || K % 8 != 0 || K <= 0 || N2 % 2 != 0 || !(limit > 0.f)) return (int)hipErrorInvalidValue;
+    NormFold fold = {};
+    fold.act_bias = (const bf16_t*)bias;
+    fold.act_limit = limit;
+    if (launch_skinny_stream<true, false, bf16_t>((const bf16_t*)X, (const bf16_t*)W, (bf16_t*)C, M, N2, K, fold, stream))
+        LLE_RETURN_LAUNCH_STATUS();
+    return launch_skinny<bf16_t, 2, true>((const bf16_t*)X, (const bf16_t*)W, (bf16_t*)C, M, N2, K, stream, fold);
 }
 
 // The product BEFORE a folded norm: delta = X W^T [M, N] is added into `hidden` (float32 [M, N],

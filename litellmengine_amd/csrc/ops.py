@@ -747,6 +747,27 @@ class HipOps:
             return out
         return self.silu_mul(self.linear(x, weight))
 
+    def gate_up_clamped(self, x, weight, bias, limit: float) -> torch.Tensor:
+        """x [M, K], weight [2 I, K] (gate rows, then up rows), bias [2 I] or None -> [M, I]: with g = min(x gate^T + b,
+        limit) and u = clamp(x up^T + b, -limit, limit) the result is g sigmoid(1.702 g) (u + 1).  Few bfloat16 rows run as
+        ONE weight-streaming launch with the activation in its epilogue; otherwise the product and bias_act."""
+        _dev(x, "x")
+        _dev(weight, "weight", x.dtype)
+        M, K = x.shape
+        N2 = weight.shape[0]
+        _need(weight.shape[1] == K and N2 % 2 == 0, f"weight {list(weight.shape)} does not fit x [{M}, {K}]")
+        if bias is not None:
+            _dev(bias, "bias", x.dtype)
+            _need(bias.shape == (N2,), "bias must cover the whole weight")
+        few = M <= self.tuning.skinny_max_rows or (M <= 32 and N2 * K <= self.tuning.skinny_small_weight)
+        if x.dtype == torch.bfloat16 and few and K % 8 == 0 and not self.force_library_gemm:
+            _need(limit > 0.0, "a clamped activation has a positive limit")
+            out = torch.empty((M, N2 // 2), dtype=x.dtype, device=x.device)
+            self._run("gemm", "lle_gemm_skinny_clamped_bf16", [_P, _P, _P, _F, _P, _I, _I, _I, _P],
+                      _ptr(x), _ptr(weight), _ptr(bias), float(limit), _ptr(out), M, N2, K)
+            return out
+        return self.bias_act(self.linear(x, weight), "clamp", True, bias=bias, limit=limit)
+
     # -- arrangements that norm a sublayer's output ------------------------------------
     def cast(self, x, dtype) -> torch.Tensor:
         """x in `dtype` (x itself where it has that type already)."""
@@ -1671,12 +1692,16 @@ class HipOps:
     SSD_CHUNK = 64  # tokens of a chunk (lle_ssd_chunk)
     SSD_WALK = 32  # most tokens of a request that are walked one by one (lle_ssd_walk)
 
-    def ssd_conv(self, u, col0: int, taps, bias, state, token_seq, cu_tokens, seq_slots, single: bool = False) -> torch.Tensor:
+    def ssd_conv(self, u, col0: int, taps, bias, state, token_seq, cu_tokens, seq_slots, single: bool = False, x=None,
+                 dt_w=None):
         """The columns col0 .. col0 + C - 1 of u [N, cols] convolved over time channel by channel with J taps (float32
         [C, J]; the last tap meets the token itself) + bias (float32 [C] or None), then silu -> float32 [N, C].  Tokens
         ahead of the step come from the request's state row (float32 [slots + 1, >= (J - 1) C]: the last J - 1 inputs of
         earlier steps, oldest first; None for J = 1), which moves on by the step's tokens.  `single`: every request of the
-        step has one token (the row then moves on in the same launch)."""
+        step has one token (the row then moves on in the same launch).  With x [N, K] and dt_w [H, K] the result is (that,
+        x dt_w^T float32 [N, H]): in the same launch for single tokens and up to 8 taps, else a product of its own."""
+        if x is not None and not (single and taps.shape[1] <= 8):
+            return self.ssd_conv(u, col0, taps, bias, state, token_seq, cu_tokens, seq_slots, single), self.linear(x, dt_w, torch.float32)
         _dev(u, "u")
         _dev(taps, "taps", torch.float32)
         for t, name in ((token_seq, "token_seq"), (cu_tokens, "cu_tokens"), (seq_slots, "seq_slots")):
@@ -1694,11 +1719,19 @@ class HipOps:
             _rows(state, "state", torch.float32)
             _need(state.shape[1] >= (J - 1) * C, "a state row holds J - 1 inputs")
         out = torch.empty((N, C), dtype=torch.float32, device=u.device)
-        self._run("ssd", "lle_ssd_conv", [_P, _I, _I, _P, _I, _P, _P, _L, _P, _P, _P, _P, _I, _I, _I, _I, _I, _P],
+        dt, K, H = None, 0, 0
+        if x is not None:
+            _dev(x, "x", u.dtype)
+            _dev(dt_w, "dt_w", u.dtype)
+            K, H = x.shape[1], dt_w.shape[0]
+            _need(x.shape[0] == N and dt_w.shape == (H, K), "x must be [N, K], dt_w [H, K]")
+            dt = torch.empty((N, H), dtype=torch.float32, device=u.device)
+        self._run("ssd", "lle_ssd_conv",
+                  [_P, _I, _I, _P, _I, _P, _P, _L, _P, _P, _P, _P, _I, _I, _I, _I, _P, _P, _P, _I, _I, _I, _P],
                   _ptr(u), cols, int(col0), _ptr(taps), J, _ptr(bias), _ptr(state) if J > 1 else None,
                   state.stride(0) if J > 1 else 0, _ptr(token_seq), _ptr(cu_tokens), _ptr(seq_slots), _ptr(out), N, S, C,
-                  1 if single else 0, dtype_code(u.dtype))
-        return out
+                  1 if single else 0, _ptr(x), _ptr(dt_w), _ptr(dt), K, H, dtype_code(u.dtype))
+        return out if x is None else (out, dt)
 
     def ssd_heads_a_group(self, heads: int, groups: int, chunks: int) -> int:
         """Heads of a group that one workgroup of the chunks' second pass takes (they share C . B): as many as leave

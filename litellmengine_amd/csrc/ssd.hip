@@ -45,11 +45,45 @@ struct SsdConvArgs {
     const int32_t *token_seq, *cu_tokens, *seq_slots;
     float* out;  // [N, CC]
     int N, CC, J, run;
+    // steps of single tokens: workgroups behind the convolution's make the step sizes' product, dt = x dt_w^T
+    const void* x;     // [N, K] or null
+    const void* dt_w;  // [H, K]
+    float* dt;         // [N, H]
+    int K, H, conv_blocks;
 };
+
+// dt[n, h] = sum_k x[n, k] dt_w[h, k] in 32-bit: a wavefront has one head and up to SSD_DT_TOKENS tokens
+#define SSD_DT_TOKENS 4
+template <typename T>
+__device__ __forceinline__ void ssd_step_products(const SsdConvArgs& a, int block) {
+    const int wave = block * 4 + threadIdx.x / LLE_WAVE, lane = threadIdx.x % LLE_WAVE;
+    const int h = wave % a.H, n0 = wave / a.H * SSD_DT_TOKENS;
+    if (n0 >= a.N) return;
+    const T* w = (const T*)a.dt_w + (int64_t)h * a.K;
+    const T* x = (const T*)a.x;
+    float acc[SSD_DT_TOKENS];
+#pragma unroll
+    for (int t = 0; t < SSD_DT_TOKENS; ++t) acc[t] = 0.f;
+#pragma unroll 4
+    for (int k = lane; k < a.K; k += LLE_WAVE) {
+        const float wv = to_f32<T>(w[k]);
+#pragma unroll
+        for (int t = 0; t < SSD_DT_TOKENS; ++t) acc[t] = fmaf(to_f32<T>(x[(int64_t)min(n0 + t, a.N - 1) * a.K + k]), wv, acc[t]);
+    }
+#pragma unroll
+    for (int t = 0; t < SSD_DT_TOKENS; ++t) {
+        const float sum = wave_sum(acc[t]);
+        if (lane == 0 && n0 + t < a.N) a.dt[(int64_t)(n0 + t) * a.H + h] = sum;
+    }
+}
 
 template <typename T, int J, bool ADVANCE>
 __global__ __launch_bounds__(256) void ssd_conv_run_kernel(SsdConvArgs a) {
     constexpr int W = J > 1 ? J - 1 : 1;
+    if (ADVANCE && (int)blockIdx.y >= a.conv_blocks) {
+        ssd_step_products<T>(a, (blockIdx.y - a.conv_blocks) * gridDim.x + blockIdx.x);
+        return;
+    }
     const int ch = blockIdx.y * 256 + threadIdx.x;
     if (ch >= a.CC) return;
     const int n0 = blockIdx.x * a.run, n1 = min(a.N, n0 + a.run);
@@ -128,7 +162,12 @@ static bool ssd_conv_runs(SsdConvArgs a, bool advance, hipStream_t stream) {
     const int blocks = (a.CC + 255) / 256;
     int run = (int)((int64_t)a.N * blocks / 2048);  // runs that load taps and windows seldom, and fill the chip
     a.run = run < 1 ? 1 : run > 16 ? 16 : run;
-    const dim3 grid((a.N + a.run - 1) / a.run, blocks);
+    dim3 grid((a.N + a.run - 1) / a.run, blocks);
+    a.conv_blocks = blocks;
+    if (advance && a.x) {
+        const int waves = a.H * ((a.N + SSD_DT_TOKENS - 1) / SSD_DT_TOKENS);
+        grid.y += ((waves + 3) / 4 + grid.x - 1) / grid.x;
+    }
 #define SSD_CONV_CASE(JJ)                                                             \
     case JJ:                                                                          \
         if (advance) ssd_conv_run_kernel<T, JJ, true><<<grid, 256, 0, stream>>>(a);   \
@@ -144,14 +183,17 @@ static bool ssd_conv_runs(SsdConvArgs a, bool advance, hipStream_t stream) {
 
 // u [N, cols] in `dtype`; taps float32 [CC, J], bias float32 [CC] or null; state rows of state_stride floats whose first
 // (J - 1) CC hold the kept rows; out float32 [N, CC].  The state is advanced: by this launch where every request of the
-// step has one token (`single` != 0), else by one behind it.
+// step has one token (`single` != 0), else by one behind it.  With `single` and J <= 8 the launch also makes dt = x dt_w^T
+// (x [N, K] and dt_w [H, K] in `dtype`, dt float32 [N, H]) where x is given.
 extern "C" int lle_ssd_conv(const void* u, int cols, int col0, const void* taps, int J, const void* bias, void* state,
                             int64_t state_stride, const void* token_seq, const void* cu_tokens, const void* seq_slots, void* out,
-                            int N, int S, int CC, int single, int dtype, hipStream_t stream) {
+                            int N, int S, int CC, int single, const void* x, const void* dt_w, void* dt, int K, int H, int dtype,
+                            hipStream_t stream) {
     if (N <= 0 || CC <= 0) return 0;
     if (J < 1 || (J > 1 && !state) || col0 < 0 || col0 + CC > cols || (CC + 255) / 256 > 65535 || S <= 0) return (int)hipErrorInvalidValue;
+    if (x && (!single || J > 8 || !dt_w || !dt || K <= 0 || H <= 0)) return (int)hipErrorInvalidValue;
     const SsdConvArgs a{u, cols, col0, (const float*)taps, (const float*)bias, (float*)state, state_stride, (const int32_t*)token_seq,
-                        (const int32_t*)cu_tokens, (const int32_t*)seq_slots, (float*)out, N, CC, J, 1};
+                        (const int32_t*)cu_tokens, (const int32_t*)seq_slots, (float*)out, N, CC, J, 1, x, dt_w, (float*)dt, K, H, 0};
     const bool advance = single && J <= 8;
     const bool done = dtype == LLE_F32 ? ssd_conv_runs<float>(a, advance, stream) : ssd_conv_runs<bf16_t>(a, advance, stream);
     const int blocks = (CC + 255) / 256;

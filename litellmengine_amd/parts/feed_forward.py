@@ -61,8 +61,10 @@ class GatedMLP(FeedForward):
         ops = self.ctx.ops
         if self.fused:
             return self.down.forward(ops.gate_up_silu(x, self.gate_up.weight), fold=fold)
-        a = ops.bias_act(ops.linear(x, self.gate_up.weight), self.activation, gated=True, bias=self.gate_up.bias,
-                         **({} if self.limit is None else {"limit": self.limit}))
+        if self.limit is not None:
+            a = ops.gate_up_clamped(x, self.gate_up.weight, self.gate_up.bias, self.limit)
+        else:
+            a = ops.bias_act(ops.linear(x, self.gate_up.weight), self.activation, gated=True, bias=self.gate_up.bias)
         y = self.down.forward(a)
         return y if self.late_bias is None else Injected(y, self.late_bias, None, ops)
 

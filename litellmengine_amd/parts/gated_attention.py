@@ -124,10 +124,18 @@ class GatedAttention(Mixer):
         elif self.talking:
             self.talk = torch.eye(self.nq, dtype=torch.float32, device=ctx.device)
 
-    def forward(self, x, step, cache):
+    def input_weight(self):
+        """The rows that a mixer beside this one may stack with its own (see SideBySideMixer); the kernels want them first."""
+        return self.qkvg.weight
+
+    def take_input_weight(self, weight) -> None:
+        self.qkvg.weight = weight
+
+    def forward(self, x, step, cache, projected=None):
+        """`projected` = (u, 0): the input projection's result is the first columns of u."""
         ops = self.ctx.ops
         group = cache.group
-        u = self.qkvg.forward(x)
+        u = self.qkvg.forward(x) if projected is None else projected[0]
         turn = None if self.rotation is None else self.rotation.table(step)
         value_turn = None if self.value_rotation is None else self.value_rotation.table(step)
         q = ops.pair_rope_write(u, self.bias, group.slot_mapping, turn, value_turn, cache.kv, self.nq, self.nkv, self.dim,

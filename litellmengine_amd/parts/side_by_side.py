@@ -10,6 +10,9 @@ by the norm's kernel that adds it into the stream (pre-norm arrangements).  At m
 of the two may keep a per-token cache; the fixed-size states of both lie one behind the other in
 one state row of the request, and each mixer sees its own columns of it.
 
+Where both mixers say which weight their input meets first (`input_weight`), the two are stacked and one product makes
+both inputs; each mixer then gets the result with the column that its own begins at.
+
 In a decode step of many requests (one that is captured into a graph) each mixer is a chain of launches that leave most of the chip
 idle: the right mixer's chain then runs on a stream of its own, forked from and joined to the step's.  Whatever either
 chain allocates is used by nobody else before the join, and the next fork comes after the launches that read their
@@ -62,6 +65,8 @@ class SideBySideMixer(Mixer):
             self._columns.append((at, spec.shape[0]))
             at += spec.shape[0]
         self._state_width = at
+        self.stacked: Optional[torch.Tensor] = None
+        self.right_col = 0
 
     def cache_spec(self) -> Optional[CacheSpec]:
         return self.left.cache_spec() or self.right.cache_spec()
@@ -76,6 +81,12 @@ class SideBySideMixer(Mixer):
         self.ctx = ctx
         self.left.bind(weights, ctx)
         self.right.bind(weights, ctx)
+        if all(hasattr(m, "input_weight") for m in (self.left, self.right)):
+            a, b = self.left.input_weight(), self.right.input_weight()
+            self.stacked = torch.cat([a, b], dim=0).contiguous()
+            self.right_col = a.shape[0]
+            self.left.take_input_weight(self.stacked[: self.right_col])  # (rows of the stack: nothing is held twice)
+            self.right.take_input_weight(self.stacked[self.right_col:])
 
     def _share(self, cache, which: int):
         columns = self._columns[which]
@@ -84,14 +95,19 @@ class SideBySideMixer(Mixer):
 
     def forward(self, x, step, cache):
         """-> (left's result, right's result): a pair that a norm's kernel adds up; with factors a ScaledSum."""
+        shares = [{}, {}]
+        if self.stacked is not None:
+            u = self.ctx.ops.linear(x, self.stacked)
+            shares = [{"projected": (u, 0)}, {"projected": (u, self.right_col)}]
+        run = lambda which, mixer: mixer.forward(x, step, self._share(cache, which), **shares[which])
         if step.seqs is None and x.is_cuda and step.num_seqs >= self.ABREAST_MIN_REQUESTS:  # (no host-side view: a step for a graph)
             here, side = torch.cuda.current_stream(x.device), _side_stream(x.device)
             side.wait_stream(here)
             with torch.cuda.stream(side):
-                right = self.right.forward(x, step, self._share(cache, 1))
-            left = self.left.forward(x, step, self._share(cache, 0))
+                right = run(1, self.right)
+            left = run(0, self.left)
             here.wait_stream(side)
             y = left, right
         else:
-            y = self.left.forward(x, step, self._share(cache, 0)), self.right.forward(x, step, self._share(cache, 1))
+            y = run(0, self.left), run(1, self.right)
         return y if self.scales is None else ScaledSum(*y, *self.scales)

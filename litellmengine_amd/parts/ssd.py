@@ -9,7 +9,7 @@
 
 The state is one float32 row per request slot (`StateSpec`): the heads' matrices (transposed, [head][value][state], the
 way the kernels read them) and, behind them, the last J - 1 rows of the convolution's inputs.  The step sizes' rows of
-W_in are a product of their own whose result stays in 32-bit; what enters the recurrence beyond the projections and
+W_in are a product of their own (in steps of single tokens part of the convolution's launch) whose result stays in 32-bit; what enters the recurrence beyond the projections and
 the convolution is 32-bit in every mode.  Requests with few tokens in a step are walked token by token, longer portions
 are cut into chunks that are worked on side by side, whatever the mix.
 """
@@ -89,14 +89,21 @@ class StateSpaceMixer(Mixer):
         self.dt_bias, self.a_log, self.D, self.norm_w = (flat(n) for n in (self.dt_bias_name, self.a_log_name, self.d_name,
                                                                           self.norm_name))
 
-    def forward(self, x, step, cache):
+    def input_weight(self):
+        """The rows that a mixer beside this one may stack with its own (see SideBySideMixer)."""
+        return self.zxbc
+
+    def take_input_weight(self, weight) -> None:
+        self.zxbc = weight
+
+    def forward(self, x, step, cache, projected=None):
+        """`projected` = (u, col): the input projection's result is the columns from `col` on of u."""
         ops = self.ctx.ops
         state = cache.state
         kept = state[:, self.matrix_floats:] if self.kept_rows else None  # (a view: the kernels take a row stride)
-        u = ops.linear(x, self.zxbc)
-        dt = ops.linear(x, self.dt_w, torch.float32)
-        c = ops.ssd_conv(u, self.inner, self.conv_w, self.conv_b, kept, step.token_seq, step.cu_tokens, step.seq_slots,
-                         single=step.max_q_len == 1)
+        u, col = projected if projected is not None else (ops.linear(x, self.zxbc), 0)
+        c, dt = ops.ssd_conv(u, col + self.inner, self.conv_w, self.conv_b, kept, step.token_seq, step.cu_tokens, step.seq_slots,
+                             single=step.max_q_len == 1, x=x, dt_w=self.dt_w)
         y = ops.ssd_scan(c, dt, self.dt_bias, self.a_log, self.D, state, self.H, self.G, self.vdim, self.N, step.seq_slots,
                          step.cu_tokens, step.min_q_len, step.max_q_len)
-        return self.o.forward(ops.ssd_gate_norm(y, u, 0, self.norm_w, self.eps, self.norm_groups))
+        return self.o.forward(ops.ssd_gate_norm(y, u, col, self.norm_w, self.eps, self.norm_groups))

@@ -85,6 +85,16 @@ def test_clamped_gate(dtype, F):
             close(o.bias_act(z, "clamp", True, bias=bias, limit=limit), REF.bias_act(z, "clamp", True, bias=bias, limit=limit), tol(dtype, 20))
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("M,K,F", [(1, 64, 40), (8, 2048, 8192), (16, 1024, 96), (5, 72, 50), (31, 256, 64), (40, 128, 64), (3, 50, 24), (9, 4096, 12288)])
+def test_clamped_gate_behind_its_product(dtype, M, K, F):
+    """One launch with the activation in its epilogue where there are few rows, the product and the activation elsewhere."""
+    o = ops()
+    x, w, b = rnd((M, K), dtype, 1), rnd((2 * F, K), dtype, 2, K ** -0.5), rnd((2 * F,), dtype, 3)
+    for limit, bias in ((0.6, b), (3.0, None)):
+        close(o.gate_up_clamped(x, w, bias, limit), REF.gate_up_clamped(x, w, bias, limit), tol(dtype, 4))
+
+
 # -- attention with capped scores ---------------------------------------------------------------------
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("nq,nkv,D,P", [(6, 2, 64, 16), (4, 4, 32, 16), (8, 1, 96, 32), (5, 5, 128, 16), (2, 1, 256, 16), (3, 1, 160, 16), (6, 3, 40, 8)])
@@ -257,6 +267,22 @@ def test_ssd_convolution(dtype, C, J, q_lens):
     close(torch.cat(rows), got[:n0], 1e-6)
     if n0 == q_lens[0]:
         close(st[int(seq_slots[0])], b[int(seq_slots[0])], 1e-7)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("N,K,H,C,J", [(1, 50, 3, 40, 4), (8, 2048, 64, 700, 4), (5, 100, 7, 77, 1), (70, 128, 12, 64, 3), (3, 64, 4, 64, 9), (200, 72, 1, 300, 2)])
+def test_step_sizes_made_beside_the_convolution(dtype, N, K, H, C, J):
+    o = ops()
+    u, taps, state = rnd((N, C), dtype, 1), rnd((C, J), torch.float32, 2, 0.5), rnd((N + 1, max(1, J - 1) * C), torch.float32, 3)
+    x, w = rnd((N, K), dtype, 4), rnd((H, K), dtype, 5)
+    where = (ints(list(range(N))), ints(list(range(N + 1))), ints(list(range(N))[::-1]))
+    a, b = state.clone(), state.clone()
+    want = REF.ssd_conv(u, 0, taps, None, a, *where, x=x, dt_w=w)
+    got = o.ssd_conv(u, 0, taps, None, b, *where, single=True, x=x, dt_w=w)
+    close(got[0], want[0], 2e-5)
+    close(got[1], want[1], 1e-4 * max(1.0, K ** 0.5 / 8))
+    close(a, b, 1e-7)
+    assert torch.equal(o.ssd_conv(u, 0, taps, None, state.clone(), *where, single=True), got[0])
 
 
 def ssd_case(H, G, vdim, n, q_lens, seed=1, steep=1.0):

@@ -367,6 +367,9 @@ class TorchOps:
             out = out * torch.sigmoid(t[:, col].to(self.cd))[:, None]
         return out.to(z.dtype)
 
+    def gate_up_clamped(self, x, weight, bias, limit):
+        return self.bias_act(self.linear(x, weight, torch.float32), "clamp", True, bias, limit=limit).to(x.dtype)
+
     def softcap_(self, x, cap):
         x.copy_((cap * torch.tanh(x.to(self.cd) / cap)).to(x.dtype))
         return x
@@ -552,7 +555,10 @@ class TorchOps:
         return (x * gg).reshape(N, heads * vdim).to(out_dtype or gate.dtype)
 
     # -- the state-space recurrence of Mamba-2 --------------------------------------------------
-    def ssd_conv(self, u, col0, taps, bias, state, token_seq, cu_tokens, seq_slots, single=False):
+    def ssd_conv(self, u, col0, taps, bias, state, token_seq, cu_tokens, seq_slots, single=False, x=None, dt_w=None):
+        if x is not None:
+            return (self.ssd_conv(u, col0, taps, bias, state, token_seq, cu_tokens, seq_slots, single),
+                    self.linear(x, dt_w, torch.float32))
         N, (C, J) = u.shape[0], taps.shape
         x = u[:, col0 : col0 + C].to(self.cd)
         y = torch.zeros((N, C), dtype=self.cd, device=u.device)
