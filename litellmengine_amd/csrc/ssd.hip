@@ -511,6 +511,11 @@ __global__ __launch_bounds__(256) void ssd_chunk_out_kernel(SsdArgs a) {
     }
     for (int hh = 0; hh < a.heads_a_group; ++hh) {
         const int h = h0 + hh;
+        // the entry state's first rows are asked for now, the later ones while the rows before them are multiplied
+        const float* S = a.part + (slot * a.H + h) * (int64_t)vdim * n;
+        ssd_f32x4 sv[NQ];
+#pragma unroll
+        for (int q = 0; q < NQ; ++q) sv[q] = ssd_quad<WIDE>(S + (int64_t)min(r, vdim - 1) * n, 16 * q + 4 * c, n);
         float dt, hi, lo;  // of token `lane` of the chunk (every wavefront makes them for itself)
         ssd_chunk_steps(a, h, t0, nt, dt, hi, lo);
         if (hh > 0) __syncthreads();  // (the head before has been read)
@@ -543,25 +548,34 @@ __global__ __launch_bounds__(256) void ssd_chunk_out_kernel(SsdArgs a) {
             }
         }
         const float entry = expf(hi_t), D = a.D[h];
-        const float* S = a.part + (slot * a.H + h) * (int64_t)vdim * n;
         for (int jt = 0; jt * 16 < vdim; ++jt) {
-            ssd_f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-            const float* srow = S + (int64_t)min(jt * 16 + r, vdim - 1) * n;
+            // (two chains of sums: a product waits for the one before it in its own chain only)
+            ssd_f32x4 acc = {0.f, 0.f, 0.f, 0.f}, acc2 = acc;
 #pragma unroll
             for (int q = 0; q < NQ; ++q) {
-                const ssd_f32x4 sv = ssd_quad<WIDE>(srow, 16 * q + 4 * c, n);
 #pragma unroll
-                for (int e = 0; e < 4; ++e) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(sv[e], C[q][e], acc, 0, 0, 0);
+                for (int e = 0; e < 4; e += 2) {
+                    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(sv[q][e], C[q][e], acc, 0, 0, 0);
+                    acc2 = __builtin_amdgcn_mfma_f32_16x16x4f32(sv[q][e + 1], C[q][e + 1], acc2, 0, 0, 0);
+                }
             }
-            acc *= entry;
+            const float* next = S + (int64_t)min((jt + 1) * 16 + r, vdim - 1) * n;
+#pragma unroll
+            for (int q = 0; q < NQ; ++q) sv[q] = ssd_quad<WIDE>(next, 16 * q + 4 * c, n);
+            acc = (acc + acc2) * entry;
+            acc2 = ssd_f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int st = 0; st < 4; ++st) {
                 if (st <= wave) {  // (the same for the whole wavefront)
 #pragma unroll
-                    for (int e = 0; e < 4; ++e)
-                        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(s_x[(st * 16 + 4 * c + e) * XS + jt * 16 + r], m[st][e], acc, 0, 0, 0);
+                    for (int e = 0; e < 4; e += 2) {
+                        const float* x2 = s_x + (st * 16 + 4 * c + e) * XS + jt * 16 + r;
+                        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x2[0], m[st][e], acc, 0, 0, 0);
+                        acc2 = __builtin_amdgcn_mfma_f32_16x16x4f32(x2[XS], m[st][e + 1], acc2, 0, 0, 0);
+                    }
                 }
             }
+            acc += acc2;
             if (tok < nt) {
                 const int j = jt * 16 + 4 * c;
                 const float* x = rows + (int64_t)tok * a.CC + h * vdim;
