@@ -184,6 +184,35 @@ def test_long_decoding_in_a_batch_with_slots_used_again(tmp_path, dtype):
     print(f"long decoding {dtype}: worst relative error {worst:.3g}")
 
 
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_many_requests_decode_side_by_side(tmp_path, dtype):
+    """Twenty-one requests of unequal lengths decode forty tokens each (one graph replayed; batches of sixteen and more run
+    the two mixers' chains on two streams), some of them ending early, so that the batch passes that size on its way
+    down: every row of every step against the plain model."""
+    d = make_model_dir(tmp_path, "B", seed=11, dtype=torch.bfloat16)
+    sharpen(d, SHARP[dtype], memory=1.6, skip=GENTLE[dtype])
+    vocab = CONFIGS["B"]["vocab"]
+    heads = {f"r{i}": 3 + 2 * i for i in range(21)}  # tokens ahead of the decoding
+    tails = {r: 40 if i % 3 else 15 + i for i, r in enumerate(heads)}
+    requests = {r: random_tokens(heads[r] + tails[r], vocab, 90 + i) for i, r in enumerate(heads)}
+    tb = TraceBuilder()
+    tb.step([(r, requests[r][: heads[r]], [heads[r] - 1]) for r in heads])
+    live, at = list(heads), dict(heads)
+    while live:
+        entries, end = [], []
+        for r in list(live):
+            entries.append((r, [requests[r][at[r]]], [0]))
+            at[r] += 1
+            if at[r] == len(requests[r]):
+                end.append(r)
+                live.remove(r)
+        tb.step(entries, end)
+    out = str(tmp_path / "out")
+    run_tool(d, dtype, out, tb, page_size=16, max_requests=21)
+    worst = check_dumps(out, tb, plain_logits(d, requests), 1.5e-4 if dtype == "float32" else 1e-1)
+    print(f"many side by side {dtype}: worst relative error {worst:.3g}")
+
+
 @pytest.mark.parametrize("which", ["A", "B"])
 def test_greedy_generation_through_the_entry_point(tmp_path, which):
     from litellmengine_amd.entrypoints.generate import generate
