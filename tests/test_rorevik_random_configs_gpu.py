@@ -51,7 +51,7 @@ def draw_layer(rng):
 def draw(seed: int):
     rng = random.Random(seed)
     layers = [draw_layer(rng) for _ in range(rng.randint(2, 5))]
-    spec = {"architecture": "Rorevik", "vocab": rng.choice([50, 97, 256, 311, 576]), "max_positions": rng.choice([260, 300, 1000]),
+    spec = {"architecture": "Rorevik", "vocab": rng.choice([50, 97, 256, 311, 533]), "max_positions": rng.choice([260, 300, 1000]),
             "width": rng.choice([64, 72, 96, 128, 136, 200, 256, 52, 90]), "norm": {"eps": rng.choice([1e-6, 1e-5, 3e-6])},
             "embedding": {"scale": rng.choice([1.0, 0.3, 5.0, 16.0])}, "layers": layers}
     if rng.random() < 0.8:
